@@ -33,9 +33,10 @@ import numpy as np
 import torch
 
 from .. import ops
-from ..models.configs import ModelConfig, get_model_config
-from ..models.llama import ForwardBatch, LlamaModel
-from .kvcache import PagedKVCache
+from ..models import build_model
+from ..models.batch import ForwardBatch, Segments
+from ..models.configs import HybridConfig, ModelConfig, get_model_config
+from .kvcache import fit_num_blocks, make_cache
 
 logger = logging.getLogger(__name__)
 
@@ -151,7 +152,7 @@ class EngineRequest:
 class LLMEngine:
     def __init__(
         self,
-        model: str | ModelConfig = "llama-3-8b",
+        model: str | ModelConfig | HybridConfig = "llama-3-8b",
         device: torch.device | str = "cpu",
         dtype: torch.dtype = torch.bfloat16,
         block_size: int = 64,
@@ -191,7 +192,7 @@ class LLMEngine:
 
         if self.device.type == "cuda":
             torch.cuda.set_device(self.device)
-        self.model = LlamaModel(
+        self.model = build_model(
             config, device=self.device, dtype=dtype, seed=seed,
             tp_group=tp_group, tp_rank=tp_rank, tp_size=tp_size,
             full_config=full_config,
@@ -199,13 +200,16 @@ class LLMEngine:
         if kv_dtype == "auto":
             kv_dtype = os.environ.get("LLMAPI_KV_DTYPE", "auto")
         if num_blocks is None:
-            num_blocks = PagedKVCache.fit_num_blocks(
-                config, block_size, self.device, dtype, hbm_fraction,
-                kv_dtype=kv_dtype,
+            num_blocks = fit_num_blocks(
+                config, block_size, self.device, dtype, hbm_fraction, kv_dtype,
+                max_batch_size,
             )
-        self.kv = PagedKVCache(
-            config, num_blocks, block_size, self.device, dtype,
-            prefix_caching=prefix_caching, kv_dtype=kv_dtype,
+        # a prefix's pages stand for the prefix only if they are its whole
+        # state: recurrent layers have no state to resume from mid-sequence
+        prefix_caching = prefix_caching and config.prefix_cacheable
+        self.kv = make_cache(
+            config, num_blocks, block_size, self.device, dtype, prefix_caching,
+            kv_dtype, max_batch_size,
         )
         self.prefix_caching = prefix_caching
         if prefill_budget == 4096:  # default: allow env tuning
@@ -232,12 +236,9 @@ class LLMEngine:
 
             self.graph_runner = DecodeGraphRunner(
                 self.model,
-                self.kv.k_caches,
-                self.kv.v_caches,
+                self.kv,
                 max_batch=max_batch_size,
                 max_blocks=(self.max_model_len + block_size - 1) // block_size,
-                k_scales=self.kv.k_scales if self.kv.fp8 else None,
-                v_scales=self.kv.v_scales if self.kv.fp8 else None,
             )
 
         # deferred sampling (GPU): the sampled-token fetch of decode step s
@@ -391,18 +392,33 @@ class LLMEngine:
             req.state = "running"
             req.prefill_start_time = time.monotonic()
             req.prefill_pos = req.num_cached
-            req.bt_slot = self._slot_pool.pop()
-            self._bt_np[req.bt_slot, : len(req.block_table)] = req.block_table
+            self._claim_slot(req)
             self._slot_ntok[req.bt_slot] = len(req.prompt_ids)
             self._slot_last[req.bt_slot] = req.prompt_ids[-1]
             self._slot_maxt[req.bt_slot] = len(req.prompt_ids) + req.params.max_tokens
-            self._slot_nblk[req.bt_slot] = len(req.block_table)
             self._slot_flags[req.bt_slot] = (
                 (1 if req.params.ignore_eos else 0)
                 | (2 if req.params.stop else 0)
             )
             admitted.append(req)
         return admitted
+
+    def _claim_slot(self, req: EngineRequest) -> None:
+        """Give the request its row: of the block tables, of the per-slot
+        bookkeeping and of the recurrent state."""
+        req.bt_slot = self._slot_pool.pop()
+        self._bt_np[req.bt_slot, : len(req.block_table)] = req.block_table
+        self._slot_nblk[req.bt_slot] = len(req.block_table)
+
+    def _extend_blocks(self, req: EngineRequest, old: int, new: int) -> None:
+        """Grow the request's block table from old to new tokens."""
+        before = len(req.block_table)
+        self.kv.manager.extend(req.block_table, old, new)
+        if len(req.block_table) != before:
+            self._bt_np[req.bt_slot, before : len(req.block_table)] = (
+                req.block_table[before:]
+            )
+            self._slot_nblk[req.bt_slot] = len(req.block_table)
 
     def _free_slot(self, req: EngineRequest) -> None:
         if req.bt_slot is not None:
@@ -482,6 +498,117 @@ class LLMEngine:
         self.stats["steps"] += 1
         return produced
 
+    def _varlen_logits(
+        self, spans: List[tuple], dec: List[tuple], logits_idx: Optional[np.ndarray] = None
+    ) -> torch.Tensor:
+        """One forward over prompt portions and decode rows together.
+
+        spans: (bt_slot, start, tokens), consecutive tokens of a sequence
+        from position start, which attend to its earlier positions through
+        the cache; dec: (bt_slot, position, token), one token each. Logits
+        come back for the rows of logits_idx (flat: spans, then dec), by
+        default the last row of every span and every dec row."""
+        device = self.device
+        bs = self.kv.block_size
+        starts = np.asarray([s for _, s, _ in spans], dtype=np.int64)
+        lens = np.asarray([len(t) for _, _, t in spans], dtype=np.int64)
+        rows = np.asarray([r for r, _, _ in spans], dtype=np.intp)
+        nd = len(dec)
+        d_rows = np.asarray([r for r, _, _ in dec], dtype=np.intp)
+        d_pos = np.asarray([p for _, p, _ in dec], dtype=np.int64)
+
+        Tp = int(lens.sum())
+        all_rows = np.concatenate([rows, d_rows])
+        all_starts = np.concatenate([starts, d_pos])
+        all_lens = np.concatenate([lens, np.ones(nd, dtype=np.int64)])
+        seg_cu = np.zeros(len(all_lens) + 1, dtype=np.int32)
+        np.cumsum(all_lens, out=seg_cu[1:])
+        token_ids = np.concatenate(
+            [np.asarray(t, dtype=np.int64) for _, _, t in spans]
+            + [np.asarray([t for _, _, t in dec], dtype=np.int64)]
+        )
+        row_seg = np.repeat(np.arange(len(all_lens), dtype=np.int32), all_lens)
+        positions = all_starts[row_seg] + np.arange(Tp + nd) - seg_cu[row_seg]
+        slots = (
+            self._bt_np[all_rows[row_seg], positions // bs].astype(np.int64) * bs
+            + positions % bs
+        )
+        if logits_idx is None:
+            logits_idx = seg_cu[1:].astype(np.int64) - 1
+
+        seg_tables = torch.from_numpy(self._bt_np[all_rows]).to(device)
+        cu = torch.from_numpy(seg_cu).to(device)
+        S = len(spans)
+        kw = {}
+        if starts.any():
+            kw.update(
+                block_tables=seg_tables[:S],
+                cached_lens=torch.from_numpy(starts.astype(np.int32)).to(device),
+            )
+        if nd:
+            kw.update(
+                dec_block_tables=seg_tables[S:],
+                dec_context_lens=torch.from_numpy((d_pos + 1).astype(np.int32)).to(device),
+            )
+        tile_seq, tile_off = ops.build_prefill_tiles(lens, device)
+        batch = ForwardBatch(
+            kind="mixed" if nd else "prefill",
+            token_ids=torch.from_numpy(token_ids).to(device),
+            positions=torch.from_numpy(positions).to(device),
+            slot_mapping=torch.from_numpy(slots).to(device),
+            cu_seqlens=cu[: S + 1],
+            max_seqlen=int(lens.max(initial=0)),
+            tile_seq=tile_seq,
+            tile_off=tile_off,
+            n_prefill_tokens=Tp,
+            logits_indices=torch.from_numpy(logits_idx).to(device),
+            segs=Segments(
+                cu=cu,
+                slots=torch.from_numpy(all_rows.astype(np.int32)).to(device),
+                tables=seg_tables,
+                row_seg=torch.from_numpy(row_seg).to(device),
+                block_size=bs, starts=all_starts, lens=all_lens, n_prefill=S,
+            ),
+            **kw,
+        )
+        return self.model.step(batch, self.kv)
+
+    def _decode_logits(self, slot_rows: np.ndarray, pos: np.ndarray, tokens) -> torch.Tensor:
+        """One forward over one token per sequence (rows slot_rows, at
+        positions pos), through the captured graph where there is one.
+        tokens: int64 array, or device tensor (deferred sampling)."""
+        device, bs, n = self.device, self.kv.block_size, len(slot_rows)
+        tables_np = self._bt_np[slot_rows]  # [n, maxb] vectorized gather
+        slots = tables_np[np.arange(n), pos // bs].astype(np.int64) * bs + pos % bs
+        ctx = (pos + 1).astype(np.int32)
+        if self.graph_runner is not None:
+            try:
+                logits = self.graph_runner.run(tokens, pos, slots, tables_np, ctx, slot_rows)
+                self.stats["graph_steps"] += 1
+                return logits
+            except Exception:
+                logger.exception("hipGraph decode failed; falling back to eager")
+                self.graph_runner = None
+        tables = torch.from_numpy(tables_np).to(device)
+        seg_cu = torch.arange(n + 1, dtype=torch.int32, device=device)
+        batch = ForwardBatch(
+            kind="decode",
+            token_ids=tokens
+            if isinstance(tokens, torch.Tensor)
+            else torch.from_numpy(tokens).to(device),
+            positions=torch.from_numpy(pos).to(device),
+            slot_mapping=torch.from_numpy(slots).to(device),
+            block_tables=tables,
+            context_lens=torch.from_numpy(ctx).to(device),
+            logits_indices=None,
+            segs=Segments(
+                cu=seg_cu,
+                slots=torch.from_numpy(slot_rows.astype(np.int32)).to(device),
+                tables=tables, row_seg=seg_cu[:n], block_size=bs,
+            ),
+        )
+        return self.model.step(batch, self.kv)
+
     def _prefill_step(self) -> int:
         """One forward over up to prefill_budget prompt tokens of the
         prefilling set PLUS one decode row for every running sequence (a
@@ -491,9 +618,6 @@ class LLMEngine:
         chunk reaches the end of its prompt samples its first token and
         joins the running set. Deferred-sampling state is always flushed
         before this step, so decode inputs are host-visible."""
-        device = self.device
-        bs = self.kv.block_size
-
         with self._lock:
             budget = self.prefill_budget
             work: List[tuple] = []  # (req, start, end, final)
@@ -521,13 +645,7 @@ class LLMEngine:
                 while i < len(self.running):
                     req = self.running[i]
                     try:
-                        before = len(req.block_table)
-                        self.kv.manager.extend(req.block_table, req.num_tokens, req.num_tokens + 1)
-                        if len(req.block_table) != before:
-                            self._bt_np[req.bt_slot, before : len(req.block_table)] = (
-                                req.block_table[before:]
-                            )
-                            self._slot_nblk[req.bt_slot] = len(req.block_table)
+                        self._extend_blocks(req, req.num_tokens, req.num_tokens + 1)
                         i += 1
                     except RuntimeError:
                         if not self._preempt_youngest():
@@ -537,76 +655,18 @@ class LLMEngine:
             return 0
 
         reqs = [w[0] for w in work]
-        starts = [w[1] for w in work]
-        lens = [w[2] - w[1] for w in work]
-        cu = np.zeros(len(reqs) + 1, dtype=np.int32)
-        np.cumsum(lens, out=cu[1:])
-        token_ids = np.concatenate(
-            [np.asarray(r.prompt_ids[s : s + L], dtype=np.int64)
-             for r, s, L in zip(reqs, starts, lens)]
-        )
-        positions = np.concatenate(
-            [np.arange(s, s + L, dtype=np.int64) for s, L in zip(starts, lens)]
-        )
-        slots = np.empty(int(cu[-1]), dtype=np.int64)
-        for i, (req, s, L) in enumerate(zip(reqs, starts, lens)):
-            p = np.arange(s, s + L, dtype=np.int64)
-            bt = np.asarray(req.block_table, dtype=np.int64)
-            slots[cu[i] : cu[i + 1]] = bt[p // bs] * bs + p % bs
-        logits_idx = (cu[1:] - 1).astype(np.int64)
-
-        cached_lens_t = None
-        block_tables_t = None
-        if any(starts):
-            rows = np.fromiter((req.bt_slot for req in reqs), dtype=np.intp, count=len(reqs))
-            block_tables_t = torch.from_numpy(self._bt_np[rows]).to(device)
-            cached_lens_t = torch.from_numpy(
-                np.asarray(starts, dtype=np.int32)
-            ).to(device)
-
-        # decode rows appended after the prefill rows (mixed step)
-        Tp = int(cu[-1])
         nd = len(dec_reqs)
-        dec_bt_t = dec_ctx_t = None
-        if nd:
-            d_tokens = np.fromiter(
-                ((r.out_ids[-1] if r.out_ids else r.prompt_ids[-1]) for r in dec_reqs),
-                dtype=np.int64, count=nd,
-            )
-            d_pos = np.fromiter((r.num_tokens - 1 for r in dec_reqs), dtype=np.int64, count=nd)
-            d_rows = np.fromiter((r.bt_slot for r in dec_reqs), dtype=np.intp, count=nd)
-            d_tables = self._bt_np[d_rows]
-            d_slots = d_tables[np.arange(nd), d_pos // bs].astype(np.int64) * bs + d_pos % bs
-            token_ids = np.concatenate([token_ids, d_tokens])
-            positions = np.concatenate([positions, d_pos])
-            slots = np.concatenate([slots, d_slots])
-            logits_idx = np.concatenate([logits_idx, Tp + np.arange(nd, dtype=np.int64)])
-            dec_bt_t = torch.from_numpy(d_tables).to(device)
-            dec_ctx_t = torch.from_numpy((d_pos + 1).astype(np.int32)).to(device)
-
-        tile_seq, tile_off = ops.build_prefill_tiles(lens, device)
-        batch = ForwardBatch(
-            kind="mixed" if nd else "prefill",
-            token_ids=torch.from_numpy(token_ids).to(device),
-            positions=torch.from_numpy(positions).to(device),
-            slot_mapping=torch.from_numpy(slots).to(device),
-            cu_seqlens=torch.from_numpy(cu).to(device),
-            max_seqlen=max(lens),
-            tile_seq=tile_seq,
-            tile_off=tile_off,
-            block_tables=block_tables_t,
-            cached_lens=cached_lens_t,
-            n_prefill_tokens=Tp,
-            dec_block_tables=dec_bt_t,
-            dec_context_lens=dec_ctx_t,
-            logits_indices=torch.from_numpy(logits_idx).to(device),
-        )
+        Tp = sum(w[2] - w[1] for w in work)
+        spans = [
+            (req.bt_slot, start, req.prompt_ids[start:end])
+            for req, start, end, _ in work
+        ]
+        dec = [
+            (r.bt_slot, r.num_tokens - 1, r.out_ids[-1] if r.out_ids else r.prompt_ids[-1])
+            for r in dec_reqs
+        ]
         self.stats["mixed_steps" if nd else "prefill_steps"] += 1
-        logits = self.model.forward(
-            batch, self.kv.k_caches, self.kv.v_caches,
-            k_scales=self.kv.k_scales if self.kv.fp8 else None,
-            v_scales=self.kv.v_scales if self.kv.fp8 else None,
-        )
+        logits = self._varlen_logits(spans, dec)
         sample_reqs = reqs + dec_reqs
         deliver_mask = [w[3] for w in work] + [True] * nd
         tokens = self._sample(logits, sample_reqs, deliver_mask)
@@ -645,7 +705,6 @@ class LLMEngine:
         return len(finals) + nd
 
     def _decode_step(self) -> int:
-        device = self.device
         bs = self.kv.block_size
         with self._lock:
             reqs_now = list(self.running)
@@ -694,13 +753,7 @@ class LLMEngine:
                     continue
                 nt = int(self._slot_ntok[req.bt_slot]) + inflight
                 try:
-                    before = len(req.block_table)
-                    self.kv.manager.extend(req.block_table, nt, nt + 1)
-                    if len(req.block_table) != before:
-                        self._bt_np[req.bt_slot, before : len(req.block_table)] = (
-                            req.block_table[before:]
-                        )
-                        self._slot_nblk[req.bt_slot] = len(req.block_table)
+                    self._extend_blocks(req, nt, nt + 1)
                 except RuntimeError:
                     if inflight:
                         i = 0  # flush below, then retry the whole step
@@ -712,13 +765,7 @@ class LLMEngine:
                         r2 = self.running[j]
                         nt2 = r2.num_tokens + inflight
                         try:
-                            b2 = len(r2.block_table)
-                            self.kv.manager.extend(r2.block_table, nt2, nt2 + 1)
-                            if len(r2.block_table) != b2:
-                                self._bt_np[r2.bt_slot, b2 : len(r2.block_table)] = (
-                                    r2.block_table[b2:]
-                                )
-                                self._slot_nblk[r2.bt_slot] = len(r2.block_table)
+                            self._extend_blocks(r2, nt2, nt2 + 1)
                             j += 1
                         except RuntimeError:
                             if not self._preempt_youngest():
@@ -734,44 +781,13 @@ class LLMEngine:
         n = len(reqs)
         slot_rows = np.fromiter((req.bt_slot for req in reqs), dtype=np.intp, count=n)
         pos = self._slot_ntok[slot_rows] + (inflight - 1)
-        tables_np = self._bt_np[slot_rows]  # [n, maxb] vectorized gather
-        blk = pos // bs
-        slots = tables_np[np.arange(n), blk].astype(np.int64) * bs + pos % bs
-        ctx = (pos + 1).astype(np.int32)
         if inflight:
             last_tokens = self._pend_tokens_dev  # device int64 [n], aligned
         else:
             last_tokens = self._slot_last[slot_rows].copy()
 
         self.stats["decode_steps"] += 1
-        logits = None
-        if self.graph_runner is not None:
-            try:
-                logits = self.graph_runner.run(last_tokens, pos, slots, tables_np, ctx)
-                self.stats["graph_steps"] += 1
-            except Exception:
-                logger.exception("hipGraph decode failed; falling back to eager")
-                self.graph_runner = None
-        if logits is None:
-            tok_t = (
-                last_tokens
-                if isinstance(last_tokens, torch.Tensor)
-                else torch.from_numpy(last_tokens).to(device)
-            )
-            batch = ForwardBatch(
-                kind="decode",
-                token_ids=tok_t,
-                positions=torch.from_numpy(pos).to(device),
-                slot_mapping=torch.from_numpy(slots).to(device),
-                block_tables=torch.from_numpy(tables_np).to(device),
-                context_lens=torch.from_numpy(ctx).to(device),
-                logits_indices=None,
-            )
-            logits = self.model.forward(
-                batch, self.kv.k_caches, self.kv.v_caches,
-                k_scales=self.kv.k_scales if self.kv.fp8 else None,
-                v_scales=self.kv.v_scales if self.kv.fp8 else None,
-            )
+        logits = self._decode_logits(slot_rows, pos, last_tokens)
 
         tokens_dev = self._sample_dev(
             logits, reqs, noise_pos=[len(r.out_ids) + inflight for r in reqs]

@@ -7,7 +7,7 @@ itself. Capturing the whole decode forward per batch-size bucket replays it
 as ONE hipGraph launch.
 
 Mechanics: persistent device buffers (token ids, positions, slot mapping,
-block tables, context lens) sized at max batch; per-bucket graphs captured
+block tables, context lens, state slots) sized at max batch; per-bucket graphs captured
 lazily on first use (standard side-stream warmup then capture); each step
 fills pinned staging, async-copies into the static buffers and replays.
 Padding rows use slot=-1 (kv write kernel skips) and context_len=1.
@@ -20,19 +20,15 @@ from typing import Dict, List, Optional
 
 import torch
 
-from ..models.llama import ForwardBatch
+from ..models.batch import ForwardBatch, Segments
 
 logger = logging.getLogger(__name__)
 
 
 class DecodeGraphRunner:
-    def __init__(self, model, k_caches, v_caches, max_batch: int, max_blocks: int,
-                 k_scales=None, v_scales=None):
+    def __init__(self, model, cache, max_batch: int, max_blocks: int):
         self.model = model
-        self.k_caches = k_caches
-        self.v_caches = v_caches
-        self.k_scales = k_scales
-        self.v_scales = v_scales
+        self.cache = cache
         self.device = model.device
         self.max_batch = max_batch
         self.max_blocks = max_blocks
@@ -47,6 +43,8 @@ class DecodeGraphRunner:
         self.slot_mapping = torch.full((B,), -1, dtype=torch.long, device=dev)
         self.block_tables = torch.zeros(B, NB, dtype=torch.int32, device=dev)
         self.context_lens = torch.ones(B, dtype=torch.int32, device=dev)
+        self.state_slots = torch.full((B,), -1, dtype=torch.int32, device=dev)
+        self.seg_cu = torch.arange(B + 1, dtype=torch.int32, device=dev)
 
         pin = dev.type == "cuda"
         self.h_token_ids = torch.zeros(B, dtype=torch.long, pin_memory=pin)
@@ -54,10 +52,12 @@ class DecodeGraphRunner:
         self.h_slot_mapping = torch.full((B,), -1, dtype=torch.long, pin_memory=pin)
         self.h_block_tables = torch.zeros(B, NB, dtype=torch.int32, pin_memory=pin)
         self.h_context_lens = torch.ones(B, dtype=torch.int32, pin_memory=pin)
+        self.h_state_slots = torch.full((B,), -1, dtype=torch.int32, pin_memory=pin)
 
         self.graphs: Dict[int, torch.cuda.CUDAGraph] = {}
         self.graph_logits: Dict[int, torch.Tensor] = {}
         self.pool = None
+        self._staged: Optional[torch.cuda.Event] = None
 
     def _batch_view(self, b: int) -> ForwardBatch:
         return ForwardBatch(
@@ -68,25 +68,34 @@ class DecodeGraphRunner:
             block_tables=self.block_tables[:b],
             context_lens=self.context_lens[:b],
             logits_indices=None,
+            segs=Segments(
+                cu=self.seg_cu[: b + 1], slots=self.state_slots[:b],
+                tables=self.block_tables[:b], row_seg=self.seg_cu[:b],
+                block_size=self.cache.block_size,
+            ),
         )
 
     def _capture(self, bucket: int) -> None:
         logger.info("capturing decode hipGraph for batch bucket %d", bucket)
         batch = self._batch_view(bucket)
+        # the warmup steps run for real: as padding rows they write no KV
+        # and advance no recurrent state
+        self.slot_mapping.fill_(-1)
+        self.state_slots.fill_(-1)
+        self.positions.zero_()
+        self.context_lens.fill_(1)
         # warmup on a side stream (cuBLAS/hipBLASLt workspace allocs etc.)
         s = torch.cuda.Stream(device=self.device)
         s.wait_stream(torch.cuda.current_stream(self.device))
         with torch.cuda.stream(s):
             for _ in range(2):
-                self.model.forward(batch, self.k_caches, self.v_caches,
-                                   k_scales=self.k_scales, v_scales=self.v_scales)
+                self.model.step(batch, self.cache)
         torch.cuda.current_stream(self.device).wait_stream(s)
         torch.cuda.synchronize(self.device)
 
         graph = torch.cuda.CUDAGraph()
         with torch.cuda.graph(graph, pool=self.pool):
-            logits = self.model.forward(batch, self.k_caches, self.v_caches,
-                                        k_scales=self.k_scales, v_scales=self.v_scales)
+            logits = self.model.step(batch, self.cache)
         if self.pool is None:
             self.pool = graph.pool()  # share the memory pool across buckets
         self.graphs[bucket] = graph
@@ -115,22 +124,32 @@ class DecodeGraphRunner:
         slots,           # np.int64 [n]
         block_tables,    # np.int32 [n, <=max_blocks]
         context_lens,    # np.int32 [n]
+        state_slots,     # np.int32 [n]
     ) -> torch.Tensor:
         n = len(tokens)
         bucket = self.bucket_for(n)
+        if bucket not in self.graphs:
+            self._capture(bucket)
+        if self._staged is not None:
+            self._staged.synchronize()  # the last step's copies have left staging
 
         # fill pinned staging via numpy views (no per-request tensors)
         if isinstance(tokens, torch.Tensor):
             self.token_ids[:n].copy_(tokens[:n])  # device-to-device
         else:
             self.h_token_ids.numpy()[:n] = tokens
-        self.h_positions.numpy()[:n] = positions
+        hp = self.h_positions.numpy()
+        hp[:n] = positions
+        hp[n:bucket] = 0
         sm = self.h_slot_mapping.numpy()
         sm[:n] = slots
         sm[n:bucket] = -1
         cl = self.h_context_lens.numpy()
         cl[:n] = context_lens
         cl[n:bucket] = 1  # padding rows read 1 stale key; output discarded
+        ss = self.h_state_slots.numpy()
+        ss[:n] = state_slots
+        ss[n:bucket] = -1  # padding rows touch no state
         self.h_block_tables.numpy()[:n, : block_tables.shape[1]] = block_tables
 
         if not isinstance(tokens, torch.Tensor):
@@ -138,9 +157,10 @@ class DecodeGraphRunner:
         self.positions[:bucket].copy_(self.h_positions[:bucket], non_blocking=True)
         self.slot_mapping[:bucket].copy_(self.h_slot_mapping[:bucket], non_blocking=True)
         self.context_lens[:bucket].copy_(self.h_context_lens[:bucket], non_blocking=True)
+        self.state_slots[:bucket].copy_(self.h_state_slots[:bucket], non_blocking=True)
         self.block_tables[:bucket].copy_(self.h_block_tables[:bucket], non_blocking=True)
 
-        if bucket not in self.graphs:
-            self._capture(bucket)
+        self._staged = torch.cuda.Event()
+        self._staged.record()
         self.graphs[bucket].replay()
         return self.graph_logits[bucket][:n]

@@ -1,4 +1,4 @@
-"""Paged KV cache: HBM-resident cache tensors + block allocator.
+"""Caches: HBM-resident paged KV, recurrent state slots, block allocator.
 
 Replaces the reference's httpx connection bookkeeping as the per-request
 resource being managed. Layout per layer:
@@ -12,16 +12,25 @@ is built — the native runtime path) and a pure-Python fallback. Sizing: on
 GPU the default number of blocks is computed from *free HBM after model
 weights* × settings.engine_hbm_fraction (288 GB per MI355X makes this the
 dominant tensor).
+
+Hybrid decoders (models/hybrid.py) keep a HybridCache: pages of latent rows
+for their attention layers, allocated by the same BlockManager, and for
+their recurrent layers one state slot per live sequence. The slot is the
+engine's row of the sequence (EngineRequest.bt_slot), so it is claimed and
+given back with the pages; a sequence's first token starts from empty
+state, so a slot needs no clearing between two owners.
 """
 
 from __future__ import annotations
 
 import logging
+import math
 from typing import List, Optional
 
 import torch
 
-from ..models.configs import ModelConfig
+from ..models.configs import HybridConfig, ModelConfig
+from ..models.mixers import MIXERS
 
 logger = logging.getLogger(__name__)
 
@@ -48,10 +57,10 @@ class _PyBlockAllocator:
 
 def make_block_allocator(num_blocks: int):
     try:
-        from ..ops import _C  # type: ignore
+        from ..ops.native import shared_native
 
-        return _C.BlockAllocator(num_blocks)
-    except Exception:
+        return shared_native().BlockAllocator(num_blocks)
+    except RuntimeError:
         return _PyBlockAllocator(num_blocks)
 
 
@@ -271,3 +280,118 @@ class PagedKVCache:
             n * per_block / (1 << 30),
         )
         return int(n)
+
+
+class HybridCache:
+    """Per layer run (a looped layer counts once per pass): ``runs[r]`` maps
+    a name to pages ``[num_blocks, block_size, row]`` in the compute dtype,
+    or to state ``[num_slots, ...]``, fp32 where the recurrence lives."""
+
+    fp8 = False
+
+    def __init__(
+        self,
+        config: HybridConfig,
+        num_blocks: int,
+        block_size: int,
+        device: torch.device | str,
+        dtype: torch.dtype = torch.bfloat16,
+        prefix_caching: bool = False,
+        kv_dtype: str = "auto",
+        num_slots: int = 64,
+    ):
+        if kv_dtype != "auto":
+            raise ValueError(f"{config.name}: kv_dtype '{kv_dtype}' is not supported")
+        self.config = config
+        self.block_size = block_size
+        self.num_blocks = num_blocks
+        self.num_slots = num_slots
+        self.runs: List[dict] = []
+        for spec in _run_specs(config):
+            views = {
+                name: torch.zeros(num_blocks, block_size, row, dtype=dtype, device=device)
+                for name, row in spec.pages.items()
+            }
+            for name, (shape, wide) in spec.state.items():
+                views[name] = torch.zeros(
+                    (num_slots, *shape), dtype=torch.float32 if wide else dtype,
+                    device=device,
+                )
+            self.runs.append(views)
+        self.manager = BlockManager(num_blocks, block_size, prefix_caching=prefix_caching)
+
+    @staticmethod
+    def block_bytes(
+        config: HybridConfig, block_size: int, dtype: torch.dtype, kv_dtype: str = "auto"
+    ) -> int:
+        elem = torch.empty(0, dtype=dtype).element_size()
+        return block_size * elem * sum(
+            row for spec in _run_specs(config) for row in spec.pages.values()
+        )
+
+    @staticmethod
+    def slot_bytes(config: HybridConfig, dtype: torch.dtype) -> int:
+        elem = torch.empty(0, dtype=dtype).element_size()
+        return sum(
+            math.prod(shape) * (4 if wide else elem)
+            for spec in _run_specs(config) for shape, wide in spec.state.values()
+        )
+
+    @classmethod
+    def fit_num_blocks(
+        cls,
+        config: HybridConfig,
+        block_size: int,
+        device: torch.device,
+        dtype: torch.dtype,
+        hbm_fraction: float = 0.90,
+        max_blocks: Optional[int] = None,
+        kv_dtype: str = "auto",
+        num_slots: int = 64,
+    ) -> int:
+        """Blocks that fit next to the state slots; never more than the
+        slots' sequences can fill."""
+        if device.type == "cuda":
+            free, _total = torch.cuda.mem_get_info(device)
+            budget = int(free * hbm_fraction) - num_slots * cls.slot_bytes(config, dtype)
+        else:
+            budget = 256 * 1024 * 1024
+        most = num_slots * -(-config.max_positions // block_size)
+        n = min(most, max(budget, 0) // max(cls.block_bytes(config, block_size, dtype), 1))
+        if max_blocks is not None:
+            n = min(n, max_blocks)
+        return int(max(n, 16))
+
+
+def _run_specs(config: HybridConfig):
+    return [
+        MIXERS[config.layers[i].type].cache_spec(config.layers[i].mixer)
+        for i, _ in config.runs()
+    ]
+
+
+def fit_num_blocks(config, block_size, device, dtype, hbm_fraction, kv_dtype, num_slots):
+    """How many pages of this model's cache the device holds."""
+    if isinstance(config, HybridConfig):
+        return HybridCache.fit_num_blocks(
+            config, block_size, device, dtype, hbm_fraction, kv_dtype=kv_dtype,
+            num_slots=num_slots,
+        )
+    return PagedKVCache.fit_num_blocks(
+        config, block_size, device, dtype, hbm_fraction, kv_dtype=kv_dtype
+    )
+
+
+def make_cache(
+    config, num_blocks, block_size, device, dtype, prefix_caching, kv_dtype, num_slots
+):
+    """The cache a configuration's model steps over."""
+    if isinstance(config, HybridConfig):
+        return HybridCache(
+            config, num_blocks, block_size, device, dtype,
+            prefix_caching=prefix_caching, kv_dtype=kv_dtype, num_slots=num_slots,
+        )
+    return PagedKVCache(
+        config, num_blocks, block_size, device, dtype,
+        prefix_caching=prefix_caching, kv_dtype=kv_dtype,
+    )

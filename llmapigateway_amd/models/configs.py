@@ -1,12 +1,17 @@
-"""Model architecture presets (random-init; no network for checkpoints).
+"""Model configurations: architecture presets and checkpoint folders.
 
 Shapes match the public architectures named by BASELINE.json's configs
 (Llama-3-8B / Llama-3-70B / Mistral-7B), plus tiny presets for CPU tests.
+A model can also be a checkpoint folder: its config.json names the
+architecture that reads it.
 """
 
 from __future__ import annotations
 
+import json
+import os
 from dataclasses import dataclass, replace
+from typing import Any, Dict, List, Optional, Tuple
 
 
 @dataclass(frozen=True)
@@ -23,6 +28,11 @@ class ModelConfig:
     rms_eps: float = 1e-5
     max_positions: int = 8192
     tie_embeddings: bool = False
+
+    @property
+    def prefix_cacheable(self) -> bool:
+        """Whether a sequence's cache pages alone are its whole state."""
+        return True
 
     @property
     def q_size(self) -> int:
@@ -42,6 +52,137 @@ class ModelConfig:
             num_kv_heads=self.num_kv_heads // tp,
             intermediate_size=self.intermediate_size // tp,
         )
+
+
+@dataclass(frozen=True)
+class HybridLayer:
+    """One layer of a hybrid decoder: a mixer (its kind and sizes) and an
+    optional feed-forward."""
+
+    type: str
+    mixer: Dict[str, Any]
+    mlp: Optional[Dict[str, Any]] = None
+
+
+@dataclass(frozen=True)
+class HybridConfig:
+    """A decoder whose layers each name their mixer (latent attention,
+    Mamba-2, mLSTM), with an optional loop: layers [start, stop) run
+    ``times`` times with the same weights, each pass with its own cache.
+
+    The field set is what the Lelisun config.json gives; ``max_positions``
+    is the framework's own bound (nothing in the design limits it) and
+    ``weights_dir`` says where the checkpoint lies (None: random init)."""
+
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: Tuple[HybridLayer, ...]
+    norm_eps: float = 1e-5
+    embed_scale: float = 1.0
+    loop: Optional[Tuple[int, int, int]] = None  # (start, stop, times)
+    max_positions: int = 32768
+    weights_dir: Optional[str] = None
+
+    def __post_init__(self):
+        if self.loop is not None:
+            start, stop, times = self.loop
+            if not (0 <= start < stop <= len(self.layers) and times >= 1):
+                raise ValueError(f"bad loop {self.loop} over {len(self.layers)} layers")
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if layer.type == "latent_attention":
+                if m["rot"]["dims"] != m["rot_dim"] or m["rot_dim"] % 2:
+                    raise ValueError(f"layer {i}: rot.dims must be rot_dim, an even number")
+            elif layer.type == "mamba2":
+                if m["heads"] % m["groups"] or (m["heads"] * m["vdim"]) % m["norm_groups"]:
+                    raise ValueError(f"layer {i}: groups do not divide the heads")
+            elif layer.type != "mlstm":
+                raise ValueError(f"layer {i}: unknown mixer '{layer.type}'")
+            if layer.mlp is not None and layer.mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward '{layer.mlp['kind']}'")
+
+    @classmethod
+    def from_json(cls, raw: Dict[str, Any], name: str, weights_dir: Optional[str] = None):
+        loop = raw.get("loop")
+        return cls(
+            name=name,
+            vocab_size=raw["vocab"],
+            hidden_size=raw["width"],
+            layers=tuple(
+                HybridLayer(type=e["type"], mixer=e["mixer"], mlp=e.get("mlp"))
+                for e in raw["layers"]
+            ),
+            norm_eps=raw["norm"]["eps"],
+            embed_scale=raw["embedding"]["scale"],
+            loop=(loop["start"], loop["stop"], loop["times"]) if loop else None,
+            weights_dir=weights_dir,
+        )
+
+    def runs(self) -> List[Tuple[int, Optional[int]]]:
+        """The layers in the order they run, as (layer index, t): t is the
+        number of the loop pass that this layer begins, None elsewhere."""
+        if self.loop is None:
+            return [(i, None) for i in range(len(self.layers))]
+        start, stop, times = self.loop
+        out: List[Tuple[int, Optional[int]]] = [(i, None) for i in range(start)]
+        for t in range(times):
+            out += [(i, t if i == start else None) for i in range(start, stop)]
+        return out + [(i, None) for i in range(stop, len(self.layers))]
+
+    @property
+    def prefix_cacheable(self) -> bool:
+        return all(layer.type == "latent_attention" for layer in self.layers)
+
+    def scaled_for_tp(self, tp: int) -> "HybridConfig":
+        raise NotImplementedError(f"{self.name}: hybrid decoders run on one GPU (tp=1)")
+
+
+# config.json "architecture" -> reader(raw, name, weights_dir)
+ARCHITECTURES = {"Lelisun": HybridConfig.from_json}
+
+
+def load_model_dir(path: str):
+    """The configuration of a checkpoint folder (config.json +
+    model.safetensors)."""
+    with open(os.path.join(path, "config.json")) as f:
+        raw = json.load(f)
+    arch = raw.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise KeyError(f"Unknown architecture '{arch}' in {path}. Known: {sorted(ARCHITECTURES)}")
+    path = os.path.abspath(path)
+    return ARCHITECTURES[arch](raw, os.path.basename(path), path)
+
+
+def _lelisun_preset(
+    name: str, width: int, vocab: int, ff: int, heads: int, dim: int, rot_dim: int,
+    kv_rank: int, q_rank: int, ssm_heads: int, ssm_vdim: int, state: int, groups: int,
+    mem_heads: int, mem_dim: int, mem_vdim: int, times: int, repeat: int = 1,
+    max_positions: int = 32768,
+) -> HybridConfig:
+    """A Lelisun of [latent attention, Mamba-2] looped, then mLSTM and
+    latent attention; ``repeat`` widens the looped stretch."""
+    attn = HybridLayer(
+        "latent_attention",
+        dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=dim, kv_rank=kv_rank,
+             q_rank=q_rank, scale=(dim + rot_dim) ** -0.5,
+             rot=dict(base=500000.0, dims=rot_dim)),
+        dict(kind="dense", ff=ff),
+    )
+    ssm = HybridLayer(
+        "mamba2",
+        dict(heads=ssm_heads, vdim=ssm_vdim, state=state, groups=groups, conv=4,
+             norm_groups=groups),
+    )
+    mem = HybridLayer(
+        "mlstm", dict(heads=mem_heads, dim=mem_dim, vdim=mem_vdim, gate_cap=15.0)
+    )
+    looped = (attn, ssm) * repeat
+    return HybridConfig(
+        name=name, vocab_size=vocab, hidden_size=width, layers=looped + (mem, attn),
+        embed_scale=width ** 0.5, loop=(0, len(looped), times),
+        max_positions=max_positions,
+    )
 
 
 MODEL_PRESETS = {
@@ -124,6 +265,23 @@ MODEL_PRESETS = {
         rope_theta=10000.0,
         max_positions=512,
     ),
+    # looped hybrid decoder (latent attention + Mamba-2 + mLSTM)
+    "tiny-lelisun": _lelisun_preset(
+        "tiny-lelisun", width=96, vocab=320, ff=112, heads=3, dim=24, rot_dim=8,
+        kv_rank=40, q_rank=56, ssm_heads=6, ssm_vdim=20, state=24, groups=3,
+        mem_heads=2, mem_dim=16, mem_vdim=40, times=2, max_positions=1024,
+    ),
+    # layers of the size of llama-1b's and llama-3-8b's
+    "lelisun-1b": _lelisun_preset(
+        "lelisun-1b", width=2048, vocab=128256, ff=8192, heads=16, dim=128, rot_dim=64,
+        kv_rank=512, q_rank=768, ssm_heads=64, ssm_vdim=64, state=128, groups=8,
+        mem_heads=4, mem_dim=256, mem_vdim=512, times=2, repeat=3,
+    ),
+    "lelisun-8b": _lelisun_preset(
+        "lelisun-8b", width=4096, vocab=128256, ff=14336, heads=32, dim=128, rot_dim=64,
+        kv_rank=512, q_rank=1536, ssm_heads=128, ssm_vdim=64, state=128, groups=8,
+        mem_heads=8, mem_dim=256, mem_vdim=512, times=2, repeat=6,
+    ),
     # small-but-real shape for 1-GPU kernel shakedown
     "llama-1b": ModelConfig(
         name="llama-1b",
@@ -139,7 +297,11 @@ MODEL_PRESETS = {
 }
 
 
-def get_model_config(name: str) -> ModelConfig:
+def get_model_config(name: str):
+    """The configuration of a preset, or of a checkpoint folder when
+    ``name`` is the path of one."""
+    if os.path.isfile(os.path.join(name, "config.json")):
+        return load_model_dir(name)
     key = name.lower()
     if key not in MODEL_PRESETS:
         raise KeyError(f"Unknown model preset '{name}'. Known: {sorted(MODEL_PRESETS)}")

@@ -23,7 +23,6 @@ row-sharded with an RCCL all-reduce over xGMI after each (2 per layer).
 from __future__ import annotations
 
 import math
-from dataclasses import dataclass
 from typing import Dict, List, Optional
 
 import torch
@@ -31,35 +30,9 @@ import torch.distributed as dist
 import torch.nn.functional as F
 
 from .. import ops
+from .batch import ForwardBatch
 from .configs import ModelConfig
-
-
-@dataclass
-class ForwardBatch:
-    kind: str  # "prefill" | "decode" | "mixed"
-    token_ids: torch.Tensor          # [T] int64
-    positions: torch.Tensor          # [T] int64
-    slot_mapping: torch.Tensor       # [T] int64 (global KV slots; -1 = don't write)
-    # prefill:
-    cu_seqlens: Optional[torch.Tensor] = None   # [B+1] int32
-    max_seqlen: int = 0
-    tile_seq: Optional[torch.Tensor] = None     # [ntiles] int32 (GPU kernel tile map)
-    tile_off: Optional[torch.Tensor] = None
-    # decode:
-    block_tables: Optional[torch.Tensor] = None  # [B, max_blocks] int32
-    context_lens: Optional[torch.Tensor] = None  # [B] int32
-    # prefill with cached prefix (prefix caching): per-seq number of
-    # positions already in the paged cache (block_tables set too)
-    cached_lens: Optional[torch.Tensor] = None   # [B] int32
-    # rows of the flat batch at which logits are needed (last token per seq)
-    logits_indices: Optional[torch.Tensor] = None  # [B] int64
-    # mixed steps: rows [0, n_prefill_tokens) are prefill (cu_seqlens etc.
-    # apply to them), rows [n_prefill_tokens, T) are decode rows with their
-    # own tables/lens (decode never shares block_tables with the cached-
-    # prefill phase in a mixed step)
-    n_prefill_tokens: int = 0
-    dec_block_tables: Optional[torch.Tensor] = None  # [Bd, max_blocks] int32
-    dec_context_lens: Optional[torch.Tensor] = None  # [Bd] int32
+from .twins import add_decode_twins
 
 
 class LlamaModel:
@@ -139,54 +112,8 @@ class LlamaModel:
         self.final_norm = torch.ones(hidden, dtype=self.dtype, device=self.device)
         self.lm_head = self.embed if c.tie_embeddings else mk(self.full_config.vocab_size, hidden, std)
 
-        # Fragment-major twins of the decode projections for the
-        # macro-tile LDS-staged GEMM (ops/csrc/gemm_m256.hip) — ON by
-        # default: the twin copy costs ~weights-again for the projections
-        # (~14 GB for llama-3-8b, cheap against 288 GB HBM) and buys the
-        # decode step its dominant GEMM time back from the library
-        # (profiles/r02_gemm_m256_probe.md). LLMAPI_NO_FRAG_WEIGHTS=1
-        # opts out; LLMAPI_SWZ_WEIGHTS=1 selects the legacy k-major twins
-        # (gemm_skinny streaming form) for comparison runs.
-        import os as _os
-
-        if self.device.type == "cuda" and not _os.environ.get("LLMAPI_NO_FRAG_WEIGHTS"):
-            legacy = bool(_os.environ.get("LLMAPI_SWZ_WEIGHTS"))
-            for layer in self.layers:
-                for name in ("qkv", "o", "gate_up", "down"):
-                    w = layer[name]
-                    if legacy:
-                        if w.shape[0] % 64 == 0 and w.shape[1] % 32 == 0:
-                            layer[name + "_swz"] = ops.swizzle_weight(w)
-                    elif (
-                        w.shape[0] % 64 == 0
-                        and w.shape[1] % 64 == 0
-                        # only shapes the measured dispatch actually routes to
-                        # the custom kernel get a twin — qkv/gate_up twins
-                        # would be dead HBM (the library wins those shapes),
-                        # ~9 GB at 8B and ~89 GB at 70B
-                        and ops._m256_config(256, w.shape[0], w.shape[1]) is not None
-                        # gate_up with a fused-swiglu twin never uses the
-                        # plain twin — don't hold both in HBM
-                        and not (
-                            name == "gate_up"
-                            and ops._m256_swiglu_config(
-                                256, w.shape[0], w.shape[1]
-                            )
-                            is not None
-                        )
-                    ):
-                        layer[name + "_swz"] = ops.swizzle_weight_frag(w)
-                gu = layer["gate_up"]
-                if (
-                    not legacy
-                    and ops._m256_swiglu_config(256, gu.shape[0], gu.shape[1])
-                    is not None
-                ):
-                    # block-16 interleaved twin for the FUSED gate_up+swiglu
-                    # decode path (ops.swiglu_linear)
-                    layer["gate_up_int"] = ops.swizzle_weight_frag(
-                        ops.interleave_gate_up(gu)
-                    )
+        for layer in self.layers:
+            add_decode_twins(layer)
 
     def param_bytes(self) -> int:
         total = self.embed.numel() + self.final_norm.numel()
@@ -224,6 +151,14 @@ class LlamaModel:
         h1.wait()
         h2.wait()
         return torch.cat([y1, y2], dim=0)
+
+    def step(self, batch: ForwardBatch, cache) -> torch.Tensor:
+        """forward() over the engine's cache object."""
+        return self.forward(
+            batch, cache.k_caches, cache.v_caches,
+            k_scales=cache.k_scales if cache.fp8 else None,
+            v_scales=cache.v_scales if cache.fp8 else None,
+        )
 
     @torch.inference_mode()
     def forward(

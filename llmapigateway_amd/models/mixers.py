@@ -1,0 +1,215 @@
+"""Token mixers of the hybrid decoders, each built from its sizes and
+constants and its checkpoint tensors.
+
+A mixer reads the normed rows of a flat batch, keeps what it must remember
+in its own cache view (pages for attention, one state slot per sequence for
+recurrences; engine/kvcache.py allocates them from ``cache_spec``) and
+returns the rows to be added to the residual stream. Projections that read
+the same rows are stacked into one product. What enters a recurrence (gate
+and step-size pre-activations) leaves its product in fp32.
+"""
+
+from __future__ import annotations
+
+from typing import Callable, Dict, NamedTuple, Tuple
+
+import torch
+
+from .. import ops
+from .batch import ForwardBatch
+from .twins import add_decode_twins
+
+Getter = Callable[[str], torch.Tensor]
+
+
+class CacheSpec(NamedTuple):
+    """What one run of a layer keeps: ``pages`` name -> row width (one row
+    per token, compute dtype); ``state`` name -> (shape, fp32?) per
+    sequence slot."""
+
+    pages: Dict[str, int]
+    state: Dict[str, Tuple[Tuple[int, ...], bool]]
+
+
+def _pad8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+class LatentAttention:
+    """Attention whose keys and values unfold from one cached latent per
+    token, plus one rotated key part that all heads share; the softmax has
+    a learned sink per head in its denominator.
+
+    Two equivalent forms: folded (queries are taken into the latent space,
+    scores and sums run over the cached rows themselves; decode and short
+    portions) and unfolded (per-head keys and values are made from the
+    latents; long portions)."""
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.m, self.eps = m, eps
+        self.H, self.dim, self.rot = m["heads"], m["dim"], m["rot_dim"]
+        self.vdim, self.rank, self.q_rank = m["vdim"], m["kv_rank"], m["q_rank"]
+        self.scale = float(m["scale"])
+        self.row = _pad8(self.rank + self.rot)  # cached row, zero-padded
+        self.cos_sin = rope(m["rot"]["base"], m["rot"]["dims"])
+        self.q_norm, self.kv_norm = vec("dq.norm"), vec("dkv.norm")
+        self.sink = vec("sink")
+        uk = get("uk").view(self.H, self.dim, self.rank)
+        uv = get("uv")
+        self.w = {
+            "down": torch.cat([get("dq"), get("dkv")]),
+            "uq": get("uq"),
+            "ukv": torch.cat([uk.reshape(-1, self.rank), uv]),
+            "o": get("o"),
+        }
+        self.uk_t = uk.transpose(1, 2).contiguous()            # [H, rank, dim]
+        self.uv = uv.view(self.H, self.vdim, self.rank)        # [H, vdim, rank]
+        add_decode_twins(self.w, ("down", "uq", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H = m["heads"]
+        return {
+            "dq": (m["q_rank"], width), "dq.norm": (m["q_rank"],),
+            "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]),
+            "dkv": (m["kv_rank"] + m["rot_dim"], width), "dkv.norm": (m["kv_rank"],),
+            "uk": (H * m["dim"], m["kv_rank"]), "uv": (H * m["vdim"], m["kv_rank"]),
+            "sink": (H,), "o": (width, H * m["vdim"]),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict) -> CacheSpec:
+        return CacheSpec({"latent": _pad8(m["kv_rank"] + m["rot_dim"])}, {})
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        T, w = h.shape[0], self.w
+        d = ops.linear(h, w["down"], w.get("down_swz"))
+        latent = cache["latent"]
+        cq = ops.latent_rows(
+            d, self.q_norm, self.kv_norm, self.eps, self.rot,
+            batch.positions, self.cos_sin, latent, batch.slot_mapping,
+        )
+        q = ops.linear(cq, w["uq"], w.get("uq_swz")).view(T, self.H, self.dim + self.rot)
+        if plan.unfold is not None:
+            out = ops.latent_attention_unfolded(
+                q, latent, w["ukv"], self.sink, self.scale, self.dim, self.vdim,
+                self.rank, self.cos_sin, batch.positions, plan.unfold,
+            )
+            Tu = plan.unfold.rows
+            if Tu < T:
+                out[Tu:] = self._folded(q[Tu:], latent, batch, plan)
+        else:
+            out = self._folded(q, latent, batch, plan)
+        return ops.linear(out.view(T, self.H * self.vdim), w["o"], w.get("o_swz"))
+
+    def _folded(self, q, latent, batch, plan) -> torch.Tensor:
+        pos = batch.positions[plan.folded_from :]
+        ql = ops.fold_queries(q, self.uk_t, self.row, self.cos_sin, pos)
+        o = ops.latent_attention_folded(
+            ql, latent, self.rank, self.sink, self.scale, pos, batch.segs,
+            plan.folded_from,
+        )
+        return ops.head_linear(o, self.uv)
+
+
+class Mamba2:
+    """State-space duality layer: short causal convolution, scalar decay
+    per head, B and C shared by the heads of a group, gated group norm."""
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.m, self.eps = m, eps
+        self.H, self.P, self.N, self.G = m["heads"], m["vdim"], m["state"], m["groups"]
+        self.inner = self.H * self.P
+        self.norm_groups = m["norm_groups"]
+        w_in = get("in")
+        self.w = {"in": w_in[: -self.H].contiguous(), "o": get("o")}
+        self.w_dt = w_in[-self.H :].contiguous()
+        self.conv, self.conv_b = vec("conv"), vec("conv.b")
+        self.dt_bias, self.A_log, self.D = vec("dt_bias"), vec("A_log"), vec("D")
+        self.norm = vec("norm")
+        add_decode_twins(self.w, ("in", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H, inner, gn = m["heads"], m["heads"] * m["vdim"], m["groups"] * m["state"]
+        return {
+            "in": (2 * inner + 2 * gn + H, width), "conv": (inner + 2 * gn, m["conv"]),
+            "conv.b": (inner + 2 * gn,), "dt_bias": (H,), "A_log": (H,), "D": (H,),
+            "norm": (inner,), "o": (width, inner),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict) -> CacheSpec:
+        channels = m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]
+        return CacheSpec({}, {
+            "S": ((m["heads"], m["vdim"], m["state"]), True),
+            "conv": ((m["conv"] - 1, channels), False),
+        })
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        dt = ops.linear_f32(h, self.w_dt)
+        xbc = ops.causal_conv(
+            u[:, self.inner :], self.conv, self.conv_b, cache["conv"],
+            batch.positions, batch.segs, plan,
+        )
+        y = ops.ssd(
+            xbc, dt, self.dt_bias, self.A_log, self.D, self.H, self.P, self.N, self.G,
+            cache["S"], batch.positions, batch.segs, plan,
+        )
+        y = ops.gated_norm(
+            y, u[:, : self.inner], self.norm, self.norm_groups, self.eps, gate_first=True
+        )
+        return ops.linear(y, w["o"], w.get("o_swz"))
+
+
+class MLSTM:
+    """Matrix-memory recurrence with exponential gates kept in range by a
+    running maximum, a normaliser state, head-wise norm and output gate."""
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.m, self.eps = m, eps
+        self.H, self.dk, self.dv = m["heads"], m["dim"], m["vdim"]
+        self.cap = float(m["gate_cap"])
+        self.w = {
+            "qkvg": torch.cat([get("q"), get("k"), get("v"), get("g")]),
+            "o": get("o"),
+        }
+        self.w_if = torch.cat([get("i"), get("f")])
+        self.if_bias = torch.cat([vec("i.b"), vec("f.b")])
+        self.norm = vec("norm")
+        add_decode_twins(self.w, ("qkvg", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H, dk, dv = m["heads"], m["dim"], m["vdim"]
+        return {
+            "q": (H * dk, width), "k": (H * dk, width), "v": (H * dv, width),
+            "g": (H * dv, width), "o": (width, H * dv), "norm": (H * dv,),
+            "i": (H, width), "i.b": (H,), "f": (H, width), "f.b": (H,),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict) -> CacheSpec:
+        H, dk, dv = m["heads"], m["dim"], m["vdim"]
+        return CacheSpec({}, {
+            "S": ((H, dv, dk), True), "n": ((H, dk), True), "m": ((H,), True),
+        })
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w, kq, vv = self.w, self.H * self.dk, self.H * self.dv
+        u = ops.linear(h, w["qkvg"], w.get("qkvg_swz"))
+        gates = ops.linear_f32(h, self.w_if)
+        y = ops.mlstm(
+            u[:, :kq], u[:, kq : 2 * kq], u[:, 2 * kq : 2 * kq + vv], gates,
+            self.if_bias, self.cap, self.H, self.dk, self.dv,
+            cache["S"], cache["n"], cache["m"], batch.positions, batch.segs, plan,
+        )
+        y = ops.gated_norm(
+            y, u[:, 2 * kq + vv :], self.norm, self.H, self.eps, gate_first=False
+        )
+        return ops.linear(y, w["o"], w.get("o_swz"))
+
+
+MIXERS = {"latent_attention": LatentAttention, "mamba2": Mamba2, "mlstm": MLSTM}

@@ -43,28 +43,11 @@ if torch.version.hip and os.path.exists(_TUNE_BASE.replace(".csv", "0.csv")):
 from . import reference
 from .reference import build_rope_cache  # re-export (host-side table builder)
 
-_C = None
-_C_ERR: Optional[str] = None
-try:
-    import importlib
-
-    _C = importlib.import_module("._C", __name__)
-except ImportError as e:  # extension not built (CPU-only envs are fine)
-    _C_ERR = str(e)
+from .native import _C, _H, dense_native as _native, shared_native as _shared
 
 
 def have_native() -> bool:
-    return _C is not None
-
-
-def _native():
-    if _C is None:
-        raise RuntimeError(
-            "llmapigateway_amd.ops._C (gfx950 HIP extension) is not built but a GPU tensor "
-            "reached the ops layer. Build it with `python setup.py build_ext --inplace` "
-            f"(import error: {_C_ERR})"
-        )
-    return _C
+    return _C is not None and _H is not None
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float = 1e-5) -> torch.Tensor:
@@ -101,7 +84,7 @@ def swiglu(x: torch.Tensor) -> torch.Tensor:
         out = torch.empty(
             (*x.shape[:-1], inter), dtype=x.dtype, device=x.device
         )
-        _native().swiglu(out, x)
+        _shared().swiglu(out, x)
         return out
     return reference.swiglu(x)
 
@@ -529,13 +512,13 @@ def linear(
             y = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
             nsk = _skinny_nsk(N, K)
             ws = _skinny_scratch(x.device, nsk * M * N) if nsk > 1 else None
-            _native().gemm_skinny(y, x, w_swz, ws, nsk, True)
+            _shared().gemm_skinny(y, x, w_swz, ws, nsk, True)
             return y
         if M <= _SKINNY_MAX_M:
             y = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
             nsk = _skinny_nsk(N, K)
             ws = _skinny_scratch(x.device, nsk * M * N) if nsk > 1 else None
-            _native().gemm_skinny(y, x, w, ws, nsk, False)
+            _shared().gemm_skinny(y, x, w, ws, nsk, False)
             return y
     return torch.nn.functional.linear(x, w)
 
@@ -565,6 +548,24 @@ def sample(
     return reference.sample(logits, temperature, noise)
 
 
+from .hybrid import (  # noqa: E402
+    add_cast,
+    add_layernorm,
+    build_pair_rope_cache,
+    causal_conv,
+    embed_scaled,
+    fold_queries,
+    gated_norm,
+    head_linear,
+    latent_attention_folded,
+    latent_attention_unfolded,
+    latent_rows,
+    linear_f32,
+    mlstm,
+    plan_segments,
+    ssd,
+)
+
 __all__ = [
     "have_native",
     "build_rope_cache",
@@ -583,4 +584,19 @@ __all__ = [
     "sample",
     "topk_topp_filter",
     "reference",
+    "add_cast",
+    "add_layernorm",
+    "build_pair_rope_cache",
+    "causal_conv",
+    "embed_scaled",
+    "fold_queries",
+    "gated_norm",
+    "head_linear",
+    "latent_attention_folded",
+    "latent_attention_unfolded",
+    "latent_rows",
+    "linear_f32",
+    "mlstm",
+    "plan_segments",
+    "ssd",
 ]

@@ -1,0 +1,263 @@
+"""Ops of the hybrid decoders: gfx950 kernels (the ``_H`` extension) on GPU
+tensors, ops/reference_hybrid.py on CPU tensors.
+
+Rows are those of a flat batch; ``segs`` (models/batch.py Segments) says
+which sequence each belongs to, where its pages and state are. Every op
+takes any split of a sequence into segments.
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import Optional
+
+import numpy as np
+import torch
+
+from . import reference_hybrid as ref
+from .native import hybrid_native
+from .reference_hybrid import build_pair_rope_cache
+
+
+# ---------------------------------------------------------------- planning
+@dataclass
+class Unfold:
+    """Prefill rows [0, rows) attend through per-head keys and values made
+    from ``keys`` latents, gathered from the pages sequence by sequence."""
+
+    rows: int
+    keys: int
+    key_slots: torch.Tensor   # [keys] int64 global cache rows
+    cu_q: torch.Tensor        # [S+1] int32
+    cu_k: torch.Tensor        # [S+1] int32
+    tile_seg: torch.Tensor    # [ntiles] int32
+    tile_off: torch.Tensor    # [ntiles] int32
+
+
+@dataclass
+class Chunks:
+    """Segments long enough for the chunked form of the recurrences."""
+
+    segs: torch.Tensor        # [L] int32 segment of each
+    first: torch.Tensor       # [L+1] int32 first chunk of each
+    chunk_seg: torch.Tensor   # [n] int32
+    chunk_off: torch.Tensor   # [n] int32 first row within the segment
+    short: torch.Tensor       # int32 segments that are run token by token
+    count: int
+
+
+@dataclass
+class SegmentPlan:
+    """How a step's rows go through the kernels; made once per step."""
+
+    folded_from: int = 0
+    unfold: Optional[Unfold] = None
+    chunks: Optional[Chunks] = None
+
+
+CHUNK = 64            # rows per chunk of the chunked recurrences
+CHUNK_MIN_ROWS = 32   # shorter segments run token by token
+UNFOLD_RATIO = 16     # query-key pairs per key from which unfolding pays
+
+
+def plan_segments(batch, dtype) -> SegmentPlan:
+    segs = batch.segs
+    plan = SegmentPlan()
+    if batch.kind == "decode" or segs.lens is None:
+        return plan
+    if not batch.token_ids.is_cuda or dtype != torch.bfloat16:
+        return plan
+    dev = batch.token_ids.device
+    lens, starts = segs.lens, segs.starts
+    nseg_p = segs.n_prefill
+    parts, fields = [], []
+
+    def put(name, a):
+        fields.append((name, len(a)))
+        parts.append(np.asarray(a, dtype=np.int32))
+
+    pl, ps = lens[:nseg_p], starts[:nseg_p]
+    keys = int((pl + ps).sum())
+    pairs = float((pl * (ps + pl / 2.0)).sum())
+    unfold = nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
+    if unfold:
+        put("cu_q", np.concatenate([[0], np.cumsum(pl)]))
+        put("cu_k", np.concatenate([[0], np.cumsum(pl + ps)]))
+        put("tile_seg", np.repeat(np.arange(nseg_p), (pl + 63) // 64))
+        put("tile_off", np.concatenate([np.arange(0, n, 64) for n in pl]))
+    long = np.nonzero(lens >= CHUNK_MIN_ROWS)[0]
+    nchunk = (lens[long] + CHUNK - 1) // CHUNK
+    if len(long):
+        put("segs", long)
+        put("first", np.concatenate([[0], np.cumsum(nchunk)]))
+        put("chunk_seg", np.repeat(long, nchunk))
+        put("chunk_off", np.concatenate([np.arange(n) * CHUNK for n in nchunk]))
+        put("short", np.nonzero(lens < CHUNK_MIN_ROWS)[0])
+    if not parts:
+        return plan
+    flat = torch.from_numpy(np.concatenate(parts)).to(dev)  # one copy for all maps
+    got, at = {}, 0
+    for name, n in fields:
+        got[name] = flat[at : at + n]
+        at += n
+    if unfold:
+        tables = segs.tables[:nseg_p]
+        cu_k = got["cu_k"].long()
+        seg = torch.repeat_interleave(
+            torch.arange(nseg_p, device=dev), cu_k.diff(), output_size=keys
+        )
+        pos = torch.arange(keys, device=dev) - cu_k[seg]
+        bs = segs.block_size
+        plan.unfold = Unfold(
+            rows=batch.n_prefill_tokens, keys=keys,
+            key_slots=tables[seg, pos // bs].long() * bs + pos % bs,
+            cu_q=got["cu_q"], cu_k=got["cu_k"],
+            tile_seg=got["tile_seg"], tile_off=got["tile_off"],
+        )
+        plan.folded_from = batch.n_prefill_tokens
+    if len(long):
+        plan.chunks = Chunks(
+            segs=got["segs"], first=got["first"], chunk_seg=got["chunk_seg"],
+            chunk_off=got["chunk_off"], short=got["short"], count=int(nchunk.sum()),
+        )
+    return plan
+
+
+# ------------------------------------------------------ stream and products
+def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w.T with the fp32 accumulator as the result."""
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, w)
+    if x.is_cuda:
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return torch.nn.functional.linear(x.float(), w.float())
+
+
+def embed_scaled(tokens, embed, scale: float, x0: Optional[torch.Tensor]) -> torch.Tensor:
+    """fp32 embed[token] * scale; x0 (compute dtype, may be strided)
+    receives the same rows."""
+    if not embed.is_cuda:
+        return ref.embed_scaled(tokens, embed, scale, x0)
+    x = torch.empty(tokens.shape[0], embed.shape[1], dtype=torch.float32, device=embed.device)
+    hybrid_native().embed_scaled(x, x0, tokens, embed, float(scale))
+    return x
+
+
+def add_layernorm(x, delta, w, b, eps: float, dtype, vec=None, replace: bool = False):
+    """x (fp32 stream, in place) += delta [+ vec], or = delta [+ vec] with
+    ``replace``; returns layer norm(x) * w + b in ``dtype``."""
+    if not x.is_cuda:
+        return ref.add_layernorm(x, delta, w, b, eps, dtype, vec, replace)
+    out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    hybrid_native().add_layernorm(out, x, delta, vec, w, b, float(eps), replace)
+    return out
+
+
+def add_cast(x, delta, out) -> None:
+    """x += delta; out (compute dtype, may be strided) = x."""
+    if not x.is_cuda:
+        return ref.add_cast(x, delta, out)
+    hybrid_native().add_cast(out, x, delta)
+
+
+def head_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """y[t, h] = w[h] @ x[t, h]: x [T, H, K], w [H, N, K]."""
+    if not x.is_cuda:
+        return ref.head_linear(x, w)
+    y = torch.empty(x.shape[0], w.shape[0], w.shape[1], dtype=x.dtype, device=x.device)
+    hybrid_native().head_linear(y, x, w)
+    return y
+
+
+# ---------------------------------------------------------- latent attention
+def latent_rows(d, q_norm, kv_norm, eps, rot, positions, cos_sin, latent, slot_mapping):
+    """d [T, q_rank + kv_rank + rot]: returns the normed query latent; writes
+    [normed kv latent | rotated key part] into the paged cache."""
+    if not d.is_cuda:
+        return ref.latent_rows(
+            d, q_norm, kv_norm, eps, rot, positions, cos_sin, latent, slot_mapping
+        )
+    cq = torch.empty(d.shape[0], q_norm.numel(), dtype=d.dtype, device=d.device)
+    hybrid_native().latent_rows(
+        cq, latent, d, q_norm, kv_norm, float(eps), rot, positions, cos_sin, slot_mapping
+    )
+    return cq
+
+
+def fold_queries(q, uk_t, row: int, cos_sin, positions) -> torch.Tensor:
+    """[T, H, row]: W_uk^T q_unrotated, the rotated part, zeros up to row."""
+    if not q.is_cuda:
+        return ref.fold_queries(q, uk_t, row, positions, cos_sin)
+    H, rank, dim = uk_t.shape
+    out = torch.empty(q.shape[0], H, row, dtype=q.dtype, device=q.device)
+    hybrid_native().head_linear(out[..., :rank], q[..., :dim], uk_t)
+    hybrid_native().rotate_pairs(out[..., rank:], q[..., dim:], positions, cos_sin)
+    return out
+
+
+def latent_attention_folded(ql, latent, rank, sink, scale, positions, segs, row0: int):
+    """Row t (row row0 + t of the flat batch) against its sequence's cached
+    rows 0..positions[t]; returns the latent-space sums [T, H, rank]."""
+    if not ql.is_cuda:
+        return ref.latent_attention_folded(
+            ql, latent, rank, sink, scale, positions, segs, row0
+        )
+    out = torch.empty(ql.shape[0], ql.shape[1], rank, dtype=ql.dtype, device=ql.device)
+    hybrid_native().latent_attention_folded(
+        out, ql, latent, sink, float(scale), positions, segs.row_seg[row0:], segs.tables
+    )
+    return out
+
+
+def latent_attention_unfolded(
+    q, latent, w_ukv, sink, scale, dim, vdim, rank, cos_sin, positions, u: Unfold
+):
+    raise NotImplementedError
+
+
+# --------------------------------------------------------------- recurrences
+def causal_conv(x, w, b, state, positions, segs, plan) -> torch.Tensor:
+    """silu of the causal per-channel convolution of x [T, C] (may be
+    strided); state [slots, taps-1, C] carries the last inputs."""
+    if not x.is_cuda:
+        return ref.causal_conv(x, w, b, state, positions, segs)
+    y = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    hybrid_native().causal_conv(
+        y, x, w, b, state, positions, segs.cu, segs.slots, segs.row_seg
+    )
+    return y
+
+
+def ssd(xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs, plan):
+    """Mamba-2 recurrence over xbc [T, H*P + 2*G*N] and raw dt [T, H]
+    (fp32); state S [slots, H, P, N]."""
+    if not xbc.is_cuda:
+        return ref.ssd(xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs)
+    y = torch.empty(xbc.shape[0], H * P, dtype=xbc.dtype, device=xbc.device)
+    hybrid_native().ssd_scan(
+        y, xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs.cu, segs.slots, None
+    )
+    return y
+
+
+def mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs, plan):
+    """mLSTM recurrence; gates [T, 2H] fp32 raw input and forget gates,
+    states S [slots, H, dv, dk], n [slots, H, dk], m [slots, H]."""
+    if not q.is_cuda:
+        return ref.mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs)
+    y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    hybrid_native().mlstm_scan(
+        y, q, k, v, gates, bias, float(cap), H, dk, dv, S, n, m, positions,
+        segs.cu, segs.slots, None,
+    )
+    return y
+
+
+def gated_norm(y, gate, w, groups: int, eps: float, gate_first: bool):
+    """RMS norm of y in ``groups`` equal parts, times w; multiplied by
+    silu(gate) before the norm, or by sigmoid(gate) after it."""
+    if not y.is_cuda:
+        return ref.gated_norm(y, gate, w, groups, eps, gate_first)
+    out = torch.empty_like(y)
+    hybrid_native().gated_norm(out, y, gate, w, groups, float(eps), gate_first)
+    return out
