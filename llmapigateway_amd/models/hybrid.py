@@ -25,6 +25,8 @@ from .weights import open_checkpoint
 
 
 class HybridModel:
+    extension = "_H"  # the HIP extension its kernels are in
+
     def __init__(
         self,
         config: HybridConfig,

@@ -36,6 +36,8 @@ from .twins import add_decode_twins
 
 
 class LlamaModel:
+    extension = "_C"  # the HIP extension its kernels are in
+
     def __init__(
         self,
         config: ModelConfig,

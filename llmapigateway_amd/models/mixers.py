@@ -124,7 +124,8 @@ class Mamba2:
         w_in = get("in")
         self.w = {"in": w_in[: -self.H].contiguous(), "o": get("o")}
         self.w_dt = w_in[-self.H :].contiguous()
-        self.conv, self.conv_b = vec("conv"), vec("conv.b")
+        self.conv_t = vec("conv").t().contiguous()  # [taps, channels]
+        self.conv_b = vec("conv.b")
         self.dt_bias, self.A_log, self.D = vec("dt_bias"), vec("A_log"), vec("D")
         self.norm = vec("norm")
         add_decode_twins(self.w, ("in", "o"))
@@ -151,7 +152,7 @@ class Mamba2:
         u = ops.linear(h, w["in"], w.get("in_swz"))
         dt = ops.linear_f32(h, self.w_dt)
         xbc = ops.causal_conv(
-            u[:, self.inner :], self.conv, self.conv_b, cache["conv"],
+            u[:, self.inner :], self.conv_t, self.conv_b, cache["conv"],
             batch.positions, batch.segs, plan,
         )
         y = ops.ssd(
@@ -194,7 +195,9 @@ class MLSTM:
     def cache_spec(m: dict) -> CacheSpec:
         H, dk, dv = m["heads"], m["dim"], m["vdim"]
         return CacheSpec({}, {
-            "S": ((H, dv, dk), True), "n": ((H, dk), True), "m": ((H,), True),
+            # every tile of 64 value rows carries its own n and m
+            "S": ((H, dv, dk), True), "n": ((-(-dv // 64), H, dk), True),
+            "m": ((-(-dv // 64), H), True),
         })
 
     def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:

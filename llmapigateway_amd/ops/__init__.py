@@ -1,9 +1,9 @@
 """Op dispatch: gfx950 HIP kernels on GPU, PyTorch reference on CPU.
 
-The HIP extension (llmapigateway_amd/ops/_C*.so, built in-tree by
-``python setup.py build_ext --inplace`` / __graft_entry__.build) is the ONLY
-compute path on GPU tensors — if a CUDA tensor reaches an op and the
-extension is missing, we raise instead of silently falling back to eager
+The HIP extensions (llmapigateway_amd/ops/_C*.so and _H*.so, built in-tree by
+``python setup.py build_ext --inplace`` / __graft_entry__.build; see native.py)
+are the ONLY compute path on GPU tensors — if a CUDA tensor reaches an op and
+its extension is missing, we raise instead of silently falling back to eager
 PyTorch. CPU tensors use ops.reference (fp32 semantics contract).
 """
 
@@ -43,11 +43,7 @@ if torch.version.hip and os.path.exists(_TUNE_BASE.replace(".csv", "0.csv")):
 from . import reference
 from .reference import build_rope_cache  # re-export (host-side table builder)
 
-from .native import _C, _H, dense_native as _native, shared_native as _shared
-
-
-def have_native() -> bool:
-    return _C is not None and _H is not None
+from .native import dense_native as _native, have_native, shared_native as _shared
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float = 1e-5) -> torch.Tensor:

@@ -51,6 +51,16 @@ __device__ __forceinline__ uint16_t f2bfbits(float v) {
     return static_cast<uint16_t>(rounded >> 16);
 }
 
+// element access for kernels templated on the compute dtype (bf16 or fp32)
+__device__ __forceinline__ float ldf(const float* p) { return *p; }
+__device__ __forceinline__ float ldf(const bf16* p) {
+    return bfbits2f(*reinterpret_cast<const uint16_t*>(p));
+}
+__device__ __forceinline__ void stf(float* p, float v) { *p = v; }
+__device__ __forceinline__ void stf(bf16* p, float v) {
+    *reinterpret_cast<uint16_t*>(p) = f2bfbits(v);
+}
+
 // unpack a uint32 holding 2 bf16
 __device__ __forceinline__ void unpack2(uint32_t p, float& lo, float& hi) {
     lo = bfbits2f(static_cast<uint16_t>(p & 0xFFFFu));

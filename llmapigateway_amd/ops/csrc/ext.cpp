@@ -4,45 +4,22 @@
 // this file validates tensors, extracts strides and dispatches on the
 // current HIP stream.
 
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
-
-#include <vector>
-
-#include "kv_manager.cpp"
+#include "bind_shared.h"
 
 extern "C" {
 hipError_t launch_rmsnorm(void*, const void*, const void*, float, int, int, hipStream_t);
 hipError_t launch_rmsnorm_residual(void*, const void*, void*, const void*, float, int, int, hipStream_t);
 hipError_t launch_rope(void*, void*, const int64_t*, const float*, int, int64_t, int64_t, int, int, int, hipStream_t);
-hipError_t launch_swiglu(void*, const void*, int, int, hipStream_t);
 hipError_t launch_kv_cache_write(const void*, const void*, void*, void*, float*, float*, const int64_t*, int, int64_t, int64_t, int, int, int, hipStream_t);
 hipError_t launch_rope_kv(void*, void*, const void*, void*, void*, float*, float*, const int64_t*, const float*, const int64_t*, int, int64_t, int64_t, int64_t, int, int, int, int, hipStream_t);
 hipError_t launch_attention_decode(void*, const void*, const void*, const void*, const float*, const float*, const int*, const int*, float, int, int, int, int, int, int, int64_t, float*, float*, int, int, hipStream_t);
 hipError_t launch_attention_prefill(void*, const void*, const void*, const void*, const int*, const int*, const int*, int, float, int, int, int, int64_t, int64_t, int64_t, const void*, const void*, const float*, const float*, const int*, const int*, int, int, hipStream_t);
 hipError_t launch_sample(int64_t*, const float*, const float*, const float*, float*, int*, int, int, hipStream_t);
 hipError_t launch_topk_topp_filter(float*, const float*, const int*, int, int, hipStream_t);
-hipError_t launch_gemm_skinny(void*, float*, const void*, const void*, int, int, int, int, int, hipStream_t);
 hipError_t launch_gemm_m256(void*, float*, const void*, const void*, int, int, int, int, int, int, int, int, hipStream_t);
 }
 
 namespace {
-
-#define CHECK_HIP(call)                                                        \
-    do {                                                                       \
-        hipError_t err = (call);                                               \
-        TORCH_CHECK(err == hipSuccess, "HIP kernel failed: ",                  \
-                    hipGetErrorString(err));                                   \
-    } while (0)
-
-hipStream_t current_stream() {
-    return at::hip::getCurrentHIPStream().stream();
-}
-
-void check_bf16(const torch::Tensor& t, const char* name) {
-    TORCH_CHECK(t.is_cuda(), name, " must be on GPU");
-    TORCH_CHECK(t.scalar_type() == torch::kBFloat16, name, " must be bf16");
-}
 
 // fp8 KV caches are stored as uint8 (e4m3 bits) with fp32 row scales
 void check_cache(const torch::Tensor& t, const char* name) {
@@ -94,15 +71,6 @@ void rope_inplace(torch::Tensor q, torch::Tensor k, torch::Tensor positions,
                           positions.data_ptr<int64_t>(),
                           cos_sin.data_ptr<float>(), T, q.stride(0), k.stride(0),
                           q.size(1), k.size(1), q.size(2), current_stream()));
-}
-
-void swiglu(torch::Tensor out, torch::Tensor x) {
-    check_bf16(x, "x");
-    TORCH_CHECK(x.is_contiguous() && out.is_contiguous());
-    const int I = out.size(-1);
-    TORCH_CHECK(x.size(-1) == 2 * I, "x last dim must be 2*I");
-    const int T = x.numel() / (2 * I);
-    CHECK_HIP(launch_swiglu(out.data_ptr(), x.data_ptr(), T, I, current_stream()));
 }
 
 void kv_cache_write(torch::Tensor k, torch::Tensor v, torch::Tensor k_cache,
@@ -281,36 +249,6 @@ void topk_topp_filter(torch::Tensor logits, torch::Tensor topp, torch::Tensor to
                                       current_stream()));
 }
 
-void gemm_skinny(torch::Tensor y, torch::Tensor x, torch::Tensor w,
-                 c10::optional<torch::Tensor> workspace, int64_t nsk,
-                 bool swizzled) {
-    check_bf16(x, "x");
-    check_bf16(w, "w");
-    check_bf16(y, "y");
-    TORCH_CHECK(x.is_contiguous() && w.is_contiguous() && y.is_contiguous());
-    TORCH_CHECK(x.dim() == 2 && y.dim() == 2);
-    const int M = x.size(0), K = x.size(1);
-    int N;
-    if (swizzled) {  // w is [K/32, N, 32]
-        TORCH_CHECK(w.dim() == 3 && w.size(0) == K / 32 && w.size(2) == 32);
-        N = w.size(1);
-    } else {
-        TORCH_CHECK(w.dim() == 2 && w.size(1) == K);
-        N = w.size(0);
-    }
-    TORCH_CHECK(y.size(0) == M && y.size(1) == N);
-    float* ws = nullptr;
-    if (workspace.has_value() && workspace->defined()) {
-        TORCH_CHECK(workspace->scalar_type() == torch::kFloat32 &&
-                    workspace->numel() >= nsk * (int64_t)M * N,
-                    "workspace must be fp32 with >= nsk*M*N elements");
-        ws = workspace->data_ptr<float>();
-    }
-    CHECK_HIP(launch_gemm_skinny(y.data_ptr(), ws, x.data_ptr(), w.data_ptr(),
-                                 M, N, K, (int)nsk, swizzled ? 1 : 0,
-                                 current_stream()));
-}
-
 void gemm_m256(torch::Tensor y, torch::Tensor x, torch::Tensor w_frag,
                c10::optional<torch::Tensor> workspace, int64_t nsk,
                int64_t nf, int64_t variant, int64_t pipe, int64_t swiglu) {
@@ -347,7 +285,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("rmsnorm", &rmsnorm, "RMSNorm (gfx950)");
     m.def("rmsnorm_residual", &rmsnorm_residual, "fused residual-add RMSNorm");
     m.def("rope_inplace", &rope_inplace, "rotate-half RoPE in place");
-    m.def("swiglu", &swiglu, "fused SiLU-gate multiply");
     m.def("kv_cache_write", &kv_cache_write, "paged KV cache scatter");
     m.def("rope_kv_write", &rope_kv_write, "fused RoPE + paged KV scatter");
     m.def("attention_decode", &attention_decode, "paged decode attention");
@@ -355,15 +292,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("sample", &sample, "greedy / gumbel-max sampling");
     m.def("topk_topp_filter", &topk_topp_filter,
           "in-place top-k/top-p logit filtering (histogram threshold)");
-    m.def("gemm_skinny", &gemm_skinny,
-          "skinny-M weight-streaming GEMM y = x @ w.T (decode projections)");
     m.def("gemm_m256", &gemm_m256,
           "macro-tile LDS-staged decode GEMM y = x @ w.T (M <= 256)");
-
-    pybind11::class_<BlockAllocator>(m, "BlockAllocator")
-        .def(pybind11::init<int64_t>())
-        .def("num_free", &BlockAllocator::num_free)
-        .def("allocate", &BlockAllocator::allocate)
-        .def("free", &BlockAllocator::free_blocks)
-        .def_property_readonly("num_blocks", &BlockAllocator::capacity);
+    bind_shared(m);
 }

@@ -1,0 +1,528 @@
+// Row kernels of the hybrid decoders for gfx950: scaled embedding, residual
+// add + layer norm over an fp32 stream, latent norms + rotation + page
+// write, gated group norm, causal convolution with carried state.
+//
+// Every kernel is templated on the compute dtype (bf16 or fp32) and takes
+// any width; widths and strides that allow it are moved 16 bytes a lane.
+// Sums and transcendentals are fp32.
+
+#include "common.h"
+
+namespace {
+
+template <int VEC>
+__device__ __forceinline__ void load_vec(const float* p, float* f) {
+    if (VEC == 8) {
+        const float4 a = reinterpret_cast<const float4*>(p)[0];
+        const float4 b = reinterpret_cast<const float4*>(p)[1];
+        f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+        f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+    } else {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) f[j] = p[j];
+    }
+}
+template <int VEC>
+__device__ __forceinline__ void load_vec(const bf16* p, float* f) {
+    if (VEC == 8) {
+        const uint4 v = *reinterpret_cast<const uint4*>(p);
+        unpack2(v.x, f[0], f[1]);
+        unpack2(v.y, f[2], f[3]);
+        unpack2(v.z, f[4], f[5]);
+        unpack2(v.w, f[6], f[7]);
+    } else {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) f[j] = ldf(p + j);
+    }
+}
+template <int VEC>
+__device__ __forceinline__ void store_vec(float* p, const float* f) {
+    if (VEC == 8) {
+        reinterpret_cast<float4*>(p)[0] = make_float4(f[0], f[1], f[2], f[3]);
+        reinterpret_cast<float4*>(p)[1] = make_float4(f[4], f[5], f[6], f[7]);
+    } else {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) p[j] = f[j];
+    }
+}
+template <int VEC>
+__device__ __forceinline__ void store_vec(bf16* p, const float* f) {
+    if (VEC == 8) {
+        uint4 v;
+        v.x = pack2(f[0], f[1]);
+        v.y = pack2(f[2], f[3]);
+        v.z = pack2(f[4], f[5]);
+        v.w = pack2(f[6], f[7]);
+        *reinterpret_cast<uint4*>(p) = v;
+    } else {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) stf(p + j, f[j]);
+    }
+}
+
+__device__ __forceinline__ float block_sum(float v, float* red) {
+    v = wave_reduce_sum(v);
+    const int wave = threadIdx.x >> 6, n = (blockDim.x + 63) >> 6;
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[wave] = v;
+    __syncthreads();
+    float t = 0.f;
+    for (int w = 0; w < n; ++w) t += red[w];
+    return t;
+}
+
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+
+// threads per row: enough for VEC elements each, whole waves, at most 512
+inline int row_threads(int width, int vec) {
+    int t = (width + vec - 1) / vec;
+    t = (t + 63) / 64 * 64;
+    return t < 64 ? 64 : (t > 512 ? 512 : t);
+}
+
+}  // namespace
+
+// ---------------------------------------------------------------------------
+// x[t] = embed[token] * scale (fp32); x0[t] (compute dtype) the same
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void embed_scaled_kernel(
+    float* __restrict__ x, T* __restrict__ x0, int64_t ld0,
+    const int64_t* __restrict__ tokens, const T* __restrict__ embed, float scale, int W) {
+    const size_t t = blockIdx.x;
+    const T* src = embed + (size_t)tokens[t] * W;
+    for (int i = threadIdx.x * VEC; i < W; i += blockDim.x * VEC) {
+        float f[VEC];
+        load_vec<VEC>(src + i, f);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) f[j] *= scale;
+        store_vec<VEC>(x + t * W + i, f);
+        if (x0 != nullptr) store_vec<VEC>(x0 + t * ld0 + i, f);
+    }
+}
+
+// ---------------------------------------------------------------------------
+// x = (REPLACE ? 0 : x) + delta + vec, kept in the fp32 stream; then
+//   norm:  out = (x - mean) / sqrt(var + eps) * w + b   (w given)
+//   cast:  out = x                                      (w null)
+// One pass over memory: a row stays in registers between the sums (widths
+// beyond 16384 re-read it).
+// ---------------------------------------------------------------------------
+template <typename T, typename D, int VEC>
+__launch_bounds__(512)
+__global__ void stream_norm_kernel(
+    T* __restrict__ out, int64_t ld_out, float* __restrict__ x,
+    const D* __restrict__ delta, const float* __restrict__ vec,
+    const float* __restrict__ w, const float* __restrict__ b, float eps, int replace,
+    int W) {
+    __shared__ float red[8];
+    constexpr int HELD = 32 / VEC;
+    const size_t t = blockIdx.x;
+    float* xr = x + t * W;
+    const D* dr = delta + t * W;
+    T* orow = out + t * ld_out;
+    const int step = blockDim.x * VEC, i0 = threadIdx.x * VEC;
+    float held[HELD][VEC];
+    float sum = 0.f;
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= W) continue;
+        float* f = held[k];
+        if (replace) {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) f[j] = 0.f;
+        } else {
+            load_vec<VEC>(xr + i, f);
+        }
+        float g[VEC];
+        if (delta != nullptr) {
+            load_vec<VEC>(dr + i, g);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) f[j] += g[j];
+        }
+        if (vec != nullptr) {
+            load_vec<VEC>(vec + i, g);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) f[j] += g[j];
+        }
+        if (delta != nullptr || vec != nullptr) store_vec<VEC>(xr + i, f);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) sum += f[j];
+        if (w == nullptr) store_vec<VEC>(orow + i, f);
+    }
+    if (w == nullptr) return;
+    const float mean = block_sum(sum, red) / (float)W;
+    float ssq = 0.f;
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        if (i0 + k * step >= W) continue;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            held[k][j] -= mean;
+            ssq += held[k][j] * held[k][j];
+        }
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, red) / (float)W + eps);
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= W) continue;
+        float wv[VEC], bv[VEC];
+        load_vec<VEC>(w + i, wv);
+        load_vec<VEC>(b + i, bv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[k][j] = held[k][j] * inv * wv[j] + bv[j];
+        store_vec<VEC>(orow + i, held[k]);
+    }
+}
+
+// ---------------------------------------------------------------------------
+// One row of d = [query latent | kv latent | rotated key part]: RMS norm of
+// the first two, pair rotation of the third; the query latent goes to cq,
+// the rest to the row's cache page slot (-1: not kept).
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void latent_rows_kernel(
+    T* __restrict__ cq, T* __restrict__ latent, int row_w, const T* __restrict__ d,
+    const float* __restrict__ q_norm, const float* __restrict__ kv_norm, float eps,
+    int q_rank, int rank, int rot, const int64_t* __restrict__ positions,
+    const float* __restrict__ cos_sin, const int64_t* __restrict__ slot_mapping) {
+    __shared__ float red[8];
+    const size_t t = blockIdx.x;
+    const T* src = d + t * (q_rank + rank + rot);
+    float sq = 0.f, sc = 0.f;
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
+        const float f = ldf(src + i);
+        sq += f * f;
+    }
+    for (int i = threadIdx.x; i < rank; i += blockDim.x) {
+        const float f = ldf(src + q_rank + i);
+        sc += f * f;
+    }
+    const float iq = 1.f / sqrtf(block_sum(sq, red) / (float)q_rank + eps);
+    const float ic = 1.f / sqrtf(block_sum(sc, red) / (float)rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
+        stf(cq + t * q_rank + i, ldf(src + i) * iq * q_norm[i]);
+    const int64_t slot = slot_mapping[t];
+    if (slot < 0) return;
+    T* dst = latent + (size_t)slot * row_w;
+    for (int i = threadIdx.x; i < rank; i += blockDim.x)
+        stf(dst + i, ldf(src + q_rank + i) * ic * kv_norm[i]);
+    const int half = rot / 2;
+    const float* cs = cos_sin + (size_t)positions[t] * rot;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) {
+        const float u = ldf(src + q_rank + rank + 2 * i);
+        const float v = ldf(src + q_rank + rank + 2 * i + 1);
+        stf(dst + rank + 2 * i, u * cs[i] - v * cs[half + i]);
+        stf(dst + rank + 2 * i + 1, v * cs[i] + u * cs[half + i]);
+    }
+}
+
+// ---------------------------------------------------------------------------
+// out[t, h, :width] = pair rotation of x[t, h, :rot], zeros from rot on
+// (x may be out). Strides in elements; the last dimension is dense.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void rotate_pairs_kernel(
+    T* out, int64_t ot, int64_t oh, int width, const T* x, int64_t xt, int64_t xh, int rot,
+    int H, const int64_t* __restrict__ positions, const float* __restrict__ cos_sin) {
+    const size_t t = blockIdx.x;
+    const int half = rot / 2;
+    const float* cs = cos_sin + (size_t)positions[t] * rot;
+    for (int e = threadIdx.x; e < H * half; e += blockDim.x) {
+        const int h = e / half, i = e % half;
+        const T* p = x + t * xt + h * xh + 2 * i;
+        T* o = out + t * ot + h * oh + 2 * i;
+        const float u = ldf(p), v = ldf(p + 1);
+        stf(o, u * cs[i] - v * cs[half + i]);
+        stf(o + 1, v * cs[i] + u * cs[half + i]);
+    }
+    const int pad = width - rot;
+    for (int e = threadIdx.x; e < H * pad; e += blockDim.x)
+        stf(out + t * ot + (e / pad) * oh + rot + e % pad, 0.f);
+}
+
+// ---------------------------------------------------------------------------
+// Group norm with a gate: y (dense rows) in `groups` equal parts.
+//   GATE_FIRST: out = rms(y * silu(gate)) * w
+//   else:       out = rms(y) * w * sigmoid(gate)
+// One workgroup per (row, group).
+// ---------------------------------------------------------------------------
+template <typename T, int VEC, bool GATE_FIRST>
+__launch_bounds__(512)
+__global__ void gated_norm_kernel(
+    T* __restrict__ out, const T* __restrict__ y, const T* __restrict__ gate, int64_t ld_gate,
+    const float* __restrict__ w, float eps, int groups, int gs) {
+    __shared__ float red[8];
+    constexpr int HELD = 32 / VEC;
+    const size_t t = blockIdx.x;
+    const int g = blockIdx.y;
+    const size_t base = t * (size_t)groups * gs + (size_t)g * gs;
+    const T* yr = y + base;
+    const T* gr = gate + t * ld_gate + (size_t)g * gs;
+    const float* wr = w + (size_t)g * gs;
+    const int step = blockDim.x * VEC, i0 = threadIdx.x * VEC;
+    float held[HELD][VEC];
+    float ssq = 0.f;
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= gs) continue;
+        load_vec<VEC>(yr + i, held[k]);
+        if (GATE_FIRST) {
+            float z[VEC];
+            load_vec<VEC>(gr + i, z);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) held[k][j] *= z[j] * sigmoid_f(z[j]);
+        }
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ssq += held[k][j] * held[k][j];
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, red) / (float)gs + eps);
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= gs) continue;
+        float wv[VEC];
+        load_vec<VEC>(wr + i, wv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[k][j] *= inv * wv[j];
+        if (!GATE_FIRST) {
+            float z[VEC];
+            load_vec<VEC>(gr + i, z);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) held[k][j] *= sigmoid_f(z[j]);
+        }
+        store_vec<VEC>(out + base + i, held[k]);
+    }
+}
+
+// ---------------------------------------------------------------------------
+// Causal per-channel convolution + silu over the rows of each segment; taps
+// before the segment come from state [slots, taps-1, C] (zeros when the
+// segment starts its sequence). w_t is [taps, C].
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void causal_conv_kernel(
+    T* __restrict__ y, const T* __restrict__ x, int64_t ldx, const float* __restrict__ w_t,
+    const float* __restrict__ b, const T* __restrict__ state,
+    const int64_t* __restrict__ positions, const int* __restrict__ cu,
+    const int* __restrict__ slots, const int* __restrict__ row_seg, int C, int taps) {
+    const size_t t = blockIdx.x;
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
+    if (c >= C) return;
+    const int s = row_seg[t];
+    const int slot = slots[s];
+    const int j0 = (int)t - cu[s];
+    float acc[VEC];
+    load_vec<VEC>(b + c, acc);
+    const bool fresh = slot < 0 || positions[t] == j0;
+    for (int k = 0; k < taps; ++k) {
+        const int src = j0 - (taps - 1) + k;
+        float f[VEC], wv[VEC];
+        if (src >= 0)
+            load_vec<VEC>(x + (t - j0 + src) * ldx + c, f);
+        else if (!fresh)
+            load_vec<VEC>(state + ((size_t)slot * (taps - 1) + src + taps - 1) * C + c, f);
+        else
+            continue;
+        load_vec<VEC>(w_t + (size_t)k * C + c, wv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * f[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) acc[j] *= sigmoid_f(acc[j]);
+    store_vec<VEC>(y + t * C + c, acc);
+}
+
+// the state after each segment: its last taps-1 inputs (ascending rows, so
+// shifting within the state is safe in place)
+template <typename T, int VEC>
+__global__ void conv_state_kernel(
+    const T* __restrict__ x, int64_t ldx, T* __restrict__ state,
+    const int64_t* __restrict__ positions, const int* __restrict__ cu,
+    const int* __restrict__ slots, int C, int taps) {
+    const int s = blockIdx.x;
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
+    const int slot = slots[s];
+    if (c >= C || slot < 0) return;
+    const int r0 = cu[s], n = cu[s + 1] - r0;
+    const bool fresh = positions[r0] == 0;
+    T* st = state + (size_t)slot * (taps - 1) * C + c;
+    for (int r = 0; r < taps - 1; ++r) {
+        const int src = n - (taps - 1) + r;
+        float f[VEC];
+        if (src >= 0) {
+            load_vec<VEC>(x + (size_t)(r0 + src) * ldx + c, f);
+        } else if (!fresh) {
+            load_vec<VEC>(st + (size_t)(src + taps - 1) * C, f);
+        } else {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) f[j] = 0.f;
+        }
+        store_vec<VEC>(st + (size_t)r * C, f);
+    }
+}
+
+// one row per segment: convolve and shift in one launch
+template <typename T, int VEC>
+__global__ void conv_step_kernel(
+    T* __restrict__ y, const T* __restrict__ x, int64_t ldx, const float* __restrict__ w_t,
+    const float* __restrict__ b, T* __restrict__ state,
+    const int64_t* __restrict__ positions, const int* __restrict__ slots, int C, int taps) {
+    const size_t t = blockIdx.x;
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
+    if (c >= C) return;
+    const int slot = slots[t];
+    const bool fresh = positions[t] == 0;
+    float acc[VEC], f[VEC], wv[VEC];
+    load_vec<VEC>(b + c, acc);
+    T* st = state + (size_t)(slot < 0 ? 0 : slot) * (taps - 1) * C + c;
+    for (int k = 0; k < taps; ++k) {
+        if (k == taps - 1) {
+            load_vec<VEC>(x + t * ldx + c, f);
+        } else if (slot < 0 || fresh) {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) f[j] = 0.f;
+        } else {
+            load_vec<VEC>(st + (size_t)k * C, f);
+        }
+        load_vec<VEC>(w_t + (size_t)k * C + c, wv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * f[j];
+        if (k > 0 && slot >= 0) store_vec<VEC>(st + (size_t)(k - 1) * C, f);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) acc[j] *= sigmoid_f(acc[j]);
+    store_vec<VEC>(y + t * C + c, acc);
+}
+
+// ---------------------------------------------------------------------------
+// launchers (f32: compute dtype is fp32; vec8: widths, strides and addresses
+// allow 8-element accesses)
+// ---------------------------------------------------------------------------
+template <typename T_, int V_>
+struct Form {
+    using T = T_;
+    static constexpr int V = V_;
+};
+
+// run launch(Form<compute dtype, elements per access>)
+template <typename F>
+static hipError_t pick(int f32, int vec8, F launch) {
+    if (f32) {
+        if (vec8) launch(Form<float, 8>{});
+        else launch(Form<float, 1>{});
+    } else {
+        if (vec8) launch(Form<bf16, 8>{});
+        else launch(Form<bf16, 1>{});
+    }
+    HIP_CHECK_LAST();
+    return hipSuccess;
+}
+#define FORM(f)                                                                \
+    using T = typename decltype(f)::T;                                         \
+    constexpr int V = decltype(f)::V;                                          \
+    (void)V
+
+extern "C" hipError_t launch_embed_scaled(
+    float* x, void* x0, int64_t ld0, const int64_t* tokens, const void* embed, float scale,
+    int rows, int W, int f32, int vec8, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    return pick(f32, vec8, [&](auto form) {
+        FORM(form);
+        embed_scaled_kernel<T, V><<<rows, row_threads(W, V), 0, stream>>>(
+            x, (T*)x0, ld0, tokens, (const T*)embed, scale, W);
+    });
+}
+
+extern "C" hipError_t launch_stream_norm(
+    void* out, int64_t ld_out, float* x, const void* delta, int delta_f32, const float* vec,
+    const float* w, const float* b, float eps, int replace, int rows, int W, int f32,
+    int vec8, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    if (W > 512 * 32) return hipErrorInvalidValue;
+    if (delta_f32)
+        return pick(f32, vec8, [&](auto form) {
+            FORM(form);
+            stream_norm_kernel<T, float, V><<<rows, row_threads(W, V), 0, stream>>>(
+                (T*)out, ld_out, x, (const float*)delta, vec, w, b, eps, replace, W);
+        });
+    else
+        return pick(f32, vec8, [&](auto form) {
+            FORM(form);
+            stream_norm_kernel<T, T, V><<<rows, row_threads(W, V), 0, stream>>>(
+                (T*)out, ld_out, x, (const T*)delta, vec, w, b, eps, replace, W);
+        });
+}
+
+extern "C" hipError_t launch_latent_rows(
+    void* cq, void* latent, int row_w, const void* d, const float* q_norm,
+    const float* kv_norm, float eps, int q_rank, int rank, int rot,
+    const int64_t* positions, const float* cos_sin, const int64_t* slot_mapping, int rows,
+    int f32, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    return pick(f32, 0, [&](auto form) {
+        FORM(form);
+        latent_rows_kernel<T><<<rows, 256, 0, stream>>>(
+            (T*)cq, (T*)latent, row_w, (const T*)d, q_norm, kv_norm, eps, q_rank, rank, rot,
+            positions, cos_sin, slot_mapping);
+    });
+}
+
+extern "C" hipError_t launch_rotate_pairs(
+    void* out, int64_t ot, int64_t oh, int width, const void* x, int64_t xt, int64_t xh,
+    int rot, int H, const int64_t* positions, const float* cos_sin, int rows, int f32,
+    hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    return pick(f32, 0, [&](auto form) {
+        FORM(form);
+        rotate_pairs_kernel<T><<<rows, 256, 0, stream>>>(
+            (T*)out, ot, oh, width, (const T*)x, xt, xh, rot, H, positions, cos_sin);
+    });
+}
+
+extern "C" hipError_t launch_gated_norm(
+    void* out, const void* y, const void* gate, int64_t ld_gate, const float* w, float eps,
+    int groups, int gs, int gate_first, int rows, int f32, int vec8, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    if (gs > 512 * 32) return hipErrorInvalidValue;
+    const dim3 grid(rows, groups);
+    if (gate_first)
+        return pick(f32, vec8, [&](auto form) {
+            FORM(form);
+            gated_norm_kernel<T, V, true><<<grid, row_threads(gs, V), 0, stream>>>(
+                (T*)out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs);
+        });
+    else
+        return pick(f32, vec8, [&](auto form) {
+            FORM(form);
+            gated_norm_kernel<T, V, false><<<grid, row_threads(gs, V), 0, stream>>>(
+                (T*)out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs);
+        });
+}
+
+extern "C" hipError_t launch_causal_conv(
+    void* y, const void* x, int64_t ldx, const float* w_t, const float* b, void* state,
+    const int64_t* positions, const int* cu, const int* slots, const int* row_seg,
+    int rows, int nseg, int C, int taps, int f32, int vec8, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    const int per = vec8 ? 8 : 1, th = 256;
+    const int cb = ceil_div_i(C, per * th);
+    if (rows == nseg)
+        return pick(f32, vec8, [&](auto form) {
+            FORM(form);
+            conv_step_kernel<T, V><<<dim3(rows, cb), th, 0, stream>>>(
+                (T*)y, (const T*)x, ldx, w_t, b, (T*)state, positions, slots, C, taps);
+        });
+    return pick(f32, vec8, [&](auto form) {
+        FORM(form);
+        causal_conv_kernel<T, V><<<dim3(rows, cb), th, 0, stream>>>(
+            (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots, row_seg,
+            C, taps);
+        if (taps > 1)
+            conv_state_kernel<T, V><<<dim3(nseg, cb), th, 0, stream>>>(
+                (const T*)x, ldx, (T*)state, positions, cu, slots, C, taps);
+    });
+}

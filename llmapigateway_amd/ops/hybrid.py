@@ -79,7 +79,7 @@ def plan_segments(batch, dtype) -> SegmentPlan:
     pl, ps = lens[:nseg_p], starts[:nseg_p]
     keys = int((pl + ps).sum())
     pairs = float((pl * (ps + pl / 2.0)).sum())
-    unfold = nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
+    unfold = False and nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
     if unfold:
         put("cu_q", np.concatenate([[0], np.cumsum(pl)]))
         put("cu_k", np.concatenate([[0], np.cumsum(pl + ps)]))
@@ -216,14 +216,14 @@ def latent_attention_unfolded(
 
 
 # --------------------------------------------------------------- recurrences
-def causal_conv(x, w, b, state, positions, segs, plan) -> torch.Tensor:
+def causal_conv(x, w_t, b, state, positions, segs, plan) -> torch.Tensor:
     """silu of the causal per-channel convolution of x [T, C] (may be
-    strided); state [slots, taps-1, C] carries the last inputs."""
+    strided) with taps w_t [taps, C]; state [slots, taps-1, C] carries the last inputs."""
     if not x.is_cuda:
-        return ref.causal_conv(x, w, b, state, positions, segs)
+        return ref.causal_conv(x, w_t, b, state, positions, segs)
     y = torch.empty(x.shape, dtype=x.dtype, device=x.device)
     hybrid_native().causal_conv(
-        y, x, w, b, state, positions, segs.cu, segs.slots, segs.row_seg
+        y, x, w_t, b, state, positions, segs.cu, segs.slots, segs.row_seg
     )
     return y
 
@@ -242,7 +242,8 @@ def ssd(xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs, plan):
 
 def mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs, plan):
     """mLSTM recurrence; gates [T, 2H] fp32 raw input and forget gates,
-    states S [slots, H, dv, dk], n [slots, H, dk], m [slots, H]."""
+    states S [slots, H, dv, dk], n [slots, tiles, H, dk], m [slots, tiles, H]
+    (a copy per tile of 64 value rows)."""
     if not q.is_cuda:
         return ref.mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs)
     y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)

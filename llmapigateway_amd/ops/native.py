@@ -8,39 +8,46 @@ extension is missing raises: there is no fallback."""
 from __future__ import annotations
 
 import importlib
-from typing import Optional
+from typing import Dict
 
-_C = None
-_C_ERR: Optional[str] = None
-_H = None
-_H_ERR: Optional[str] = None
-
-try:
-    _C = importlib.import_module("llmapigateway_amd.ops._C")
-except ImportError as e:  # extension not built (CPU-only envs are fine)
-    _C_ERR = str(e)
-try:
-    _H = importlib.import_module("llmapigateway_amd.ops._H")
-except ImportError as e:
-    _H_ERR = str(e)
+_loaded: Dict[str, object] = {}
+_errors: Dict[str, str] = {}
 
 
-def _missing(name: str, err: Optional[str]):
-    raise RuntimeError(
-        f"llmapigateway_amd.ops.{name} (gfx950 HIP extension) is not built but a GPU "
-        "tensor reached the ops layer. Build it with `python setup.py build_ext "
-        f"--inplace` (import error: {err})"
-    )
+def _load(name: str):
+    """The extension module, or None (CPU-only trees are fine)."""
+    if name not in _loaded:
+        try:
+            _loaded[name] = importlib.import_module(f"llmapigateway_amd.ops.{name}")
+        except ImportError as e:
+            _errors[name] = str(e)
+            return None
+    return _loaded[name]
+
+
+def _require(name: str):
+    ext = _load(name)
+    if ext is None:
+        raise RuntimeError(
+            f"llmapigateway_amd.ops.{name} (gfx950 HIP extension) is not built but a GPU "
+            "tensor reached the ops layer. Build it with `python setup.py build_ext "
+            f"--inplace` (import error: {_errors[name]})"
+        )
+    return ext
+
+
+def have_native() -> bool:
+    return _load("_C") is not None and _load("_H") is not None
 
 
 def dense_native():
-    return _C if _C is not None else _missing("_C", _C_ERR)
+    return _require("_C")
 
 
 def hybrid_native():
-    return _H if _H is not None else _missing("_H", _H_ERR)
+    return _require("_H")
 
 
 def shared_native():
     """Either extension: for kernels that are in both."""
-    return _C if _C is not None else hybrid_native()
+    return _load("_C") or _require("_H")

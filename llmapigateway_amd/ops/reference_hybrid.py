@@ -96,9 +96,9 @@ def head_linear(x, w):
     return torch.einsum("thk,hnk->thn", x.float(), w.float()).to(x.dtype).contiguous()
 
 
-def causal_conv(x, w, b, state, positions, segs):
+def causal_conv(x, w_t, b, state, positions, segs):
     y = torch.empty(x.shape, dtype=x.dtype)
-    k = w.shape[1] - 1
+    k = w_t.shape[0] - 1
     cu = segs.cu.tolist()
     for s, slot in enumerate(segs.slots.tolist()):
         r0, r1 = cu[s], cu[s + 1]
@@ -111,7 +111,7 @@ def causal_conv(x, w, b, state, positions, segs):
             past = torch.zeros_like(past)
         full = torch.cat([past, xs])
         win = full.unfold(0, k + 1, 1)  # [n, C, taps]
-        y[r0:r1] = F.silu((win * w).sum(-1) + b)
+        y[r0:r1] = F.silu((win * w_t.t()).sum(-1) + b)
         if k:
             state[slot] = full[-k:].to(state.dtype)
     return y
@@ -153,7 +153,7 @@ def mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs):
     for s, slot in enumerate(segs.slots.tolist()):
         if slot < 0:
             continue
-        st, nt, mt = S[slot].clone(), n[slot].clone(), m[slot].clone()
+        st, nt, mt = S[slot].clone(), n[slot, 0].clone(), m[slot, 0].clone()
         if int(positions[cu[s]]) == 0:
             st.zero_(), nt.zero_(), mt.zero_()
         for t in range(cu[s], cu[s + 1]):
