@@ -64,6 +64,7 @@ class LatentAttention:
         }
         self.uk_t = uk.transpose(1, 2).contiguous()            # [H, rank, dim]
         self.uv = uv.view(self.H, self.vdim, self.rank)        # [H, vdim, rank]
+        self.unfolds = ops.can_unfold(self.dim, self.rot, self.vdim, self.rank)
         add_decode_twins(self.w, ("down", "uq", "o"))
 
     @staticmethod
@@ -90,24 +91,24 @@ class LatentAttention:
             batch.positions, self.cos_sin, latent, batch.slot_mapping,
         )
         q = ops.linear(cq, w["uq"], w.get("uq_swz")).view(T, self.H, self.dim + self.rot)
-        if plan.unfold is not None:
+        if plan.unfold is not None and self.unfolds:
             out = ops.latent_attention_unfolded(
                 q, latent, w["ukv"], self.sink, self.scale, self.dim, self.vdim,
                 self.rank, self.cos_sin, batch.positions, plan.unfold,
             )
             Tu = plan.unfold.rows
             if Tu < T:
-                out[Tu:] = self._folded(q[Tu:], latent, batch, plan)
+                out[Tu:] = self._folded(q[Tu:], latent, batch, Tu)
         else:
-            out = self._folded(q, latent, batch, plan)
+            out = self._folded(q, latent, batch, 0)
         return ops.linear(out.view(T, self.H * self.vdim), w["o"], w.get("o_swz"))
 
-    def _folded(self, q, latent, batch, plan) -> torch.Tensor:
-        pos = batch.positions[plan.folded_from :]
+    def _folded(self, q, latent, batch, row0: int) -> torch.Tensor:
+        pos = batch.positions[row0:]
         ql = ops.fold_queries(q, self.uk_t, self.row, self.cos_sin, pos)
         o = ops.latent_attention_folded(
             ql, latent, self.rank, self.sink, self.scale, pos, batch.segs,
-            plan.folded_from,
+            row0,
         )
         return ops.head_linear(o, self.uv)
 

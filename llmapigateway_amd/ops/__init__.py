@@ -548,6 +548,7 @@ from .hybrid import (  # noqa: E402
     add_cast,
     add_layernorm,
     build_pair_rope_cache,
+    can_unfold,
     causal_conv,
     embed_scaled,
     fold_queries,
@@ -583,6 +584,7 @@ __all__ = [
     "add_cast",
     "add_layernorm",
     "build_pair_rope_cache",
+    "can_unfold",
     "causal_conv",
     "embed_scaled",
     "fold_queries",

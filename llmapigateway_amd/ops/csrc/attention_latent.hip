@@ -2,9 +2,9 @@
 // latent rows [c (rank) | rotated key part | zero pad].
 //
 // Folded form: queries are already in the latent space, one cached row is
-// key and value of every head.
+// key and value of every head. Unfolded form: per-head keys and values.
 
-#include "common.h"
+#include "mfma.h"
 
 #define LA_THREADS 256
 
@@ -113,4 +113,406 @@ extern "C" hipError_t launch_latent_folded_any(
                                    rows, H, rank, row_w, block_size, max_blocks, stream)
                : folded_any<bf16>(out, q, latent, sink, scale, positions, row_seg, tables,
                                   rows, H, rank, row_w, block_size, max_blocks, stream);
+}
+
+// ---------------------------------------------------------------------------
+// Folded form on MFMA (bf16). One workgroup: one row, 16 heads, one split of
+// the row's keys; tiles of 64 keys, 16 a wave.
+//   scores: a wave's own 16 cached rows come from global memory straight as
+//     B fragments (prefetched a tile ahead) against the query fragments;
+//   sums: the same registers go to LDS once, and every wave multiplies the
+//     tile's weights with its share of the latent dimensions (transposing
+//     LDS reads).
+// One split writes the output (softmax started from the sink); several write
+// partials that latent_combine_kernel merges with the sink. Splits divide
+// the row's own key count, so a launch of fixed shape (captured graphs)
+// balances at every context length.
+// ---------------------------------------------------------------------------
+#define LF_KT 64
+#define LA_NEG (-1e30f)
+
+template <int NKC>  // 32-wide chunks that cover a cached row
+__launch_bounds__(256)
+__global__ void latent_folded_mfma_kernel(
+    bf16* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml,
+    const bf16* __restrict__ q, const bf16* __restrict__ latent,
+    const float* __restrict__ sink, float scale, const int64_t* __restrict__ positions,
+    const int* __restrict__ row_seg, const int* __restrict__ tables, int max_blocks,
+    int block_size, int H, int rank, int row_w, int nsplit) {
+    constexpr int LDK = NKC * 32 + 8;
+    constexpr int NT = (NKC * 32 + 63) / 64;  // 16-dim tiles of the sums per wave
+    __shared__ bf16 k_lds[LF_KT][LDK];
+    __shared__ bf16 p_lds[16][LF_KT + 8];
+    __shared__ float mx_lds[2][4][16];
+    __shared__ float l_lds[4][16];
+    const size_t t = blockIdx.x;
+    const int h0 = blockIdx.y * 16, split = blockIdx.z;
+    const int n = (int)positions[t] + 1;
+    const int span = (n + nsplit * LF_KT - 1) / (nsplit * LF_KT) * LF_KT;
+    const int key_lo = split * span, key_hi = min(n, key_lo + span);
+    const int* bt = tables + (size_t)row_seg[t] * max_blocks;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int r16 = lane & 15, g = lane >> 4;
+
+    bf16x8 qf[NKC];
+    {
+        const bf16* qr = q + (t * H + min(h0 + r16, H - 1)) * row_w;
+#pragma unroll
+        for (int c = 0; c < NKC; ++c) {
+            uint4 v = {0, 0, 0, 0};
+            if (c * 32 + g * 8 < row_w)
+                v = *reinterpret_cast<const uint4*>(qr + c * 32 + g * 8);
+            qf[c] = as_frag(v);
+        }
+    }
+    float m[4], l[4];
+    f32x4 acc[NT];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const int h = min(h0 + g * 4 + r, H - 1);
+        m[r] = nsplit == 1 ? sink[h] : LA_NEG;
+        l[r] = nsplit == 1 && wave == 0 && r16 == 0 ? 1.f : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+
+    uint4 kr[NKC];
+    auto load_tile = [&](int k0) {
+        const int key = k0 + wave * 16 + r16;
+        const bool in = key < key_hi;
+        const bf16* src = latent;
+        if (in) src += ((size_t)bt[key / block_size] * block_size + key % block_size) * row_w;
+#pragma unroll
+        for (int c = 0; c < NKC; ++c) {
+            kr[c] = (uint4){0, 0, 0, 0};
+            if (in && c * 32 + g * 8 < row_w)
+                kr[c] = *reinterpret_cast<const uint4*>(src + c * 32 + g * 8);
+        }
+    };
+    if (key_lo < key_hi) load_tile(key_lo);
+    int par = 0;
+    for (int k0 = key_lo; k0 < key_hi; k0 += LF_KT, par ^= 1) {
+        f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int c = 0; c < NKC; ++c) s = mfma16(qf[c], as_frag(kr[c]), s);
+#pragma unroll
+        for (int c = 0; c < NKC; ++c)
+            *reinterpret_cast<uint4*>(&k_lds[wave * 16 + r16][c * 32 + g * 8]) = kr[c];
+        if (k0 + LF_KT < key_hi) load_tile(k0 + LF_KT);
+        const bool in = k0 + wave * 16 + r16 < key_hi;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            s[r] = in ? s[r] * scale : LA_NEG;
+            const float v = group16_reduce_max(s[r]);
+            if (r16 == 0) mx_lds[par][wave][g * 4 + r] = v;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int row = g * 4 + r;
+            const float m_new = fmaxf(
+                m[r], fmaxf(fmaxf(mx_lds[par][0][row], mx_lds[par][1][row]),
+                            fmaxf(mx_lds[par][2][row], mx_lds[par][3][row])));
+            const float f = __expf(m[r] - m_new);
+            const float p = in ? __expf(s[r] - m_new) : 0.f;
+            l[r] = l[r] * f + p;
+            m[r] = m_new;
+            p_lds[row][wave * 16 + r16] = f2bf(p);
+#pragma unroll
+            for (int j = 0; j < NT; ++j) acc[j][r] *= f;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int c = 0; c < LF_KT / 32; ++c) {
+            const bf16x8 pf = *reinterpret_cast<const bf16x8*>(&p_lds[r16][c * 32 + g * 8]);
+#pragma unroll
+            for (int j = 0; j < NT; ++j) {
+                const int d0 = (wave * NT + j) * 16;
+                if (d0 < rank)
+                    acc[j] = mfma16(pf, tr_frag(&k_lds[0][0], LDK, c * 32, d0), acc[j]);
+            }
+        }
+        __syncthreads();
+    }
+    // the waves' shares of the denominator
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const float v = group16_reduce_sum(l[r]);
+        if (r16 == 0) l_lds[wave][g * 4 + r] = v;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const int row = g * 4 + r, h = h0 + row;
+        if (h >= H) continue;
+        const float lt = l_lds[0][row] + l_lds[1][row] + l_lds[2][row] + l_lds[3][row];
+        const size_t th = t * H + h, pb = th * nsplit + split;
+        const float inv = 1.f / lt;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            const int d = (wave * NT + j) * 16 + r16;
+            if (d >= rank) continue;
+            if (nsplit == 1) stf(out + th * rank + d, acc[j][r] * inv);
+            else part_acc[pb * rank + d] = acc[j][r];
+        }
+        if (nsplit > 1 && wave == 0 && r16 == 0) {
+            part_ml[pb * 2] = m[r];
+            part_ml[pb * 2 + 1] = lt;
+        }
+    }
+}
+
+__global__ void latent_combine_kernel(
+    bf16* __restrict__ out, const float* __restrict__ part_acc,
+    const float* __restrict__ part_ml, const float* __restrict__ sink, int H, int rank,
+    int nsplit) {
+    const size_t th = blockIdx.x;
+    const float sk = sink[th % H];
+    float M = sk;
+    for (int s = 0; s < nsplit; ++s) M = fmaxf(M, part_ml[(th * nsplit + s) * 2]);
+    float den = __expf(sk - M);
+    for (int s = 0; s < nsplit; ++s)
+        den += part_ml[(th * nsplit + s) * 2 + 1] * __expf(part_ml[(th * nsplit + s) * 2] - M);
+    for (int d = threadIdx.x; d < rank; d += blockDim.x) {
+        float a = 0.f;
+        for (int s = 0; s < nsplit; ++s)
+            a += part_acc[(th * nsplit + s) * rank + d] *
+                 __expf(part_ml[(th * nsplit + s) * 2] - M);
+        stf(out + th * rank + d, a / den);
+    }
+}
+
+extern "C" hipError_t launch_latent_folded_mfma(
+    void* out, float* part_acc, float* part_ml, const void* q, const void* latent,
+    const float* sink, float scale, const int64_t* positions, const int* row_seg,
+    const int* tables, int rows, int H, int rank, int row_w, int block_size, int max_blocks,
+    int nsplit, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    if (row_w % 8 || row_w > 576 || (nsplit > 1 && (!part_acc || !part_ml)))
+        return hipErrorInvalidValue;
+    const dim3 grid(rows, ceil_div_i(H, 16), nsplit);
+#define GO(NKC)                                                                           \
+    latent_folded_mfma_kernel<NKC><<<grid, 256, 0, stream>>>(                             \
+        (bf16*)out, part_acc, part_ml, (const bf16*)q, (const bf16*)latent, sink, scale,  \
+        positions, row_seg, tables, max_blocks, block_size, H, rank, row_w, nsplit)
+    if (row_w <= 128) GO(4);
+    else if (row_w <= 192) GO(6);
+    else if (row_w <= 320) GO(10);
+    else GO(18);
+#undef GO
+    HIP_CHECK_LAST();
+    if (nsplit > 1) {
+        latent_combine_kernel<<<rows * H, 128, 0, stream>>>(
+            (bf16*)out, part_acc, part_ml, sink, H, rank, nsplit);
+        HIP_CHECK_LAST();
+    }
+    return hipSuccess;
+}
+
+// ---------------------------------------------------------------------------
+// Unfolded form (bf16): flash attention over per-head keys [unrotated |
+// shared rotated part] and values. Query rows of a segment are its last
+// cu_q[s+1]-cu_q[s] positions, its keys all cu_k[s+1]-cu_k[s]. One workgroup:
+// 64*MR query rows of one head, 16*MR a wave; keys in tiles of 64, loaded to
+// registers a tile ahead and staged in LDS (values are read transposed). The
+// head varies fastest over the grid, so a head's keys stay in one XCD's L2.
+// ---------------------------------------------------------------------------
+template <int NDQ, int NDV, int MR>  // 32-chunks of a query, 16-tiles of a value
+__launch_bounds__(256)
+__global__ void latent_unfolded_kernel(
+    bf16* __restrict__ out, const bf16* __restrict__ q, const bf16* __restrict__ kv,
+    const bf16* __restrict__ lat, int64_t lat_row, const float* __restrict__ sink, float scale,
+    const int* __restrict__ cu_q, const int* __restrict__ cu_k,
+    const int* __restrict__ tile_seg, const int* __restrict__ tile_off, int H, int dim,
+    int rot, int vdim, int rank) {
+    constexpr int LDQ = NDQ * 32 + 8, LDV = NDV * 16 + 8, LDP = 64 + 8;
+    __shared__ bf16 k_lds[64][LDQ];
+    __shared__ bf16 v_lds[64][LDV];
+    __shared__ bf16 p_lds[4][16 * MR][LDP];
+    const int h = blockIdx.x % H, tile = blockIdx.x / H;
+    const int seg = tile_seg[tile], off = tile_off[tile];
+    const int q0 = cu_q[seg], nq = cu_q[seg + 1] - q0;
+    const int kbase = cu_k[seg], nk = cu_k[seg + 1] - kbase;
+    const int ctx = nk - nq;  // position of the segment's first query row
+    const int dq = dim + rot;
+    const size_t ldkv = (size_t)H * (dim + vdim);
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int r16 = lane & 15, g = lane >> 4;
+    const int wrow0 = off + wave * 16 * MR;
+
+    bf16x8 qf[MR][NDQ];
+#pragma unroll
+    for (int i = 0; i < MR; ++i) {
+        const bf16* qr = q + ((size_t)(q0 + min(wrow0 + i * 16 + r16, nq - 1)) * H + h) * dq;
+#pragma unroll
+        for (int c = 0; c < NDQ; ++c) {
+            uint4 v = {0, 0, 0, 0};
+            if (c * 32 + g * 8 < dq) v = *reinterpret_cast<const uint4*>(qr + c * 32 + g * 8);
+            qf[i][c] = as_frag(v);
+        }
+    }
+    float m[MR][4], l[MR][4];
+    f32x4 acc[MR][NDV];
+    const float sk = sink[h];
+#pragma unroll
+    for (int i = 0; i < MR; ++i) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            m[i][r] = sk;
+            l[i][r] = r16 == 0 ? 1.f : 0.f;  // the sink, once per row
+        }
+#pragma unroll
+        for (int j = 0; j < NDV; ++j) acc[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    }
+    constexpr int KV = (64 * NDQ * 4) / 256, VV = (64 * NDV * 2) / 256;
+    uint4 kreg[KV], vreg[VV];
+    auto load_tile = [&](int k0) {
+#pragma unroll
+        for (int c = 0; c < KV; ++c) {
+            const int e = tid + c * 256, key = k0 + e / (NDQ * 4), d = e % (NDQ * 4) * 8;
+            kreg[c] = (uint4){0, 0, 0, 0};
+            if (key < nk && d < dq) {
+                const bf16* src = d < dim
+                    ? kv + (size_t)(kbase + key) * ldkv + (size_t)h * dim + d
+                    : lat + (size_t)(kbase + key) * lat_row + rank + d - dim;
+                kreg[c] = *reinterpret_cast<const uint4*>(src);
+            }
+        }
+#pragma unroll
+        for (int c = 0; c < VV; ++c) {
+            const int e = tid + c * 256, key = k0 + e / (NDV * 2), d = e % (NDV * 2) * 8;
+            vreg[c] = (uint4){0, 0, 0, 0};
+            if (key < nk && d < vdim)
+                vreg[c] = *reinterpret_cast<const uint4*>(
+                    kv + (size_t)(kbase + key) * ldkv + (size_t)H * dim + (size_t)h * vdim + d);
+        }
+    };
+    const int key_end = ctx + min(nq, off + 64 * MR);  // keys any row here sees
+    load_tile(0);
+    for (int k0 = 0; k0 < key_end; k0 += 64) {
+        __syncthreads();
+#pragma unroll
+        for (int c = 0; c < KV; ++c) {
+            const int e = tid + c * 256;
+            *reinterpret_cast<uint4*>(&k_lds[e / (NDQ * 4)][e % (NDQ * 4) * 8]) = kreg[c];
+        }
+#pragma unroll
+        for (int c = 0; c < VV; ++c) {
+            const int e = tid + c * 256;
+            *reinterpret_cast<uint4*>(&v_lds[e / (NDV * 2)][e % (NDV * 2) * 8]) = vreg[c];
+        }
+        __syncthreads();
+        if (k0 + 64 < key_end) load_tile(k0 + 64);
+        if (k0 > ctx + wrow0 + 16 * MR - 1) continue;  // all masked for this wave
+        f32x4 s[MR][4];
+#pragma unroll
+        for (int i = 0; i < MR; ++i)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) s[i][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int c = 0; c < NDQ; ++c) {
+                const bf16x8 kf =
+                    *reinterpret_cast<const bf16x8*>(&k_lds[u * 16 + r16][c * 32 + g * 8]);
+#pragma unroll
+                for (int i = 0; i < MR; ++i) s[i][u] = mfma16(qf[i][c], kf, s[i][u]);
+            }
+        const bool edge = k0 + 63 > ctx + wrow0;  // some row does not see all keys
+#pragma unroll
+        for (int i = 0; i < MR; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int pos = ctx + wrow0 + i * 16 + g * 4 + r;
+                float mx = LA_NEG;
+#pragma unroll
+                for (int u = 0; u < 4; ++u) {
+                    float v = s[i][u][r] * scale;
+                    if (edge && k0 + u * 16 + r16 > pos) v = LA_NEG;
+                    s[i][u][r] = v;
+                    mx = fmaxf(mx, v);
+                }
+                const float m_new = fmaxf(m[i][r], group16_reduce_max(mx));
+                const float f = __expf(m[i][r] - m_new);
+                m[i][r] = m_new;
+                float sum = 0.f;
+#pragma unroll
+                for (int u = 0; u < 4; ++u) {
+                    const float p = __expf(s[i][u][r] - m_new);
+                    sum += p;
+                    p_lds[wave][i * 16 + g * 4 + r][u * 16 + r16] = f2bf(p);
+                }
+                l[i][r] = l[i][r] * f + sum;
+#pragma unroll
+                for (int j = 0; j < NDV; ++j) acc[i][j][r] *= f;
+            }
+        // a wave reads back its own weights: no barrier
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+            bf16x8 pf[MR];
+#pragma unroll
+            for (int i = 0; i < MR; ++i)
+                pf[i] = *reinterpret_cast<const bf16x8*>(
+                    &p_lds[wave][i * 16 + r16][c * 32 + g * 8]);
+#pragma unroll
+            for (int j = 0; j < NDV; ++j) {
+                const bf16x8 vf = tr_frag(&v_lds[0][0], LDV, c * 32, j * 16);
+#pragma unroll
+                for (int i = 0; i < MR; ++i) acc[i][j] = mfma16(pf[i], vf, acc[i][j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < MR; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float inv = 1.f / group16_reduce_sum(l[i][r]);
+            const int row = wrow0 + i * 16 + g * 4 + r;
+            if (row >= nq) continue;
+            bf16* o = out + ((size_t)(q0 + row) * H + h) * vdim;
+#pragma unroll
+            for (int j = 0; j < NDV; ++j)
+                if (j * 16 + r16 < vdim) stf(o + j * 16 + r16, acc[i][j][r] * inv);
+        }
+}
+
+template <int NDQ, int NDV>
+static void unfolded_go(
+    bf16* out, const bf16* q, const bf16* kv, const bf16* lat, int64_t lat_row,
+    const float* sink, float scale, const int* cu_q, const int* cu_k, const int* tile_seg,
+    const int* tile_off, int ntiles, int tile_rows, int H, int dim, int rot, int vdim,
+    int rank, hipStream_t stream) {
+    if (tile_rows == 128)
+        latent_unfolded_kernel<NDQ, NDV, 2><<<ntiles * H, 256, 0, stream>>>(
+            out, q, kv, lat, lat_row, sink, scale, cu_q, cu_k, tile_seg, tile_off, H, dim,
+            rot, vdim, rank);
+    else
+        latent_unfolded_kernel<NDQ, NDV, 1><<<ntiles * H, 256, 0, stream>>>(
+            out, q, kv, lat, lat_row, sink, scale, cu_q, cu_k, tile_seg, tile_off, H, dim,
+            rot, vdim, rank);
+}
+
+extern "C" hipError_t launch_latent_unfolded(
+    void* out, const void* q, const void* kv, const void* lat, int64_t lat_row,
+    const float* sink, float scale, const int* cu_q, const int* cu_k, const int* tile_seg,
+    const int* tile_off, int ntiles, int tile_rows, int H, int dim, int rot, int vdim,
+    int rank, hipStream_t stream) {
+    if (ntiles <= 0) return hipSuccess;
+    if (dim % 8 || rot % 8 || vdim % 8 || rank % 8 || lat_row % 8 ||
+        (tile_rows != 64 && tile_rows != 128))
+        return hipErrorInvalidValue;
+    const int dq = dim + rot;
+#define GO(A, B)                                                                         \
+    unfolded_go<A, B>((bf16*)out, (const bf16*)q, (const bf16*)kv, (const bf16*)lat,     \
+                      lat_row, sink, scale, cu_q, cu_k, tile_seg, tile_off, ntiles,      \
+                      tile_rows, H, dim, rot, vdim, rank, stream)
+    if (dq <= 64 && vdim <= 64) GO(2, 4);
+    else if (dq <= 96 && vdim <= 64) GO(3, 4);
+    else if (dq <= 128 && vdim <= 128) GO(4, 8);
+    else if (dq <= 192 && vdim <= 128) GO(6, 8);
+    else if (dq <= 256 && vdim <= 256) GO(8, 16);
+    else return hipErrorInvalidValue;
+#undef GO
+    HIP_CHECK_LAST();
+    return hipSuccess;
 }

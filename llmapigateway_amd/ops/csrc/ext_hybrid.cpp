@@ -13,6 +13,8 @@ hipError_t launch_gated_norm(void*, const void*, const void*, int64_t, const flo
 hipError_t launch_causal_conv(void*, const void*, int64_t, const float*, const float*, void*, const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_head_linear(void*, int64_t, int64_t, const void*, int64_t, int64_t, const void*, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_latent_folded_any(void*, const void*, const void*, const float*, float, const int64_t*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
+hipError_t launch_latent_folded_mfma(void*, float*, float*, const void*, const void*, const float*, float, const int64_t*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
+hipError_t launch_latent_unfolded(void*, const void*, const void*, const void*, int64_t, const float*, float, const int*, const int*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_ssd_scan(void*, const void*, int64_t, const float*, const float*, const float*, const float*, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
 hipError_t launch_mlstm_scan(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*, const float*, float, float, int, int, int, float*, float*, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
 }
@@ -174,7 +176,8 @@ void head_linear(Tensor y, Tensor x, Tensor w) {
 }
 
 void latent_attention_folded(Tensor out, Tensor q, Tensor latent, Tensor sink, double scale,
-                             Tensor positions, Tensor row_seg, Tensor tables) {
+                             Tensor positions, Tensor row_seg, Tensor tables,
+                             int64_t nsplit, OptTensor part_acc, OptTensor part_ml) {
     const bool f32 = is_f32(q, "q");
     same_type(q, latent, "latent");
     same_type(q, out, "out");
@@ -183,11 +186,54 @@ void latent_attention_folded(Tensor out, Tensor q, Tensor latent, Tensor sink, d
     const int64_t T = q.size(0), H = q.size(1), rank = out.size(2);
     TORCH_CHECK(out.size(0) == T && out.size(1) == H && rank <= latent.size(2));
     TORCH_CHECK(tables.dim() == 2);
+    if (nsplit > 0) {  // MFMA form
+        float *pa = nullptr, *pm = nullptr;
+        if (nsplit > 1) {
+            TORCH_CHECK(has(part_acc) && has(part_ml));
+            TORCH_CHECK(part_acc->numel() >= T * H * nsplit * rank &&
+                        part_ml->numel() >= T * H * nsplit * 2, "folded: scratch too small");
+            f32_ptr(*part_acc, part_acc->numel(), "part_acc");
+            f32_ptr(*part_ml, part_ml->numel(), "part_ml");
+            pa = part_acc->data_ptr<float>();
+            pm = part_ml->data_ptr<float>();
+        }
+        TORCH_CHECK(!f32 && vec8({&q, &latent}, {q.size(2)}) && q.size(2) <= 576);
+        CHECK_HIP(launch_latent_folded_mfma(
+            out.data_ptr(), pa, pm, q.data_ptr(), latent.data_ptr(), f32_ptr(sink, H, "sink"),
+            (float)scale, i64_ptr(positions, T, "positions"),
+            i32_ptr(row_seg, T, "row_seg"), i32_ptr(tables, 1, "tables"), T, H, rank,
+            q.size(2), latent.size(1), tables.size(1), nsplit, current_stream()));
+        return;
+    }
     CHECK_HIP(launch_latent_folded_any(
         out.data_ptr(), q.data_ptr(), latent.data_ptr(), f32_ptr(sink, H, "sink"),
         (float)scale, i64_ptr(positions, T, "positions"), i32_ptr(row_seg, T, "row_seg"),
         i32_ptr(tables, 1, "tables"), T, H, rank, q.size(2), latent.size(1), tables.size(1),
         f32, current_stream()));
+}
+
+void latent_attention_unfolded(Tensor out, Tensor q, Tensor kv, Tensor lat, Tensor sink,
+                               double scale, Tensor cu_q, Tensor cu_k, Tensor tile_seg,
+                               Tensor tile_off, int64_t tile_rows, int64_t dim, int64_t vdim,
+                               int64_t rank) {
+    check_bf16(q, "q");
+    check_bf16(kv, "kv");
+    check_bf16(lat, "lat");
+    check_bf16(out, "out");
+    TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && out.is_contiguous());
+    const int64_t H = q.size(1), rot = q.size(2) - dim, keys = lat.size(0);
+    TORCH_CHECK(rot > 0 && out.numel() >= q.size(0) * H * vdim);
+    TORCH_CHECK(kv.is_contiguous() && kv.dim() == 2 && kv.size(0) == keys &&
+                kv.size(1) == H * (dim + vdim));
+    TORCH_CHECK(lat.is_contiguous() && lat.dim() == 2 && lat.size(1) >= rank + rot);
+    TORCH_CHECK(vec8({&q, &kv, &lat}, {dim, rot, vdim, rank, lat.size(1)}));
+    const int64_t S = cu_q.numel() - 1, nt = tile_seg.numel();
+    CHECK_HIP(launch_latent_unfolded(
+        out.data_ptr(), q.data_ptr(), kv.data_ptr(), lat.data_ptr(), lat.size(1),
+        f32_ptr(sink, H, "sink"), (float)scale, i32_ptr(cu_q, S + 1, "cu_q"),
+        i32_ptr(cu_k, S + 1, "cu_k"), i32_ptr(tile_seg, nt, "tile_seg"),
+        i32_ptr(tile_off, nt, "tile_off"), nt, tile_rows, H, dim, rot, vdim, rank,
+        current_stream()));
 }
 
 void causal_conv(Tensor y, Tensor x, Tensor w_t, Tensor b, Tensor state, Tensor positions,
@@ -291,6 +337,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("head_linear", &head_linear, "per-head products");
     m.def("latent_attention_folded", &latent_attention_folded,
           "paged attention in the latent space, with a sink");
+    m.def("latent_attention_unfolded", &latent_attention_unfolded,
+          "varlen causal attention over per-head keys and values, with a sink");
     m.def("causal_conv", &causal_conv, "segmented causal convolution + silu");
     m.def("ssd_scan", &ssd_scan, "Mamba-2 recurrence, token by token");
     m.def("mlstm_scan", &mlstm_scan, "mLSTM recurrence, token by token");

@@ -1,0 +1,39 @@
+// bf16 MFMA fragments on gfx950 (v_mfma_f32_16x16x32_bf16):
+//   A: lane l holds A[row = l&15][k = (l>>4)*8 + j], j = 0..7
+//   B: lane l holds B[k = (l>>4)*8 + j][col = l&15]
+//   C: lane l holds C[row = (l>>4)*4 + r][col = l&15], r = 0..3
+#pragma once
+
+#include "common.h"
+
+typedef __attribute__((__vector_size__(8 * sizeof(short)))) short bf16x8;
+typedef __attribute__((__vector_size__(4 * sizeof(short)))) short bf16x4;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4;
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+__device__ __forceinline__ bf16x8 as_frag(const uint4& v) {
+    return *reinterpret_cast<const bf16x8*>(&v);
+}
+
+// Fragment whose k runs over the rows of a row-major LDS tile (a B operand
+// stored [k][col], or an A operand stored [k][row]): rows k0..k0+31, columns
+// c0..c0+15. ds_read_b64_tr_b16 hands each lane of a 16-lane group one column
+// of a 4x16 block, so two reads make the 8 k values. Rows and c0 must keep
+// 8-byte alignment.
+__device__ __forceinline__ bf16x8 tr_frag(const bf16* tile, int stride, int k0, int c0) {
+    typedef __attribute__((address_space(3))) bf16x4* lds_ptr;
+    const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15;
+    const bf16* p = tile + (k0 + g * 8 + (i >> 2)) * stride + c0 + (i & 3) * 4;
+    const bf16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p);
+    const bf16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)(p + 4 * stride));
+    return (bf16x8){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+}
+
+// fp32 as a sum of two bf16 (16 mantissa bits): products of a fp32 operand
+// with bf16 data keep fp32-like accuracy in two MFMAs
+__device__ __forceinline__ void split_bf16(float v, uint16_t& hi, uint16_t& lo) {
+    hi = f2bfbits(v);
+    lo = f2bfbits(v - bfbits2f(hi));
+}

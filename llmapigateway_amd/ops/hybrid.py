@@ -32,6 +32,7 @@ class Unfold:
     cu_k: torch.Tensor        # [S+1] int32
     tile_seg: torch.Tensor    # [ntiles] int32
     tile_off: torch.Tensor    # [ntiles] int32
+    tile_rows: int            # query rows per tile
 
 
 @dataclass
@@ -50,7 +51,6 @@ class Chunks:
 class SegmentPlan:
     """How a step's rows go through the kernels; made once per step."""
 
-    folded_from: int = 0
     unfold: Optional[Unfold] = None
     chunks: Optional[Chunks] = None
 
@@ -79,12 +79,16 @@ def plan_segments(batch, dtype) -> SegmentPlan:
     pl, ps = lens[:nseg_p], starts[:nseg_p]
     keys = int((pl + ps).sum())
     pairs = float((pl * (ps + pl / 2.0)).sum())
-    unfold = False and nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
+    unfold = nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
     if unfold:
         put("cu_q", np.concatenate([[0], np.cumsum(pl)]))
         put("cu_k", np.concatenate([[0], np.cumsum(pl + ps)]))
-        put("tile_seg", np.repeat(np.arange(nseg_p), (pl + 63) // 64))
-        put("tile_off", np.concatenate([np.arange(0, n, 64) for n in pl]))
+        tile_rows = 128 if int(pl.max()) > 64 else 64
+        seg = np.repeat(np.arange(nseg_p), -(-pl // tile_rows))
+        off = np.concatenate([np.arange(0, n, tile_rows) for n in pl])
+        order = np.argsort(-(ps[seg] + off), kind="stable")  # longest first
+        put("tile_seg", seg[order])
+        put("tile_off", off[order])
     long = np.nonzero(lens >= CHUNK_MIN_ROWS)[0]
     nchunk = (lens[long] + CHUNK - 1) // CHUNK
     if len(long):
@@ -113,8 +117,8 @@ def plan_segments(batch, dtype) -> SegmentPlan:
             key_slots=tables[seg, pos // bs].long() * bs + pos % bs,
             cu_q=got["cu_q"], cu_k=got["cu_k"],
             tile_seg=got["tile_seg"], tile_off=got["tile_off"],
+            tile_rows=tile_rows,
         )
-        plan.folded_from = batch.n_prefill_tokens
     if len(long):
         plan.chunks = Chunks(
             segs=got["segs"], first=got["first"], chunk_seg=got["chunk_seg"],
@@ -202,17 +206,67 @@ def latent_attention_folded(ql, latent, rank, sink, scale, positions, segs, row0
         return ref.latent_attention_folded(
             ql, latent, rank, sink, scale, positions, segs, row0
         )
-    out = torch.empty(ql.shape[0], ql.shape[1], rank, dtype=ql.dtype, device=ql.device)
+    T, H, row = ql.shape
+    out = torch.empty(T, H, rank, dtype=ql.dtype, device=ql.device)
+    nsplit, pa, pm = 0, None, None
+    if ql.dtype == torch.bfloat16 and row <= 576:
+        # fill the chip: splits only from shapes, so captured graphs hold
+        max_tiles = -(-segs.tables.shape[1] * latent.shape[1] // 64)
+        nsplit = max(1, min(512 // (T * -(-H // 16)), 16, max_tiles))
+        if nsplit > 1:
+            pa, pm = _folded_scratch(ql.device, T * H * nsplit * rank, T * H * nsplit * 2)
     hybrid_native().latent_attention_folded(
-        out, ql, latent, sink, float(scale), positions, segs.row_seg[row0:], segs.tables
+        out, ql, latent, sink, float(scale), positions, segs.row_seg[row0:], segs.tables,
+        nsplit, pa, pm,
     )
     return out
 
 
-def latent_attention_unfolded(
-    q, latent, w_ukv, sink, scale, dim, vdim, rank, cos_sin, positions, u: Unfold
-):
-    raise NotImplementedError
+_scratch: dict = {}
+_scratch_retired: list = []
+
+
+def _folded_scratch(device, n_acc: int, n_ml: int):
+    """fp32 scratch shared by all launches of a device (stream order)."""
+    ws = _scratch.get(device.index)
+    if ws is None or ws[0].numel() < n_acc or ws[1].numel() < n_ml:
+        if ws is not None:
+            _scratch_retired.append(ws)  # captured graphs may still use it
+            n_acc, n_ml = max(n_acc, ws[0].numel()), max(n_ml, ws[1].numel())
+        ws = (
+            torch.empty(n_acc, dtype=torch.float32, device=device),
+            torch.empty(n_ml, dtype=torch.float32, device=device),
+        )
+        _scratch[device.index] = ws
+    return ws
+
+
+def can_unfold(dim: int, rot: int, vdim: int, rank: int) -> bool:
+    """Whether latent_attention_unfolded has a kernel for these sizes."""
+    return (
+        all(d % 8 == 0 for d in (dim, rot, vdim, rank)) and dim + rot <= 256 and vdim <= 256
+    )
+
+
+def latent_attention_unfolded(q, latent, w_ukv, sink, scale, dim, vdim, rank, cos_sin,
+                              positions, u: Unfold) -> torch.Tensor:
+    """Rows [0, u.rows) of q [T, H, dim + rot] (rotated in place) against
+    keys and values unfolded from their sequences' latents by w_ukv
+    [H*dim | H*vdim, rank]; returns [T, H, vdim], later rows unset. bf16 on
+    the GPU only: the folded form is the same function."""
+    T, H = q.shape[0], q.shape[1]
+    ext = hybrid_native()
+    ext.rotate_pairs(
+        q[: u.rows, :, dim:], q[: u.rows, :, dim:], positions[: u.rows], cos_sin
+    )
+    lat = latent.view(-1, latent.shape[-1])[u.key_slots]
+    kv = torch.nn.functional.linear(lat[:, :rank], w_ukv)
+    out = torch.empty(T, H, vdim, dtype=q.dtype, device=q.device)
+    ext.latent_attention_unfolded(
+        out, q, kv, lat, sink, float(scale), u.cu_q, u.cu_k, u.tile_seg, u.tile_off,
+        u.tile_rows, dim, vdim, rank,
+    )
+    return out
 
 
 # --------------------------------------------------------------- recurrences
