@@ -17,6 +17,8 @@ hipError_t launch_latent_folded_mfma(void*, float*, float*, const void*, const v
 hipError_t launch_latent_unfolded(void*, const void*, const void*, const void*, int64_t, const float*, float, const int*, const int*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_ssd_scan(void*, const void*, int64_t, const float*, const float*, const float*, const float*, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
 hipError_t launch_mlstm_scan(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*, const float*, float, float, int, int, int, float*, float*, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
+hipError_t launch_ssd_chunked(void*, const void*, int64_t, const float*, const float*, const float*, const float*, int, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, const int*, const int*, const int*, int, int, float*, void*, hipStream_t);
+hipError_t launch_mlstm_chunked(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*, const float*, float, float, int, int, int, int, float*, float*, float*, const int64_t*, const int*, const int*, const int*, const int*, const int*, const int*, int, int, float*, void*, float*, float*, hipStream_t);
 }
 
 namespace {
@@ -311,6 +313,69 @@ void mlstm_scan(Tensor y, Tensor q, Tensor k, Tensor v, Tensor gates, Tensor bia
         current_stream()));
 }
 
+// the chunked forms: segs/first/chunk_seg/chunk_off cut long segments into
+// chunks of 64 rows (segment segs[i] has chunks first[i]..first[i+1])
+void ssd_chunked(Tensor y, Tensor xbc, Tensor dt, Tensor dt_bias, Tensor A_log, Tensor D,
+                 int64_t H, int64_t P, int64_t N, int64_t G, Tensor state, Tensor positions,
+                 Tensor cu, Tensor slots, Tensor segs, Tensor first, Tensor chunk_seg,
+                 Tensor chunk_off) {
+    check_bf16(xbc, "xbc");
+    check_bf16(y, "y");
+    const int64_t T = xbc.size(0), S = slots.numel();
+    const int64_t L = segs.numel(), nc = chunk_seg.numel();
+    check_rows(xbc, T, H * P + 2 * G * N, "xbc");
+    TORCH_CHECK(G > 0 && H % G == 0 && y.is_contiguous() && y.numel() == T * H * P);
+    TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == P && state.size(3) == N);
+    TORCH_CHECK(vec8({&xbc}, {P, N}));
+    f32_ptr(state, state.numel(), "state");
+    const auto dev = xbc.options();
+    auto Fb = torch::empty({2, H, T}, dev.dtype(torch::kFloat32));
+    auto planes = torch::empty({2, nc, H, P, N}, dev);
+    CHECK_HIP(launch_ssd_chunked(
+        y.data_ptr(), xbc.data_ptr(), xbc.stride(0), f32_ptr(dt, T * H, "dt"),
+        f32_ptr(dt_bias, H, "dt_bias"), f32_ptr(A_log, H, "A_log"), f32_ptr(D, H, "D"), T, H,
+        P, N, G, state.data_ptr<float>(), i64_ptr(positions, T, "positions"),
+        i32_ptr(cu, S + 1, "cu"), i32_ptr(slots, S, "slots"), i32_ptr(segs, L, "segs"),
+        i32_ptr(first, L + 1, "first"), i32_ptr(chunk_seg, nc, "chunk_seg"),
+        i32_ptr(chunk_off, nc, "chunk_off"), L, nc, Fb.data_ptr<float>(), planes.data_ptr(),
+        current_stream()));
+}
+
+void mlstm_chunked(Tensor y, Tensor q, Tensor k, Tensor v, Tensor gates, Tensor bias,
+                   double cap, int64_t H, int64_t dk, int64_t dv, Tensor S, Tensor n, Tensor m,
+                   Tensor positions, Tensor cu, Tensor slots, Tensor segs, Tensor first,
+                   Tensor chunk_seg, Tensor chunk_off) {
+    check_bf16(q, "q");
+    check_bf16(k, "k");
+    check_bf16(v, "v");
+    check_bf16(y, "y");
+    const int64_t T = q.size(0), ns = slots.numel(), tiles = (dv + 63) / 64;
+    const int64_t L = segs.numel(), nc = chunk_seg.numel();
+    check_rows(q, T, H * dk, "q");
+    check_rows(k, T, H * dk, "k");
+    check_rows(v, T, H * dv, "v");
+    TORCH_CHECK(y.is_contiguous() && y.numel() == T * H * dv);
+    TORCH_CHECK(S.dim() == 4 && S.size(1) == H && S.size(2) == dv && S.size(3) == dk);
+    TORCH_CHECK(vec8({&q, &k, &v}, {dk, dv}));
+    f32_ptr(S, S.numel(), "S");
+    f32_ptr(n, S.size(0) * tiles * H * dk, "n");
+    f32_ptr(m, S.size(0) * tiles * H, "m");
+    const auto f32 = q.options().dtype(torch::kFloat32);
+    auto Fb = torch::empty({2, H, T}, f32);
+    auto planes = torch::empty({2, nc, H, dv, dk}, q.options());
+    auto n_in = torch::empty({nc, H, dk}, f32);
+    auto m_in = torch::empty({nc, H}, f32);
+    CHECK_HIP(launch_mlstm_chunked(
+        y.data_ptr(), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(),
+        v.stride(0), f32_ptr(gates, T * 2 * H, "gates"), f32_ptr(bias, 2 * H, "bias"),
+        (float)cap, 1.0f / std::sqrt((float)dk), T, H, dk, dv, S.data_ptr<float>(),
+        n.data_ptr<float>(), m.data_ptr<float>(), i64_ptr(positions, T, "positions"),
+        i32_ptr(cu, ns + 1, "cu"), i32_ptr(slots, ns, "slots"), i32_ptr(segs, L, "segs"),
+        i32_ptr(first, L + 1, "first"), i32_ptr(chunk_seg, nc, "chunk_seg"),
+        i32_ptr(chunk_off, nc, "chunk_off"), L, nc, Fb.data_ptr<float>(), planes.data_ptr(),
+        n_in.data_ptr<float>(), m_in.data_ptr<float>(), current_stream()));
+}
+
 void gated_norm(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t groups, double eps,
                 bool gate_first) {
     const bool f32 = is_f32(y, "y");
@@ -342,6 +407,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("causal_conv", &causal_conv, "segmented causal convolution + silu");
     m.def("ssd_scan", &ssd_scan, "Mamba-2 recurrence, token by token");
     m.def("mlstm_scan", &mlstm_scan, "mLSTM recurrence, token by token");
+    m.def("ssd_chunked", &ssd_chunked, "Mamba-2 recurrence, chunked");
+    m.def("mlstm_chunked", &mlstm_chunked, "mLSTM recurrence, chunked");
     m.def("gated_norm", &gated_norm, "group RMS norm with a gate");
     bind_shared(m);
 }

@@ -7,7 +7,7 @@
 // segment, one head, 64 value rows (16 lane groups x 4 rows); state stays in
 // registers over the segment's tokens. Bandwidth bound at one token.
 
-#include "common.h"
+#include "recurrence.h"
 
 #define SCAN_ROWS 64  // value rows per workgroup
 
@@ -16,14 +16,6 @@ __device__ __forceinline__ float sum16(float v) {
     for (int off = 8; off > 0; off >>= 1) v += __shfl_xor(v, off, WAVE_SIZE);
     return v;
 }
-// log(1 + e^z) without overflow
-__device__ __forceinline__ float softplus_f(float z) {
-    return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
-}
-__device__ __forceinline__ float log_sigmoid_f(float z) {
-    return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
-}
-
 // lane's key dims: 64 * e4 + 4 * l16 + j
 template <typename T, int E4>
 __device__ __forceinline__ void load_dims(const T* p, int l16, int dk, float (*f)[4]) {
@@ -153,8 +145,8 @@ __global__ void scan_kernel(ScanArgs a) {
         for (int r = 0; r < 4; ++r) v[r] = row0 + r < dv ? ldf(vp + row0 + r) : 0.f;
         if (MLSTM) {
             const float* g = a.gates + (size_t)t * 2 * H;
-            const float i = a.cap * tanhf((g[h] + a.bias[h]) / a.cap);
-            const float f = log_sigmoid_f(a.cap * tanhf((g[H + h] + a.bias[H + h]) / a.cap));
+            const float i = soft_cap_f(g[h] + a.bias[h], a.cap);
+            const float f = log_sigmoid_f(soft_cap_f(g[H + h] + a.bias[H + h], a.cap));
             const float m_new = fmaxf(f + m, i);
             keep = expf(f + m - m_new);
             add = expf(i - m_new);

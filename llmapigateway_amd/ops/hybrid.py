@@ -9,7 +9,7 @@ takes any split of a sequence into segments.
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Optional
+from typing import Optional, Tuple
 
 import numpy as np
 import torch
@@ -39,12 +39,10 @@ class Unfold:
 class Chunks:
     """Segments long enough for the chunked form of the recurrences."""
 
-    segs: torch.Tensor        # [L] int32 segment of each
-    first: torch.Tensor       # [L+1] int32 first chunk of each
-    chunk_seg: torch.Tensor   # [n] int32
-    chunk_off: torch.Tensor   # [n] int32 first row within the segment
-    short: torch.Tensor       # int32 segments that are run token by token
-    count: int
+    # int32: the segments, the first chunk of each (and the end), then per
+    # chunk its segment and its first row within it
+    maps: Tuple[torch.Tensor, torch.Tensor, torch.Tensor, torch.Tensor]
+    short: Optional[torch.Tensor]  # int32 segments that run token by token
 
 
 @dataclass
@@ -121,8 +119,8 @@ def plan_segments(batch, dtype) -> SegmentPlan:
         )
     if len(long):
         plan.chunks = Chunks(
-            segs=got["segs"], first=got["first"], chunk_seg=got["chunk_seg"],
-            chunk_off=got["chunk_off"], short=got["short"], count=int(nchunk.sum()),
+            maps=tuple(got[k] for k in ("segs", "first", "chunk_seg", "chunk_off")),
+            short=got["short"] if got["short"].numel() else None,
         )
     return plan
 
@@ -288,9 +286,14 @@ def ssd(xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs, plan):
     if not xbc.is_cuda:
         return ref.ssd(xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs)
     y = torch.empty(xbc.shape[0], H * P, dtype=xbc.dtype, device=xbc.device)
-    hybrid_native().ssd_scan(
-        y, xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs.cu, segs.slots, None
-    )
+    ext, ch = hybrid_native(), plan.chunks
+    args = (y, xbc, dt, dt_bias, A_log, D, H, P, N, G, S, positions, segs.cu, segs.slots)
+    if ch is not None and P % 8 == 0 and N % 8 == 0:
+        ext.ssd_chunked(*args, *ch.maps)
+        if ch.short is not None:
+            ext.ssd_scan(*args, ch.short)
+    else:
+        ext.ssd_scan(*args, None)
     return y
 
 
@@ -301,10 +304,15 @@ def mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs, plan):
     if not q.is_cuda:
         return ref.mlstm(q, k, v, gates, bias, cap, H, dk, dv, S, n, m, positions, segs)
     y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
-    hybrid_native().mlstm_scan(
-        y, q, k, v, gates, bias, float(cap), H, dk, dv, S, n, m, positions,
-        segs.cu, segs.slots, None,
-    )
+    ext, ch = hybrid_native(), plan.chunks
+    args = (y, q, k, v, gates, bias, float(cap), H, dk, dv, S, n, m, positions, segs.cu,
+            segs.slots)
+    if ch is not None and dk % 8 == 0 and dv % 8 == 0:
+        ext.mlstm_chunked(*args, *ch.maps)
+        if ch.short is not None:
+            ext.mlstm_scan(*args, ch.short)
+    else:
+        ext.mlstm_scan(*args, None)
     return y
 
 
