@@ -42,7 +42,7 @@ class EngineSpec(BaseModel):
     from a ``local://<model>?device=N&...`` baseUrl.
     """
 
-    model: str = "llama-3-8b"           # architecture preset name (models/configs.py)
+    model: str = "llama-3-8b"           # preset name (models/configs.py) or checkpoint folder
     device: int = 0                      # GPU ordinal (cuda:N == MI355X N)
     tp: int = 1                          # tensor-parallel degree over xGMI
     dtype: str = "bfloat16"
@@ -72,6 +72,8 @@ class ProviderDetails(BaseModel):
             updates: Dict[str, Any] = {}
             if u.netloc:
                 updates["model"] = u.netloc
+            elif u.path:
+                updates["model"] = u.path
             q = parse_qs(u.query)
             for key in ("device", "tp", "max_batch_size", "kv_block_size", "fail_requests"):
                 if key in q:

@@ -29,6 +29,7 @@ from fastapi.responses import StreamingResponse
 
 from ..config.loader import EngineSpec
 from ..config.settings import Settings
+from ..models.configs import get_model_config
 from .engine import EngineRequest, LLMEngine, SamplingParams
 from .tokenizer import ByteTokenizer
 
@@ -154,7 +155,9 @@ class EngineRegistry:
             handle = self._engines.get(key)
             if handle is not None:
                 return handle
+            config = get_model_config(spec.model)
             if spec.tp > 1:
+                config.scaled_for_tp(spec.tp)  # raises if the model cannot be sharded
                 from .tp_group import TPEngineClient
 
                 if torch.cuda.is_available() and torch.cuda.device_count() < spec.tp:
@@ -177,8 +180,10 @@ class EngineRegistry:
             dtype = torch.bfloat16 if device.startswith("cuda") else torch.float32
             if spec.dtype in ("float16", "fp16"):
                 dtype = torch.float16
+            elif spec.dtype in ("float32", "fp32"):
+                dtype = torch.float32
             engine = LLMEngine(
-                model=spec.model,
+                model=config,
                 device=device,
                 dtype=dtype,
                 block_size=spec.kv_block_size or self.settings.engine_kv_block_size,

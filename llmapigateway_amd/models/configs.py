@@ -271,14 +271,14 @@ MODEL_PRESETS = {
         kv_rank=40, q_rank=56, ssm_heads=6, ssm_vdim=20, state=24, groups=3,
         mem_heads=2, mem_dim=16, mem_vdim=40, times=2, max_positions=1024,
     ),
-    # layers of the size of llama-1b's and llama-3-8b's
-    "lelisun-1b": _lelisun_preset(
-        "lelisun-1b", width=2048, vocab=128256, ff=8192, heads=16, dim=128, rot_dim=64,
+    # layers as wide as llama-1b's and llama-3-8b's
+    "lelisun-small": _lelisun_preset(
+        "lelisun-small", width=2048, vocab=128256, ff=8192, heads=16, dim=128, rot_dim=64,
         kv_rank=512, q_rank=768, ssm_heads=64, ssm_vdim=64, state=128, groups=8,
         mem_heads=4, mem_dim=256, mem_vdim=512, times=2, repeat=3,
     ),
-    "lelisun-8b": _lelisun_preset(
-        "lelisun-8b", width=4096, vocab=128256, ff=14336, heads=32, dim=128, rot_dim=64,
+    "lelisun-base": _lelisun_preset(
+        "lelisun-base", width=4096, vocab=128256, ff=14336, heads=32, dim=128, rot_dim=64,
         kv_rank=512, q_rank=1536, ssm_heads=128, ssm_vdim=64, state=128, groups=8,
         mem_heads=8, mem_dim=256, mem_vdim=512, times=2, repeat=6,
     ),
