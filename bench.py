@@ -31,11 +31,13 @@ import statistics
 import sys
 import time
 
+import numpy as np
 import torch
 
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
 from llmapigateway_amd.engine import LLMEngine, EngineRequest, SamplingParams  # noqa: E402
+from llmapigateway_amd.models import ModelConfig, get_model_config  # noqa: E402
 
 
 def parse_args():
@@ -55,10 +57,19 @@ def parse_args():
     p.add_argument("--top-p", type=float, default=1.0)
     p.add_argument("--top-k", type=int, default=0)
     p.add_argument(
-        "--mode", choices=["qps", "wave"], default="qps",
+        "--mode", choices=["qps", "wave", "layers"], default="qps",
         help="qps = open-loop Poisson arrivals at --qps (the BASELINE "
-        "metric); wave = round-1 closed-loop waves",
+        "metric); wave = round-1 closed-loop waves; layers = prefill and "
+        "decode throughput of Lelisun beside a Llama of equal width, "
+        "feed-forward and number of layer runs",
     )
+    p.add_argument("--sizes", default="small,base", help="--mode layers: lelisun-<size> presets, or any hybrid model")
+    p.add_argument("--sides", default="lelisun,llama", help="--mode layers: which models")
+    p.add_argument("--prefill-shapes", default="4x1024,1x4096,1x8192",
+                   help="--mode layers: prompts x tokens (steps of 4096 tokens)")
+    p.add_argument("--decode-batches", default="16,64,256",
+                   help="--mode layers: sequences decoding after --decode-context tokens")
+    p.add_argument("--decode-context", type=int, default=1024)
     p.add_argument("--debug-stats", action="store_true")
     p.add_argument(
         "--qps", default="auto",
@@ -139,8 +150,134 @@ def run_open_loop(engine: LLMEngine, prompts, gen_tokens: int, qps: float, seed:
     return ttfts, elapsed
 
 
+class StepDriver:
+    """Sequences of random tokens stepped through the engine's own forwards,
+    without sampling or delivery."""
+
+    def __init__(self, engine: LLMEngine, n: int):
+        self.engine = engine
+        self.seqs = [EngineRequest([], SamplingParams()) for _ in range(n)]
+        for r in self.seqs:
+            engine._claim_slot(r)
+        self.rows = np.asarray([r.bt_slot for r in self.seqs], dtype=np.int64)
+        self.pos = np.zeros(n, dtype=np.int64)
+        self.rng = np.random.default_rng(0)
+
+    def _tokens(self, n: int):
+        vocab = self.engine.full_config.vocab_size
+        return self.rng.integers(3, min(vocab, 4096), n, dtype=np.int64)
+
+    def prefill(self, length: int, which=None) -> None:
+        """``length`` more tokens of each of these sequences in one step."""
+        which = range(len(self.seqs)) if which is None else which
+        spans = []
+        for i in which:
+            p = int(self.pos[i])
+            self.engine._extend_blocks(self.seqs[i], p, p + length)
+            spans.append((self.seqs[i].bt_slot, p, self._tokens(length)))
+            self.pos[i] += length
+        self.engine._varlen_logits(spans, [])
+
+    def decode(self) -> None:
+        for r, p in zip(self.seqs, self.pos):
+            self.engine._extend_blocks(r, int(p), int(p) + 1)
+        self.engine._decode_logits(self.rows, self.pos.copy(), self._tokens(len(self.rows)))
+        self.pos += 1
+
+    def restart(self) -> None:
+        self.pos[:] = 0
+
+    def close(self) -> None:
+        for r in self.seqs:
+            self.engine.kv.manager.free(r.block_table)
+            self.engine._free_slot(r)
+
+
+def run_layers(args) -> None:
+    """Prefill and decode tokens/s of Lelisun at a few sizes, each beside the
+    closest dense model at equal width: as many Llama layers as Lelisun runs
+    layers."""
+    device = "cuda:0" if torch.cuda.is_available() else "cpu"
+    context = args.decode_context
+    batches = [int(b) for b in args.decode_batches.split(",") if b]
+    shapes = [x for x in args.prefill_shapes.split(",") if x]
+    budget = 4096  # tokens per prefill step
+
+    def llama_like(c):
+        ff = next(e.mlp["ff"] for e in c.layers if e.mlp)
+        heads = c.hidden_size // 128 or 1
+        return ModelConfig(
+            name=f"llama of {c.name}", hidden_size=c.hidden_size, intermediate_size=ff,
+            num_layers=len(c.runs()), num_heads=heads, num_kv_heads=min(8, heads),
+            vocab_size=c.vocab_size, max_positions=16384,
+        )
+
+    def sync():
+        if device != "cpu":
+            torch.cuda.synchronize()
+
+    def timed(fn, steps):
+        sync()
+        t = time.monotonic()
+        for _ in range(steps):
+            fn()
+        sync()
+        return (time.monotonic() - t) / steps
+
+    results = []
+    for size in args.sizes.split(","):
+        config = get_model_config(f"lelisun-{size}" if size in ("small", "base") else size)
+        for side in args.sides.split(","):
+            c = config if side == "lelisun" else llama_like(config)
+            eng = LLMEngine(
+                model=c, device=device, num_blocks=8192 if device != "cpu" else 256,
+                dtype=torch.bfloat16 if device != "cpu" else torch.float32,
+                max_batch_size=max(batches + [8]), max_model_len=min(8320, c.max_positions), seed=1,
+            )
+            row = {"model": c.name, "layer_runs": len(config.runs()), "prefill": {}, "decode": {}}
+            for name in shapes:
+                n, length = map(int, name.split("x"))
+                portion = min(length, budget // n)
+                d = StepDriver(eng, n)
+
+                def whole():
+                    d.restart()
+                    for _ in range(0, length, portion):
+                        d.prefill(portion)
+
+                for _ in range(max(1, args.warmup)):
+                    whole()
+                s = timed(whole, args.steps)
+                row["prefill"][name] = {"tok_s": round(n * length / s), "ms": round(s * 1e3, 2)}
+                d.close()
+            for b in batches:
+                d = StepDriver(eng, b)
+                group = max(1, budget // context)
+                for i in range(0, b, group):
+                    d.prefill(context, range(i, min(b, i + group)))
+                for _ in range(3 * max(1, args.warmup)):
+                    d.decode()
+                s = timed(d.decode, 10 * args.steps)
+                row["decode"][f"b{b}"] = {"tok_s": round(b / s), "ms": round(s * 1e3, 3)}
+                d.close()
+            results.append(row)
+            print(json.dumps(row), file=sys.stderr, flush=True)
+            del d, eng
+            if device != "cpu":
+                torch.cuda.empty_cache()
+    print(json.dumps({
+        "metric": "prefill and decode tokens/s per model", "unit": "tokens/s", "n_gpus": 1,
+        "steps": args.steps, "warmup": args.warmup, "higher_is_better": True,
+        "dtype": "bf16" if device != "cpu" else "fp32",
+        "data": "synthetic (random token prompts, random-init weights)",
+        "decode_context": context, "results": results,
+    }))
+
+
 def main():
     args = parse_args()
+    if args.mode == "layers":
+        return run_layers(args)
     world_size = int(os.environ.get("WORLD_SIZE", "1"))
     rank = int(os.environ.get("RANK", "0"))
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))
