@@ -116,170 +116,281 @@ extern "C" hipError_t launch_latent_folded_any(
 }
 
 // ---------------------------------------------------------------------------
-// Folded form on MFMA (bf16). One workgroup: one row, 16 heads, one split of
-// the row's keys; tiles of 64 keys, 16 a wave.
-//   scores: a wave's own 16 cached rows come from global memory straight as
-//     B fragments (prefetched a tile ahead) against the query fragments;
-//   sums: the same registers go to LDS once, and every wave multiplies the
-//     tile's weights with its share of the latent dimensions (transposing
-//     LDS reads).
+// Folded form on MFMA (bf16). One workgroup: one row, 16*HT heads, one split
+// of the row's keys, 4*HT waves, tiles of 64 keys. Cached rows stream through
+// two LDS buffers by global_load_lds (a tile in flight behind the one in
+// use); 16-byte chunks are XOR-swizzled by row, on the source address, so
+// that row-wise and transposing reads both spread over the banks.
+//   scores: wave (ht, kq) takes 16 heads x 16 keys;
+//   sums: a wave takes its share of the latent dimensions for all heads.
 // One split writes the output (softmax started from the sink); several write
 // partials that latent_combine_kernel merges with the sink. Splits divide
 // the row's own key count, so a launch of fixed shape (captured graphs)
 // balances at every context length.
 // ---------------------------------------------------------------------------
 #define LF_KT 64
+#define LF_PAGES 512  // page ids held in LDS (a tile has at most 64)
 #define LA_NEG (-1e30f)
 
-template <int NKC>  // 32-wide chunks that cover a cached row
-__launch_bounds__(256)
+// lds_barrier: LDS data of the workgroup's waves is visible after it, while
+// transfers of dma16 stay in flight across it; dma_barrier: they too have
+// landed.
+__device__ __forceinline__ void lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+__device__ __forceinline__ void dma_barrier() {
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+// 16 bytes a lane from global memory to LDS at lds (wave-uniform) + 16*lane.
+// As asm: the compiler would let every later LDS read wait for the transfer;
+// here only dma_barrier does. (Wait counts it places for its own loads are
+// only stricter for the transfers it does not see.)
+__device__ __forceinline__ void dma16(const bf16* src, const bf16* lds) {
+    const uint32_t at = __builtin_amdgcn_readfirstlane(
+        (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) bf16*)lds);
+    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
+                 ::"s"(at), "v"(src) : "memory", "m0");
+}
+
+// NKC: 32-wide chunks that cover a cached row (even); RT: 16-wide tiles that
+// cover the rank (a multiple of 4, at most 2*NKC)
+template <int NKC, int RT, int HT>
+__launch_bounds__(256 * HT)
 __global__ void latent_folded_mfma_kernel(
     bf16* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml,
     const bf16* __restrict__ q, const bf16* __restrict__ latent,
     const float* __restrict__ sink, float scale, const int64_t* __restrict__ positions,
     const int* __restrict__ row_seg, const int* __restrict__ tables, int max_blocks,
-    int block_size, int H, int rank, int row_w, int nsplit) {
-    constexpr int LDK = NKC * 32 + 8;
-    constexpr int NT = (NKC * 32 + 63) / 64;  // 16-dim tiles of the sums per wave
-    __shared__ bf16 k_lds[LF_KT][LDK];
-    __shared__ bf16 p_lds[16][LF_KT + 8];
-    __shared__ float mx_lds[2][4][16];
-    __shared__ float l_lds[4][16];
+    int page_shift, int H, int rank, int row_w, int nsplit) {
+    constexpr int WAVES = 4 * HT;
+    constexpr int RC = NKC * 4;                   // 16-byte chunks per LDS row
+    constexpr int TILE = LF_KT * RC * 8;          // elements per buffer
+    constexpr int NI = RC / WAVES;                // transfers per wave and tile
+    constexpr int NT = (RT + WAVES - 1) / WAVES;  // rank tiles per wave
+    __shared__ __align__(16) bf16 k_lds[2 * TILE];
+    __shared__ bf16 p_lds[16 * HT][LF_KT + 8];
+    __shared__ float mx_lds[2][4][16 * HT];
+    __shared__ float l_lds[4][16 * HT];
+    __shared__ int page_lds[LF_PAGES];
     const size_t t = blockIdx.x;
-    const int h0 = blockIdx.y * 16, split = blockIdx.z;
+    const int h0 = blockIdx.y * 16 * HT, split = blockIdx.z;
     const int n = (int)positions[t] + 1;
     const int span = (n + nsplit * LF_KT - 1) / (nsplit * LF_KT) * LF_KT;
     const int key_lo = split * span, key_hi = min(n, key_lo + span);
     const int* bt = tables + (size_t)row_seg[t] * max_blocks;
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int ht = wave >> 2, kq = wave & 3;
     const int r16 = lane & 15, g = lane >> 4;
+
+    // page ids from the page of key k0 on
+    int page0 = 0;
+    auto load_pages = [&](int k0) {
+        page0 = k0 >> page_shift;
+        const int pages = ((key_hi - 1) >> page_shift) + 1 - page0;
+        for (int i = tid; i < min(pages, LF_PAGES); i += 64 * WAVES) page_lds[i] = bt[page0 + i];
+        __syncthreads();
+    };
+    // LDS chunk e of a tile holds chunk (e % RC) ^ swizzle(row) of row e / RC.
+    // Past the last key: any row, its weight is 0; past the row's end: any
+    // column, the queries are 0 there.
+    auto stage = [&](int k0, int buf) {
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int e0 = (wave * NI + i) * 64, e = e0 + lane;
+            const int row = e / RC, c = (e % RC) ^ ((row >> 1) & 7);
+            const int key = min(k0 + row, key_hi - 1);
+            const uint32_t at =
+                ((uint32_t)page_lds[(key >> page_shift) - page0] << page_shift) +
+                (key & ((1 << page_shift) - 1));
+            dma16(latent + (size_t)at * row_w + (c * 8 < row_w ? c * 8 : 0),
+                  k_lds + buf * TILE + e0 * 8);
+        }
+    };
+    if (key_lo < key_hi) {
+        load_pages(key_lo);
+        stage(key_lo, 0);
+    }
 
     bf16x8 qf[NKC];
     {
-        const bf16* qr = q + (t * H + min(h0 + r16, H - 1)) * row_w;
+        const bf16* qr = q + (t * H + min(h0 + ht * 16 + r16, H - 1)) * row_w;
 #pragma unroll
         for (int c = 0; c < NKC; ++c) {
-            uint4 v = {0, 0, 0, 0};
-            if (c * 32 + g * 8 < row_w)
-                v = *reinterpret_cast<const uint4*>(qr + c * 32 + g * 8);
+            const bool in = c * 32 + g * 8 < row_w;
+            uint4 v = *reinterpret_cast<const uint4*>(qr + (in ? c * 32 + g * 8 : 0));
+            if (!in) v = (uint4){0, 0, 0, 0};
             qf[c] = as_frag(v);
         }
     }
-    float m[4], l[4];
-    f32x4 acc[NT];
+    float m[HT][4], l[4];
+    f32x4 acc[HT][NT];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const int h = min(h0 + g * 4 + r, H - 1);
-        m[r] = nsplit == 1 ? sink[h] : LA_NEG;
-        l[r] = nsplit == 1 && wave == 0 && r16 == 0 ? 1.f : 0.f;
+    for (int i = 0; i < HT; ++i) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            m[i][r] = nsplit == 1 ? sink[min(h0 + i * 16 + g * 4 + r, H - 1)] : LA_NEG;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
     }
 #pragma unroll
-    for (int j = 0; j < NT; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int r = 0; r < 4; ++r) l[r] = nsplit == 1 && kq == 0 && r16 == 0 ? 1.f : 0.f;
 
-    uint4 kr[NKC];
-    auto load_tile = [&](int k0) {
-        const int key = k0 + wave * 16 + r16;
-        const bool in = key < key_hi;
-        const bf16* src = latent;
-        if (in) src += ((size_t)bt[key / block_size] * block_size + key % block_size) * row_w;
-#pragma unroll
-        for (int c = 0; c < NKC; ++c) {
-            kr[c] = (uint4){0, 0, 0, 0};
-            if (in && c * 32 + g * 8 < row_w)
-                kr[c] = *reinterpret_cast<const uint4*>(src + c * 32 + g * 8);
+    dma_barrier();
+    int buf = 0;
+#pragma unroll 1
+    for (int k0 = key_lo; k0 < key_hi; k0 += LF_KT, buf ^= 1) {
+        if (k0 + LF_KT < key_hi) {
+            if (((min(k0 + 2 * LF_KT, key_hi) - 1) >> page_shift) - page0 >= LF_PAGES)
+                load_pages(k0 + LF_KT);
+            stage(k0 + LF_KT, buf ^ 1);
         }
-    };
-    if (key_lo < key_hi) load_tile(key_lo);
-    int par = 0;
-    for (int k0 = key_lo; k0 < key_hi; k0 += LF_KT, par ^= 1) {
+        const bf16* kt = k_lds + buf * TILE;
         f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
+        {
+            const int row = kq * 16 + r16, sw = (row >> 1) & 7;
+            const bf16* even = kt + (row * RC + (g ^ sw)) * 8;
+            const bf16* odd = kt + (row * RC + ((4 + g) ^ sw)) * 8;
 #pragma unroll
-        for (int c = 0; c < NKC; ++c) s = mfma16(qf[c], as_frag(kr[c]), s);
-#pragma unroll
-        for (int c = 0; c < NKC; ++c)
-            *reinterpret_cast<uint4*>(&k_lds[wave * 16 + r16][c * 32 + g * 8]) = kr[c];
-        if (k0 + LF_KT < key_hi) load_tile(k0 + LF_KT);
-        const bool in = k0 + wave * 16 + r16 < key_hi;
+            for (int c = 0; c < NKC; ++c)
+                s = mfma16(qf[c], *reinterpret_cast<const bf16x8*>(
+                                      (c & 1 ? odd : even) + (c >> 1) * 64), s);
+        }
+        const bool in = k0 + kq * 16 + r16 < key_hi;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             s[r] = in ? s[r] * scale : LA_NEG;
-            const float v = group16_reduce_max(s[r]);
-            if (r16 == 0) mx_lds[par][wave][g * 4 + r] = v;
+            const float v = row16_max(s[r]);
+            if (r16 == 0) mx_lds[buf][kq][ht * 16 + g * 4 + r] = v;
         }
-        __syncthreads();
+        lds_barrier();
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int row = g * 4 + r;
-            const float m_new = fmaxf(
-                m[r], fmaxf(fmaxf(mx_lds[par][0][row], mx_lds[par][1][row]),
-                            fmaxf(mx_lds[par][2][row], mx_lds[par][3][row])));
-            const float f = __expf(m[r] - m_new);
-            const float p = in ? __expf(s[r] - m_new) : 0.f;
-            l[r] = l[r] * f + p;
-            m[r] = m_new;
-            p_lds[row][wave * 16 + r16] = f2bf(p);
+        for (int i = 0; i < HT; ++i)
 #pragma unroll
-            for (int j = 0; j < NT; ++j) acc[j][r] *= f;
-        }
-        __syncthreads();
+            for (int r = 0; r < 4; ++r) {
+                const int row = i * 16 + g * 4 + r;
+                const float m_new = fmaxf(
+                    m[i][r], fmaxf(fmaxf(mx_lds[buf][0][row], mx_lds[buf][1][row]),
+                                   fmaxf(mx_lds[buf][2][row], mx_lds[buf][3][row])));
+                const float f = __expf(m[i][r] - m_new);
+                m[i][r] = m_new;
+                if (i == ht) {
+                    const float p = in ? __expf(s[r] - m_new) : 0.f;
+                    l[r] = l[r] * f + p;
+                    p_lds[row][kq * 16 + r16] = f2bf(p);
+                }
+#pragma unroll
+                for (int j = 0; j < NT; ++j) acc[i][j][r] *= f;
+            }
+        lds_barrier();
 #pragma unroll
         for (int c = 0; c < LF_KT / 32; ++c) {
-            const bf16x8 pf = *reinterpret_cast<const bf16x8*>(&p_lds[r16][c * 32 + g * 8]);
+            bf16x8 pf[HT];
+#pragma unroll
+            for (int i = 0; i < HT; ++i)
+                pf[i] = *reinterpret_cast<const bf16x8*>(
+                    &p_lds[i * 16 + r16][c * 32 + g * 8]);
+            // transposing reads of rows k, k+4 (see tr_frag), swizzled
+            const int row = c * 32 + g * 8 + (r16 >> 2);
+            const int sw0 = (row >> 1) & 7, sw1 = ((row + 4) >> 1) & 7;
+            const bf16* r0 = kt + row * RC * 8 + (r16 & 1) * 4;
 #pragma unroll
             for (int j = 0; j < NT; ++j) {
-                const int d0 = (wave * NT + j) * 16;
-                if (d0 < rank)
-                    acc[j] = mfma16(pf, tr_frag(&k_lds[0][0], LDK, c * 32, d0), acc[j]);
+                // the last wave's tiles may lie past RT: repeat one, unused
+                const int tile = NT * WAVES == RT ? wave * NT + j : min(wave * NT + j, RT - 1);
+                const int ch = tile * 2 + ((r16 >> 1) & 1);
+                const bf16x8 vf =
+                    tr_pair(r0 + (ch ^ sw0) * 8, r0 + 4 * RC * 8 + (ch ^ sw1) * 8);
+#pragma unroll
+                for (int i = 0; i < HT; ++i) acc[i][j] = mfma16(pf[i], vf, acc[i][j]);
             }
         }
-        __syncthreads();
+        dma_barrier();
     }
     // the waves' shares of the denominator
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-        const float v = group16_reduce_sum(l[r]);
-        if (r16 == 0) l_lds[wave][g * 4 + r] = v;
+        const float v = row16_sum(l[r]);
+        if (r16 == 0) l_lds[kq][ht * 16 + g * 4 + r] = v;
     }
     __syncthreads();
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const int row = g * 4 + r, h = h0 + row;
-        if (h >= H) continue;
-        const float lt = l_lds[0][row] + l_lds[1][row] + l_lds[2][row] + l_lds[3][row];
-        const size_t th = t * H + h, pb = th * nsplit + split;
-        const float inv = 1.f / lt;
+    for (int i = 0; i < HT; ++i)
 #pragma unroll
-        for (int j = 0; j < NT; ++j) {
-            const int d = (wave * NT + j) * 16 + r16;
-            if (d >= rank) continue;
-            if (nsplit == 1) stf(out + th * rank + d, acc[j][r] * inv);
-            else part_acc[pb * rank + d] = acc[j][r];
+        for (int r = 0; r < 4; ++r) {
+            const int row = i * 16 + g * 4 + r, h = h0 + row;
+            if (h >= H) continue;
+            const float lt = l_lds[0][row] + l_lds[1][row] + l_lds[2][row] + l_lds[3][row];
+            const size_t th = t * H + h, pb = th * nsplit + split;
+            const float inv = 1.f / lt;
+#pragma unroll
+            for (int j = 0; j < NT; ++j) {
+                const int d = (wave * NT + j) * 16 + r16;
+                if (d >= rank) continue;
+                if (nsplit == 1) stf(out + th * rank + d, acc[i][j][r] * inv);
+                else part_acc[pb * rank + d] = acc[i][j][r];
+            }
+            if (nsplit > 1 && wave == 0 && r16 == 0) {
+                part_ml[pb * 2] = m[i][r];
+                part_ml[pb * 2 + 1] = lt;
+            }
         }
-        if (nsplit > 1 && wave == 0 && r16 == 0) {
-            part_ml[pb * 2] = m[r];
-            part_ml[pb * 2 + 1] = lt;
-        }
-    }
 }
 
+// one workgroup per (row, head); a thread owns 4 latent dimensions when the
+// rank allows
 __global__ void latent_combine_kernel(
     bf16* __restrict__ out, const float* __restrict__ part_acc,
     const float* __restrict__ part_ml, const float* __restrict__ sink, int H, int rank,
     int nsplit) {
     const size_t th = blockIdx.x;
     const float sk = sink[th % H];
+    const float2* ml = reinterpret_cast<const float2*>(part_ml) + th * nsplit;
     float M = sk;
-    for (int s = 0; s < nsplit; ++s) M = fmaxf(M, part_ml[(th * nsplit + s) * 2]);
+    for (int s = 0; s < nsplit; ++s) M = fmaxf(M, ml[s].x);
     float den = __expf(sk - M);
-    for (int s = 0; s < nsplit; ++s)
-        den += part_ml[(th * nsplit + s) * 2 + 1] * __expf(part_ml[(th * nsplit + s) * 2] - M);
+    for (int s = 0; s < nsplit; ++s) den += ml[s].y * __expf(ml[s].x - M);
+    const float inv = 1.f / den;
+    const float* pa = part_acc + th * nsplit * rank;
+    if (rank % 4 == 0) {
+        for (int d = threadIdx.x * 4; d < rank; d += blockDim.x * 4) {
+            float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+            for (int s = 0; s < nsplit; ++s) {
+                const float w = __expf(ml[s].x - M) * inv;
+                const float4 v = *reinterpret_cast<const float4*>(pa + (size_t)s * rank + d);
+                a.x = fmaf(v.x, w, a.x);
+                a.y = fmaf(v.y, w, a.y);
+                a.z = fmaf(v.z, w, a.z);
+                a.w = fmaf(v.w, w, a.w);
+            }
+            *reinterpret_cast<uint2*>(out + th * rank + d) =
+                make_uint2(pack2(a.x, a.y), pack2(a.z, a.w));
+        }
+        return;
+    }
     for (int d = threadIdx.x; d < rank; d += blockDim.x) {
         float a = 0.f;
         for (int s = 0; s < nsplit; ++s)
-            a += part_acc[(th * nsplit + s) * rank + d] *
-                 __expf(part_ml[(th * nsplit + s) * 2] - M);
-        stf(out + th * rank + d, a / den);
+            a += pa[(size_t)s * rank + d] * __expf(ml[s].x - M);
+        stf(out + th * rank + d, a * inv);
     }
+}
+
+template <int NKC, int RT>
+static void folded_go(
+    bf16* out, float* part_acc, float* part_ml, const bf16* q, const bf16* latent,
+    const float* sink, float scale, const int64_t* positions, const int* row_seg,
+    const int* tables, int rows, int H, int rank, int row_w, int page_shift, int max_blocks,
+    int nsplit, hipStream_t stream) {
+    if (H > 16)
+        latent_folded_mfma_kernel<NKC, RT, 2>
+            <<<dim3(rows, ceil_div_i(H, 32), nsplit), 512, 0, stream>>>(
+                out, part_acc, part_ml, q, latent, sink, scale, positions, row_seg, tables,
+                max_blocks, page_shift, H, rank, row_w, nsplit);
+    else
+        latent_folded_mfma_kernel<NKC, RT, 1><<<dim3(rows, 1, nsplit), 256, 0, stream>>>(
+            out, part_acc, part_ml, q, latent, sink, scale, positions, row_seg, tables,
+            max_blocks, page_shift, H, rank, row_w, nsplit);
 }
 
 extern "C" hipError_t launch_latent_folded_mfma(
@@ -288,17 +399,18 @@ extern "C" hipError_t launch_latent_folded_mfma(
     const int* tables, int rows, int H, int rank, int row_w, int block_size, int max_blocks,
     int nsplit, hipStream_t stream) {
     if (rows <= 0) return hipSuccess;
-    if (row_w % 8 || row_w > 576 || (nsplit > 1 && (!part_acc || !part_ml)))
+    if (block_size & (block_size - 1)) return hipErrorInvalidValue;
+    const int page_shift = __builtin_ctz(block_size);
+    if (row_w % 8 || row_w > 576 || rank > row_w || (nsplit > 1 && (!part_acc || !part_ml)))
         return hipErrorInvalidValue;
-    const dim3 grid(rows, ceil_div_i(H, 16), nsplit);
-#define GO(NKC)                                                                           \
-    latent_folded_mfma_kernel<NKC><<<grid, 256, 0, stream>>>(                             \
-        (bf16*)out, part_acc, part_ml, (const bf16*)q, (const bf16*)latent, sink, scale,  \
-        positions, row_seg, tables, max_blocks, block_size, H, rank, row_w, nsplit)
-    if (row_w <= 128) GO(4);
-    else if (row_w <= 192) GO(6);
-    else if (row_w <= 320) GO(10);
-    else GO(18);
+#define GO(NKC, RT)                                                                       \
+    folded_go<NKC, RT>((bf16*)out, part_acc, part_ml, (const bf16*)q,                     \
+                       (const bf16*)latent, sink, scale, positions, row_seg, tables, rows, \
+                       H, rank, row_w, page_shift, max_blocks, nsplit, stream)
+    if (row_w <= 128) GO(4, 8);
+    else if (row_w <= 192) { if (rank <= 128) GO(6, 8); else GO(6, 12); }
+    else if (row_w <= 320) { if (rank <= 256) GO(10, 16); else GO(10, 20); }
+    else { if (rank <= 512) GO(18, 32); else GO(18, 36); }
 #undef GO
     HIP_CHECK_LAST();
     if (nsplit > 1) {
@@ -432,7 +544,7 @@ __global__ void latent_unfolded_kernel(
                     s[i][u][r] = v;
                     mx = fmaxf(mx, v);
                 }
-                const float m_new = fmaxf(m[i][r], group16_reduce_max(mx));
+                const float m_new = fmaxf(m[i][r], row16_max(mx));
                 const float f = __expf(m[i][r] - m_new);
                 m[i][r] = m_new;
                 float sum = 0.f;
@@ -466,7 +578,7 @@ __global__ void latent_unfolded_kernel(
     for (int i = 0; i < MR; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const float inv = 1.f / group16_reduce_sum(l[i][r]);
+            const float inv = 1.f / row16_sum(l[i][r]);
             const int row = wrow0 + i * 16 + g * 4 + r;
             if (row >= nq) continue;
             bf16* o = out + ((size_t)(q0 + row) * H + h) * vdim;

@@ -7,7 +7,7 @@
 extern "C" {
 hipError_t launch_embed_scaled(float*, void*, int64_t, const int64_t*, const void*, float, int, int, int, int, hipStream_t);
 hipError_t launch_stream_norm(void*, int64_t, float*, const void*, int, const float*, const float*, const float*, float, int, int, int, int, int, hipStream_t);
-hipError_t launch_latent_rows(void*, void*, int, const void*, const float*, const float*, float, int, int, int, const int64_t*, const float*, const int64_t*, int, int, hipStream_t);
+hipError_t launch_latent_rows(void*, void*, int, const void*, const float*, const float*, float, int, int, int, const int64_t*, const float*, const int64_t*, int, int, int, hipStream_t);
 hipError_t launch_rotate_pairs(void*, int64_t, int64_t, int, const void*, int64_t, int64_t, int, int, const int64_t*, const float*, int, int, hipStream_t);
 hipError_t launch_gated_norm(void*, const void*, const void*, int64_t, const float*, float, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_causal_conv(void*, const void*, int64_t, const float*, const float*, void*, const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
@@ -142,7 +142,7 @@ void latent_rows(Tensor cq, Tensor latent, Tensor d, Tensor q_norm, Tensor kv_no
         f32_ptr(q_norm, qr, "q_norm"), f32_ptr(kv_norm, rank, "kv_norm"), (float)eps, qr,
         rank, rot, i64_ptr(positions, T, "positions"),
         f32_ptr(cos_sin, cos_sin.numel(), "cos_sin"), i64_ptr(slot_mapping, T, "slots"), T,
-        f32, current_stream()));
+        f32, vec8({&d, &cq, &latent, &q_norm, &kv_norm}, {qr, rank}), current_stream()));
 }
 
 void check_heads(const Tensor& t, int64_t T, int64_t H, const char* name) {
@@ -253,7 +253,7 @@ void causal_conv(Tensor y, Tensor x, Tensor w_t, Tensor b, Tensor state, Tensor 
         y.data_ptr(), x.data_ptr(), x.stride(0), f32_ptr(w_t, taps * C, "w_t"),
         f32_ptr(b, C, "b"), state.data_ptr(), i64_ptr(positions, T, "positions"),
         i32_ptr(cu, S + 1, "cu"), i32_ptr(slots, S, "slots"), i32_ptr(row_seg, T, "row_seg"),
-        T, S, C, taps, f32, vec8({&x, &y, &w_t, &b}, {C}), current_stream()));
+        T, S, C, taps, f32, vec8({&x, &y, &w_t, &b, &state}, {C}), current_stream()));
 }
 
 const int* seg_list_ptr(const OptTensor& list, int64_t S, int64_t& nseg) {

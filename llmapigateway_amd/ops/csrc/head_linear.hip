@@ -12,8 +12,8 @@
 typedef __attribute__((__vector_size__(8 * sizeof(short)))) short bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4;
 
-// WM waves along rows, 4/WM along columns; a wave owns 16 rows x 64 columns
-template <int WM>
+// WM waves along rows, 4/WM along columns; a wave owns 16 rows x 16*NJ columns
+template <int WM, int NJ>
 __launch_bounds__(256)
 __global__ void head_linear_mfma_kernel(
     bf16* __restrict__ y, int64_t yt, int64_t yh, const bf16* __restrict__ x, int64_t xt,
@@ -22,35 +22,36 @@ __global__ void head_linear_mfma_kernel(
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int r = lane & 15, g = lane >> 4;
     const int m0 = (blockIdx.x * WM + wave % WM) * 16;
-    const int n0 = (blockIdx.y * (4 / WM) + wave / WM) * 64;
+    const int n0 = (blockIdx.y * (4 / WM) + wave / WM) * (16 * NJ);
     if (m0 >= M || n0 >= N) return;
     // rows and columns past the end read the last one; nothing of them is kept
     const bf16* xr = x + (size_t)min(m0 + r, M - 1) * xt + h * xh;
-    const bf16* wr[4];
+    const bf16* wr[NJ];
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+    for (int j = 0; j < NJ; ++j)
         wr[j] = w + ((size_t)h * N + min(n0 + j * 16 + r, N - 1)) * K;
-    f32x4 acc[4];
+    f32x4 acc[NJ];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < NJ; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
     for (int k0 = 0; k0 < K; k0 += 32) {
         const int k = k0 + g * 8;
-        uint4 av = {0, 0, 0, 0}, bv[4];
+        uint4 av = {0, 0, 0, 0}, bv[NJ];
         const bool in = k < K;  // K is a multiple of 8
         if (in) av = *reinterpret_cast<const uint4*>(xr + k);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
+        for (int j = 0; j < NJ; ++j) {
             bv[j] = (uint4){0, 0, 0, 0};
             if (in) bv[j] = *reinterpret_cast<const uint4*>(wr[j] + k);
         }
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
+        for (int j = 0; j < NJ; ++j)
             acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
                 *reinterpret_cast<const bf16x8*>(&av),
                 *reinterpret_cast<const bf16x8*>(&bv[j]), acc[j], 0, 0, 0);
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
+    for (int j = 0; j < NJ; ++j) {
         const int n = n0 + j * 16 + r;
         if (n >= N) continue;
 #pragma unroll
@@ -76,6 +77,16 @@ __global__ void head_linear_any_kernel(
     stf(y + t * yt + h * yh + n, acc);
 }
 
+template <int WM, int NJ>
+static void head_linear_go(
+    bf16* y, int64_t yt, int64_t yh, const bf16* x, int64_t xt, int64_t xh, const bf16* w,
+    int M, int N, int K, int H, hipStream_t stream) {
+    const dim3 grid(ceil_div_i(M, 16 * WM), ceil_div_i(N, 16 * NJ * (4 / WM)), H);
+    head_linear_mfma_kernel<WM, NJ><<<grid, 256, 0, stream>>>(
+        y, yt, yh, x, xt, xh, w, M, N, K);
+}
+#define ARGS (bf16*)y, yt, yh, (const bf16*)x, xt, xh, (const bf16*)w, M, N, K, H, stream
+
 extern "C" hipError_t launch_head_linear(
     void* y, int64_t yt, int64_t yh, const void* x, int64_t xt, int64_t xh, const void* w,
     int M, int N, int K, int H, int f32, int vec8, hipStream_t stream) {
@@ -86,13 +97,17 @@ extern "C" hipError_t launch_head_linear(
     else if (!vec8)
         head_linear_any_kernel<bf16><<<dim3(M, ceil_div_i(N, 64), H), 64, 0, stream>>>(
             (bf16*)y, yt, yh, (const bf16*)x, xt, xh, (const bf16*)w, N, K);
-    else if (M <= 16)
-        head_linear_mfma_kernel<1><<<dim3(1, ceil_div_i(N, 256), H), 256, 0, stream>>>(
-            (bf16*)y, yt, yh, (const bf16*)x, xt, xh, (const bf16*)w, M, N, K);
-    else
-        head_linear_mfma_kernel<4><<<dim3(ceil_div_i(M, 64), ceil_div_i(N, 64), H), 256, 0,
-                                     stream>>>(
-            (bf16*)y, yt, yh, (const bf16*)x, xt, xh, (const bf16*)w, M, N, K);
+    else if (M <= 16) {
+        // narrower column tiles until the chip is filled
+        if (ceil_div_i(N, 256) * H >= 256) head_linear_go<1, 4>(ARGS);
+        else if (ceil_div_i(N, 128) * H >= 256) head_linear_go<1, 2>(ARGS);
+        else head_linear_go<1, 1>(ARGS);
+    } else {
+        const int mt = ceil_div_i(M, 64);
+        if (mt * ceil_div_i(N, 64) * H >= 512) head_linear_go<4, 4>(ARGS);
+        else if (mt * ceil_div_i(N, 32) * H >= 512) head_linear_go<4, 2>(ARGS);
+        else head_linear_go<4, 1>(ARGS);
+    }
     HIP_CHECK_LAST();
     return hipSuccess;
 }

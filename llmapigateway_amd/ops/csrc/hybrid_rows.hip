@@ -182,38 +182,53 @@ __global__ void stream_norm_kernel(
 // the first two, pair rotation of the third; the query latent goes to cq,
 // the rest to the row's cache page slot (-1: not kept).
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, int VEC>
+__launch_bounds__(512)
 __global__ void latent_rows_kernel(
     T* __restrict__ cq, T* __restrict__ latent, int row_w, const T* __restrict__ d,
     const float* __restrict__ q_norm, const float* __restrict__ kv_norm, float eps,
     int q_rank, int rank, int rot, const int64_t* __restrict__ positions,
     const float* __restrict__ cos_sin, const int64_t* __restrict__ slot_mapping) {
     __shared__ float red[8];
+    constexpr int HELD = 32 / VEC;
     const size_t t = blockIdx.x;
     const T* src = d + t * (q_rank + rank + rot);
+    const int W = q_rank + rank, step = blockDim.x * VEC, i0 = threadIdx.x * VEC;
+    float held[HELD][VEC];
     float sq = 0.f, sc = 0.f;
-    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
-        const float f = ldf(src + i);
-        sq += f * f;
-    }
-    for (int i = threadIdx.x; i < rank; i += blockDim.x) {
-        const float f = ldf(src + q_rank + i);
-        sc += f * f;
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= W) continue;
+        load_vec<VEC>(src + i, held[k]);
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss += held[k][j] * held[k][j];
+        if (i < q_rank) sq += ss;
+        else sc += ss;
     }
     const float iq = 1.f / sqrtf(block_sum(sq, red) / (float)q_rank + eps);
     const float ic = 1.f / sqrtf(block_sum(sc, red) / (float)rank + eps);
-    for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
-        stf(cq + t * q_rank + i, ldf(src + i) * iq * q_norm[i]);
     const int64_t slot = slot_mapping[t];
+    T* dst = latent + (size_t)(slot < 0 ? 0 : slot) * row_w;
+#pragma unroll
+    for (int k = 0; k < HELD; ++k) {
+        const int i = i0 + k * step;
+        if (i >= W) continue;
+        const bool is_q = i < q_rank;
+        float wv[VEC];
+        load_vec<VEC>(is_q ? q_norm + i : kv_norm + i - q_rank, wv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[k][j] *= (is_q ? iq : ic) * wv[j];
+        if (is_q) store_vec<VEC>(cq + t * q_rank + i, held[k]);
+        else if (slot >= 0) store_vec<VEC>(dst + i - q_rank, held[k]);
+    }
     if (slot < 0) return;
-    T* dst = latent + (size_t)slot * row_w;
-    for (int i = threadIdx.x; i < rank; i += blockDim.x)
-        stf(dst + i, ldf(src + q_rank + i) * ic * kv_norm[i]);
     const int half = rot / 2;
     const float* cs = cos_sin + (size_t)positions[t] * rot;
     for (int i = threadIdx.x; i < half; i += blockDim.x) {
-        const float u = ldf(src + q_rank + rank + 2 * i);
-        const float v = ldf(src + q_rank + rank + 2 * i + 1);
+        const float u = ldf(src + W + 2 * i);
+        const float v = ldf(src + W + 2 * i + 1);
         stf(dst + rank + 2 * i, u * cs[i] - v * cs[half + i]);
         stf(dst + rank + 2 * i + 1, v * cs[i] + u * cs[half + i]);
     }
@@ -334,6 +349,58 @@ __global__ void causal_conv_kernel(
 #pragma unroll
     for (int j = 0; j < VEC; ++j) acc[j] *= sigmoid_f(acc[j]);
     store_vec<VEC>(y + t * C + c, acc);
+}
+
+// the same for CONV_ROWS consecutive rows a thread, the window in registers
+#define CONV_ROWS 8
+template <typename T, int TAPS>
+__global__ void causal_conv_rows_kernel(
+    T* __restrict__ y, const T* __restrict__ x, int64_t ldx, const float* __restrict__ w_t,
+    const float* __restrict__ b, const T* __restrict__ state,
+    const int64_t* __restrict__ positions, const int* __restrict__ cu,
+    const int* __restrict__ slots, const int* __restrict__ row_seg, int rows, int C) {
+    constexpr int P = TAPS - 1;  // rows of the past in the window
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
+    if (c >= C) return;
+    float w[TAPS][8], bias[8], win[TAPS][8];
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) load_vec<8>(w_t + (size_t)k * C + c, w[k]);
+    load_vec<8>(b + c, bias);
+    int prev = -1;
+    for (int i = 0; i < CONV_ROWS; ++i) {
+        const int t = blockIdx.x * CONV_ROWS + i;
+        if (t >= rows) return;
+        const int s = row_seg[t];
+        if (s != prev) {  // fill the window from the segment or the state
+            prev = s;
+            const int slot = slots[s], j0 = t - cu[s];
+            const bool fresh = slot < 0 || positions[t] == j0;
+#pragma unroll
+            for (int k = 0; k < P; ++k) {
+                const int src = j0 - P + k;
+                if (src >= 0) {
+                    load_vec<8>(x + (size_t)(t - P + k) * ldx + c, win[k]);
+                } else if (!fresh) {
+                    load_vec<8>(state + ((size_t)slot * P + src + P) * C + c, win[k]);
+                } else {
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) win[k][j] = 0.f;
+                }
+            }
+        }
+        load_vec<8>(x + (size_t)t * ldx + c, win[P]);
+        float acc[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            acc[j] = bias[j];
+#pragma unroll
+            for (int k = 0; k < TAPS; ++k) acc[j] = fmaf(w[k][j], win[k][j], acc[j]);
+            acc[j] *= sigmoid_f(acc[j]);
+#pragma unroll
+            for (int k = 0; k < P; ++k) win[k][j] = win[k + 1][j];
+        }
+        store_vec<8>(y + (size_t)t * C + c, acc);
+    }
 }
 
 // the state after each segment: its last taps-1 inputs (ascending rows, so
@@ -461,11 +528,12 @@ extern "C" hipError_t launch_latent_rows(
     void* cq, void* latent, int row_w, const void* d, const float* q_norm,
     const float* kv_norm, float eps, int q_rank, int rank, int rot,
     const int64_t* positions, const float* cos_sin, const int64_t* slot_mapping, int rows,
-    int f32, hipStream_t stream) {
+    int f32, int vec8, hipStream_t stream) {
     if (rows <= 0) return hipSuccess;
-    return pick(f32, 0, [&](auto form) {
+    if (q_rank + rank > 512 * 32) return hipErrorInvalidValue;
+    return pick(f32, vec8, [&](auto form) {
         FORM(form);
-        latent_rows_kernel<T><<<rows, 256, 0, stream>>>(
+        latent_rows_kernel<T, V><<<rows, row_threads(q_rank + rank, V), 0, stream>>>(
             (T*)cq, (T*)latent, row_w, (const T*)d, q_norm, kv_norm, eps, q_rank, rank, rot,
             positions, cos_sin, slot_mapping);
     });
@@ -518,9 +586,23 @@ extern "C" hipError_t launch_causal_conv(
         });
     return pick(f32, vec8, [&](auto form) {
         FORM(form);
-        causal_conv_kernel<T, V><<<dim3(rows, cb), th, 0, stream>>>(
-            (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots, row_seg,
-            C, taps);
+        const dim3 grid(ceil_div_i(rows, CONV_ROWS), cb);
+        if (vec8 && taps == 4)
+            causal_conv_rows_kernel<T, 4><<<grid, th, 0, stream>>>(
+                (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots,
+                row_seg, rows, C);
+        else if (vec8 && taps == 3)
+            causal_conv_rows_kernel<T, 3><<<grid, th, 0, stream>>>(
+                (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots,
+                row_seg, rows, C);
+        else if (vec8 && taps == 2)
+            causal_conv_rows_kernel<T, 2><<<grid, th, 0, stream>>>(
+                (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots,
+                row_seg, rows, C);
+        else
+            causal_conv_kernel<T, V><<<dim3(rows, cb), th, 0, stream>>>(
+                (T*)y, (const T*)x, ldx, w_t, b, (const T*)state, positions, cu, slots,
+                row_seg, C, taps);
         if (taps > 1)
             conv_state_kernel<T, V><<<dim3(nseg, cb), th, 0, stream>>>(
                 (const T*)x, ldx, (T*)state, positions, cu, slots, C, taps);

@@ -17,18 +17,42 @@ __device__ __forceinline__ bf16x8 as_frag(const uint4& v) {
     return *reinterpret_cast<const bf16x8*>(&v);
 }
 
+// sum / maximum over the 16 lanes of a fragment row, in every lane: DPP row
+// rotations stay in the vector ALU (a shuffle goes through the LDS unit)
+template <int N>
+__device__ __forceinline__ float row16_ror(float v) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(
+        0, __float_as_int(v), 0x120 + N, 0xF, 0xF, false));
+}
+__device__ __forceinline__ float row16_max(float v) {
+    v = fmaxf(v, row16_ror<8>(v));
+    v = fmaxf(v, row16_ror<4>(v));
+    v = fmaxf(v, row16_ror<2>(v));
+    return fmaxf(v, row16_ror<1>(v));
+}
+__device__ __forceinline__ float row16_sum(float v) {
+    v += row16_ror<8>(v);
+    v += row16_ror<4>(v);
+    v += row16_ror<2>(v);
+    return v + row16_ror<1>(v);
+}
+
+// ds_read_b64_tr_b16 twice: a 16-lane group's lanes address 4 rows of 16
+// columns (lane i: row i/4, columns (i%4)*4..+3) and each gets one column
+__device__ __forceinline__ bf16x8 tr_pair(const bf16* lo_rows, const bf16* hi_rows) {
+    typedef __attribute__((address_space(3))) bf16x4* lds_ptr;
+    const bf16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)lo_rows);
+    const bf16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)hi_rows);
+    return (bf16x8){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+}
+
 // Fragment whose k runs over the rows of a row-major LDS tile (a B operand
 // stored [k][col], or an A operand stored [k][row]): rows k0..k0+31, columns
-// c0..c0+15. ds_read_b64_tr_b16 hands each lane of a 16-lane group one column
-// of a 4x16 block, so two reads make the 8 k values. Rows and c0 must keep
-// 8-byte alignment.
+// c0..c0+15. Rows and c0 must keep 8-byte alignment.
 __device__ __forceinline__ bf16x8 tr_frag(const bf16* tile, int stride, int k0, int c0) {
-    typedef __attribute__((address_space(3))) bf16x4* lds_ptr;
     const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15;
     const bf16* p = tile + (k0 + g * 8 + (i >> 2)) * stride + c0 + (i & 3) * 4;
-    const bf16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p);
-    const bf16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)(p + 4 * stride));
-    return (bf16x8){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+    return tr_pair(p, p + 4 * stride);
 }
 
 // fp32 as a sum of two bf16 (16 mantissa bits): products of a fp32 operand

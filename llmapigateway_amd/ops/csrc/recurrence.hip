@@ -7,15 +7,11 @@
 // segment, one head, 64 value rows (16 lane groups x 4 rows); state stays in
 // registers over the segment's tokens. Bandwidth bound at one token.
 
+#include "mfma.h"
 #include "recurrence.h"
 
 #define SCAN_ROWS 64  // value rows per workgroup
 
-__device__ __forceinline__ float sum16(float v) {
-#pragma unroll
-    for (int off = 8; off > 0; off >>= 1) v += __shfl_xor(v, off, WAVE_SIZE);
-    return v;
-}
 // lane's key dims: 64 * e4 + 4 * l16 + j
 template <typename T, int E4>
 __device__ __forceinline__ void load_dims(const T* p, int l16, int dk, float (*f)[4]) {
@@ -167,7 +163,7 @@ __global__ void scan_kernel(ScanArgs a) {
                     nv[e][j] = keep * nv[e][j] + add * k[e][j];
                     nq = fmaf(nv[e][j], q[e][j], nq);
                 }
-            den = fmaxf(fabsf(sum16(nq)), expf(-m)) + 1e-6f;
+            den = fmaxf(fabsf(row16_sum(nq)), expf(-m)) + 1e-6f;
         }
         float o[4];
 #pragma unroll
@@ -181,7 +177,7 @@ __global__ void scan_kernel(ScanArgs a) {
                     S[r][e][j] = fmaf(av, k[e][j], keep * S[r][e][j]);
                     s = fmaf(S[r][e][j], q[e][j], s);
                 }
-            o[r] = sum16(s);
+            o[r] = row16_sum(s);
         }
         const float dh = MLSTM ? 0.f : a.D[h];
 #pragma unroll

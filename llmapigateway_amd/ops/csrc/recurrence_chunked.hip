@@ -120,7 +120,13 @@ __global__ void state_pass_kernel(ChunkArgs a) {
     }
 
     uint4 kreg[2], vreg[2];
+    float F_last, F_row, b_row;  // of the chunk that is loaded, a row per lane
     auto load_rows = [&](int r0) {
+        const size_t at = (size_t)h * a.T + r0;
+        const int last = min(CH, row_hi - r0) - 1;
+        F_last = a.F[at + last];
+        F_row = a.F[at + min(lane, last)];
+        b_row = a.b[at + min(lane, last)];
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
             const int e = tid + u * 256, r = r0 + e / 8, d = e % 8 * 8;
@@ -162,18 +168,15 @@ __global__ void state_pass_kernel(ChunkArgs a) {
         // weights of the chunk's rows at its end
         float keep, m_out = 0.f;
         {
-            const size_t at = (size_t)h * a.T + r0;
-            const float FL = a.F[at + n - 1];
-            const float b = lane < n ? a.b[at + lane] : (MLSTM ? -INFINITY : 0.f);
             float w;
             if (MLSTM) {
-                const float gl = fmaxf(m, wave_reduce_max(b));
-                w = lane < n ? expf(b - gl) : 0.f;
+                const float gl = fmaxf(m, wave_reduce_max(b_row));
+                w = lane < n ? expf(b_row - gl) : 0.f;
                 keep = expf(m - gl);
-                m_out = FL + gl;
+                m_out = F_last + gl;
             } else {
-                w = lane < n ? expf(FL - a.F[at + lane]) * b : 0.f;
-                keep = expf(FL);
+                w = lane < n ? expf(F_last - F_row) * b_row : 0.f;
+                keep = expf(F_last);
             }
             __syncthreads();  // the previous chunk's tiles have been read
             if (wave == 0) w_lds[lane] = w;
@@ -383,7 +386,7 @@ __global__ void chunk_out_kernel(ChunkArgs a) {
             *reinterpret_cast<uint16_t*>(p_lo + row * LDT + s) = lo;
         }
         if (MLSTM) {
-            const float nq = group16_reduce_sum(sum) + inter * __shfl(qn, row, WAVE_SIZE);
+            const float nq = row16_sum(sum) + inter * __shfl(qn, row, WAVE_SIZE);
             den[r] = 1.f / (fmaxf(fabsf(nq), expf(-(Ft + gt))) + 1e-6f);
         } else {
             den[r] = 1.f;

@@ -207,10 +207,11 @@ def latent_attention_folded(ql, latent, rank, sink, scale, positions, segs, row0
     T, H, row = ql.shape
     out = torch.empty(T, H, rank, dtype=ql.dtype, device=ql.device)
     nsplit, pa, pm = 0, None, None
-    if ql.dtype == torch.bfloat16 and row <= 576:
+    page = latent.shape[1]
+    if ql.dtype == torch.bfloat16 and row <= 576 and page & (page - 1) == 0:
         # fill the chip: splits only from shapes, so captured graphs hold
-        max_tiles = -(-segs.tables.shape[1] * latent.shape[1] // 64)
-        nsplit = max(1, min(512 // (T * -(-H // 16)), 16, max_tiles))
+        max_tiles = -(-segs.tables.shape[1] * page // 64)
+        nsplit = max(1, min(-(-256 // (T * -(-H // 32))), 16, max_tiles))
         if nsplit > 1:
             pa, pm = _folded_scratch(ql.device, T * H * nsplit * rank, T * H * nsplit * 2)
     hybrid_native().latent_attention_folded(
