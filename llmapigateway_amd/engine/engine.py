@@ -536,19 +536,28 @@ class LLMEngine:
         if logits_idx is None:
             logits_idx = seg_cu[1:].astype(np.int64) - 1
 
-        seg_tables = torch.from_numpy(self._bt_np[all_rows]).to(device)
         cu = torch.from_numpy(seg_cu).to(device)
         S = len(spans)
         kw = {}
+        if starts.any() or nd or self.model.uses_segments:
+            tables = torch.from_numpy(self._bt_np[all_rows]).to(device)
         if starts.any():
             kw.update(
-                block_tables=seg_tables[:S],
+                block_tables=tables[:S],
                 cached_lens=torch.from_numpy(starts.astype(np.int32)).to(device),
             )
         if nd:
             kw.update(
-                dec_block_tables=seg_tables[S:],
+                dec_block_tables=tables[S:],
                 dec_context_lens=torch.from_numpy((d_pos + 1).astype(np.int32)).to(device),
+            )
+        if self.model.uses_segments:
+            kw["segs"] = Segments(
+                cu=cu,
+                slots=torch.from_numpy(all_rows.astype(np.int32)).to(device),
+                tables=tables,
+                row_seg=torch.from_numpy(row_seg).to(device),
+                block_size=bs, starts=all_starts, lens=all_lens, n_prefill=S,
             )
         tile_seq, tile_off = ops.build_prefill_tiles(lens, device)
         batch = ForwardBatch(
@@ -562,13 +571,6 @@ class LLMEngine:
             tile_off=tile_off,
             n_prefill_tokens=Tp,
             logits_indices=torch.from_numpy(logits_idx).to(device),
-            segs=Segments(
-                cu=cu,
-                slots=torch.from_numpy(all_rows.astype(np.int32)).to(device),
-                tables=seg_tables,
-                row_seg=torch.from_numpy(row_seg).to(device),
-                block_size=bs, starts=all_starts, lens=all_lens, n_prefill=S,
-            ),
             **kw,
         )
         return self.model.step(batch, self.kv)

@@ -26,6 +26,7 @@ from .weights import open_checkpoint
 
 class HybridModel:
     extension = "_H"  # the HIP extension its kernels are in
+    uses_segments = True  # steps over ForwardBatch.segs
 
     def __init__(
         self,

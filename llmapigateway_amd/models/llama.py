@@ -37,6 +37,7 @@ from .twins import add_decode_twins
 
 class LlamaModel:
     extension = "_C"  # the HIP extension its kernels are in
+    uses_segments = False  # steps without ForwardBatch.segs
 
     def __init__(
         self,

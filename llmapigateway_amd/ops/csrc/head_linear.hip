@@ -7,10 +7,7 @@
 // between them). fp32 and shapes that are no multiple of 8: one output a
 // thread.
 
-#include "common.h"
-
-typedef __attribute__((__vector_size__(8 * sizeof(short)))) short bf16x8;
-typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4;
+#include "mfma.h"
 
 // WM waves along rows, 4/WM along columns; a wave owns 16 rows x 16*NJ columns
 template <int WM, int NJ>
@@ -33,22 +30,25 @@ __global__ void head_linear_mfma_kernel(
     f32x4 acc[NJ];
 #pragma unroll
     for (int j = 0; j < NJ; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int k0 = 0; k0 < K; k0 += 32) {
-        const int k = k0 + g * 8;
-        uint4 av = {0, 0, 0, 0}, bv[NJ];
-        const bool in = k < K;  // K is a multiple of 8
-        if (in) av = *reinterpret_cast<const uint4*>(xr + k);
+    // U k-steps of loads in flight; past K the activations are 0
+    constexpr int U = NJ == 1 ? 8 : 4;
+    for (int k0 = 0; k0 < K; k0 += 32 * U) {
+        uint4 av[U], bv[U][NJ];
 #pragma unroll
-        for (int j = 0; j < NJ; ++j) {
-            bv[j] = (uint4){0, 0, 0, 0};
-            if (in) bv[j] = *reinterpret_cast<const uint4*>(wr[j] + k);
+        for (int u = 0; u < U; ++u) {
+            const bool in = k0 + u * 32 + g * 8 < K;  // K is a multiple of 8
+            const int k = in ? k0 + u * 32 + g * 8 : 0;
+            av[u] = *reinterpret_cast<const uint4*>(xr + k);
+            if (!in) av[u] = (uint4){0, 0, 0, 0};
+#pragma unroll
+            for (int j = 0; j < NJ; ++j)
+                bv[u][j] = *reinterpret_cast<const uint4*>(wr[j] + k);
         }
 #pragma unroll
-        for (int j = 0; j < NJ; ++j)
-            acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                *reinterpret_cast<const bf16x8*>(&av),
-                *reinterpret_cast<const bf16x8*>(&bv[j]), acc[j], 0, 0, 0);
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int j = 0; j < NJ; ++j)
+                acc[j] = mfma16(as_frag(av[u]), as_frag(bv[u][j]), acc[j]);
     }
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
