@@ -57,6 +57,15 @@ def test_wave_mode():
     assert d["config"]["mode"] == "closed-loop-waves"
 
 
+def test_layers_mode():
+    d = run_bench(["--mode", "layers", "--sizes", "tiny-lelisun", "--prefill-shapes", "2x16",
+                   "--decode-batches", "2", "--decode-context", "16"])
+    assert [r["model"] for r in d["results"]] == ["tiny-lelisun", "llama of tiny-lelisun"]
+    for r in d["results"]:
+        assert r["layer_runs"] == 6
+        assert r["prefill"]["2x16"]["tok_s"] > 0 and r["decode"]["b2"]["tok_s"] > 0
+
+
 @pytest.mark.timeout(420)
 def test_two_rank_launch_matches_driver_shape():
     env = dict(os.environ)
