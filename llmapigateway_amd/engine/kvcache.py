@@ -13,8 +13,8 @@ GPU the default number of blocks is computed from *free HBM after model
 weights* × settings.engine_hbm_fraction (288 GB per MI355X makes this the
 dominant tensor).
 
-Hybrid decoders (models/hybrid.py) keep a HybridCache: pages of latent rows
-for their attention layers, allocated by the same BlockManager, and for
+Hybrid decoders (models/hybrid.py) keep a HybridCache: pages of key, value
+or latent rows for their attention layers, allocated by the same BlockManager, and for
 their recurrent layers one state slot per live sequence. The slot is the
 engine's row of the sequence (EngineRequest.bt_slot), so it is claimed and
 given back with the pages; a sequence's first token starts from empty
@@ -365,7 +365,7 @@ class HybridCache:
 
 def _run_specs(config: HybridConfig):
     return [
-        MIXERS[config.layers[i].type].cache_spec(config.layers[i].mixer)
+        MIXERS[config.layers[i].type].cache_spec(config.layers[i].mixer, config.hidden_size)
         for i, _ in config.runs()
     ]
 

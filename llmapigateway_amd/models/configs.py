@@ -66,21 +66,28 @@ class HybridLayer:
 
 @dataclass(frozen=True)
 class HybridConfig:
-    """A decoder whose layers each name their mixer (latent attention,
-    Mamba-2, mLSTM), with an optional loop: layers [start, stop) run
-    ``times`` times with the same weights, each pass with its own cache.
+    """A decoder whose layers each name their mixer (models/mixers.py) and
+    their feed-forward (models/feedforward.py), with an optional loop: layers
+    [start, stop) run ``times`` times with the same weights, each pass with
+    its own cache.
 
-    The field set is what the Lelisun config.json gives; ``max_positions``
-    is the framework's own bound (nothing in the design limits it) and
-    ``weights_dir`` says where the checkpoint lies (None: random init)."""
+    The field set is what the Lelisun and Filinex config.json files give and
+    what their designs fix; ``max_positions`` is the framework's own bound
+    (nothing in the designs limits it) and ``weights_dir`` says where the
+    checkpoint lies (None: random init)."""
 
     name: str
     vocab_size: int
     hidden_size: int
     layers: Tuple[HybridLayer, ...]
     norm_eps: float = 1e-5
+    norm: str = "layernorm"       # of the stream: "layernorm" | "tanh" (dynamic tanh)
+    post_norm: bool = False       # a norm on every sublayer's output, too
+    embed_norm: bool = False
     embed_scale: float = 1.0
     loop: Optional[Tuple[int, int, int]] = None  # (start, stop, times)
+    loop_step: bool = True        # a learned vector per loop pass
+    logit_softcap: Optional[float] = None
     max_positions: int = 32768
     weights_dir: Optional[str] = None
 
@@ -89,34 +96,81 @@ class HybridConfig:
             start, stop, times = self.loop
             if not (0 <= start < stop <= len(self.layers) and times >= 1):
                 raise ValueError(f"bad loop {self.loop} over {len(self.layers)} layers")
+        if self.norm not in ("layernorm", "tanh"):
+            raise ValueError(f"unknown norm '{self.norm}'")
+        if self.norm != "tanh" and (self.post_norm or self.embed_norm):
+            raise ValueError("norms of sublayer outputs and of the embedding: dynamic tanh only")
         for i, layer in enumerate(self.layers):
-            m = layer.mixer
-            if layer.type == "latent_attention":
-                if m["rot"]["dims"] != m["rot_dim"] or m["rot_dim"] % 2:
-                    raise ValueError(f"layer {i}: rot.dims must be rot_dim, an even number")
-            elif layer.type == "mamba2":
-                if m["heads"] % m["groups"] or (m["heads"] * m["vdim"]) % m["norm_groups"]:
-                    raise ValueError(f"layer {i}: groups do not divide the heads")
-            elif layer.type != "mlstm":
-                raise ValueError(f"layer {i}: unknown mixer '{layer.type}'")
-            if layer.mlp is not None and layer.mlp["kind"] != "dense":
-                raise ValueError(f"layer {i}: unknown feed-forward '{layer.mlp['kind']}'")
+            try:
+                self._check_layer(layer)
+            except ValueError as e:
+                raise ValueError(f"layer {i}: {e}") from None
+
+    @staticmethod
+    def _check_layer(layer: HybridLayer) -> None:
+        m = layer.mixer
+        if layer.type == "latent_attention":
+            if m["rot"]["dims"] != m["rot_dim"] or m["rot_dim"] % 2:
+                raise ValueError("rot.dims must be rot_dim, an even number")
+        elif layer.type == "mamba2":
+            if m["heads"] % m["groups"] or (m["heads"] * m["vdim"]) % m["norm_groups"]:
+                raise ValueError("groups do not divide the heads")
+        elif layer.type == "parallel":
+            if m["left"]["heads"] % m["left"]["kv_heads"]:
+                raise ValueError("kv_heads does not divide the heads")
+            if not m["left"]["softcap"] > 0 or not m["right"]["tau"] > 0:
+                raise ValueError("softcap and tau are positive")
+        elif layer.type not in ("mlstm", "wkv"):
+            raise ValueError(f"unknown mixer '{layer.type}'")
+        if layer.mlp is None:
+            return
+        if layer.mlp["kind"] == "moe":
+            r = layer.mlp["router"]
+            if not 1 <= r["top"] <= r["experts"]:
+                raise ValueError(f"router: top {r['top']} of {r['experts']} experts")
+        elif layer.mlp["kind"] != "dense":
+            raise ValueError(f"unknown feed-forward '{layer.mlp['kind']}'")
+
+    @staticmethod
+    def _common(raw: Dict[str, Any], layers) -> Dict[str, Any]:
+        loop = raw.get("loop")
+        return dict(
+            vocab_size=raw["vocab"], hidden_size=raw["width"], layers=tuple(layers),
+            norm_eps=raw["norm"]["eps"],
+            loop=(loop["start"], loop["stop"], loop["times"]) if loop else None,
+        )
 
     @classmethod
     def from_json(cls, raw: Dict[str, Any], name: str, weights_dir: Optional[str] = None):
-        loop = raw.get("loop")
+        """Lelisun's config.json."""
+        layers = [
+            HybridLayer(type=e["type"], mixer=e["mixer"], mlp=e.get("mlp"))
+            for e in raw["layers"]
+        ]
         return cls(
-            name=name,
-            vocab_size=raw["vocab"],
-            hidden_size=raw["width"],
-            layers=tuple(
-                HybridLayer(type=e["type"], mixer=e["mixer"], mlp=e.get("mlp"))
-                for e in raw["layers"]
-            ),
-            norm_eps=raw["norm"]["eps"],
-            embed_scale=raw["embedding"]["scale"],
-            loop=(loop["start"], loop["stop"], loop["times"]) if loop else None,
-            weights_dir=weights_dir,
+            name=name, embed_scale=raw["embedding"]["scale"], weights_dir=weights_dir,
+            **cls._common(raw, layers),
+        )
+
+    @classmethod
+    def from_filinex_json(cls, raw: Dict[str, Any], name: str, weights_dir: Optional[str] = None):
+        """Filinex's config.json. The ranks of the decay projections are only
+        in the checkpoint's shapes: they join the mixers' sizes here."""
+        from .weights import open_checkpoint
+
+        ckpt = open_checkpoint(weights_dir)
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            m = dict(e["mixer"])
+            if e["type"] == "parallel":
+                m["right"] = dict(m["right"], decay_rank=ckpt.shape(f"l{i}.mix.right.a1")[0])
+            elif e["type"] == "wkv":
+                m["decay_rank"] = ckpt.shape(f"l{i}.mix.w1")[0]
+            layers.append(HybridLayer(type=e["type"], mixer=m, mlp=e.get("mlp")))
+        return cls(
+            name=name, norm="tanh", post_norm=True, embed_norm=True, loop_step=False,
+            logit_softcap=raw["logit_softcap"], weights_dir=weights_dir,
+            **cls._common(raw, layers),
         )
 
     def runs(self) -> List[Tuple[int, Optional[int]]]:
@@ -139,7 +193,10 @@ class HybridConfig:
 
 
 # config.json "architecture" -> reader(raw, name, weights_dir)
-ARCHITECTURES = {"Lelisun": HybridConfig.from_json}
+ARCHITECTURES = {
+    "Lelisun": HybridConfig.from_json,
+    "Filinex": HybridConfig.from_filinex_json,
+}
 
 
 def load_model_dir(path: str):
@@ -182,6 +239,34 @@ def _lelisun_preset(
         name=name, vocab_size=vocab, hidden_size=width, layers=looped + (mem, attn),
         embed_scale=width ** 0.5, loop=(0, len(looped), times),
         max_positions=max_positions,
+    )
+
+
+def _filinex_preset(
+    name: str, width: int, vocab: int, heads: int, kv_heads: int, dim: int, lin_heads: int,
+    lin_dim: int, lin_vdim: int, wkv_dim: int, rank: int, experts: int, top: int, ff: int,
+    shared_ff: int, times: int, repeat: int = 1, max_positions: int = 32768,
+) -> HybridConfig:
+    """A Filinex of [parallel, wkv] pairs, all but the last layer looped."""
+    mlp = dict(
+        kind="moe", router=dict(experts=experts, top=top), expert=dict(ff=ff, limit=7.0),
+        shared=dict(ff=shared_ff, limit=7.0),
+    )
+    par = HybridLayer(
+        "parallel",
+        dict(left=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5,
+                       softcap=30.0),
+             right=dict(heads=lin_heads, dim=lin_dim, vdim=lin_vdim, tau=16.0,
+                        decay_rank=rank),
+             left_scale=1.0, right_scale=1.0),
+        mlp,
+    )
+    mem = HybridLayer("wkv", dict(heads=width // wkv_dim, dim=wkv_dim, decay_rank=4 * rank), mlp)
+    layers = (par, mem) * repeat
+    return HybridConfig(
+        name=name, vocab_size=vocab, hidden_size=width, layers=layers, norm="tanh",
+        post_norm=True, embed_norm=True, loop=(0, len(layers) - 1, times), loop_step=False,
+        logit_softcap=30.0, max_positions=max_positions,
     )
 
 
@@ -281,6 +366,23 @@ MODEL_PRESETS = {
         "lelisun-base", width=4096, vocab=128256, ff=14336, heads=32, dim=128, rot_dim=64,
         kv_rank=512, q_rank=1536, ssm_heads=128, ssm_vdim=64, state=128, groups=8,
         mem_heads=8, mem_dim=256, mem_vdim=512, times=2, repeat=6,
+    ),
+    # looped hybrid decoder (attention beside linear attention, WKV, experts)
+    "tiny-filinex": _filinex_preset(
+        "tiny-filinex", width=96, vocab=320, heads=4, kv_heads=2, dim=24, lin_heads=3,
+        lin_dim=16, lin_vdim=40, wkv_dim=32, rank=8, experts=6, top=2, ff=40, shared_ff=56,
+        times=2, max_positions=1024,
+    ),
+    # layers as wide as llama-1b's and llama-3-8b's
+    "filinex-small": _filinex_preset(
+        "filinex-small", width=2048, vocab=128256, heads=16, kv_heads=4, dim=128,
+        lin_heads=8, lin_dim=128, lin_vdim=256, wkv_dim=64, rank=16, experts=32, top=4,
+        ff=1536, shared_ff=2048, times=2, repeat=3,
+    ),
+    "filinex-base": _filinex_preset(
+        "filinex-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=128,
+        lin_heads=16, lin_dim=128, lin_vdim=256, wkv_dim=64, rank=16, experts=64, top=6,
+        ff=1536, shared_ff=5120, times=2, repeat=4,
     ),
     # small-but-real shape for 1-GPU kernel shakedown
     "llama-1b": ModelConfig(

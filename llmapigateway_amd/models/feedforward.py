@@ -1,0 +1,85 @@
+"""Feed-forwards of the hybrid decoders, each built from its sizes and
+constants and its checkpoint tensors; called with the normed rows, they
+return what is to be added to the residual stream: a tensor, or the experts'
+parts of it (ops.ExpertSum), which the next stream kernel adds up."""
+
+from __future__ import annotations
+
+from typing import Callable, Dict, Tuple
+
+import torch
+
+from .. import ops
+from .twins import add_decode_twins
+
+Getter = Callable[[str], torch.Tensor]
+
+
+class DenseFF:
+    """W_down (silu(W_gate h) * W_up h)."""
+
+    def __init__(self, m: dict, get: Getter, vec: Getter):
+        self.w = {"gate_up": torch.cat([get("gate"), get("up")]), "down": get("down")}
+        add_decode_twins(self.w, ("gate_up", "down"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        ff = m["ff"]
+        return {"gate": (ff, width), "up": (ff, width), "down": (width, ff)}
+
+    def __call__(self, h: torch.Tensor) -> torch.Tensor:
+        w = self.w
+        return ops.linear(
+            ops.swiglu_linear(h, w["gate_up"], w.get("gate_up_swz"), w.get("gate_up_int")),
+            w["down"], w.get("down_swz"),
+        )
+
+
+class ExpertFF:
+    """Clamped-SwiGLU experts of which a router picks ``top`` per token
+    (weights: softmax over the chosen logits), and a shared one for every
+    token. Expert: g = min(W_gate h, limit), u = clamp(W_up h, +-limit),
+    W_down (g sigmoid(1.702 g) (u + 1))."""
+
+    def __init__(self, m: dict, get: Getter, vec: Getter):
+        E = m["router"]["experts"]
+        self.top = m["router"]["top"]
+        self.limit = float(m["expert"]["limit"])
+        self.w_router, self.b_router = get("router"), vec("router.b")
+        self.experts = ops.pack_experts(
+            m["expert"]["ff"], self.w_router.shape[1], E,
+            lambda e: (get(f"e{e}.gate"), get(f"e{e}.up"), get(f"e{e}.down")),
+        )
+        self.shared = None
+        if m.get("shared") is not None:
+            self.shared_limit = float(m["shared"]["limit"])
+            self.shared = {
+                "gate_up": torch.cat([get("shared.gate"), get("shared.up")]),
+                "down": get("shared.down"),
+            }
+            add_decode_twins(self.shared, ("down",))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        E = m["router"]["experts"]
+        out: Dict[str, Tuple[int, ...]] = {"router": (E, width), "router.b": (E,)}
+        parts = [(f"e{e}", m["expert"]["ff"]) for e in range(E)]
+        if m.get("shared") is not None:
+            parts.append(("shared", m["shared"]["ff"]))
+        for name, ff in parts:
+            out[f"{name}.gate"] = out[f"{name}.up"] = (ff, width)
+            out[f"{name}.down"] = (width, ff)
+        return out
+
+    def __call__(self, h: torch.Tensor) -> "ops.ExpertSum":
+        routing = ops.route_experts(h, self.w_router, self.b_router, self.top, self.experts)
+        rows = ops.expert_rows(h, routing, self.experts, self.limit)
+        shared = None
+        if self.shared is not None:
+            s = self.shared
+            act = ops.clamped_glu(ops.linear(h, s["gate_up"]), self.shared_limit)
+            shared = ops.linear(act, s["down"], s.get("down_swz"))
+        return ops.ExpertSum(rows, routing.slot, routing.weights, shared)
+
+
+FEEDFORWARDS = {"dense": DenseFF, "moe": ExpertFF}

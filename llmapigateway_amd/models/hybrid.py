@@ -1,13 +1,14 @@
 """Hybrid decoder: every layer names its mixer; a stretch of layers can run
 several times in a row with the same weights.
 
-The residual stream is fp32; a sublayer's output stays pending and is added
-by the next norm's kernel (ops.add_layernorm). A loop pass starts by
-replacing the stream with W [stream; embedding output] + step[t]; each pass
-of a layer has its own cache view.
+The residual stream is fp32; a sublayer's output stays pending, with its own
+norm where the design has one, and is added by the next norm's kernel
+(ops.add_layernorm, ops.add_tanh_norm). A loop pass starts by replacing the
+stream with W [stream; embedding output] (+ step[t]); each pass of a layer
+has its own cache view.
 
-Serves Lelisun; another design built from these mixers needs only a
-configuration.
+Serves Lelisun and Filinex; another design built from these mixers and
+feed-forwards needs only a configuration.
 """
 
 from __future__ import annotations
@@ -19,8 +20,8 @@ import torch
 from .. import ops
 from .batch import ForwardBatch
 from .configs import HybridConfig
+from .feedforward import FEEDFORWARDS
 from .mixers import MIXERS
-from .twins import add_decode_twins
 from .weights import open_checkpoint
 
 
@@ -49,6 +50,7 @@ class HybridModel:
         self.dtype = dtype
         self.max_positions = max_positions or config.max_positions
         self._ropes: Dict[tuple, torch.Tensor] = {}
+        self.plans = {p for layer in config.layers for p in MIXERS[layer.type].plans}
         self._build(self._source(seed))
 
     # ---- weights ----
@@ -56,19 +58,30 @@ class HybridModel:
     def tensor_shapes(config: HybridConfig) -> Dict[str, tuple]:
         """Checkpoint tensor name -> shape."""
         W, V = config.hidden_size, config.vocab_size
-        out = {"embed": (V, W), "final.norm": (W,), "final.norm.b": (W,), "head": (V, W)}
+        out = {"embed": (V, W), "head": (V, W)}
+
+        def norm(name: str) -> None:
+            out[name] = out[name + ".b"] = (W,)
+            if config.norm == "tanh":
+                out[name + ".alpha"] = ()
+
+        norm("final.norm")
+        if config.embed_norm:
+            norm("embed.norm")
         if config.loop is not None:
             out["loop.in"] = (W, 2 * W)
-            out["loop.step"] = (config.loop[2], W)
+            if config.loop_step:
+                out["loop.step"] = (config.loop[2], W)
         for i, layer in enumerate(config.layers):
-            out[f"l{i}.norm1"] = out[f"l{i}.norm1.b"] = (W,)
             for k, s in MIXERS[layer.type].shapes(layer.mixer, W).items():
                 out[f"l{i}.mix.{k}"] = s
             if layer.mlp is not None:
-                ff = layer.mlp["ff"]
-                out[f"l{i}.norm2"] = out[f"l{i}.norm2.b"] = (W,)
-                out[f"l{i}.mlp.gate"] = out[f"l{i}.mlp.up"] = (ff, W)
-                out[f"l{i}.mlp.down"] = (W, ff)
+                for k, s in FEEDFORWARDS[layer.mlp["kind"]].shapes(layer.mlp, W).items():
+                    out[f"l{i}.mlp.{k}"] = s
+            for n in "12" if layer.mlp is not None else "1":
+                norm(f"l{i}.norm{n}")
+                if config.post_norm:
+                    norm(f"l{i}.norm{n}b")
         return out
 
     def _source(self, seed: int):
@@ -91,12 +104,16 @@ class HybridModel:
         def draw(name: str) -> torch.Tensor:
             shape, leaf = shapes[name], name.rsplit(".", 1)[-1]
             t = torch.empty(shape, dtype=torch.float32, device=device)
-            if leaf in ("norm", "norm1", "norm2", "D"):
+            if leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b", "D", "alpha"):
                 return t.fill_(1.0)
             if leaf == "b" or leaf == "A_log":
-                return t.fill_(2.0 if name.endswith(".f.b") else 0.0)
+                return t.fill_(2.0 if name.endswith((".f.b", ".a2.b")) else 0.0)
             if leaf == "dt_bias":
                 return t.fill_(-2.0)
+            if leaf == "w0":
+                return t.normal_(-1.5, 1.0, generator=gen)
+            if ".mu." in name:
+                return t.uniform_(0.0, 1.0, generator=gen)
             std = 1.0 / scale if name == "embed" else 0.02 if name == "loop.step" else (
                 1.0 if len(shape) == 1 else shape[-1] ** -0.5
             )
@@ -113,15 +130,22 @@ class HybridModel:
         def vec(name: str) -> torch.Tensor:  # small vectors and taps: fp32
             return source(name).to(self.device).float().contiguous()
 
+        def norm(name: str):
+            parts = (vec(name), vec(name + ".b"))
+            return parts + (float(source(name + ".alpha")),) if c.norm == "tanh" else parts
+
         self.embed = mat("embed")
+        self.embed_norm = norm("embed.norm") if c.embed_norm else None
         self.loop_in = self.loop_step = None
         if c.loop is not None:
-            self.loop_in, self.loop_step = mat("loop.in"), vec("loop.step")
+            self.loop_in = mat("loop.in")
+            self.loop_step = vec("loop.step") if c.loop_step else [None] * c.loop[2]
         self.layers: List[dict] = []
         for i, layer in enumerate(c.layers):
             p = f"l{i}."
             ent = {
-                "norm1": (vec(p + "norm1"), vec(p + "norm1.b")),
+                "norm1": norm(p + "norm1"),
+                "norm1b": norm(p + "norm1b") if c.post_norm else None,
                 "mixer": MIXERS[layer.type](
                     layer.mixer, c.norm_eps,
                     lambda n, p=p: mat(f"{p}mix.{n}"), lambda n, p=p: vec(f"{p}mix.{n}"),
@@ -130,14 +154,14 @@ class HybridModel:
                 "mlp": None,
             }
             if layer.mlp is not None:
-                ent["norm2"] = (vec(p + "norm2"), vec(p + "norm2.b"))
-                ent["mlp"] = {
-                    "gate_up": torch.cat([mat(p + "mlp.gate"), mat(p + "mlp.up")]),
-                    "down": mat(p + "mlp.down"),
-                }
-                add_decode_twins(ent["mlp"], ("gate_up", "down"))
+                ent["norm2"] = norm(p + "norm2")
+                ent["norm2b"] = norm(p + "norm2b") if c.post_norm else None
+                ent["mlp"] = FEEDFORWARDS[layer.mlp["kind"]](
+                    layer.mlp,
+                    lambda n, p=p: mat(f"{p}mlp.{n}"), lambda n, p=p: vec(f"{p}mlp.{n}"),
+                )
             self.layers.append(ent)
-        self.final_norm = (vec("final.norm"), vec("final.norm.b"))
+        self.final_norm = norm("final.norm")
         self.head = mat("head")
 
     def _rope(self, base: float, dims: int) -> torch.Tensor:
@@ -149,42 +173,58 @@ class HybridModel:
         return self._ropes[key]
 
     # ---- forward ----
+    def _norm(self, x, delta, post, norm, vec=None, replace=False) -> torch.Tensor:
+        """Add the pending sublayer output (through its own norm, ``post``)
+        to the stream, or replace the stream by it; the normed rows."""
+        if self.config.norm == "tanh":
+            return ops.add_tanh_norm(x, delta, post, norm, self.dtype, replace=replace)
+        return ops.add_layernorm(
+            x, delta, *norm, self.config.norm_eps, self.dtype, vec=vec, replace=replace
+        )
+
+    def _cast(self, x, delta, post, out) -> None:
+        """The same addition; the stream itself goes to ``out``."""
+        if self.config.norm == "tanh":
+            ops.add_tanh_norm(x, delta, post, None, self.dtype, out=out)
+        else:
+            ops.add_cast(x, delta, out)
+
     @torch.inference_mode()
     def step(self, batch: ForwardBatch, cache) -> torch.Tensor:
         """Logits [B, vocab] (fp32) at batch.logits_indices (every row if
         that is None); the caches take in the batch's rows."""
-        c, eps, W = self.config, self.config.norm_eps, self.config.hidden_size
-        plan = ops.plan_segments(batch, self.dtype)
+        c, W = self.config, self.config.hidden_size
+        plan = ops.plan_segments(batch, self.dtype, self.plans)
         T = batch.token_ids.shape[0]
         both = x0 = None
         if c.loop is not None:  # [stream; embedding output], the loop's input
             both = torch.empty(T, 2 * W, dtype=self.dtype, device=self.device)
             x0 = both[:, W:]
-        x = ops.embed_scaled(batch.token_ids, self.embed, c.embed_scale, x0)
-        delta = None
+        if self.embed_norm is None:
+            x = ops.embed_scaled(batch.token_ids, self.embed, c.embed_scale, x0)
+        else:
+            x = ops.embed_tanh_norm(batch.token_ids, self.embed, self.embed_norm, x0)
+        delta = post = None
         for r, (i, t) in enumerate(c.runs()):
             layer = self.layers[i]
             if t is None:
-                h = ops.add_layernorm(x, delta, *layer["norm1"], eps, self.dtype)
+                h = self._norm(x, delta, post, layer["norm1"])
             else:
-                ops.add_cast(x, delta, both[:, :W])
-                h = ops.add_layernorm(
-                    x, ops.linear_f32(both, self.loop_in), *layer["norm1"], eps,
-                    self.dtype, vec=self.loop_step[t], replace=True,
+                self._cast(x, delta, post, both[:, :W])
+                h = self._norm(
+                    x, ops.linear_f32(both, self.loop_in), None, layer["norm1"],
+                    vec=self.loop_step[t], replace=True,
                 )
-            delta = layer["mixer"](h, batch, cache.runs[r], plan)
+            delta, post = layer["mixer"](h, batch, cache.runs[r], plan), layer["norm1b"]
             if layer["mlp"] is not None:
-                m = layer["mlp"]
-                h = ops.add_layernorm(x, delta, *layer["norm2"], eps, self.dtype)
-                delta = ops.linear(
-                    ops.swiglu_linear(
-                        h, m["gate_up"], m.get("gate_up_swz"), m.get("gate_up_int")
-                    ),
-                    m["down"], m.get("down_swz"),
-                )
+                h = self._norm(x, delta, post, layer["norm2"])
+                delta, post = layer["mlp"](h), layer["norm2b"]
         if batch.logits_indices is not None:
             x, delta = x[batch.logits_indices], delta[batch.logits_indices]
             if x.shape[0] == 0:
                 return torch.empty(0, c.vocab_size, dtype=torch.float32, device=self.device)
-        h = ops.add_layernorm(x, delta, *self.final_norm, eps, self.dtype)
-        return ops.linear_f32(h, self.head)
+        h = self._norm(x, delta, post, self.final_norm)
+        logits = ops.linear_f32(h, self.head)
+        if c.logit_softcap is not None:
+            ops.soft_cap_(logits, c.logit_softcap)
+        return logits

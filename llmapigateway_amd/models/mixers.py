@@ -35,6 +35,21 @@ def _pad8(n: int) -> int:
     return (n + 7) // 8 * 8
 
 
+def _stack(parts):
+    """Weights [n, width] stacked to one, every part at a multiple of 8 rows
+    and all of it a multiple of 64 (zero rows in between); the parts' row
+    ranges by name."""
+    rows, cut, at = [], {}, 0
+    for i, (name, w) in enumerate(parts):
+        cut[name] = (at, at + w.shape[0])
+        end = (at + w.shape[0] + 7) // 8 * 8
+        if i + 1 == len(parts):
+            end = (end + 63) // 64 * 64
+        rows += [w, w.new_zeros(end - cut[name][1], w.shape[1])]
+        at = end
+    return torch.cat(rows), cut
+
+
 class LatentAttention:
     """Attention whose keys and values unfold from one cached latent per
     token, plus one rotated key part that all heads share; the softmax has
@@ -44,6 +59,8 @@ class LatentAttention:
     scores and sums run over the cached rows themselves; decode and short
     portions) and unfolded (per-head keys and values are made from the
     latents; long portions)."""
+
+    plans = ("unfold",)  # what it uses of a step's plan
 
     def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
         self.m, self.eps = m, eps
@@ -79,7 +96,7 @@ class LatentAttention:
         }
 
     @staticmethod
-    def cache_spec(m: dict) -> CacheSpec:
+    def cache_spec(m: dict, width: int) -> CacheSpec:
         return CacheSpec({"latent": _pad8(m["kv_rank"] + m["rot_dim"])}, {})
 
     def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
@@ -117,6 +134,8 @@ class Mamba2:
     """State-space duality layer: short causal convolution, scalar decay
     per head, B and C shared by the heads of a group, gated group norm."""
 
+    plans = ("chunks",)  # what it uses of a step's plan
+
     def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
         self.m, self.eps = m, eps
         self.H, self.P, self.N, self.G = m["heads"], m["vdim"], m["state"], m["groups"]
@@ -141,7 +160,7 @@ class Mamba2:
         }
 
     @staticmethod
-    def cache_spec(m: dict) -> CacheSpec:
+    def cache_spec(m: dict, width: int) -> CacheSpec:
         channels = m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]
         return CacheSpec({}, {
             "S": ((m["heads"], m["vdim"], m["state"]), True),
@@ -170,6 +189,8 @@ class MLSTM:
     """Matrix-memory recurrence with exponential gates kept in range by a
     running maximum, a normaliser state, head-wise norm and output gate."""
 
+    plans = ("chunks",)  # what it uses of a step's plan
+
     def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
         self.m, self.eps = m, eps
         self.H, self.dk, self.dv = m["heads"], m["dim"], m["vdim"]
@@ -193,7 +214,7 @@ class MLSTM:
         }
 
     @staticmethod
-    def cache_spec(m: dict) -> CacheSpec:
+    def cache_spec(m: dict, width: int) -> CacheSpec:
         H, dk, dv = m["heads"], m["dim"], m["vdim"]
         return CacheSpec({}, {
             # every tile of 64 value rows carries its own n and m
@@ -216,4 +237,175 @@ class MLSTM:
         return ops.linear(y, w["o"], w.get("o_swz"))
 
 
-MIXERS = {"latent_attention": LatentAttention, "mamba2": Mamba2, "mlstm": MLSTM}
+class GatedAttention:
+    """Grouped-query attention without rotation: soft-capped scores, a
+    learned sink per head in the softmax's denominator, and a sigmoid gate
+    per head on its output. Leaves the heads' outputs in the rows it is
+    given; the projections around it belong to the mixer that holds it."""
+
+    def __init__(self, m: dict, get: Getter, vec: Getter, out_scale: float):
+        self.H, self.G, self.dim, self.vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.scale, self.cap = float(m["scale"]), float(m["softcap"])
+        self.sink, self.out_scale = vec("sink"), out_scale
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H, G = m["heads"], m["kv_heads"]
+        return {
+            "q": (H * m["dim"], width), "k": (G * m["dim"], width),
+            "v": (G * m["vdim"], width), "sink": (H,), "g": (H, width),
+            "o": (width, H * m["vdim"]),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        return CacheSpec({"k": m["kv_heads"] * m["dim"], "v": m["kv_heads"] * m["vdim"]}, {})
+
+    def __call__(self, q, k, v, gate, out, batch: ForwardBatch, cache, plan) -> None:
+        ops.page_write(k, v, cache["k"], cache["v"], batch.slot_mapping)
+        ops.paged_attention(
+            out, q, cache["k"], cache["v"], self.H, self.G, self.sink, self.scale, self.cap,
+            gate, self.out_scale, batch.positions, batch.segs, plan,
+        )
+
+
+class GatedLinearAttention:
+    """Linear attention with a decay per key channel, sigmoid(z)^(1/tau) of a
+    low-rank projection z, head-wise RMS norm and a silu gate."""
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, out_scale: float):
+        self.H, self.dk, self.dv, self.eps = m["heads"], m["dim"], m["vdim"], eps
+        self.tau = float(m["tau"])
+        self.a2, self.a2_bias = get("a2"), vec("a2.b")
+        # the norm's weight, shared by the heads, takes the output's scale
+        self.norm = (vec("norm") * out_scale).repeat(self.H)
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        kk, vv, rank = m["heads"] * m["dim"], m["heads"] * m["vdim"], m["decay_rank"]
+        return {
+            "q": (kk, width), "k": (kk, width), "v": (vv, width), "g": (vv, width),
+            "o": (width, vv), "norm": (m["vdim"],), "a1": (rank, width), "a2": (kk, rank),
+            "a2.b": (kk,),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        return CacheSpec({}, {"S": ((m["heads"], m["vdim"], m["dim"]), True)})
+
+    def __call__(self, q, k, v, gate, a, out, batch: ForwardBatch, cache, plan) -> None:
+        logw = ops.decay_logs(a, self.a2, self.a2_bias, "sigmoid", self.tau)
+        y = ops.decayed_kv(
+            q, k, v, logw, None, self.dk ** -0.5, self.H, self.dk, self.dv, cache["S"],
+            batch.positions, batch.segs, plan,
+        )
+        ops.head_norm_gate(out, y, gate, self.norm, self.H, self.eps)
+
+
+class Parallel:
+    """Gated attention (left) and gated linear attention (right) side by
+    side on the same rows: one product projects for both, and one product of
+    their joined outputs, each scaled already, sums both output projections."""
+
+    plans = ("tiles", "chunks")  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        def side(f, name):
+            return lambda n: f(f"{name}.{n}")
+
+        gl, gr = side(get, "left"), side(get, "right")
+        self.left = GatedAttention(m["left"], gl, side(vec, "left"), float(m["left_scale"]))
+        self.right = GatedLinearAttention(
+            m["right"], eps, gr, side(vec, "right"), float(m["right_scale"])
+        )
+        w_in, self.cut = _stack([
+            ("q", gl("q")), ("k", gl("k")), ("v", gl("v")), ("rq", gr("q")), ("rk", gr("k")),
+            ("rv", gr("v")), ("rg", gr("g")), ("a", gr("a1")), ("g", gl("g")),
+        ])
+        o_l, o_r = gl("o"), gr("o")
+        self.n_left, self.n_right = o_l.shape[1], o_r.shape[1]
+        pad = _pad8(self.n_left) - self.n_left  # the right half starts aligned
+        self.w = {
+            "in": w_in, "o": torch.cat([o_l, o_l.new_zeros(o_l.shape[0], pad), o_r], 1),
+        }
+        add_decode_twins(self.w, ("in", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        out = {f"left.{k}": s for k, s in GatedAttention.shapes(m["left"], width).items()}
+        for k, s in GatedLinearAttention.shapes(m["right"], width).items():
+            out[f"right.{k}"] = s
+        return out
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        left = GatedAttention.cache_spec(m["left"], width)
+        right = GatedLinearAttention.cache_spec(m["right"], width)
+        return CacheSpec({**left.pages, **right.pages}, {**left.state, **right.state})
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        p = {name: u[:, lo:hi] for name, (lo, hi) in self.cut.items()}
+        K = w["o"].shape[1]
+        both = torch.empty(h.shape[0], K, dtype=h.dtype, device=h.device)
+        if K != self.n_left + self.n_right:
+            both.zero_()  # the columns between the halves
+        self.left(p["q"], p["k"], p["v"], p["g"], both[:, : self.n_left], batch, cache, plan)
+        self.right(
+            p["rq"], p["rk"], p["rv"], p["rg"], p["a"], both[:, K - self.n_right :],
+            batch, cache, plan,
+        )
+        return ops.linear(both, w["o"], w.get("o_swz"))
+
+
+class WKV:
+    """RWKV-style time mixing: every projection reads its own mix of a
+    token's row and the previous one; a data-dependent decay per key channel,
+    exp(-exp(.)), and a bonus for the current token only."""
+
+    plans = ("chunks",)  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.H, self.d, self.eps = m["heads"], m["dim"], eps
+        self.mu = torch.stack([vec(f"mu.{s}") for s in "rkvgw"])
+        self.w = {s: get(s) for s in ("r", "k", "v", "g", "w1", "o")}
+        self.w2, self.w0, self.u = get("w2"), vec("w0"), vec("u")
+        self.norm = vec("norm")
+        add_decode_twins(self.w, ("r", "k", "v", "g", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        n, rank = m["heads"] * m["dim"], m["decay_rank"]
+        out: Dict[str, Tuple[int, ...]] = {f"mu.{s}": (width,) for s in "rkvgw"}
+        out.update({s: (n, width) for s in "rkvg"})
+        out.update({
+            "w1": (rank, width), "w2": (n, rank), "w0": (n,), "u": (m["heads"], m["dim"]),
+            "norm": (n,), "o": (width, n),
+        })
+        return out
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        return CacheSpec({}, {
+            "S": ((m["heads"], m["dim"], m["dim"]), True), "prev": ((width,), False),
+        })
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        mixes = ops.token_shift(h, self.mu, cache["prev"], batch.positions, batch.segs)
+        r, k, v, g = (ops.linear(mixes[i], w[s], w.get(s + "_swz")) for i, s in enumerate("rkvg"))
+        logw = ops.decay_logs(ops.linear(mixes[4], w["w1"]), self.w2, self.w0, "exp", 1.0)
+        y = ops.decayed_kv(
+            r, k, v, logw, self.u, 1.0, self.H, self.d, self.d, cache["S"],
+            batch.positions, batch.segs, plan,
+        )
+        out = torch.empty_like(y)
+        ops.head_norm_gate(out, y, g, self.norm, self.H, self.eps)
+        return ops.linear(out, w["o"], w.get("o_swz"))
+
+
+MIXERS = {
+    "latent_attention": LatentAttention, "mamba2": Mamba2, "mlstm": MLSTM,
+    "parallel": Parallel, "wkv": WKV,
+}

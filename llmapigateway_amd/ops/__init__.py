@@ -544,23 +544,35 @@ def sample(
     return reference.sample(logits, temperature, noise)
 
 
+from .experts import (  # noqa: E402
+    ExpertSum, clamped_glu, expert_rows, pack_experts, route_experts,
+)
 from .hybrid import (  # noqa: E402
     add_cast,
     add_layernorm,
+    add_tanh_norm,
     build_pair_rope_cache,
     can_unfold,
     causal_conv,
+    decay_logs,
+    decayed_kv,
     embed_scaled,
+    embed_tanh_norm,
     fold_queries,
     gated_norm,
     head_linear,
+    head_norm_gate,
     latent_attention_folded,
     latent_attention_unfolded,
     latent_rows,
     linear_f32,
     mlstm,
+    page_write,
+    paged_attention,
     plan_segments,
+    soft_cap_,
     ssd,
+    token_shift,
 )
 
 __all__ = [

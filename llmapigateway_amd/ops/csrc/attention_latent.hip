@@ -4,6 +4,7 @@
 // Folded form: queries are already in the latent space, one cached row is
 // key and value of every head. Unfolded form: per-head keys and values.
 
+#include "lds_dma.h"
 #include "mfma.h"
 
 #define LA_THREADS 256
@@ -131,26 +132,6 @@ extern "C" hipError_t launch_latent_folded_any(
 #define LF_KT 64
 #define LF_PAGES 512  // page ids held in LDS (a tile has at most 64)
 #define LA_NEG (-1e30f)
-
-// lds_barrier: LDS data of the workgroup's waves is visible after it, while
-// transfers of dma16 stay in flight across it; dma_barrier: they too have
-// landed.
-__device__ __forceinline__ void lds_barrier() {
-    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-}
-__device__ __forceinline__ void dma_barrier() {
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
-}
-// 16 bytes a lane from global memory to LDS at lds (wave-uniform) + 16*lane.
-// As asm: the compiler would let every later LDS read wait for the transfer;
-// here only dma_barrier does. (Wait counts it places for its own loads are
-// only stricter for the transfers it does not see.)
-__device__ __forceinline__ void dma16(const bf16* src, const bf16* lds) {
-    const uint32_t at = __builtin_amdgcn_readfirstlane(
-        (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) bf16*)lds);
-    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
-                 ::"s"(at), "v"(src) : "memory", "m0");
-}
 
 // NKC: 32-wide chunks that cover a cached row (even); RT: 16-wide tiles that
 // cover the rank (a multiple of 4, at most 2*NKC)

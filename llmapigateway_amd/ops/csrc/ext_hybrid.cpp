@@ -3,13 +3,16 @@
 // kernels assume them.
 
 #include "bind_shared.h"
+#include "bind_checks.h"
+
+void bind_parallel(pybind11::module_& m);  // bind_parallel.cpp
 
 extern "C" {
 hipError_t launch_embed_scaled(float*, void*, int64_t, const int64_t*, const void*, float, int, int, int, int, hipStream_t);
 hipError_t launch_stream_norm(void*, int64_t, float*, const void*, int, const float*, const float*, const float*, float, int, int, int, int, int, hipStream_t);
 hipError_t launch_latent_rows(void*, void*, int, const void*, const float*, const float*, float, int, int, int, const int64_t*, const float*, const int64_t*, int, int, int, hipStream_t);
 hipError_t launch_rotate_pairs(void*, int64_t, int64_t, int, const void*, int64_t, int64_t, int, int, const int64_t*, const float*, int, int, hipStream_t);
-hipError_t launch_gated_norm(void*, const void*, const void*, int64_t, const float*, float, int, int, int, int, int, int, hipStream_t);
+hipError_t launch_gated_norm(void*, int64_t, const void*, const void*, int64_t, const float*, float, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_causal_conv(void*, const void*, int64_t, const float*, const float*, void*, const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_head_linear(void*, int64_t, int64_t, const void*, int64_t, int64_t, const void*, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_latent_folded_any(void*, const void*, const void*, const float*, float, const int64_t*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
@@ -22,55 +25,6 @@ hipError_t launch_mlstm_chunked(void*, const void*, int64_t, const void*, int64_
 }
 
 namespace {
-
-using torch::Tensor;
-using OptTensor = c10::optional<Tensor>;
-
-bool has(const OptTensor& t) { return t.has_value() && t->defined(); }
-
-// compute dtype of an activation; returns whether it is fp32
-bool is_f32(const Tensor& t, const char* name) {
-    TORCH_CHECK(t.is_cuda(), name, " must be on GPU");
-    TORCH_CHECK(t.scalar_type() == torch::kBFloat16 || t.scalar_type() == torch::kFloat32,
-                name, " must be bf16 or fp32");
-    return t.scalar_type() == torch::kFloat32;
-}
-const float* f32_ptr(const Tensor& t, int64_t numel, const char* name) {
-    TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 && t.is_contiguous() &&
-                t.numel() == numel, name, ": fp32, dense, ", numel, " elements");
-    return t.data_ptr<float>();
-}
-const int* i32_ptr(const Tensor& t, int64_t at_least, const char* name) {
-    TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 && t.is_contiguous() &&
-                t.numel() >= at_least, name, ": int32, dense, >= ", at_least, " elements");
-    return t.data_ptr<int>();
-}
-const int64_t* i64_ptr(const Tensor& t, int64_t at_least, const char* name) {
-    TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt64 && t.is_contiguous() &&
-                t.numel() >= at_least, name, ": int64, dense, >= ", at_least, " elements");
-    return t.data_ptr<int64_t>();
-}
-void same_type(const Tensor& a, const Tensor& b, const char* what) {
-    TORCH_CHECK(a.is_cuda() && b.is_cuda() && a.scalar_type() == b.scalar_type(), what,
-                ": dtypes differ");
-}
-// rows of a 2D tensor whose last dimension is dense
-void check_rows(const Tensor& t, int64_t rows, int64_t width, const char* name) {
-    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == width &&
-                (t.stride(1) == 1 || width <= 1), name, ": [", rows, ", ", width,
-                "] with dense rows");
-}
-// 8-element accesses possible: base 16-byte aligned, strides multiples of 8
-bool vec8(std::initializer_list<const Tensor*> ts, std::initializer_list<int64_t> dims) {
-    for (int64_t d : dims)
-        if (d % 8) return false;
-    for (const Tensor* t : ts) {
-        if (reinterpret_cast<uintptr_t>(t->data_ptr()) % 16) return false;
-        for (int64_t i = 0; i + 1 < t->dim(); ++i)
-            if (t->stride(i) % 8) return false;
-    }
-    return true;
-}
 
 void embed_scaled(Tensor x, OptTensor x0, Tensor tokens, Tensor embed, double scale) {
     const bool f32 = is_f32(embed, "embed");
@@ -376,19 +330,22 @@ void mlstm_chunked(Tensor y, Tensor q, Tensor k, Tensor v, Tensor gates, Tensor 
         n_in.data_ptr<float>(), m_in.data_ptr<float>(), current_stream()));
 }
 
+// mode 0: rms(y) w sigmoid(gate), 1: rms(y silu(gate)) w, 2: rms(y) w silu(gate)
 void gated_norm(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t groups, double eps,
-                bool gate_first) {
+                int64_t mode) {
     const bool f32 = is_f32(y, "y");
     same_type(y, gate, "gate");
     same_type(y, out, "out");
     const int64_t T = y.size(0), W = y.size(1);
-    TORCH_CHECK(y.is_contiguous() && out.is_contiguous() && out.numel() == T * W);
+    TORCH_CHECK(y.is_contiguous());
+    check_rows(out, T, W, "out");
     check_rows(gate, T, W, "gate");
     TORCH_CHECK(groups > 0 && W % groups == 0);
     const int64_t gs = W / groups;
-    CHECK_HIP(launch_gated_norm(out.data_ptr(), y.data_ptr(), gate.data_ptr(), gate.stride(0),
-                                f32_ptr(w, W, "w"), (float)eps, groups, gs, gate_first, T,
-                                f32, vec8({&out, &y, &gate, &w}, {gs}), current_stream()));
+    CHECK_HIP(launch_gated_norm(out.data_ptr(), out.stride(0), y.data_ptr(), gate.data_ptr(),
+                                gate.stride(0), f32_ptr(w, W, "w"), (float)eps, groups, gs,
+                                mode, T, f32, vec8({&out, &y, &gate, &w}, {gs}),
+                                current_stream()));
 }
 
 }  // namespace
@@ -410,5 +367,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("ssd_chunked", &ssd_chunked, "Mamba-2 recurrence, chunked");
     m.def("mlstm_chunked", &mlstm_chunked, "mLSTM recurrence, chunked");
     m.def("gated_norm", &gated_norm, "group RMS norm with a gate");
+    bind_parallel(m);
     bind_shared(m);
 }

@@ -6,81 +6,8 @@
 // any width; widths and strides that allow it are moved 16 bytes a lane.
 // Sums and transcendentals are fp32.
 
-#include "common.h"
+#include "rows.h"
 
-namespace {
-
-template <int VEC>
-__device__ __forceinline__ void load_vec(const float* p, float* f) {
-    if (VEC == 8) {
-        const float4 a = reinterpret_cast<const float4*>(p)[0];
-        const float4 b = reinterpret_cast<const float4*>(p)[1];
-        f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
-        f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
-    } else {
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) f[j] = p[j];
-    }
-}
-template <int VEC>
-__device__ __forceinline__ void load_vec(const bf16* p, float* f) {
-    if (VEC == 8) {
-        const uint4 v = *reinterpret_cast<const uint4*>(p);
-        unpack2(v.x, f[0], f[1]);
-        unpack2(v.y, f[2], f[3]);
-        unpack2(v.z, f[4], f[5]);
-        unpack2(v.w, f[6], f[7]);
-    } else {
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) f[j] = ldf(p + j);
-    }
-}
-template <int VEC>
-__device__ __forceinline__ void store_vec(float* p, const float* f) {
-    if (VEC == 8) {
-        reinterpret_cast<float4*>(p)[0] = make_float4(f[0], f[1], f[2], f[3]);
-        reinterpret_cast<float4*>(p)[1] = make_float4(f[4], f[5], f[6], f[7]);
-    } else {
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) p[j] = f[j];
-    }
-}
-template <int VEC>
-__device__ __forceinline__ void store_vec(bf16* p, const float* f) {
-    if (VEC == 8) {
-        uint4 v;
-        v.x = pack2(f[0], f[1]);
-        v.y = pack2(f[2], f[3]);
-        v.z = pack2(f[4], f[5]);
-        v.w = pack2(f[6], f[7]);
-        *reinterpret_cast<uint4*>(p) = v;
-    } else {
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) stf(p + j, f[j]);
-    }
-}
-
-__device__ __forceinline__ float block_sum(float v, float* red) {
-    v = wave_reduce_sum(v);
-    const int wave = threadIdx.x >> 6, n = (blockDim.x + 63) >> 6;
-    __syncthreads();
-    if ((threadIdx.x & 63) == 0) red[wave] = v;
-    __syncthreads();
-    float t = 0.f;
-    for (int w = 0; w < n; ++w) t += red[w];
-    return t;
-}
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-
-// threads per row: enough for VEC elements each, whole waves, at most 512
-inline int row_threads(int width, int vec) {
-    int t = (width + vec - 1) / vec;
-    t = (t + 63) / 64 * 64;
-    return t < 64 ? 64 : (t > 512 ? 512 : t);
-}
-
-}  // namespace
 
 // ---------------------------------------------------------------------------
 // x[t] = embed[token] * scale (fp32); x0[t] (compute dtype) the same
@@ -260,15 +187,16 @@ __global__ void rotate_pairs_kernel(
 
 // ---------------------------------------------------------------------------
 // Group norm with a gate: y (dense rows) in `groups` equal parts.
-//   GATE_FIRST: out = rms(y * silu(gate)) * w
-//   else:       out = rms(y) * w * sigmoid(gate)
+//   GATE 0: out = rms(y) * w * sigmoid(gate)
+//   GATE 1: out = rms(y * silu(gate)) * w
+//   GATE 2: out = rms(y) * w * silu(gate)
 // One workgroup per (row, group).
 // ---------------------------------------------------------------------------
-template <typename T, int VEC, bool GATE_FIRST>
+template <typename T, int VEC, int GATE>
 __launch_bounds__(512)
 __global__ void gated_norm_kernel(
-    T* __restrict__ out, const T* __restrict__ y, const T* __restrict__ gate, int64_t ld_gate,
-    const float* __restrict__ w, float eps, int groups, int gs) {
+    T* __restrict__ out, int64_t ld_out, const T* __restrict__ y, const T* __restrict__ gate,
+    int64_t ld_gate, const float* __restrict__ w, float eps, int groups, int gs) {
     __shared__ float red[8];
     constexpr int HELD = 32 / VEC;
     const size_t t = blockIdx.x;
@@ -285,7 +213,7 @@ __global__ void gated_norm_kernel(
         const int i = i0 + k * step;
         if (i >= gs) continue;
         load_vec<VEC>(yr + i, held[k]);
-        if (GATE_FIRST) {
+        if (GATE == 1) {
             float z[VEC];
             load_vec<VEC>(gr + i, z);
 #pragma unroll
@@ -303,13 +231,14 @@ __global__ void gated_norm_kernel(
         load_vec<VEC>(wr + i, wv);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) held[k][j] *= inv * wv[j];
-        if (!GATE_FIRST) {
+        if (GATE != 1) {
             float z[VEC];
             load_vec<VEC>(gr + i, z);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) held[k][j] *= sigmoid_f(z[j]);
+            for (int j = 0; j < VEC; ++j)
+                held[k][j] *= sigmoid_f(z[j]) * (GATE == 2 ? z[j] : 1.f);
         }
-        store_vec<VEC>(out + base + i, held[k]);
+        store_vec<VEC>(out + t * ld_out + (size_t)g * gs + i, held[k]);
     }
 }
 
@@ -466,33 +395,8 @@ __global__ void conv_step_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// launchers (f32: compute dtype is fp32; vec8: widths, strides and addresses
-// allow 8-element accesses)
+// launchers
 // ---------------------------------------------------------------------------
-template <typename T_, int V_>
-struct Form {
-    using T = T_;
-    static constexpr int V = V_;
-};
-
-// run launch(Form<compute dtype, elements per access>)
-template <typename F>
-static hipError_t pick(int f32, int vec8, F launch) {
-    if (f32) {
-        if (vec8) launch(Form<float, 8>{});
-        else launch(Form<float, 1>{});
-    } else {
-        if (vec8) launch(Form<bf16, 8>{});
-        else launch(Form<bf16, 1>{});
-    }
-    HIP_CHECK_LAST();
-    return hipSuccess;
-}
-#define FORM(f)                                                                \
-    using T = typename decltype(f)::T;                                         \
-    constexpr int V = decltype(f)::V;                                          \
-    (void)V
-
 extern "C" hipError_t launch_embed_scaled(
     float* x, void* x0, int64_t ld0, const int64_t* tokens, const void* embed, float scale,
     int rows, int W, int f32, int vec8, hipStream_t stream) {
@@ -552,23 +456,22 @@ extern "C" hipError_t launch_rotate_pairs(
 }
 
 extern "C" hipError_t launch_gated_norm(
-    void* out, const void* y, const void* gate, int64_t ld_gate, const float* w, float eps,
-    int groups, int gs, int gate_first, int rows, int f32, int vec8, hipStream_t stream) {
+    void* out, int64_t ld_out, const void* y, const void* gate, int64_t ld_gate,
+    const float* w, float eps, int groups, int gs, int mode, int rows, int f32, int vec8,
+    hipStream_t stream) {
     if (rows <= 0) return hipSuccess;
-    if (gs > 512 * 32) return hipErrorInvalidValue;
+    if (gs > 512 * 32 || mode < 0 || mode > 2) return hipErrorInvalidValue;
     const dim3 grid(rows, groups);
-    if (gate_first)
-        return pick(f32, vec8, [&](auto form) {
-            FORM(form);
-            gated_norm_kernel<T, V, true><<<grid, row_threads(gs, V), 0, stream>>>(
-                (T*)out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs);
-        });
-    else
-        return pick(f32, vec8, [&](auto form) {
-            FORM(form);
-            gated_norm_kernel<T, V, false><<<grid, row_threads(gs, V), 0, stream>>>(
-                (T*)out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs);
-        });
+    return pick(f32, vec8, [&](auto form) {
+        FORM(form);
+#define GO(GATE)                                                                  \
+    gated_norm_kernel<T, V, GATE><<<grid, row_threads(gs, V), 0, stream>>>(       \
+        (T*)out, ld_out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs)
+        if (mode == 0) GO(0);
+        else if (mode == 1) GO(1);
+        else GO(2);
+#undef GO
+    });
 }
 
 extern "C" hipError_t launch_causal_conv(

@@ -1,0 +1,647 @@
+// Linear recurrences with a decay per key channel for gfx950 (gated linear
+// attention, WKV): per head, with q, k in dk and v in dv dimensions,
+//
+//   GLA:  S_t = diag(w_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t
+//   WKV:  o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t,  then S_t as above
+//
+// The log decays log w come from a low-rank product (decay_logs). The state
+// is fp32, transposed [slots, H, dv, dk] as in recurrence.hip. Token by
+// token (decoding, short portions, fp32, any size) or in chunks of 64 rows
+// on MFMA. With F the chunk's inclusive sums of log w and E_t = F_t (GLA) or
+// F_(t-1) (WKV), all exponents below are <= 0:
+//
+//   o_t   = (q_t e^(E_t))^T S_in + sum_{s<t} P[t,s] v_s + d_t v_t
+//   P[t,s] = sum_i q_t[i] k_s[i] e^(E_t[i] - F_s[i]),  d_t = q_t.(u k_t), u = 1 for GLA
+//   S_out = diag(e^(F_L)) S_in + sum_s (k_s e^(F_L - F_s)) v_s^T
+//
+// P between two 16-row blocks factors through the sum R before the later one:
+// (q e^(E_t-R)).(k e^(R-F_s)); inside a block it is taken row by row.
+
+#include "mfma.h"
+#include "recurrence.h"
+
+#define CH 64  // rows per chunk
+#define LDT (CH + 8)
+
+// fp32 values as the sum of two bf16 fragments
+__device__ __forceinline__ void split_frag(const float* f, bf16x8& hi, bf16x8& lo) {
+    uint4 h, l;
+    uint32_t* hp = reinterpret_cast<uint32_t*>(&h);
+    uint32_t* lp = reinterpret_cast<uint32_t*>(&l);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        hp[i] = pack2(f[2 * i], f[2 * i + 1]);
+        float a, b;
+        unpack2(hp[i], a, b);
+        lp[i] = pack2(f[2 * i] - a, f[2 * i + 1] - b);
+    }
+    hi = as_frag(h);
+    lo = as_frag(l);
+}
+__device__ __forceinline__ void unpack8(const uint4& v, float* f) {
+    unpack2(v.x, f[0], f[1]);
+    unpack2(v.y, f[2], f[3]);
+    unpack2(v.z, f[4], f[5]);
+    unpack2(v.w, f[6], f[7]);
+}
+__device__ __forceinline__ void load8f(const float* p, float* f) {
+    const float4 a = reinterpret_cast<const float4*>(p)[0];
+    const float4 b = reinterpret_cast<const float4*>(p)[1];
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+}
+
+// ---------------------------------------------------------------------------
+// log decays from z = act(a) W2^T + bias
+//   EXP:  act = tanh, log w = -e^z          (w = exp(-exp(z)))
+//   else: act = id,   log w = log sigmoid(z) / tau
+// ---------------------------------------------------------------------------
+template <bool EXP>
+__device__ __forceinline__ float log_decay(float z, float inv_tau) {
+    // e^-80 is as good as 0, and sums of 64 of them keep their precision
+    return fmaxf(EXP ? -expf(z) : log_sigmoid_f(z) * inv_tau, -80.f);
+}
+
+#define DL_ROWS 8
+template <typename T, bool EXP>
+__launch_bounds__(256)
+__global__ void decay_logs_any_kernel(
+    float* __restrict__ out, const T* __restrict__ a, int64_t lda, const T* __restrict__ w2,
+    const float* __restrict__ bias, float inv_tau, int rows, int N, int R) {
+    extern __shared__ float act[];  // [DL_ROWS][R]
+    const int t0 = blockIdx.x * DL_ROWS, n = blockIdx.y * 256 + threadIdx.x;
+    for (int e = threadIdx.x; e < DL_ROWS * R; e += 256) {
+        const int t = t0 + e / R;
+        const float v = t < rows ? ldf(a + (size_t)t * lda + e % R) : 0.f;
+        act[e] = EXP ? tanhf(v) : v;
+    }
+    __syncthreads();
+    if (n >= N) return;
+    float z[DL_ROWS];
+#pragma unroll
+    for (int i = 0; i < DL_ROWS; ++i) z[i] = bias[n];
+    for (int r = 0; r < R; ++r) {
+        const float w = ldf(w2 + (size_t)n * R + r);
+#pragma unroll
+        for (int i = 0; i < DL_ROWS; ++i) z[i] = fmaf(act[i * R + r], w, z[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < DL_ROWS; ++i)
+        if (t0 + i < rows) out[(size_t)(t0 + i) * N + n] = log_decay<EXP>(z[i], inv_tau);
+}
+
+// MFMA form: a wave takes 16 rows x 64 channels; C fragments hold [channel][row]
+template <bool EXP>
+__launch_bounds__(256)
+__global__ void decay_logs_mfma_kernel(
+    float* __restrict__ out, const bf16* __restrict__ a, int64_t lda,
+    const bf16* __restrict__ w2, const float* __restrict__ bias, float inv_tau, int rows,
+    int N, int R) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, g = lane >> 4;
+    const int t = (blockIdx.x * 4 + wave) * 16 + r16, n0 = blockIdx.y * 64;
+    if ((blockIdx.x * 4 + wave) * 16 >= rows) return;
+    f32x4 acc[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int r0 = 0; r0 < R; r0 += 32) {
+        const int r = r0 + g * 8;
+        float f[8];
+        bf16x8 hi, lo;
+        uint4 x = {0, 0, 0, 0};
+        if (r < R && t < rows) x = *reinterpret_cast<const uint4*>(a + (size_t)t * lda + r);
+        unpack8(x, f);
+        if (EXP) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) f[i] = tanhf(f[i]);
+        }
+        split_frag(f, hi, lo);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            uint4 w = {0, 0, 0, 0};
+            const int n = n0 + j * 16 + r16;
+            if (r < R && n < N) w = *reinterpret_cast<const uint4*>(w2 + (size_t)n * R + r);
+            acc[j] = mfma16(as_frag(w), hi, acc[j]);
+            if (EXP) acc[j] = mfma16(as_frag(w), lo, acc[j]);
+        }
+    }
+    if (t >= rows) return;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int n = n0 + j * 16 + g * 4;
+        if (n >= N) continue;  // N is a multiple of 4
+        const float4 b = *reinterpret_cast<const float4*>(bias + n);
+        *reinterpret_cast<float4*>(out + (size_t)t * N + n) = make_float4(
+            log_decay<EXP>(acc[j][0] + b.x, inv_tau), log_decay<EXP>(acc[j][1] + b.y, inv_tau),
+            log_decay<EXP>(acc[j][2] + b.z, inv_tau), log_decay<EXP>(acc[j][3] + b.w, inv_tau));
+    }
+}
+
+// ---------------------------------------------------------------------------
+// Token by token: a workgroup holds 64 value rows of a head's state in
+// registers over a segment's tokens; 16 lanes share 4 value rows, a lane
+// holds key dims 64e + 4*l16 + j.
+// ---------------------------------------------------------------------------
+struct DecayArgs {
+    void* y;              // [T, H*dv]
+    const void *q, *k, *v;
+    int64_t ldq, ldk, ldv;
+    float* logw;          // [T, H*dk]
+    const float* u;       // WKV: [H, dk]
+    float qscale;
+    int T, H, dk, dv;
+    float* S;             // [slots, H, dv, dk]
+    const int64_t* positions;
+    const int *cu, *slots;
+    const int* seg_list;  // scan: nullable
+    // chunks
+    const int *segs, *first, *chunk_seg, *chunk_off;
+    uint16_t *s_hi, *s_lo;  // [chunks, H, dv, dk]
+};
+
+template <typename T, int E4, bool WKV>
+__launch_bounds__(256)
+__global__ void decay_scan_kernel(DecayArgs a) {
+    const int seg = a.seg_list ? a.seg_list[blockIdx.x] : blockIdx.x;
+    const int h = blockIdx.y, slot = a.slots[seg];
+    const int r0 = a.cu[seg], r1 = a.cu[seg + 1];
+    const int l16 = threadIdx.x & 15, grp = threadIdx.x >> 4;
+    const int row0 = blockIdx.z * 64 + grp * 4;
+    const int dk = a.dk, dv = a.dv, H = a.H;
+    T* y = (T*)a.y + (size_t)h * dv;
+    if (slot < 0) {  // padding row
+        for (int t = r0; t < r1; ++t)
+            if (l16 < 4 && row0 + l16 < dv) stf(y + (size_t)t * H * dv + row0 + l16, 0.f);
+        return;
+    }
+    const bool fresh = a.positions[r0] == 0, vec = (dk & 3) == 0;
+    float* Sp = a.S + ((size_t)slot * H + h) * dv * dk;
+    float S[4][E4][4], u[E4][4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        if (!fresh && row0 + r < dv) {
+            load_state<E4>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
+        } else {
+#pragma unroll
+            for (int e = 0; e < E4; ++e)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) S[r][e][j] = 0.f;
+        }
+    }
+    if (WKV) load_state<E4>(a.u + (size_t)h * dk, l16, dk, false, u);
+    for (int t = r0; t < r1; ++t) {
+        float k[E4][4], q[E4][4], w[E4][4], v[4], o[4];
+        load_dims<T, E4>((const T*)a.k + (size_t)t * a.ldk + (size_t)h * dk, l16, dk, k);
+        load_dims<T, E4>((const T*)a.q + (size_t)t * a.ldq + (size_t)h * dk, l16, dk, q);
+        load_state<E4>(a.logw + ((size_t)t * H + h) * dk, l16, dk, vec, w);
+        const T* vp = (const T*)a.v + (size_t)t * a.ldv + (size_t)h * dv;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = row0 + r < dv ? ldf(vp + row0 + r) : 0.f;
+        float bonus = 0.f;
+#pragma unroll
+        for (int e = 0; e < E4; ++e)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                q[e][j] *= a.qscale;
+                w[e][j] = expf(w[e][j]);
+                if (WKV) bonus = fmaf(q[e][j] * u[e][j], k[e][j], bonus);
+            }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            float s = WKV ? bonus * v[r] : 0.f;
+#pragma unroll
+            for (int e = 0; e < E4; ++e)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const float next = fmaf(v[r], k[e][j], w[e][j] * S[r][e][j]);
+                    s = fmaf(WKV ? S[r][e][j] : next, q[e][j], s);
+                    S[r][e][j] = next;
+                }
+            o[r] = row16_sum(s);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            if (l16 == r && row0 + r < dv) stf(y + (size_t)t * H * dv + row0 + r, o[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+        if (row0 + r < dv) store_state<E4>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
+}
+
+// ---------------------------------------------------------------------------
+// Chunked form. logw becomes F in place, per chunk.
+// ---------------------------------------------------------------------------
+__launch_bounds__(256)
+__global__ void decay_sums_kernel(DecayArgs a) {
+    const int c = blockIdx.x, N = a.H * a.dk, i = blockIdx.y * 256 + threadIdx.x;
+    if (i >= N) return;
+    const int seg = a.chunk_seg[c], r0 = a.cu[seg] + a.chunk_off[c];
+    const int n = min(CH, a.cu[seg + 1] - r0);
+    float* p = a.logw + (size_t)r0 * N + i;
+    float sum = 0.f;
+    for (int s0 = 0; s0 < n; s0 += 8) {
+        float f[8];
+#pragma unroll
+        for (int s = 0; s < 8; ++s) f[s] = s0 + s < n ? p[(size_t)(s0 + s) * N] : 0.f;
+#pragma unroll
+        for (int s = 0; s < 8; ++s) {
+            sum += f[s];
+            if (s0 + s < n) p[(size_t)(s0 + s) * N] = sum;
+        }
+    }
+}
+
+// grid (segments, H, dv tiles * dk tiles of 64): walks a segment's chunks and
+// leaves the state before each. C fragments hold S[dk][dv]: wave = 16 key
+// dims, lane = 4 consecutive key dims of one value dim per dv tile.
+__launch_bounds__(256)
+__global__ void decay_state_kernel(DecayArgs a) {
+    __shared__ bf16 k_hi[CH][LDT], k_lo[CH][LDT], v_lds[CH][LDT];
+    const int seg = a.segs[blockIdx.x], h = blockIdx.y;
+    const int dk = a.dk, dv = a.dv, H = a.H, N = H * dk;
+    const int nkt = (dk + 63) / 64, vt = blockIdx.z / nkt, kt = blockIdx.z % nkt;
+    const int slot = a.slots[seg], row_lo = a.cu[seg], row_hi = a.cu[seg + 1];
+    const int c_lo = a.first[blockIdx.x], c_hi = a.first[blockIdx.x + 1];
+    const bool fresh = a.positions[row_lo] == 0;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int r16 = lane & 15, g = lane >> 4;
+    const int kd = kt * 64 + wave * 16 + g * 4;  // first of this lane's key dims
+    const bf16 *kp = (const bf16*)a.k + (size_t)h * dk, *vp = (const bf16*)a.v + (size_t)h * dv;
+    const float* Fp = a.logw + (size_t)h * dk;
+    f32x4 S[4];
+    float* Sp = a.S + ((size_t)slot * H + h) * dv * dk;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int vd = vt * 64 + j * 16 + r16;
+        S[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        if (!fresh && vd < dv && kd < dk)
+            S[j] = *reinterpret_cast<const f32x4*>(Sp + (size_t)vd * dk + kd);
+    }
+    const int d8 = tid % 8 * 8, kcol = kt * 64 + d8;
+    uint4 kreg[2], vreg[2];
+    float Fr[2][8], Fl[8];
+    f32x4 keep;
+    auto load_rows = [&](int r0) {
+        const int last = min(r0 + CH, row_hi) - 1;
+        keep = (f32x4){0.f, 0.f, 0.f, 0.f};
+        if (kd < dk) keep = *reinterpret_cast<const f32x4*>(Fp + (size_t)last * N + kd);
+        if (kcol < dk) load8f(Fp + (size_t)last * N + kcol, Fl);
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int r = r0 + tid / 8 + u * 32;
+            kreg[u] = vreg[u] = (uint4){0, 0, 0, 0};
+            if (r < row_hi) {
+                if (kcol < dk) {
+                    kreg[u] = *reinterpret_cast<const uint4*>(kp + (size_t)r * a.ldk + kcol);
+                    load8f(Fp + (size_t)r * N + kcol, Fr[u]);
+                }
+                if (vt * 64 + d8 < dv)
+                    vreg[u] = *reinterpret_cast<const uint4*>(vp + (size_t)r * a.ldv + vt * 64 + d8);
+            }
+        }
+    };
+    load_rows(row_lo);
+    for (int c = c_lo; c < c_hi; ++c) {
+        const int r0 = row_lo + (c - c_lo) * CH;
+        const size_t base = ((size_t)c * H + h) * dv;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int vd = vt * 64 + j * 16 + r16;
+            if (vd < dv && kd < dk) {
+                uint16_t hi[4], lo[4];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) split_bf16(S[j][r], hi[r], lo[r]);
+                const size_t at = (base + vd) * dk + kd;
+                *reinterpret_cast<uint2*>(a.s_hi + at) = make_uint2(
+                    hi[0] | ((uint32_t)hi[1] << 16), hi[2] | ((uint32_t)hi[3] << 16));
+                *reinterpret_cast<uint2*>(a.s_lo + at) = make_uint2(
+                    lo[0] | ((uint32_t)lo[1] << 16), lo[2] | ((uint32_t)lo[3] << 16));
+            }
+        }
+        __syncthreads();  // the previous chunk's tiles have been read
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int s = tid / 8 + u * 32;
+            float f[8];
+            bf16x8 hi, lo;
+            unpack8(kreg[u], f);
+            if (r0 + s < row_hi && kcol < dk) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) f[i] *= __expf(Fl[i] - Fr[u][i]);
+            }
+            split_frag(f, hi, lo);
+            *reinterpret_cast<bf16x8*>(&k_hi[s][d8]) = hi;
+            *reinterpret_cast<bf16x8*>(&k_lo[s][d8]) = lo;
+            *reinterpret_cast<uint4*>(&v_lds[s][d8]) = vreg[u];
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float f = __expf(keep[r]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) S[j][r] *= f;
+        }
+        __syncthreads();
+        if (c + 1 < c_hi) load_rows(r0 + CH);
+#pragma unroll
+        for (int s0 = 0; s0 < CH; s0 += 32) {
+            const bf16x8 ah = tr_frag(&k_hi[0][0], LDT, s0, wave * 16);
+            const bf16x8 al = tr_frag(&k_lo[0][0], LDT, s0, wave * 16);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const bf16x8 vf = tr_frag(&v_lds[0][0], LDT, s0, j * 16);
+                S[j] = mfma16(ah, vf, S[j]);
+                S[j] = mfma16(al, vf, S[j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int vd = vt * 64 + j * 16 + r16;
+        if (vd < dv && kd < dk) *reinterpret_cast<f32x4*>(Sp + (size_t)vd * dk + kd) = S[j];
+    }
+}
+
+// ---------------------------------------------------------------------------
+// grid (chunks, H, dv / (64*NB)). First a wave takes 16 query rows: q e^E and
+// the rows of P, to LDS; then 16*NB value dims: C fragments hold [dv][row].
+// NC: 32-wide slices of the key dims.
+// ---------------------------------------------------------------------------
+template <int NC, int NB, bool WKV>
+__launch_bounds__(256)
+__global__ void decay_out_kernel(DecayArgs a) {
+    constexpr int LDK = NC * 32 + 8, LDV = NB * 64 + 8;
+    __shared__ __align__(16) bf16 q_lds[2][CH * LDK];
+    __shared__ __align__(16) bf16 p_lds[2][CH * LDT];
+    __shared__ __align__(16) bf16 v_lds[CH * LDV];
+    const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * NB * 64;
+    const int dk = a.dk, dv = a.dv, H = a.H, N = H * dk;
+    const int seg = a.chunk_seg[c], r0 = a.cu[seg] + a.chunk_off[c];
+    const int n = min(CH, a.cu[seg + 1] - r0);
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int r16 = lane & 15, g = lane >> 4;
+    const bf16 *kp = (const bf16*)a.k + (size_t)r0 * a.ldk + (size_t)h * dk;
+    const bf16 *vp = (const bf16*)a.v + (size_t)r0 * a.ldv + (size_t)h * dv;
+    const float* Fp = a.logw + (size_t)r0 * N + (size_t)h * dk;
+#pragma unroll
+    for (int u = 0; u < NB * 2; ++u) {
+        const int e = tid + u * 256, s = e / (NB * 8), d = e % (NB * 8) * 8;
+        uint4 x = {0, 0, 0, 0};
+        if (s < n && v0 + d < dv)
+            x = *reinterpret_cast<const uint4*>(vp + (size_t)s * a.ldv + v0 + d);
+        *reinterpret_cast<uint4*>(v_lds + s * LDV + d) = x;
+    }
+    {
+        const int b0 = wave * 16, t = min(b0 + r16, n - 1);  // this lane's row
+        const bf16* qr = (const bf16*)a.q + (size_t)(r0 + t) * a.ldq + (size_t)h * dk;
+        f32x4 P[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) P[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        for (int cc = 0; cc < NC; ++cc) {
+            const int d = cc * 32 + g * 8;
+            const bool in = d < dk;
+            const int dd = in ? d : 0;
+            uint4 qraw = *reinterpret_cast<const uint4*>(qr + dd);
+            if (!in) qraw = (uint4){0, 0, 0, 0};
+            float q[8], E[8], R[8], f[8];
+            bf16x8 qh, ql;
+            unpack8(qraw, q);
+            const int te = WKV ? t - 1 : t;
+            if (te >= 0) {
+                load8f(Fp + (size_t)te * N + dd, E);
+            } else {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) E[i] = 0.f;
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) f[i] = q[i] * __expf(E[i]);
+            split_frag(f, qh, ql);
+            *reinterpret_cast<bf16x8*>(&q_lds[0][(b0 + r16) * LDK + d]) = qh;
+            *reinterpret_cast<bf16x8*>(&q_lds[1][(b0 + r16) * LDK + d]) = ql;
+            if (b0 >= n) continue;  // (uniform in the wave) no rows here
+            if (wave > 0) {  // earlier blocks, through the sums before this one
+                load8f(Fp + (size_t)(b0 - 1) * N + dd, R);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) f[i] = q[i] * __expf(E[i] - R[i]);
+                split_frag(f, qh, ql);
+                for (int j = 0; j < wave; ++j) {
+                    const int s = j * 16 + r16;
+                    float Fs[8], k[8];
+                    bf16x8 kh, kl;
+                    unpack8(*reinterpret_cast<const uint4*>(kp + (size_t)s * a.ldk + dd), k);
+                    load8f(Fp + (size_t)s * N + dd, Fs);
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) k[i] *= __expf(R[i] - Fs[i]);
+                    split_frag(k, kh, kl);
+                    f32x4 p = j == 0 ? P[0] : j == 1 ? P[1] : P[2];
+                    p = mfma16(qh, kh, p);
+                    p = mfma16(qh, kl, p);
+                    p = mfma16(ql, kh, p);
+                    if (j == 0) P[0] = p;
+                    else if (j == 1) P[1] = p;
+                    else P[2] = p;
+                }
+            }
+            // this block: row tt of P is row tt of q against k_s e^(E_tt - F_s)
+            float Fs[8], k[8], u[8];
+            unpack8(*reinterpret_cast<const uint4*>(kp + (size_t)t * a.ldk + dd), k);
+            load8f(Fp + (size_t)t * N + dd, Fs);
+            if (WKV) load8f(a.u + (size_t)h * dk + dd, u);
+            const int rows = min(16, n - b0);
+#pragma unroll 4
+            for (int tt = 0; tt < rows; ++tt) {
+                const int row = b0 + tt - (WKV ? 1 : 0);
+                float Et[8];
+                load8f(Fp + (size_t)max(row, 0) * N + dd, Et);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    const float w = r16 < tt ? __expf(fminf(Et[i] - Fs[i], 0.f))
+                                             : (r16 == tt ? (WKV ? u[i] : 1.f) : 0.f);
+                    f[i] = k[i] * w;
+                }
+                bf16x8 kh, kl;
+                split_frag(f, kh, kl);
+                uint4 qm = qraw;
+                if (r16 != tt) qm = (uint4){0, 0, 0, 0};
+                P[3] = mfma16(as_frag(qm), kh, P[3]);
+                P[3] = mfma16(as_frag(qm), kl, P[3]);
+            }
+        }
+        // rows of P: blocks before this wave's, its own, zeros after
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            f32x4 p = (f32x4){0.f, 0.f, 0.f, 0.f};
+            if (j == wave) p = P[3];
+            else if (j < wave) p = P[j];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                uint16_t hi, lo;
+                split_bf16(p[r], hi, lo);
+                const int at = (b0 + g * 4 + r) * LDT + j * 16 + r16;
+                *reinterpret_cast<uint16_t*>(&p_lds[0][at]) = hi;
+                *reinterpret_cast<uint16_t*>(&p_lds[1][at]) = lo;
+            }
+        }
+    }
+    __syncthreads();
+    f32x4 o[4][NB];  // [row block][16 value dims]
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < NB; ++j) o[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const int vw = wave * NB * 16;  // first of this wave's value dims
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        bf16x8 vf[NB];
+#pragma unroll
+        for (int j = 0; j < NB; ++j) vf[j] = tr_frag(v_lds, LDV, u * 32, vw + j * 16);
+#pragma unroll
+        for (int i = u * 2; i < 4; ++i) {
+            const int at = (i * 16 + r16) * LDT + u * 32 + g * 8;
+            const bf16x8 ph = *reinterpret_cast<const bf16x8*>(&p_lds[0][at]);
+            const bf16x8 pl = *reinterpret_cast<const bf16x8*>(&p_lds[1][at]);
+#pragma unroll
+            for (int j = 0; j < NB; ++j) {
+                o[i][j] = mfma16(vf[j], ph, o[i][j]);
+                o[i][j] = mfma16(vf[j], pl, o[i][j]);
+            }
+        }
+    }
+    const size_t sbase = ((size_t)c * H + h) * dv;
+    for (int cc = 0; cc < NC; ++cc) {
+        const int d = cc * 32 + g * 8;
+        bf16x8 sh[NB], sl[NB];
+#pragma unroll
+        for (int j = 0; j < NB; ++j) {
+            const int vd = v0 + vw + j * 16 + r16;
+            uint4 x = {0, 0, 0, 0}, y = {0, 0, 0, 0};
+            if (vd < dv && d < dk) {
+                x = *reinterpret_cast<const uint4*>(a.s_hi + (sbase + vd) * dk + d);
+                y = *reinterpret_cast<const uint4*>(a.s_lo + (sbase + vd) * dk + d);
+            }
+            sh[j] = as_frag(x);
+            sl[j] = as_frag(y);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int at = (i * 16 + r16) * LDK + d;
+            const bf16x8 qh = *reinterpret_cast<const bf16x8*>(&q_lds[0][at]);
+            const bf16x8 ql = *reinterpret_cast<const bf16x8*>(&q_lds[1][at]);
+#pragma unroll
+            for (int j = 0; j < NB; ++j) {
+                o[i][j] = mfma16(sh[j], qh, o[i][j]);
+                o[i][j] = mfma16(sl[j], qh, o[i][j]);
+                o[i][j] = mfma16(sh[j], ql, o[i][j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int t = i * 16 + r16;
+        if (t >= n) continue;
+        bf16* yr = (bf16*)a.y + ((size_t)(r0 + t) * H + h) * dv;
+#pragma unroll
+        for (int j = 0; j < NB; ++j) {
+            const int vd = v0 + vw + j * 16 + g * 4;
+            if (vd < dv)
+                *reinterpret_cast<uint2*>(yr + vd) = make_uint2(
+                    pack2(o[i][j][0] * a.qscale, o[i][j][1] * a.qscale),
+                    pack2(o[i][j][2] * a.qscale, o[i][j][3] * a.qscale));
+        }
+    }
+}
+
+// ---------------------------------------------------------------------------
+// launchers
+// ---------------------------------------------------------------------------
+// vec: bf16, R a multiple of 8, N of 4, rows aligned for 16-byte loads
+extern "C" hipError_t launch_decay_logs(
+    float* out, const void* a, int64_t lda, const void* w2, const float* bias, int exp_form,
+    float inv_tau, int rows, int N, int R, int f32, int vec, hipStream_t stream) {
+    if (rows <= 0) return hipSuccess;
+    if (!f32 && vec) {
+        const dim3 grid(ceil_div_i(rows, 64), ceil_div_i(N, 64));
+        if (exp_form)
+            decay_logs_mfma_kernel<true><<<grid, 256, 0, stream>>>(
+                out, (const bf16*)a, lda, (const bf16*)w2, bias, inv_tau, rows, N, R);
+        else
+            decay_logs_mfma_kernel<false><<<grid, 256, 0, stream>>>(
+                out, (const bf16*)a, lda, (const bf16*)w2, bias, inv_tau, rows, N, R);
+        HIP_CHECK_LAST();
+        return hipSuccess;
+    }
+    const dim3 grid(ceil_div_i(rows, DL_ROWS), ceil_div_i(N, 256));
+    const size_t lds = (size_t)DL_ROWS * R * sizeof(float);
+    if (lds > 48 * 1024) return hipErrorInvalidValue;
+#define GO(T, E)                                                              \
+    decay_logs_any_kernel<T, E><<<grid, 256, lds, stream>>>(                  \
+        out, (const T*)a, lda, (const T*)w2, bias, inv_tau, rows, N, R)
+    if (f32) {
+        if (exp_form) GO(float, true);
+        else GO(float, false);
+    } else {
+        if (exp_form) GO(bf16, true);
+        else GO(bf16, false);
+    }
+#undef GO
+    HIP_CHECK_LAST();
+    return hipSuccess;
+}
+
+template <typename T, bool WKV>
+static hipError_t decay_scan_go(const DecayArgs& a, int nseg, hipStream_t stream) {
+    const dim3 grid(nseg, a.H, ceil_div_i(a.dv, 64));
+    if (a.dk <= 64) decay_scan_kernel<T, 1, WKV><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 128) decay_scan_kernel<T, 2, WKV><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 256) decay_scan_kernel<T, 4, WKV><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 512) decay_scan_kernel<T, 8, WKV><<<grid, 256, 0, stream>>>(a);
+    else return hipErrorInvalidValue;
+    HIP_CHECK_LAST();
+    return hipSuccess;
+}
+
+extern "C" hipError_t launch_decay_scan(
+    void* y, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
+    int64_t ldv, const float* logw, const float* u, float qscale, int T, int H, int dk, int dv,
+    float* S, const int64_t* positions, const int* cu, const int* slots, const int* seg_list,
+    int nseg, int f32, hipStream_t stream) {
+    if (nseg <= 0) return hipSuccess;
+    DecayArgs a = {y, q, k, v, ldq, ldk, ldv, const_cast<float*>(logw), u, qscale, T, H, dk, dv,
+                   S, positions, cu, slots, seg_list};
+    if (u)
+        return f32 ? decay_scan_go<float, true>(a, nseg, stream)
+                   : decay_scan_go<bf16, true>(a, nseg, stream);
+    return f32 ? decay_scan_go<float, false>(a, nseg, stream)
+               : decay_scan_go<bf16, false>(a, nseg, stream);
+}
+
+template <bool WKV>
+static hipError_t decay_out_go(const DecayArgs& a, int nchunks, hipStream_t stream) {
+#define GO(NC, NB)                                                                       \
+    decay_out_kernel<NC, NB, WKV>                                                        \
+        <<<dim3(nchunks, a.H, ceil_div_i(a.dv, NB * 64)), 256, 0, stream>>>(a)
+    if (a.dk <= 64) { if (a.dv <= 64) GO(2, 1); else if (a.dv <= 128) GO(2, 2); else GO(2, 4); }
+    else if (a.dk <= 128) { if (a.dv <= 128) GO(4, 2); else GO(4, 4); }
+    else GO(8, 2);
+#undef GO
+    HIP_CHECK_LAST();
+    return hipSuccess;
+}
+
+// bf16; dk (up to 256) and dv multiples of 8; scratch planes [2, chunks, H, dv, dk]
+extern "C" hipError_t launch_decay_chunked(
+    void* y, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
+    int64_t ldv, float* logw, const float* u, float qscale, int T, int H, int dk, int dv,
+    float* S, const int64_t* positions, const int* cu, const int* slots, const int* segs,
+    const int* first, const int* chunk_seg, const int* chunk_off, int nsegs, int nchunks,
+    void* planes, hipStream_t stream) {
+    if (nchunks <= 0) return hipSuccess;
+    if (dk % 8 || dv % 8 || ldq % 8 || ldk % 8 || ldv % 8 || dk > 256) return hipErrorInvalidValue;
+    DecayArgs a = {y, q, k, v, ldq, ldk, ldv, logw, u, qscale, T, H, dk, dv,
+                   S, positions, cu, slots, nullptr, segs, first, chunk_seg, chunk_off};
+    a.s_hi = (uint16_t*)planes;
+    a.s_lo = a.s_hi + (size_t)nchunks * H * dv * dk;
+    decay_sums_kernel<<<dim3(nchunks, ceil_div_i(H * dk, 256)), 256, 0, stream>>>(a);
+    HIP_CHECK_LAST();
+    decay_state_kernel<<<dim3(nsegs, H, ceil_div_i(dv, 64) * ceil_div_i(dk, 64)), 256, 0, stream>>>(a);
+    HIP_CHECK_LAST();
+    return u ? decay_out_go<true>(a, nchunks, stream) : decay_out_go<false>(a, nchunks, stream);
+}

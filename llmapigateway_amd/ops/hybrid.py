@@ -46,19 +46,33 @@ class Chunks:
 
 
 @dataclass
+class Tiles:
+    """Segments long enough for the tiled form of paged attention."""
+
+    tile_seg: torch.Tensor          # [ntiles] int32
+    tile_off: torch.Tensor          # [ntiles] int32 first row within the segment
+    tile_rows: int
+    rest: Optional[torch.Tensor]    # int32 rows of the other segments
+
+
+@dataclass
 class SegmentPlan:
     """How a step's rows go through the kernels; made once per step."""
 
     unfold: Optional[Unfold] = None
     chunks: Optional[Chunks] = None
+    tiles: Optional[Tiles] = None
 
 
 CHUNK = 64            # rows per chunk of the chunked recurrences
 CHUNK_MIN_ROWS = 32   # shorter segments run token by token
 UNFOLD_RATIO = 16     # query-key pairs per key from which unfolding pays
+TILE_MIN_ROWS = 16    # shorter segments attend row by row
+PLANS = ("unfold", "chunks", "tiles")
 
 
-def plan_segments(batch, dtype) -> SegmentPlan:
+def plan_segments(batch, dtype, parts_of=PLANS) -> SegmentPlan:
+    """parts_of: the parts that the model's mixers use."""
     segs = batch.segs
     plan = SegmentPlan()
     if batch.kind == "decode" or segs.lens is None:
@@ -77,7 +91,8 @@ def plan_segments(batch, dtype) -> SegmentPlan:
     pl, ps = lens[:nseg_p], starts[:nseg_p]
     keys = int((pl + ps).sum())
     pairs = float((pl * (ps + pl / 2.0)).sum())
-    unfold = nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
+    unfold = "unfold" in parts_of and nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
+    tiled = np.nonzero(lens >= TILE_MIN_ROWS)[0] if "tiles" in parts_of else []
     if unfold:
         put("cu_q", np.concatenate([[0], np.cumsum(pl)]))
         put("cu_k", np.concatenate([[0], np.cumsum(pl + ps)]))
@@ -87,7 +102,16 @@ def plan_segments(batch, dtype) -> SegmentPlan:
         order = np.argsort(-(ps[seg] + off), kind="stable")  # longest first
         put("tile_seg", seg[order])
         put("tile_off", off[order])
-    long = np.nonzero(lens >= CHUNK_MIN_ROWS)[0]
+    if len(tiled):
+        n = lens[tiled]
+        rows_t = 128 if int(n.max()) > 64 else 64
+        seg = np.repeat(tiled, -(-n // rows_t))
+        off = np.concatenate([np.arange(0, k, rows_t) for k in n])
+        order = np.argsort(-(starts[seg] + off), kind="stable")  # longest first
+        put("at_seg", seg[order])
+        put("at_off", off[order])
+        put("at_rest", np.nonzero(np.repeat(lens < TILE_MIN_ROWS, lens))[0])
+    long = np.nonzero(lens >= CHUNK_MIN_ROWS)[0] if "chunks" in parts_of else np.empty(0, int)
     nchunk = (lens[long] + CHUNK - 1) // CHUNK
     if len(long):
         put("segs", long)
@@ -116,6 +140,11 @@ def plan_segments(batch, dtype) -> SegmentPlan:
             cu_q=got["cu_q"], cu_k=got["cu_k"],
             tile_seg=got["tile_seg"], tile_off=got["tile_off"],
             tile_rows=tile_rows,
+        )
+    if len(tiled):
+        plan.tiles = Tiles(
+            tile_seg=got["at_seg"], tile_off=got["at_off"], tile_rows=rows_t,
+            rest=got["at_rest"] if got["at_rest"].numel() else None,
         )
     if len(long):
         plan.chunks = Chunks(
@@ -323,5 +352,138 @@ def gated_norm(y, gate, w, groups: int, eps: float, gate_first: bool):
     if not y.is_cuda:
         return ref.gated_norm(y, gate, w, groups, eps, gate_first)
     out = torch.empty_like(y)
-    hybrid_native().gated_norm(out, y, gate, w, groups, float(eps), gate_first)
+    hybrid_native().gated_norm(out, y, gate, w, groups, float(eps), 1 if gate_first else 0)
     return out
+
+
+def head_norm_gate(out, y, gate, w, heads: int, eps: float) -> None:
+    """out = RMS norm of y per head, times w, times silu(gate); out and gate
+    may be strided."""
+    if not y.is_cuda:
+        return ref.head_norm_gate(out, y, gate, w, heads, eps)
+    hybrid_native().head_norm_gate(out, y, gate, w, heads, float(eps))
+
+
+# ------------------------------------------------------------- dynamic tanh
+def add_tanh_norm(x, delta, post, norm, dtype, replace: bool = False, out=None):
+    """x (fp32 stream, in place) += post(delta), or = with ``replace``;
+    returns norm(x), or x without a norm, in ``dtype`` (written to ``out`` if
+    given, which may be strided). Norms are (w, b, alpha):
+    tanh(alpha z) * w + b. delta: None, a tensor, or an ExpertSum."""
+    if not x.is_cuda:
+        return ref.add_tanh_norm(x, delta, post, norm, dtype, replace, out)
+    if out is None:
+        out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    parts = (delta, None, None, None, None)
+    if isinstance(delta, ExpertSum):
+        parts = (None, delta.rows, delta.slot, delta.weights, delta.shared)
+    none = (None, None, 1.0)
+    hybrid_native().stream_tanh(out, x, *parts, *(post or none), *(norm or none), replace)
+    return out
+
+
+def embed_tanh_norm(tokens, embed, norm, x0: Optional[torch.Tensor]) -> torch.Tensor:
+    """fp32 norm(embed[token]); x0 as in embed_scaled."""
+    if not embed.is_cuda:
+        return ref.embed_tanh_norm(tokens, embed, norm, x0)
+    x = torch.empty(tokens.shape[0], embed.shape[1], dtype=torch.float32, device=embed.device)
+    hybrid_native().embed_tanh(x, x0, tokens, embed, *norm)
+    return x
+
+
+def soft_cap_(x: torch.Tensor, cap: float) -> None:
+    """x (fp32) = cap * tanh(x / cap) in place."""
+    if not x.is_cuda:
+        return ref.soft_cap_(x, cap)
+    hybrid_native().soft_cap(x, float(cap))
+
+
+# ------------------------------------------------- attention over k/v pages
+def page_write(k, v, k_pages, v_pages, slot_mapping) -> None:
+    """Rows of keys and values (may be strided) into their cache slots."""
+    if not k.is_cuda:
+        return ref.page_write(k, v, k_pages, v_pages, slot_mapping)
+    hybrid_native().page_write(k, v, k_pages, v_pages, slot_mapping)
+
+
+def paged_attention(out, q, k_pages, v_pages, H: int, G: int, sink, scale: float, cap: float,
+                    gate, out_scale: float, positions, segs, plan: SegmentPlan) -> None:
+    """Causal attention of every row to its sequence's pages (its own token
+    among them): scores cap*tanh(scale q.k/cap), a sink per head in the
+    denominator; out [T, H*vdim] is multiplied by sigmoid(gate [T, H]) and
+    out_scale. q, gate and out may be strided."""
+    if not q.is_cuda:
+        return ref.paged_attention(
+            out, q, k_pages, v_pages, H, G, sink, scale, cap, gate, out_scale, positions, segs
+        )
+    ext = hybrid_native()
+    page, dim, vdim = k_pages.shape[1], k_pages.shape[2] // G, v_pages.shape[2] // G
+    head = (out, q, k_pages, v_pages, H, G, sink, float(scale), float(cap), gate,
+            float(out_scale), positions)
+    mfma = (
+        q.dtype == torch.bfloat16 and page >= 16 and page & (page - 1) == 0
+        and dim % 8 == 0 and vdim % 8 == 0 and dim <= 256 and vdim <= 256
+    )
+    rows, n = None, q.shape[0]
+    if mfma and plan.tiles is not None:
+        t = plan.tiles
+        ext.paged_tiles(
+            *head, segs.tables, segs.cu, t.tile_seg, t.tile_off, t.tile_rows
+        )
+        if t.rest is None:
+            return
+        rows, n = t.rest, t.rest.numel()
+    nsplit, pa, pm = 0, None, None
+    if mfma:
+        # fill the chip: splits only from shapes, so captured graphs hold
+        groups = n * G * -(-(H // G) // 16)
+        max_tiles = -(-segs.tables.shape[1] * page // 128)
+        nsplit = max(1, min(-(-512 // groups), 16, max_tiles))
+        if nsplit > 1:
+            pa, pm = _folded_scratch(q.device, n * H * nsplit * vdim, n * H * nsplit * 2)
+    ext.paged_rows(*head, segs.row_seg, segs.tables, rows, nsplit, pa, pm)
+
+
+# -------------------------------------- recurrences with a decay per channel
+def decay_logs(a, w2, bias, kind: str, tau: float) -> torch.Tensor:
+    """fp32 log decays [T, N] from a [T, rank] (may be strided): "sigmoid":
+    log sigmoid(z) / tau with z = a w2^T + bias; "exp": -e^z with
+    z = tanh(a) w2^T + bias."""
+    if not a.is_cuda:
+        return ref.decay_logs(a, w2, bias, kind, tau)
+    out = torch.empty(a.shape[0], w2.shape[0], dtype=torch.float32, device=a.device)
+    hybrid_native().decay_logs(out, a, w2, bias, kind == "exp", float(tau))
+    return out
+
+
+def token_shift(h, mu, prev, positions, segs) -> torch.Tensor:
+    """[mixes, T, W]: h + (h' - h) * mu[m] with h' the sequence's previous
+    row (zeros before the first); prev [slots, W] carries each sequence's
+    last row."""
+    if not h.is_cuda:
+        return ref.token_shift(h, mu, prev, positions, segs)
+    out = torch.empty(mu.shape[0], *h.shape, dtype=h.dtype, device=h.device)
+    hybrid_native().token_shift(out, h, mu, prev, positions, segs.cu, segs.slots, segs.row_seg)
+    return out
+
+
+def decayed_kv(q, k, v, logw, u, qscale: float, H: int, dk: int, dv: int, S, positions, segs,
+               plan: SegmentPlan) -> torch.Tensor:
+    """S = diag(e^logw) S + k v^T per head, read out by q: after the update
+    (u None), or before it with a bonus u for the current token. q, k, v may
+    be strided; logw [T, H*dk] fp32 is consumed; S [slots, H, dv, dk]."""
+    if not q.is_cuda:
+        return ref.decayed_kv(q, k, v, logw, u, qscale, H, dk, dv, S, positions, segs)
+    y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    ext, ch = hybrid_native(), plan.chunks
+    args = (y, q, k, v, logw, u, float(qscale), H, dk, dv, S, positions, segs.cu, segs.slots)
+    if ch is not None and dk % 8 == 0 and dv % 8 == 0 and dk <= 256:
+        if ch.short is not None:
+            ext.decay_scan(*args, ch.short)
+        ext.decay_chunked(*args, *ch.maps)
+    else:
+        ext.decay_scan(*args, None)
+    return y
+
+
+from .experts import ExpertSum  # noqa: E402

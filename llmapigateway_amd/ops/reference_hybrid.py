@@ -177,3 +177,137 @@ def gated_norm(y, gate, w, groups, eps, gate_first):
     if not gate_first:
         yf = yf * torch.sigmoid(gf)
     return yf.to(y.dtype)
+
+
+# ------------------------------------------------------------- dynamic tanh
+def _tanh_norm(x, norm):
+    w, b, alpha = norm
+    return torch.tanh(alpha * x) * w + b
+
+
+def add_tanh_norm(x, delta, post, norm, dtype, replace, out):
+    if delta is not None:
+        d = delta.float()
+        if post is not None:
+            d = _tanh_norm(d, post)
+        x.copy_(d) if replace else x.add_(d)
+    y = x if norm is None else _tanh_norm(x, norm)
+    if out is None:
+        return y.to(dtype)
+    out.copy_(y)
+    return out
+
+
+def embed_tanh_norm(tokens, embed, norm, x0):
+    x = _tanh_norm(embed[tokens].float(), norm)
+    if x0 is not None:
+        x0.copy_(x)
+    return x
+
+
+# ---------------------------------------------------- attention over pages
+def page_write(k, v, k_pages, v_pages, slot_mapping):
+    keep = slot_mapping >= 0
+    for rows, pages in ((k, k_pages), (v, v_pages)):
+        pages.view(-1, pages.shape[-1])[slot_mapping[keep]] = rows[keep]
+
+
+def paged_attention(out, q, k_pages, v_pages, H, G, sink, scale, cap, gate, out_scale,
+                    positions, segs):
+    T, bs = q.shape[0], k_pages.shape[1]
+    dim, vdim = k_pages.shape[2] // G, v_pages.shape[2] // G
+    for t in range(T):
+        n = int(positions[t]) + 1
+        pages = segs.tables[int(segs.row_seg[t]), : (n + bs - 1) // bs].long()
+        k = k_pages[pages].reshape(-1, G, dim)[:n].float().repeat_interleave(H // G, 1)
+        v = v_pages[pages].reshape(-1, G, vdim)[:n].float().repeat_interleave(H // G, 1)
+        s = torch.einsum("hd,nhd->hn", q[t].float().view(H, dim), k) * scale
+        s = cap * torch.tanh(s / cap)
+        p = torch.softmax(torch.cat([s, sink[:, None]], -1), -1)[:, :n]
+        o = torch.einsum("hn,nhd->hd", p, v)
+        out[t] = (o * (torch.sigmoid(gate[t].float()) * out_scale)[:, None]).view(-1)
+
+
+# ------------------------------------- recurrences with a decay per channel
+def decay_logs(a, w2, bias, kind, tau):
+    a = torch.tanh(a.float()) if kind == "exp" else a.float()
+    z = a @ w2.float().t() + bias
+    return -torch.exp(z) if kind == "exp" else F.logsigmoid(z) / tau
+
+
+def token_shift(h, mu, prev, positions, segs):
+    hf = h.float()
+    last = torch.zeros_like(hf)
+    last[1:] = hf[:-1]
+    cu = segs.cu.tolist()
+    for s, slot in enumerate(segs.slots.tolist()):
+        r0 = cu[s]
+        fresh = slot < 0 or int(positions[r0]) == 0
+        last[r0] = 0.0 if fresh else prev[slot].float()
+    for s, slot in enumerate(segs.slots.tolist()):
+        if slot >= 0:
+            prev[slot] = h[cu[s + 1] - 1]
+    return (hf + (last - hf) * mu[:, None]).to(h.dtype)
+
+
+def decayed_kv(q, k, v, logw, u, qscale, H, dk, dv, S, positions, segs):
+    T = q.shape[0]
+    qf = q.float().reshape(T, H, dk) * qscale
+    kf, vf = k.float().reshape(T, H, dk), v.float().reshape(T, H, dv)
+    w = torch.exp(logw).view(T, H, 1, dk)
+    y = torch.zeros(T, H, dv)
+    cu = segs.cu.tolist()
+    for s, slot in enumerate(segs.slots.tolist()):
+        if slot < 0:
+            continue
+        st = S[slot].clone()  # [H, dv, dk]
+        if int(positions[cu[s]]) == 0:
+            st.zero_()
+        for t in range(cu[s], cu[s + 1]):
+            if u is not None:
+                bonus = (qf[t] * u * kf[t]).sum(-1, keepdim=True)
+                y[t] = (st * qf[t][:, None, :]).sum(-1) + bonus * vf[t]
+            st = w[t] * st + vf[t][:, :, None] * kf[t][:, None, :]
+            if u is None:
+                y[t] = (st * qf[t][:, None, :]).sum(-1)
+        S[slot] = st
+    return y.view(T, H * dv).to(q.dtype)
+
+
+def head_norm_gate(out, y, gate, w, heads, eps):
+    T, W = y.shape
+    yf = _rms(y.float().view(T, heads, W // heads), eps).view(T, W) * w
+    out.copy_(yf * F.silu(gate.float()))
+
+
+# ------------------------------------------------------------------- experts
+def route_experts(z, top):
+    e = torch.argsort(z, dim=-1, descending=True, stable=True)[:, :top]
+    return e, torch.softmax(z.gather(1, e), -1)
+
+
+def clamped_glu(x, limit):
+    g, u = x.float().chunk(2, -1)
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(x.dtype)
+
+
+def expert_rows(h, ids, gate_up, down, limit):
+    """[T * top, width]: row t * top + j is expert ids[t, j] on row t."""
+    T, top = ids.shape
+    out = torch.empty(T * top, down.shape[1], dtype=h.dtype)
+    flat = ids.reshape(-1)
+    for e in flat.unique().tolist():
+        rows = torch.nonzero(flat == e).view(-1)
+        act = clamped_glu(F.linear(h[rows // top], gate_up[e]), limit)
+        out[rows] = F.linear(act, down[e])
+    return out
+
+
+def expert_sum(rows, slot, weights, shared):
+    y = (rows[slot.long()].float() * weights[..., None]).sum(1)
+    return y if shared is None else y + shared.float()
+
+
+def soft_cap_(x, cap):
+    x.div_(cap).tanh_().mul_(cap)
