@@ -60,11 +60,15 @@ def parse_args():
         "--mode", choices=["qps", "wave", "layers"], default="qps",
         help="qps = open-loop Poisson arrivals at --qps (the BASELINE "
         "metric); wave = round-1 closed-loop waves; layers = prefill and "
-        "decode throughput of Lelisun beside a Llama of equal width, "
-        "feed-forward and number of layer runs",
+        "decode throughput of a hybrid decoder beside a Llama of equal "
+        "width, feed-forward (of experts: what a token uses) and number of "
+        "layer runs",
     )
-    p.add_argument("--sizes", default="small,base", help="--mode layers: lelisun-<size> presets, or any hybrid model")
-    p.add_argument("--sides", default="lelisun,llama", help="--mode layers: which models")
+    p.add_argument("--family", default="lelisun", choices=["lelisun", "filinex"],
+                   help="--mode layers: whose presets")
+    p.add_argument("--sizes", default="small,base",
+                   help="--mode layers: <family>-<size> presets, or any hybrid model")
+    p.add_argument("--sides", default="hybrid,llama", help="--mode layers: which models")
     p.add_argument("--prefill-shapes", default="4x1024,1x4096,1x8192",
                    help="--mode layers: prompts x tokens (steps of 4096 tokens)")
     p.add_argument("--decode-batches", default="16,64,256",
@@ -194,9 +198,9 @@ class StepDriver:
 
 
 def run_layers(args) -> None:
-    """Prefill and decode tokens/s of Lelisun at a few sizes, each beside the
-    closest dense model at equal width: as many Llama layers as Lelisun runs
-    layers."""
+    """Prefill and decode tokens/s of a hybrid decoder at a few sizes, each
+    beside the closest dense model at equal width: as many Llama layers as
+    the hybrid runs layers, a feed-forward as wide as what a token uses."""
     device = "cuda:0" if torch.cuda.is_available() else "cpu"
     context = args.decode_context
     batches = [int(b) for b in args.decode_batches.split(",") if b]
@@ -204,7 +208,9 @@ def run_layers(args) -> None:
     budget = 4096  # tokens per prefill step
 
     def llama_like(c):
-        ff = next(e.mlp["ff"] for e in c.layers if e.mlp)
+        m = next(e.mlp for e in c.layers if e.mlp)
+        ff = m["ff"] if m["kind"] == "dense" else (
+            m["router"]["top"] * m["expert"]["ff"] + m["shared"]["ff"])
         heads = c.hidden_size // 128 or 1
         return ModelConfig(
             name=f"llama of {c.name}", hidden_size=c.hidden_size, intermediate_size=ff,
@@ -226,9 +232,9 @@ def run_layers(args) -> None:
 
     results = []
     for size in args.sizes.split(","):
-        config = get_model_config(f"lelisun-{size}" if size in ("small", "base") else size)
+        config = get_model_config(f"{args.family}-{size}" if size in ("small", "base") else size)
         for side in args.sides.split(","):
-            c = config if side == "lelisun" else llama_like(config)
+            c = config if side == "hybrid" else llama_like(config)
             eng = LLMEngine(
                 model=c, device=device, num_blocks=8192 if device != "cpu" else 256,
                 dtype=torch.bfloat16 if device != "cpu" else torch.float32,

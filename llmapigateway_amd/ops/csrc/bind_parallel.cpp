@@ -313,36 +313,38 @@ void soft_cap(Tensor x, double cap) {
 }
 
 // z [T, E] logits -> ids, weights [T, top], and the rows' places by expert
-void route(Tensor ids, Tensor weights, Tensor slot, Tensor row_token, Tensor tile_expert,
+void route(Tensor ids, Tensor weights, Tensor slot, Tensor row_token, Tensor tile_info,
            Tensor z, Tensor bias, int64_t tile_rows) {
     TORCH_CHECK(z.dim() == 2 && ids.dim() == 2);
-    const int64_t T = z.size(0), E = z.size(1), top = ids.size(1), nt = tile_expert.numel();
+    const int64_t T = z.size(0), E = z.size(1), top = ids.size(1), nt = (tile_info.numel() - 1) / 4;
     f32_ptr(z, T * E, "z");
     i32_ptr(ids, T * top, "ids");
     f32_ptr(weights, T * top, "weights");
     i32_ptr(slot, T * top, "slot");
-    i32_ptr(tile_expert, nt, "tile_expert");
+    i32_ptr(tile_info, 4 * nt + 1, "tile_info");
     i32_ptr(row_token, nt * tile_rows, "row_token");
+    TORCH_CHECK(reinterpret_cast<uintptr_t>(tile_info.data_ptr()) % 16 == 0, "tile_info: unaligned");
     TORCH_CHECK(tile_rows > 0 && nt >= std::min(T * top, E + T * top / tile_rows),
                 "route: too few tiles");
     CHECK_HIP(launch_route_topk(ids.data_ptr<int>(), weights.data_ptr<float>(),
                                 z.data_ptr<float>(), f32_ptr(bias, E, "bias"), T, E, top,
                                 current_stream()));
     CHECK_HIP(launch_route_plan(slot.data_ptr<int>(), row_token.data_ptr<int>(),
-                                tile_expert.data_ptr<int>(), ids.data_ptr<int>(), T * top, top,
+                                tile_info.data_ptr<int>(), ids.data_ptr<int>(), T * top, top,
                                 E, tile_rows, nt, current_stream()));
 }
 
 // out[r] = w[e] x[token(r)] through the clamped GLU (glu), or w[e] x[r]
-void expert_product(Tensor out, Tensor x, Tensor w, Tensor row_token, Tensor tile_expert,
+void expert_product(Tensor out, Tensor x, Tensor w, Tensor row_token, Tensor tile_info,
                     int64_t tile_rows, bool glu, double limit) {
     const bool f32 = is_f32(x, "x"), frag = w.dim() == 5;
     same_type(x, w, "w");
     same_type(x, out, "out");
-    const int64_t nt = tile_expert.numel(), R = nt * tile_rows;
+    const int64_t nt = (tile_info.numel() - 1) / 4, R = nt * tile_rows;
     const int64_t N = out.size(1), K = x.size(1);
     check_rows(out, R, N, "out");
     check_rows(x, x.size(0), K, "x");
+    TORCH_CHECK(reinterpret_cast<uintptr_t>(tile_info.data_ptr()) % 16 == 0, "tile_info: unaligned");
     TORCH_CHECK(x.size(0) > 0 && (glu || x.size(0) == R) && w.is_contiguous());
     int64_t nfrags = 0, ksteps = 0;
     if (frag) {
@@ -354,7 +356,7 @@ void expert_product(Tensor out, Tensor x, Tensor w, Tensor row_token, Tensor til
     }
     CHECK_HIP(launch_expert_product(
         out.data_ptr(), out.stride(0), x.data_ptr(), x.stride(0), w.data_ptr(),
-        i32_ptr(row_token, R, "row_token"), i32_ptr(tile_expert, nt, "tile_expert"), N, K, glu,
+        i32_ptr(row_token, R, "row_token"), i32_ptr(tile_info, 4 * nt + 1, "tile_info"), N, K, glu,
         (float)limit, frag, nfrags, ksteps, tile_rows, nt, f32, current_stream()));
 }
 

@@ -9,7 +9,7 @@
 // The weighted sum over a token's experts is part of the stream kernel.
 //
 // Weights of the MFMA forms lie in fragments, [N/16][K/32][64 lanes][8]: one
-// wave load of 1 KiB is an operand in lane order. N is padded to 128, K to
+// wave load of 1 KiB is an operand in lane order. N is padded to 256, K to
 // 64 with zeros; gate and up rows alternate in blocks of 16.
 
 #include "lds_dma.h"
@@ -76,11 +76,13 @@ __global__ void route_topk_kernel(
 
 // ---------------------------------------------------------------------------
 // Rows by expert, in one workgroup: slot[i] is where (token, choice) i went.
-// The order within a group is arbitrary; no value depends on it.
+// The order within a group is arbitrary; no value depends on it. tile_info,
+// [4 * max_tiles + 1]: per tile its expert (-1: none), the expert's first tile,
+// how many the expert has, and the tile's rows; then the number of tiles.
 // ---------------------------------------------------------------------------
 __launch_bounds__(1024)
 __global__ void route_plan_kernel(
-    int* __restrict__ slot, int* __restrict__ row_token, int* __restrict__ tile_expert,
+    int* __restrict__ slot, int* __restrict__ row_token, int* __restrict__ tile_info,
     const int* __restrict__ ids, int n, int top, int E, int tile_rows, int max_tiles) {
     __shared__ int count[MAX_EXPERTS], end[MAX_EXPERTS], cursor[MAX_EXPERTS];
     const int tid = threadIdx.x;
@@ -99,9 +101,15 @@ __global__ void route_plan_kernel(
     }
     const int first = end[tid] - tiles;
     cursor[tid] = first * tile_rows;
-    for (int i = first; i < end[tid]; ++i) tile_expert[i] = tid;
+    for (int i = first; i < end[tid]; ++i) {
+        tile_info[4 * i] = tid;
+        tile_info[4 * i + 1] = first;
+        tile_info[4 * i + 2] = tiles;
+        tile_info[4 * i + 3] = min(tile_rows, count[tid] - (i - first) * tile_rows);
+    }
+    if (tid == 0) tile_info[4 * max_tiles] = end[1023];
     for (int r = first * tile_rows + count[tid]; r < end[tid] * tile_rows; ++r) row_token[r] = -1;
-    for (int i = end[1023] + tid; i < max_tiles; i += 1024) tile_expert[i] = -1;
+    for (int i = end[1023] + tid; i < max_tiles; i += 1024) tile_info[4 * i] = -1;
     __syncthreads();
     for (int i = tid; i < n; i += 1024) {
         const int r = atomicAdd(&cursor[ids[i]], 1);
@@ -114,7 +122,8 @@ struct ExpertArgs {
     void* out;               // [rows, ld_out]
     const void* x;           // GLU: [tokens, ldx], rows by row_token; else [rows, ldx]
     const void* w;
-    const int *row_token, *tile_expert;
+    const int *row_token, *tile_info;
+    int max_tiles;
     int64_t ldx, ld_out;
     int N, K;                // output width (GLU: of act), input width
     float limit;
@@ -127,7 +136,7 @@ template <typename T, bool GLU>
 __launch_bounds__(256)
 __global__ void expert_any_kernel(ExpertArgs a) {
     __shared__ float x_lds[16][33], w_lds[GLU ? 2 : 1][16][33];
-    const int tile = blockIdx.x, n0 = blockIdx.y * 16, e = a.tile_expert[tile];
+    const int tile = blockIdx.x, n0 = blockIdx.y * 16, e = a.tile_info[4 * tile];
     if (e < 0) return;
     const int tid = threadIdx.x, row = tid >> 4, col = tid & 15;
     const T* w = (const T*)a.w + (size_t)e * (GLU ? 2 : 1) * a.N * a.K;
@@ -179,7 +188,7 @@ template <int MF, bool GLU>
 __launch_bounds__(256)
 __global__ void expert_stream_kernel(ExpertArgs a, int nfrags, int ksteps) {
     __shared__ f32x4 red[4][MF * 4][64];
-    const int tile = blockIdx.y, e = a.tile_expert[tile];
+    const int tile = blockIdx.y, e = a.tile_info[4 * tile];
     if (e < 0) return;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int r16 = lane & 15, g = lane >> 4, nf0 = blockIdx.x * 4;
@@ -244,82 +253,104 @@ __global__ void expert_stream_kernel(ExpertArgs a, int nfrags, int ksteps) {
 }
 
 // ---------------------------------------------------------------------------
-// Many rows an expert (prompts): 128 rows x 8 weight fragments a workgroup,
-// 4 waves of 64 x 64, K in steps of 64 through two LDS buffers of fragments,
-// filled by global-to-LDS transfers a step ahead.
+// Many rows an expert (prompts): 256 rows x 16 weight fragments a workgroup,
+// 8 waves of 64 rows x 128 outputs; waves without rows only help to bring the
+// weights, and since two waves share a SIMD, one of each half, a half-empty
+// tile takes half the time. K runs in steps of 32 through a ring of LDS
+// buffers in fragment order, filled by global-to-LDS transfers RING-1 steps
+// ahead: at step s a wave waits until only its transfers of later steps are
+// under way; the barrier extends that to all waves' and frees the buffer of
+// step s-1, which the next transfers overwrite.
 // ---------------------------------------------------------------------------
+#define RING 4
 template <bool GLU>
-__launch_bounds__(256)
-__global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn, int total) {
-    // [buffer][x | w][2 * fragment + k32][64 lanes * 8]
-    __shared__ __align__(16) bf16 lds[2][2][16][512];
-    // neighbours share rows and weights: give each XCD (8, round robin) a
-    // contiguous part of the grid
-    const int per = (total + 7) / 8, b = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
-    if (b >= total) return;
-    const int tile = b / ntn, nf0 = b % ntn * 8, e = a.tile_expert[tile];
-    if (e < 0) return;
+__launch_bounds__(512)
+__global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn) {
+    // [ring][16 row fragments | 16 weight fragments][64 lanes * 8]
+    __shared__ __align__(16) bf16 lds[RING][32][512];
+    // each XCD (8, round robin) takes a contiguous part of the tiles there are;
+    // within an expert its row tiles vary fastest, so that what runs together
+    // shares rows and weights in the XCD's L2
+    const int total = a.tile_info[4 * a.max_tiles] * ntn, per = (total + 7) / 8;
+    const int b = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || b >= total) return;
+    const int4 info = reinterpret_cast<const int4*>(a.tile_info)[b / ntn];
+    const int in_e = b - info.y * ntn;
+    const int tile = info.y + in_e % info.z, nf0 = in_e / info.z * 16;
+    const int rows = reinterpret_cast<const int4*>(a.tile_info)[tile].w;
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r16 = lane & 15, g = lane >> 4;
-    const bf16* w = (const bf16*)a.w + ((size_t)e * nfrags + nf0) * ksteps * 512 + lane * 8;
-    const bf16* xr[2];  // the rows this wave brings: fragments 2*wave, 2*wave+1
+    const bf16* w =
+        (const bf16*)a.w + ((size_t)info.x * nfrags + nf0 + wave * 2) * ksteps * 512 + lane * 8;
+    const size_t wstep = (size_t)ksteps * 512;
+    // this wave brings row fragments 2*wave and 2*wave+1 if their 64 rows count
+    const bool brings = (wave >> 1) * 64 < rows, works = brings;
+    const bf16* xr[2];
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
-        int src = tile * 128 + (wave * 2 + i) * 16 + r16;
+        int src = tile * 256 + (wave * 2 + i) * 16 + r16;
         if (GLU) src = max(a.row_token[src], 0);
         xr[i] = (const bf16*)a.x + (size_t)src * a.ldx;
     }
     auto stage = [&](int s, int buf) {
-#pragma unroll
-        for (int i = 0; i < 2; ++i)
-#pragma unroll
-            for (int u = 0; u < 2; ++u) {
-                const int f = wave * 2 + i, k = (s + u) * 32 + g * 8;
-                dma16(xr[i] + (k < a.K ? k : 0), lds[buf][0][f * 2 + u]);
-                dma16(w + ((size_t)f * ksteps + s + u) * 512, lds[buf][1][f * 2 + u]);
-            }
+        const int k = s * 32 + g * 8, kk = k < a.K ? k : 0;  // past K the weights are 0
+        if (brings) {
+            dma16(xr[0] + kk, lds[buf][wave * 2]);
+            dma16(xr[1] + kk, lds[buf][wave * 2 + 1]);
+        }
+        dma16(w + (size_t)s * 512, lds[buf][16 + wave * 2]);
+        dma16(w + wstep + (size_t)s * 512, lds[buf][17 + wave * 2]);
     };
-    f32x4 acc[4][4];  // [weight fragment][row fragment]
+    f32x4 acc[8][4];  // [weight fragment][row fragment]
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+    for (int j = 0; j < 8; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) acc[j][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const int wm = (wave & 1) * 4, wn = (wave >> 1) * 4;
-    stage(0, 0);
-    dma_barrier();
+    const int wm = (wave >> 1) * 4, wn = 16 + (wave & 1) * 8;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int s = 0; s < RING - 1; ++s)
+        if (s < ksteps) stage(s, s);
     int buf = 0;
-    for (int s = 0; s < ksteps; s += 2, buf ^= 1) {
-        if (s + 2 < ksteps) stage(s + 2, buf ^ 1);
+    for (int s = 0; s < ksteps; ++s) {
+        if (s + RING - 1 > ksteps)
+            dma_barrier();
+        else if (brings)  // transfers of RING-2 later steps under way
+            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(4 * (RING - 2)) : "memory");
+        else
+            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(2 * (RING - 2)) : "memory");
+        if (s + RING - 1 < ksteps) stage(s + RING - 1, buf == 0 ? RING - 1 : buf - 1);
+        if (works) {
+            bf16x8 xf[4];
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            bf16x8 xf[4], wf[4];
+            for (int i = 0; i < 4; ++i)
+                xf[i] = *reinterpret_cast<const bf16x8*>(&lds[buf][wm + i][lane * 8]);
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                xf[i] = *reinterpret_cast<const bf16x8*>(&lds[buf][0][(wm + i) * 2 + u][lane * 8]);
-                wf[i] = *reinterpret_cast<const bf16x8*>(&lds[buf][1][(wn + i) * 2 + u][lane * 8]);
+            for (int j = 0; j < 8; ++j) {
+                const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&lds[buf][wn + j][lane * 8]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[j][i] = mfma16(wf, xf[i], acc[j][i]);
             }
-#pragma unroll
-            for (int j = 0; j < 4; ++j)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) acc[j][i] = mfma16(wf[j], xf[i], acc[j][i]);
         }
-        dma_barrier();
+        buf = buf + 1 == RING ? 0 : buf + 1;
     }
+    if (!works) return;
+    const int f0 = nf0 + wn - 16;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const int row = tile * 128 + (wm + i) * 16 + r16;
+        const int row = tile * 256 + (wm + i) * 16 + r16;
         bf16* o = (bf16*)a.out + (size_t)row * a.ld_out;
         if (GLU) {
 #pragma unroll
-            for (int j = 0; j < 2; ++j) {
-                const int n = ((nf0 + wn) / 2 + j) * 16 + g * 4;
+            for (int j = 0; j < 4; ++j) {
+                const int n = (f0 / 2 + j) * 16 + g * 4;
                 if (n < a.N) store4(o + n, glu4(acc[2 * j][i], acc[2 * j + 1][i], a.limit));
             }
         } else {
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int n = (nf0 + wn + j) * 16 + g * 4;
+            for (int j = 0; j < 8; ++j) {
+                const int n = (f0 + j) * 16 + g * 4;
                 if (n < a.N) store4(o + n, acc[j][i]);
             }
         }
@@ -345,12 +376,12 @@ extern "C" hipError_t launch_route_topk(
 }
 
 extern "C" hipError_t launch_route_plan(
-    int* slot, int* row_token, int* tile_expert, const int* ids, int n, int top, int E,
+    int* slot, int* row_token, int* tile_info, const int* ids, int n, int top, int E,
     int tile_rows, int max_tiles, hipStream_t stream) {
     if (n <= 0) return hipSuccess;
     if (E > MAX_EXPERTS) return hipErrorInvalidValue;
     route_plan_kernel<<<1, 1024, 0, stream>>>(
-        slot, row_token, tile_expert, ids, n, top, E, tile_rows, max_tiles);
+        slot, row_token, tile_info, ids, n, top, E, tile_rows, max_tiles);
     HIP_CHECK_LAST();
     return hipSuccess;
 }
@@ -358,10 +389,10 @@ extern "C" hipError_t launch_route_plan(
 // frag: weights in fragments (bf16), else dense [E, N or 2N, K] and tiles of 16 rows
 extern "C" hipError_t launch_expert_product(
     void* out, int64_t ld_out, const void* x, int64_t ldx, const void* w, const int* row_token,
-    const int* tile_expert, int N, int K, int glu, float limit, int frag, int nfrags,
+    const int* tile_info, int N, int K, int glu, float limit, int frag, int nfrags,
     int ksteps, int tile_rows, int max_tiles, int f32, hipStream_t stream) {
     if (max_tiles <= 0) return hipSuccess;
-    const ExpertArgs a = {out, x, w, row_token, tile_expert, ldx, ld_out, N, K, limit};
+    const ExpertArgs a = {out, x, w, row_token, tile_info, max_tiles, ldx, ld_out, N, K, limit};
     if (!frag) {
         if (tile_rows != 16) return hipErrorInvalidValue;
         const dim3 grid(max_tiles, ceil_div_i(N, 16));
@@ -379,15 +410,14 @@ extern "C" hipError_t launch_expert_product(
         HIP_CHECK_LAST();
         return hipSuccess;
     }
-    if (f32 || nfrags % 8 || ksteps % 2 || N % 8 || K % 8 || ldx % 8 || ld_out % 8 ||
+    if (f32 || nfrags % 16 || ksteps % 2 || N % 8 || K % 8 || ldx % 8 || ld_out % 8 ||
         ksteps * 32 < K || nfrags * 16 < (glu ? 2 : 1) * N)
         return hipErrorInvalidValue;
-    if (tile_rows == 128) {
-        const int ntn = nfrags / 8, total = max_tiles * ntn;
-        const int grid = ceil_div_i(total, 8) * 8;
-        if (glu) expert_tile_kernel<true><<<grid, 256, 0, stream>>>(a, nfrags, ksteps, ntn, total);
+    if (tile_rows == 256) {
+        const int ntn = nfrags / 16, grid = ceil_div_i(max_tiles * ntn, 8) * 8;
+        if (glu) expert_tile_kernel<true><<<grid, 512, 0, stream>>>(a, nfrags, ksteps, ntn);
         else {
-            expert_tile_kernel<false><<<grid, 256, 0, stream>>>(a, nfrags, ksteps, ntn, total);
+            expert_tile_kernel<false><<<grid, 512, 0, stream>>>(a, nfrags, ksteps, ntn);
         }
         HIP_CHECK_LAST();
         return hipSuccess;

@@ -39,7 +39,7 @@ class Routing:
     weights: torch.Tensor
     ids: torch.Tensor                            # [T, top] int32
     row_token: Optional[torch.Tensor] = None     # [rows] int32, -1: no row (GPU)
-    tile_expert: Optional[torch.Tensor] = None   # [tiles] int32, -1: no tile (GPU)
+    tile_info: Optional[torch.Tensor] = None     # [4 * tiles + 1] int32, see experts.hip
     tile_rows: int = 0
 
 
@@ -62,10 +62,10 @@ class ExpertSum:
 
 
 def _fragments(w: torch.Tensor) -> torch.Tensor:
-    """[N, K] (zero-padded to multiples of 128 and 64) -> [N/16, K/32, 64, 8]:
+    """[N, K] (zero-padded to multiples of 256 and 64) -> [N/16, K/32, 64, 8]:
     lane l of a fragment holds W[l % 16][8 (l / 16) ..]."""
     N, K = w.shape
-    w = torch.nn.functional.pad(w, (0, -K % 64, 0, -N % 128))
+    w = torch.nn.functional.pad(w, (0, -K % 64, 0, -N % 256))
     w = w.view(w.shape[0] // 16, 16, w.shape[1] // 32, 4, 8)
     return w.permute(0, 2, 3, 1, 4).reshape(w.shape[0], w.shape[2], 64, 8)
 
@@ -99,7 +99,7 @@ def _tile_rows(choices: int, w: ExpertWeights) -> int:
     if not w.fragments:
         return 16
     mean = choices / w.experts
-    return 16 if mean <= 10 else 32 if mean <= 20 else 64 if mean <= 48 else 128
+    return 16 if mean <= 10 else 32 if mean <= 20 else 64 if mean <= 48 else 256
 
 
 def route_experts(h, w_router, bias, top: int, experts: ExpertWeights) -> Routing:
@@ -116,12 +116,13 @@ def route_experts(h, w_router, bias, top: int, experts: ExpertWeights) -> Routin
     n = T * top
     rows = _tile_rows(n, experts)
     tiles = min(n, experts.experts + n // rows)
-    ints = torch.empty(2 * n + tiles * (rows + 1), dtype=torch.int32, device=dev)
-    ids, slot = ints[:n].view(T, top), ints[n : 2 * n].view(T, top)
-    row_token, tile_expert = ints[2 * n : 2 * n + tiles * rows], ints[2 * n + tiles * rows :]
+    sizes = (4 * tiles + 1, n, n, tiles * rows)
+    ints = torch.empty(sum(sizes), dtype=torch.int32, device=dev)
+    tile_info, ids, slot, row_token = ints.split(sizes)
+    ids, slot = ids.view(T, top), slot.view(T, top)
     weights = torch.empty(T, top, dtype=torch.float32, device=dev)
-    hybrid_native().route(ids, weights, slot, row_token, tile_expert, z, bias, rows)
-    return Routing(slot, weights, ids, row_token, tile_expert, rows)
+    hybrid_native().route(ids, weights, slot, row_token, tile_info, z, bias, rows)
+    return Routing(slot, weights, ids, row_token, tile_info, rows)
 
 
 def expert_rows(h, routing: Routing, w: ExpertWeights, limit: float) -> torch.Tensor:
@@ -131,7 +132,7 @@ def expert_rows(h, routing: Routing, w: ExpertWeights, limit: float) -> torch.Te
     R, ext = routing.row_token.numel(), hybrid_native()
     act = torch.empty(R, w.ff, dtype=h.dtype, device=h.device)
     out = torch.empty(R, w.width, dtype=h.dtype, device=h.device)
-    where = (routing.row_token, routing.tile_expert, routing.tile_rows)
+    where = (routing.row_token, routing.tile_info, routing.tile_rows)
     ext.expert_product(act, h, w.gate_up, *where, True, float(limit))
     ext.expert_product(out, act, w.down, *where, False, 0.0)
     return out

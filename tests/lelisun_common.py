@@ -83,7 +83,7 @@ def write_checkpoint(folder, cfg, weights):
     (folder / "config.json").write_text(json.dumps(cfg))
     header, blobs, at = {}, [], 0
     for name, t in weights.items():
-        raw = t.contiguous().view(torch.uint8).numpy().tobytes()
+        raw = t.contiguous().reshape(-1).view(torch.uint8).numpy().tobytes()
         header[name] = {"dtype": _DTYPE[t.dtype], "shape": list(t.shape),
                         "data_offsets": [at, at + len(raw)]}
         blobs.append(raw)
