@@ -120,10 +120,10 @@ struct CapExp {
 
 __device__ __forceinline__ bf16x8 weights_frag(const float* lo, const float* hi) {
     uint4 v;
-    v.x = pack2(lo[0], lo[1]);
-    v.y = pack2(lo[2], lo[3]);
-    v.z = pack2(hi[0], hi[1]);
-    v.w = pack2(hi[2], hi[3]);
+    v.x = cvt_pk_bf16(lo[0], lo[1]);
+    v.y = cvt_pk_bf16(lo[2], lo[3]);
+    v.z = cvt_pk_bf16(hi[0], hi[1]);
+    v.w = cvt_pk_bf16(hi[2], hi[3]);
     return as_frag(v);
 }
 
@@ -135,7 +135,7 @@ __device__ __forceinline__ bf16x8 weights_frag(const float* lo, const float* hi)
 // tile ahead. The waves' shares meet in LDS at the end; several splits leave
 // partials for paged_combine_kernel.
 // ONLINE: running maximum; otherwise the maximum is fixed at max(cap, sink),
-// which no score exceeds and, for caps up to 40, none is too far below.
+// which no score exceeds and, for caps up to 30, none is too far below.
 // ---------------------------------------------------------------------------
 template <int NDQ, int NDV, bool ONLINE>
 __launch_bounds__(PA_THREADS)
@@ -482,8 +482,8 @@ __global__ void paged_tiles_kernel(
             const int d = j * 16 + g * 4;  // vdim is a multiple of 8
             if (d < a.vdim)
                 *reinterpret_cast<uint2*>(o + d) = make_uint2(
-                    pack2(acc[i][j][0] * f, acc[i][j][1] * f),
-                    pack2(acc[i][j][2] * f, acc[i][j][3] * f));
+                    cvt_pk_bf16(acc[i][j][0] * f, acc[i][j][1] * f),
+                    cvt_pk_bf16(acc[i][j][2] * f, acc[i][j][3] * f));
         }
     }
 }
@@ -541,7 +541,7 @@ extern "C" hipError_t launch_paged_rows(
     const dim3 grid(nrows, G * ceil_div_i(H / G, 16), nsplit);
 #define GO(A, B)                                                                         \
     {                                                                                    \
-        if (cap > 40.f)                                                                  \
+        if (cap > 30.f)                                                                  \
             paged_rows_kernel<A, B, true><<<grid, PA_THREADS, 0, stream>>>(              \
                 a, shift, nsplit, part_acc, part_ml);                                    \
         else                                                                             \
@@ -574,7 +574,7 @@ extern "C" hipError_t launch_paged_tiles(
     const int shift = __builtin_ctz(block_size);
 #define GO2(A, B, M)                                                                     \
     {                                                                                    \
-        if (cap > 40.f)                                                                  \
+        if (cap > 30.f)                                                                  \
             paged_tiles_kernel<A, B, M, true><<<ntiles * H, PA_THREADS, 0, stream>>>(    \
                 a, shift, cu, tile_seg, tile_off);                                       \
         else                                                                             \

@@ -79,6 +79,15 @@ __device__ __forceinline__ uint32_t pack2_trunc(float lo, float hi) {
     return (a.u >> 16) | (b.u & 0xFFFF0000u);
 }
 
+// tanh by one exponential, by its series where that would lose relative
+// accuracy; both far inside bf16 rounding
+__device__ __forceinline__ float tanh_fast(float z) {
+    const float z2 = z * z;
+    const float series = z * (1.f + z2 * (-1.f / 3.f + z2 * (2.f / 15.f)));
+    const float e = 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __expf(2.f * z));
+    return z2 < 0.01f ? series : e;
+}
+
 // wave-wide reductions (64 lanes)
 __device__ __forceinline__ float wave_reduce_sum(float v) {
 #pragma unroll

@@ -170,7 +170,7 @@ __global__ void expert_any_kernel(ExpertArgs a) {
 }
 
 __device__ __forceinline__ void store4(bf16* p, const f32x4& v) {
-    *reinterpret_cast<uint2*>(p) = make_uint2(pack2(v[0], v[1]), pack2(v[2], v[3]));
+    *reinterpret_cast<uint2*>(p) = make_uint2(cvt_pk_bf16(v[0], v[1]), cvt_pk_bf16(v[2], v[3]));
 }
 __device__ __forceinline__ f32x4 glu4(const f32x4& g, const f32x4& u, float limit) {
     f32x4 o;
@@ -256,18 +256,17 @@ __global__ void expert_stream_kernel(ExpertArgs a, int nfrags, int ksteps) {
 // Many rows an expert (prompts): 256 rows x 16 weight fragments a workgroup,
 // 8 waves of 64 rows x 128 outputs; waves without rows only help to bring the
 // weights, and since two waves share a SIMD, one of each half, a half-empty
-// tile takes half the time. K runs in steps of 32 through a ring of LDS
-// buffers in fragment order, filled by global-to-LDS transfers RING-1 steps
-// ahead: at step s a wave waits until only its transfers of later steps are
-// under way; the barrier extends that to all waves' and frees the buffer of
-// step s-1, which the next transfers overwrite.
+// tile takes half the time. K runs in steps of 64 through two LDS buffers
+// filled by global-to-LDS transfers a step ahead. Weights come as fragments;
+// rows in pieces of 8 rows x 128 bytes (whole cache lines), their 16-byte
+// chunks XOR-swizzled by row on the source address, so that fragment reads
+// spread over the banks.
 // ---------------------------------------------------------------------------
-#define RING 4
 template <bool GLU>
 __launch_bounds__(512)
 __global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn) {
-    // [ring][16 row fragments | 16 weight fragments][64 lanes * 8]
-    __shared__ __align__(16) bf16 lds[RING][32][512];
+    // [buffer][32 pieces of rows | 16 weight fragments x 2][1 KiB]
+    __shared__ __align__(16) bf16 lds[2][64][512];
     // each XCD (8, round robin) takes a contiguous part of the tiles there are;
     // within an expert its row tiles vary fastest, so that what runs together
     // shares rows and weights in the XCD's L2
@@ -284,59 +283,63 @@ __global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn
     const bf16* w =
         (const bf16*)a.w + ((size_t)info.x * nfrags + nf0 + wave * 2) * ksteps * 512 + lane * 8;
     const size_t wstep = (size_t)ksteps * 512;
-    // this wave brings row fragments 2*wave and 2*wave+1 if their 64 rows count
-    const bool brings = (wave >> 1) * 64 < rows, works = brings;
-    const bf16* xr[2];
+    const bool works = (wave >> 1) * 64 < rows;  // this wave's 64 rows count
+    const bf16* xr[4];  // it brings 32 of them: lane = row lane/8 of a piece
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-        int src = tile * 256 + (wave * 2 + i) * 16 + r16;
+    for (int i = 0; i < 4; ++i) {
+        int src = tile * 256 + wave * 32 + i * 8 + (lane >> 3);
         if (GLU) src = max(a.row_token[src], 0);
         xr[i] = (const bf16*)a.x + (size_t)src * a.ldx;
     }
-    auto stage = [&](int s, int buf) {
-        const int k = s * 32 + g * 8, kk = k < a.K ? k : 0;  // past K the weights are 0
-        if (brings) {
-            dma16(xr[0] + kk, lds[buf][wave * 2]);
-            dma16(xr[1] + kk, lds[buf][wave * 2 + 1]);
+    const int chunk = ((lane & 7) ^ (lane >> 3)) * 8;
+    auto stage = [&](int s, int buf) {  // steps s and s+1 of 32
+        const int k = s * 32 + chunk, kk = k < a.K ? k : 0;  // past K the weights are 0
+        if (works) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) dma16(xr[i] + kk, lds[buf][wave * 4 + i]);
         }
-        dma16(w + (size_t)s * 512, lds[buf][16 + wave * 2]);
-        dma16(w + wstep + (size_t)s * 512, lds[buf][17 + wave * 2]);
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+                dma16(w + i * wstep + (size_t)(s + u) * 512, lds[buf][32 + (wave * 2 + i) * 2 + u]);
     };
     f32x4 acc[8][4];  // [weight fragment][row fragment]
 #pragma unroll
     for (int j = 0; j < 8; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) acc[j][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const int wm = (wave >> 1) * 4, wn = 16 + (wave & 1) * 8;
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-#pragma unroll
-    for (int s = 0; s < RING - 1; ++s)
-        if (s < ksteps) stage(s, s);
+    const int wm = (wave >> 1) * 4, wn = (wave & 1) * 8;
+    const int piece = r16 >> 3, at = (r16 & 7) * 64;  // of a 16-row fragment
+    stage(0, 0);
+    dma_barrier();
     int buf = 0;
-    for (int s = 0; s < ksteps; ++s) {
-        if (s + RING - 1 > ksteps)
-            dma_barrier();
-        else if (brings)  // transfers of RING-2 later steps under way
-            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(4 * (RING - 2)) : "memory");
-        else
-            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(2 * (RING - 2)) : "memory");
-        if (s + RING - 1 < ksteps) stage(s + RING - 1, buf == 0 ? RING - 1 : buf - 1);
+    for (int s = 0; s < ksteps; s += 2, buf ^= 1) {
+        if (s + 2 < ksteps) stage(s + 2, buf ^ 1);
         if (works) {
-            bf16x8 xf[4];
+            __builtin_amdgcn_s_setprio(1);  // before the waves that still issue transfers
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-                xf[i] = *reinterpret_cast<const bf16x8*>(&lds[buf][wm + i][lane * 8]);
+            for (int u = 0; u < 2; ++u) {
+                const int slot = ((u * 4 + g) ^ (r16 & 7)) * 8;
+                bf16x8 xf[4];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&lds[buf][wn + j][lane * 8]);
+                for (int i = 0; i < 4; ++i)
+                    xf[i] = *reinterpret_cast<const bf16x8*>(
+                        &lds[buf][(wm + i) * 2 + piece][at + slot]);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) acc[j][i] = mfma16(wf, xf[i], acc[j][i]);
+                for (int j = 0; j < 8; ++j) {
+                    const bf16x8 wf = *reinterpret_cast<const bf16x8*>(
+                        &lds[buf][32 + (wn + j) * 2 + u][lane * 8]);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) acc[j][i] = mfma16(wf, xf[i], acc[j][i]);
+                }
             }
+            __builtin_amdgcn_s_setprio(0);
         }
-        buf = buf + 1 == RING ? 0 : buf + 1;
+        dma_barrier();
     }
     if (!works) return;
-    const int f0 = nf0 + wn - 16;
+    const int f0 = nf0 + wn;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const int row = tile * 256 + (wm + i) * 16 + r16;

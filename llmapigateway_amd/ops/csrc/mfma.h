@@ -55,6 +55,14 @@ __device__ __forceinline__ bf16x8 tr_frag(const bf16* tile, int stride, int k0, 
     return tr_pair(p, p + 4 * stride);
 }
 
+// two fp32 to packed bf16, one instruction (round to nearest even)
+__device__ __forceinline__ uint32_t cvt_pk_bf16(float lo, float hi) {
+    typedef __attribute__((__vector_size__(2 * sizeof(float)))) float f32x2;
+    typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 b16x2;
+    const b16x2 v = __builtin_convertvector((f32x2){lo, hi}, b16x2);
+    return *reinterpret_cast<const uint32_t*>(&v);
+}
+
 // fp32 as a sum of two bf16 (16 mantissa bits): products of a fp32 operand
 // with bf16 data keep fp32-like accuracy in two MFMAs
 __device__ __forceinline__ void split_bf16(float v, uint16_t& hi, uint16_t& lo) {

@@ -17,6 +17,7 @@
 // P between two 16-row blocks factors through the sum R before the later one:
 // (q e^(E_t-R)).(k e^(R-F_s)); inside a block it is taken row by row.
 
+#include "lds_dma.h"
 #include "mfma.h"
 #include "recurrence.h"
 
@@ -30,10 +31,10 @@ __device__ __forceinline__ void split_frag(const float* f, bf16x8& hi, bf16x8& l
     uint32_t* lp = reinterpret_cast<uint32_t*>(&l);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        hp[i] = pack2(f[2 * i], f[2 * i + 1]);
+        hp[i] = cvt_pk_bf16(f[2 * i], f[2 * i + 1]);
         float a, b;
         unpack2(hp[i], a, b);
-        lp[i] = pack2(f[2 * i] - a, f[2 * i + 1] - b);
+        lp[i] = cvt_pk_bf16(f[2 * i] - a, f[2 * i + 1] - b);
     }
     hi = as_frag(h);
     lo = as_frag(l);
@@ -60,6 +61,16 @@ template <bool EXP>
 __device__ __forceinline__ float log_decay(float z, float inv_tau) {
     // e^-80 is as good as 0, and sums of 64 of them keep their precision
     return fmaxf(EXP ? -expf(z) : log_sigmoid_f(z) * inv_tau, -80.f);
+}
+
+// the same for bf16 steps, whose z has bf16 rounding in it: hardware exponential
+// and logarithm, log(1 + x) by its series where x is small
+template <bool EXP>
+__device__ __forceinline__ float log_decay_fast(float z, float inv_tau) {
+    if (EXP) return fmaxf(-__expf(z), -80.f);
+    const float x = __expf(-fabsf(z));
+    const float l = x < 0.02f ? x * (1.f + x * (-0.5f + x * (1.f / 3.f))) : __logf(1.f + x);
+    return fmaxf((fminf(z, 0.f) - l) * inv_tau, -80.f);
 }
 
 #define DL_ROWS 8
@@ -112,7 +123,7 @@ __global__ void decay_logs_mfma_kernel(
         unpack8(x, f);
         if (EXP) {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) f[i] = tanhf(f[i]);
+            for (int i = 0; i < 8; ++i) f[i] = tanh_fast(f[i]);
         }
         split_frag(f, hi, lo);
 #pragma unroll
@@ -131,8 +142,8 @@ __global__ void decay_logs_mfma_kernel(
         if (n >= N) continue;  // N is a multiple of 4
         const float4 b = *reinterpret_cast<const float4*>(bias + n);
         *reinterpret_cast<float4*>(out + (size_t)t * N + n) = make_float4(
-            log_decay<EXP>(acc[j][0] + b.x, inv_tau), log_decay<EXP>(acc[j][1] + b.y, inv_tau),
-            log_decay<EXP>(acc[j][2] + b.z, inv_tau), log_decay<EXP>(acc[j][3] + b.w, inv_tau));
+            log_decay_fast<EXP>(acc[j][0] + b.x, inv_tau), log_decay_fast<EXP>(acc[j][1] + b.y, inv_tau),
+            log_decay_fast<EXP>(acc[j][2] + b.z, inv_tau), log_decay_fast<EXP>(acc[j][3] + b.w, inv_tau));
     }
 }
 
@@ -277,70 +288,76 @@ __global__ void decay_state_kernel(DecayArgs a) {
             S[j] = *reinterpret_cast<const f32x4*>(Sp + (size_t)vd * dk + kd);
     }
     const int d8 = tid % 8 * 8, kcol = kt * 64 + d8;
-    uint4 kreg[2], vreg[2];
-    float Fr[2][8], Fl[8];
-    f32x4 keep;
-    auto load_rows = [&](int r0) {
+    struct Rows {  // a chunk's operands on their way to LDS
+        uint4 k[2], v[2];
+        float F[2][8], Fl[8];
+        f32x4 keep;
+    };
+    auto load_rows = [&](Rows& x, int r0) {
         const int last = min(r0 + CH, row_hi) - 1;
-        keep = (f32x4){0.f, 0.f, 0.f, 0.f};
-        if (kd < dk) keep = *reinterpret_cast<const f32x4*>(Fp + (size_t)last * N + kd);
-        if (kcol < dk) load8f(Fp + (size_t)last * N + kcol, Fl);
+        x.keep = (f32x4){0.f, 0.f, 0.f, 0.f};
+        if (kd < dk) x.keep = *reinterpret_cast<const f32x4*>(Fp + (size_t)last * N + kd);
+        if (kcol < dk) load8f(Fp + (size_t)last * N + kcol, x.Fl);
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
             const int r = r0 + tid / 8 + u * 32;
-            kreg[u] = vreg[u] = (uint4){0, 0, 0, 0};
+            x.k[u] = x.v[u] = (uint4){0, 0, 0, 0};
             if (r < row_hi) {
                 if (kcol < dk) {
-                    kreg[u] = *reinterpret_cast<const uint4*>(kp + (size_t)r * a.ldk + kcol);
-                    load8f(Fp + (size_t)r * N + kcol, Fr[u]);
+                    x.k[u] = *reinterpret_cast<const uint4*>(kp + (size_t)r * a.ldk + kcol);
+                    load8f(Fp + (size_t)r * N + kcol, x.F[u]);
                 }
                 if (vt * 64 + d8 < dv)
-                    vreg[u] = *reinterpret_cast<const uint4*>(vp + (size_t)r * a.ldv + vt * 64 + d8);
+                    x.v[u] = *reinterpret_cast<const uint4*>(vp + (size_t)r * a.ldv + vt * 64 + d8);
             }
         }
     };
-    load_rows(row_lo);
-    for (int c = c_lo; c < c_hi; ++c) {
+    // one chunk; its register set then takes the chunk after the next
+    auto run_chunk = [&](Rows& x, int c) {
         const int r0 = row_lo + (c - c_lo) * CH;
         const size_t base = ((size_t)c * H + h) * dv;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int vd = vt * 64 + j * 16 + r16;
             if (vd < dv && kd < dk) {
-                uint16_t hi[4], lo[4];
+                uint32_t hi[2], lo[2];
 #pragma unroll
-                for (int r = 0; r < 4; ++r) split_bf16(S[j][r], hi[r], lo[r]);
+                for (int r = 0; r < 2; ++r) {
+                    hi[r] = cvt_pk_bf16(S[j][2 * r], S[j][2 * r + 1]);
+                    float p, q;
+                    unpack2(hi[r], p, q);
+                    lo[r] = cvt_pk_bf16(S[j][2 * r] - p, S[j][2 * r + 1] - q);
+                }
                 const size_t at = (base + vd) * dk + kd;
-                *reinterpret_cast<uint2*>(a.s_hi + at) = make_uint2(
-                    hi[0] | ((uint32_t)hi[1] << 16), hi[2] | ((uint32_t)hi[3] << 16));
-                *reinterpret_cast<uint2*>(a.s_lo + at) = make_uint2(
-                    lo[0] | ((uint32_t)lo[1] << 16), lo[2] | ((uint32_t)lo[3] << 16));
+                *reinterpret_cast<uint2*>(a.s_hi + at) = make_uint2(hi[0], hi[1]);
+                *reinterpret_cast<uint2*>(a.s_lo + at) = make_uint2(lo[0], lo[1]);
             }
         }
-        __syncthreads();  // the previous chunk's tiles have been read
+        // barriers that leave the loads of later chunks under way
+        lds_barrier();  // the previous chunk's tiles have been read
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
             const int s = tid / 8 + u * 32;
             float f[8];
             bf16x8 hi, lo;
-            unpack8(kreg[u], f);
+            unpack8(x.k[u], f);
             if (r0 + s < row_hi && kcol < dk) {
 #pragma unroll
-                for (int i = 0; i < 8; ++i) f[i] *= __expf(Fl[i] - Fr[u][i]);
+                for (int i = 0; i < 8; ++i) f[i] *= __expf(x.Fl[i] - x.F[u][i]);
             }
             split_frag(f, hi, lo);
             *reinterpret_cast<bf16x8*>(&k_hi[s][d8]) = hi;
             *reinterpret_cast<bf16x8*>(&k_lo[s][d8]) = lo;
-            *reinterpret_cast<uint4*>(&v_lds[s][d8]) = vreg[u];
+            *reinterpret_cast<uint4*>(&v_lds[s][d8]) = x.v[u];
         }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const float f = __expf(keep[r]);
+            const float f = __expf(x.keep[r]);
 #pragma unroll
             for (int j = 0; j < 4; ++j) S[j][r] *= f;
         }
-        __syncthreads();
-        if (c + 1 < c_hi) load_rows(r0 + CH);
+        if (c + 2 < c_hi) load_rows(x, r0 + 2 * CH);
+        lds_barrier();
 #pragma unroll
         for (int s0 = 0; s0 < CH; s0 += 32) {
             const bf16x8 ah = tr_frag(&k_hi[0][0], LDT, s0, wave * 16);
@@ -352,6 +369,13 @@ __global__ void decay_state_kernel(DecayArgs a) {
                 S[j] = mfma16(al, vf, S[j]);
             }
         }
+    };
+    Rows even, odd;
+    load_rows(even, row_lo);
+    if (c_lo + 1 < c_hi) load_rows(odd, row_lo + CH);
+    for (int c = c_lo; c < c_hi; c += 2) {
+        run_chunk(even, c);
+        if (c + 1 < c_hi) run_chunk(odd, c + 1);
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -371,7 +395,7 @@ __global__ void decay_out_kernel(DecayArgs a) {
     constexpr int LDK = NC * 32 + 8, LDV = NB * 64 + 8;
     __shared__ __align__(16) bf16 q_lds[2][CH * LDK];
     __shared__ __align__(16) bf16 p_lds[2][CH * LDT];
-    __shared__ __align__(16) bf16 v_lds[CH * LDV];
+    __shared__ __align__(16) bf16 v_lds[32 * LDV];  // half of the chunk's rows
     const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * NB * 64;
     const int dk = a.dk, dv = a.dv, H = a.H, N = H * dk;
     const int seg = a.chunk_seg[c], r0 = a.cu[seg] + a.chunk_off[c];
@@ -381,17 +405,23 @@ __global__ void decay_out_kernel(DecayArgs a) {
     const bf16 *kp = (const bf16*)a.k + (size_t)r0 * a.ldk + (size_t)h * dk;
     const bf16 *vp = (const bf16*)a.v + (size_t)r0 * a.ldv + (size_t)h * dv;
     const float* Fp = a.logw + (size_t)r0 * N + (size_t)h * dk;
+    uint4 v_late[NB];  // the other half
 #pragma unroll
-    for (int u = 0; u < NB * 2; ++u) {
+    for (int u = 0; u < NB; ++u) {
         const int e = tid + u * 256, s = e / (NB * 8), d = e % (NB * 8) * 8;
         uint4 x = {0, 0, 0, 0};
-        if (s < n && v0 + d < dv)
-            x = *reinterpret_cast<const uint4*>(vp + (size_t)s * a.ldv + v0 + d);
+        v_late[u] = x;
+        if (v0 + d < dv) {
+            if (s < n) x = *reinterpret_cast<const uint4*>(vp + (size_t)s * a.ldv + v0 + d);
+            if (s + 32 < n)
+                v_late[u] = *reinterpret_cast<const uint4*>(vp + (size_t)(s + 32) * a.ldv + v0 + d);
+        }
         *reinterpret_cast<uint4*>(v_lds + s * LDV + d) = x;
     }
     {
         const int b0 = wave * 16, t = min(b0 + r16, n - 1);  // this lane's row
         const bf16* qr = (const bf16*)a.q + (size_t)(r0 + t) * a.ldq + (size_t)h * dk;
+        float* w_own = reinterpret_cast<float*>(&p_lds[0][b0 * LDT]);  // until P goes there
         f32x4 P[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) P[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -440,27 +470,45 @@ __global__ void decay_out_kernel(DecayArgs a) {
                     else P[2] = p;
                 }
             }
-            // this block: row tt of P is row tt of q against k_s e^(E_tt - F_s)
-            float Fs[8], k[8], u[8];
+            // this block: row tt of P is row tt of q against k_s w_(s+1) .. w_tt
+            // (WKV: .. w_(tt-1), and u k_tt): the decayed keys are carried from
+            // row to row, lane r16 holds key r16 (0 before its row is there)
+            float k[8], u[8], kt[8];
             unpack8(*reinterpret_cast<const uint4*>(kp + (size_t)t * a.ldk + dd), k);
-            load8f(Fp + (size_t)t * N + dd, Fs);
             if (WKV) load8f(a.u + (size_t)h * dk + dd, u);
+            {
+                float Fs[8], Fb[8];
+                load8f(Fp + (size_t)t * N + dd, Fs);
+                if (t > 0) {
+                    load8f(Fp + (size_t)(t - 1) * N + dd, Fb);
+                } else {
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) Fb[i] = 0.f;
+                }
+#pragma unroll
+                for (int i = 0; i < 8; ++i) Fs[i] = __expf(Fs[i] - Fb[i]);
+                float* wp = w_own + r16 * 32 + g * 8;
+                reinterpret_cast<float4*>(wp)[0] = make_float4(Fs[0], Fs[1], Fs[2], Fs[3]);
+                reinterpret_cast<float4*>(wp)[1] = make_float4(Fs[4], Fs[5], Fs[6], Fs[7]);
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) kt[i] = 0.f;
             const int rows = min(16, n - b0);
 #pragma unroll 4
             for (int tt = 0; tt < rows; ++tt) {
-                const int row = b0 + tt - (WKV ? 1 : 0);
-                float Et[8];
-                load8f(Fp + (size_t)max(row, 0) * N + dd, Et);
+                float w[8];
+                load8f(w_own + tt * 32 + g * 8, w);
+                const bool mine = r16 == tt;
 #pragma unroll
                 for (int i = 0; i < 8; ++i) {
-                    const float w = r16 < tt ? __expf(fminf(Et[i] - Fs[i], 0.f))
-                                             : (r16 == tt ? (WKV ? u[i] : 1.f) : 0.f);
-                    f[i] = k[i] * w;
+                    const float next = mine ? k[i] : kt[i] * w[i];
+                    f[i] = WKV ? (mine ? u[i] * k[i] : kt[i]) : next;
+                    kt[i] = next;
                 }
                 bf16x8 kh, kl;
                 split_frag(f, kh, kl);
                 uint4 qm = qraw;
-                if (r16 != tt) qm = (uint4){0, 0, 0, 0};
+                if (!mine) qm = (uint4){0, 0, 0, 0};
                 P[3] = mfma16(as_frag(qm), kh, P[3]);
                 P[3] = mfma16(as_frag(qm), kl, P[3]);
             }
@@ -490,9 +538,18 @@ __global__ void decay_out_kernel(DecayArgs a) {
     const int vw = wave * NB * 16;  // first of this wave's value dims
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
+        if (u) {
+            __syncthreads();
+#pragma unroll
+            for (int k = 0; k < NB; ++k) {
+                const int e = tid + k * 256;
+                *reinterpret_cast<uint4*>(v_lds + e / (NB * 8) * LDV + e % (NB * 8) * 8) = v_late[k];
+            }
+            __syncthreads();
+        }
         bf16x8 vf[NB];
 #pragma unroll
-        for (int j = 0; j < NB; ++j) vf[j] = tr_frag(v_lds, LDV, u * 32, vw + j * 16);
+        for (int j = 0; j < NB; ++j) vf[j] = tr_frag(v_lds, LDV, 0, vw + j * 16);
 #pragma unroll
         for (int i = u * 2; i < 4; ++i) {
             const int at = (i * 16 + r16) * LDT + u * 32 + g * 8;
@@ -543,8 +600,8 @@ __global__ void decay_out_kernel(DecayArgs a) {
             const int vd = v0 + vw + j * 16 + g * 4;
             if (vd < dv)
                 *reinterpret_cast<uint2*>(yr + vd) = make_uint2(
-                    pack2(o[i][j][0] * a.qscale, o[i][j][1] * a.qscale),
-                    pack2(o[i][j][2] * a.qscale, o[i][j][3] * a.qscale));
+                    cvt_pk_bf16(o[i][j][0] * a.qscale, o[i][j][1] * a.qscale),
+                    cvt_pk_bf16(o[i][j][2] * a.qscale, o[i][j][3] * a.qscale));
         }
     }
 }

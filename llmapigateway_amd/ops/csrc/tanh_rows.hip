@@ -7,15 +7,10 @@
 
 #include "rows.h"
 
-// tanh: the library's in fp32; in bf16 steps one exponential, a series where
-// that would lose relative accuracy (both far inside bf16 rounding)
+// tanh: the library's in fp32, the short one in bf16 steps
 template <typename T>
 __device__ __forceinline__ float tanh_of(float z) {
-    if (sizeof(T) == 4) return tanhf(z);
-    const float z2 = z * z;
-    const float series = z * (1.f + z2 * (-1.f / 3.f + z2 * (2.f / 15.f)));
-    const float e = 1.f - 2.f / (1.f + __expf(2.f * z));
-    return z2 < 0.01f ? series : e;
+    return sizeof(T) == 4 ? tanhf(z) : tanh_fast(z);
 }
 template <typename T>
 __device__ __forceinline__ float silu_of(float z) {
