@@ -57,12 +57,13 @@ def test_wave_mode():
     assert d["config"]["mode"] == "closed-loop-waves"
 
 
-def test_layers_mode():
-    d = run_bench(["--mode", "layers", "--sizes", "tiny-lelisun", "--prefill-shapes", "2x16",
-                   "--decode-batches", "2", "--decode-context", "16"])
-    assert [r["model"] for r in d["results"]] == ["tiny-lelisun", "llama of tiny-lelisun"]
+@pytest.mark.parametrize("family,runs", [("lelisun", 6), ("filinex", 3)])
+def test_layers_mode(family, runs):
+    d = run_bench(["--mode", "layers", "--family", family, "--sizes", f"tiny-{family}",
+                   "--prefill-shapes", "2x16", "--decode-batches", "2", "--decode-context", "16"])
+    assert [r["model"] for r in d["results"]] == [f"tiny-{family}", f"llama of tiny-{family}"]
     for r in d["results"]:
-        assert r["layer_runs"] == 6
+        assert r["layer_runs"] == runs
         assert r["prefill"]["2x16"]["tok_s"] > 0 and r["decode"]["b2"]["tok_s"] > 0
 
 
