@@ -360,9 +360,9 @@ class Parallel:
 
 
 class WKV:
-    """RWKV-style time mixing: every projection reads its own mix of a
-    token's row and the previous one; a data-dependent decay per key channel,
-    exp(-exp(.)), and a bonus for the current token only."""
+    """RWKV-style time mixing: five projections of different blends of a
+    token's row and the one before it; a data-dependent decay per key channel,
+    exp(-exp(.)), and an extra weight u on the current token's own key."""
 
     plans = ("chunks",)  # what it uses of a step's plan
 
