@@ -71,23 +71,25 @@ class HybridConfig:
     [start, stop) run ``times`` times with the same weights, each pass with
     its own cache.
 
-    The field set is what the Lelisun and Filinex config.json files give and
-    what their designs fix; ``max_positions`` is the framework's own bound
-    (nothing in the designs limits it) and ``weights_dir`` says where the
-    checkpoint lies (None: random init)."""
+    The field set is what the Lelisun, Filinex and Mekevik config.json files
+    give and what their designs fix; ``max_positions`` is the framework's own
+    bound (nothing in the designs limits it) and ``weights_dir`` says where
+    the checkpoint lies (None: random init)."""
 
     name: str
     vocab_size: int
     hidden_size: int
     layers: Tuple[HybridLayer, ...]
     norm_eps: float = 1e-5
-    norm: str = "layernorm"       # of the stream: "layernorm" | "tanh" (dynamic tanh)
+    norm: str = "layernorm"       # of the stream: "layernorm" | "tanh" (dynamic tanh) | "rms"
+    parallel_mlp: bool = False    # mixer and feed-forward read the same stream
     post_norm: bool = False       # a norm on every sublayer's output, too
     embed_norm: bool = False
     embed_scale: float = 1.0
     loop: Optional[Tuple[int, int, int]] = None  # (start, stop, times)
     loop_step: bool = True        # a learned vector per loop pass
     logit_softcap: Optional[float] = None
+    logit_scale: float = 1.0
     max_positions: int = 32768
     weights_dir: Optional[str] = None
 
@@ -96,8 +98,12 @@ class HybridConfig:
             start, stop, times = self.loop
             if not (0 <= start < stop <= len(self.layers) and times >= 1):
                 raise ValueError(f"bad loop {self.loop} over {len(self.layers)} layers")
-        if self.norm not in ("layernorm", "tanh"):
+        if self.norm not in ("layernorm", "tanh", "rms"):
             raise ValueError(f"unknown norm '{self.norm}'")
+        if self.norm != "rms" and self.parallel_mlp:
+            raise ValueError("mixer and feed-forward in parallel: RMS norms only")
+        if self.norm == "rms" and self.loop is not None:
+            raise ValueError("loops: layer norms and dynamic tanh only")
         if self.norm != "tanh" and (self.post_norm or self.embed_norm):
             raise ValueError("norms of sublayer outputs and of the embedding: dynamic tanh only")
         for i, layer in enumerate(self.layers):
@@ -105,6 +111,12 @@ class HybridConfig:
                 self._check_layer(layer)
             except ValueError as e:
                 raise ValueError(f"layer {i}: {e}") from None
+        shared = {
+            layer.mixer["kv_heads"] * layer.mixer["vdim"]
+            for layer in self.layers if layer.mixer.get("v_mix")
+        }
+        if len(shared) > 1:
+            raise ValueError(f"layers that mix values have {sorted(shared)} of them")
 
     @staticmethod
     def _check_layer(layer: HybridLayer) -> None:
@@ -120,6 +132,13 @@ class HybridConfig:
                 raise ValueError("kv_heads does not divide the heads")
             if not m["left"]["softcap"] > 0 or not m["right"]["tau"] > 0:
                 raise ValueError("softcap and tau are positive")
+        elif layer.type == "sigmoid_attention":
+            if m["heads"] % m["kv_heads"]:
+                raise ValueError("kv_heads does not divide the heads")
+            if not m["bias_max"] > m["bias_rows"] // 2 > 0:
+                raise ValueError(f"bias_max {m['bias_max']} for {m['bias_rows']} rows")
+            if not m["window"] >= 1:
+                raise ValueError(f"a window of {m['window']}")
         elif layer.type not in ("mlstm", "wkv"):
             raise ValueError(f"unknown mixer '{layer.type}'")
         if layer.mlp is None:
@@ -173,6 +192,29 @@ class HybridConfig:
             **cls._common(raw, layers),
         )
 
+    @classmethod
+    def from_mekevik_json(cls, raw: Dict[str, Any], name: str, weights_dir: Optional[str] = None):
+        """Mekevik's config.json. How many rows a layer's distance table has
+        is only in the checkpoint's shapes."""
+        from .weights import open_checkpoint
+
+        ckpt = open_checkpoint(weights_dir)
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            if e["type"] != "attention":
+                raise ValueError(f"layer {i}: unknown mixer '{e['type']}'")
+            m, mlp = dict(e["mixer"]), e.get("mlp")
+            m["window"] = m.pop("mask")["size"]
+            m["bias_rows"] = ckpt.shape(f"l{i}.mix.rel")[0]
+            if mlp is not None and mlp["kind"] == "moe":
+                mlp = dict(mlp, router=dict(mlp["router"], bias=False))
+            layers.append(HybridLayer(type="sigmoid_attention", mixer=m, mlp=mlp))
+        return cls(
+            name=name, norm="rms", parallel_mlp=True, embed_scale=raw["embedding"]["scale"],
+            logit_scale=raw["logit_scale"], weights_dir=weights_dir,
+            **cls._common(raw, layers),
+        )
+
     def runs(self) -> List[Tuple[int, Optional[int]]]:
         """The layers in the order they run, as (layer index, t): t is the
         number of the loop pass that this layer begins, None elsewhere."""
@@ -186,7 +228,9 @@ class HybridConfig:
 
     @property
     def prefix_cacheable(self) -> bool:
-        return all(layer.type == "latent_attention" for layer in self.layers)
+        return all(
+            layer.type in ("latent_attention", "sigmoid_attention") for layer in self.layers
+        )
 
     def scaled_for_tp(self, tp: int) -> "HybridConfig":
         raise NotImplementedError(f"{self.name}: hybrid decoders run on one GPU (tp=1)")
@@ -196,6 +240,7 @@ class HybridConfig:
 ARCHITECTURES = {
     "Lelisun": HybridConfig.from_json,
     "Filinex": HybridConfig.from_filinex_json,
+    "Mekevik": HybridConfig.from_mekevik_json,
 }
 
 
@@ -267,6 +312,30 @@ def _filinex_preset(
         name=name, vocab_size=vocab, hidden_size=width, layers=layers, norm="tanh",
         post_norm=True, embed_norm=True, loop=(0, len(layers) - 1, times), loop_step=False,
         logit_softcap=30.0, max_positions=max_positions,
+    )
+
+
+def _mekevik_preset(
+    name: str, width: int, vocab: int, heads: int, kv_heads: int, dim: int, vdim: int,
+    window: int, bias_rows: int, bias_max: int, ff: int, experts: int, top: int,
+    expert_ff: int, layers: int, max_positions: int = 32768,
+) -> HybridConfig:
+    """A Mekevik of layers with a dense feed-forward and with experts in turn."""
+    mixer = dict(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, window=window,
+        bias_rows=bias_rows, bias_max=bias_max, v_mix=True,
+    )
+    mlps = (
+        dict(kind="dense", ff=ff, limit=7.0),
+        dict(kind="moe", expert=dict(ff=expert_ff),
+             router=dict(experts=experts, top=top, scale=1.0, bias=False)),
+    )
+    return HybridConfig(
+        name=name, vocab_size=vocab, hidden_size=width, norm="rms", parallel_mlp=True,
+        layers=tuple(
+            HybridLayer("sigmoid_attention", mixer, mlps[i % 2]) for i in range(layers)
+        ),
+        embed_scale=width ** 0.5, logit_scale=0.5, max_positions=max_positions,
     )
 
 
@@ -383,6 +452,23 @@ MODEL_PRESETS = {
         "filinex-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=128,
         lin_heads=16, lin_dim=128, lin_vdim=256, wkv_dim=64, rank=16, experts=64, top=6,
         ff=1536, shared_ff=5120, times=2, repeat=4,
+    ),
+    # windowed sigmoid attention with mixed heads beside dense and expert layers
+    "tiny-mekevik": _mekevik_preset(
+        "tiny-mekevik", width=96, vocab=320, heads=6, kv_heads=3, dim=24, vdim=16, window=40,
+        bias_rows=12, bias_max=33, ff=112, experts=6, top=2, expert_ff=40, layers=3,
+        max_positions=1024,
+    ),
+    # layers as wide as llama-1b's and llama-3-8b's
+    "mekevik-small": _mekevik_preset(
+        "mekevik-small", width=2048, vocab=128256, heads=16, kv_heads=4, dim=128, vdim=128,
+        window=1024, bias_rows=32, bias_max=128, ff=8192, experts=32, top=4, expert_ff=2048,
+        layers=12,
+    ),
+    "mekevik-base": _mekevik_preset(
+        "mekevik-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=128, vdim=128,
+        window=1024, bias_rows=32, bias_max=128, ff=14336, experts=64, top=8, expert_ff=1792,
+        layers=16,
     ),
     # small-but-real shape for 1-GPU kernel shakedown
     "llama-1b": ModelConfig(

@@ -16,11 +16,14 @@ Getter = Callable[[str], torch.Tensor]
 
 
 class DenseFF:
-    """W_down (silu(W_gate h) * W_up h)."""
+    """W_down (silu(W_gate h) * W_up h); with a ``limit`` the clamped GLU of
+    the two instead: g = min(W_gate h, limit), u = clamp(W_up h, +-limit),
+    g sigmoid(1.702 g) (u + 1)."""
 
     def __init__(self, m: dict, get: Getter, vec: Getter):
+        self.limit = m.get("limit")
         self.w = {"gate_up": torch.cat([get("gate"), get("up")]), "down": get("down")}
-        add_decode_twins(self.w, ("gate_up", "down"))
+        add_decode_twins(self.w, ("gate_up", "down") if self.limit is None else ("down",))
 
     @staticmethod
     def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
@@ -29,6 +32,9 @@ class DenseFF:
 
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
         w = self.w
+        if self.limit is not None:
+            act = ops.clamped_glu(ops.linear(h, w["gate_up"]), float(self.limit))
+            return ops.linear(act, w["down"], w.get("down_swz"))
         return ops.linear(
             ops.swiglu_linear(h, w["gate_up"], w.get("gate_up_swz"), w.get("gate_up_int")),
             w["down"], w.get("down_swz"),
@@ -36,16 +42,18 @@ class DenseFF:
 
 
 class ExpertFF:
-    """Clamped-SwiGLU experts of which a router picks ``top`` per token
-    (weights: softmax over the chosen logits), and a shared one for every
-    token. Expert: g = min(W_gate h, limit), u = clamp(W_up h, +-limit),
-    W_down (g sigmoid(1.702 g) (u + 1))."""
+    """Experts of which a router picks ``top`` per token, and optionally a
+    shared one for every token. An expert is a DenseFF, with or without a
+    limit. Weights: softmax over the chosen logits (which is the softmax over
+    all of them, divided by the chosen ones' sum), times the router's
+    ``scale``; the router may have a bias."""
 
     def __init__(self, m: dict, get: Getter, vec: Getter):
-        E = m["router"]["experts"]
-        self.top = m["router"]["top"]
-        self.limit = float(m["expert"]["limit"])
-        self.w_router, self.b_router = get("router"), vec("router.b")
+        r = m["router"]
+        E, self.top, self.scale = r["experts"], r["top"], float(r.get("scale", 1.0))
+        self.limit = m["expert"].get("limit")
+        self.w_router = get("router")
+        self.b_router = vec("router.b") if r.get("bias", True) else None
         self.experts = ops.pack_experts(
             m["expert"]["ff"], self.w_router.shape[1], E,
             lambda e: (get(f"e{e}.gate"), get(f"e{e}.up"), get(f"e{e}.down")),
@@ -62,7 +70,9 @@ class ExpertFF:
     @staticmethod
     def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
         E = m["router"]["experts"]
-        out: Dict[str, Tuple[int, ...]] = {"router": (E, width), "router.b": (E,)}
+        out: Dict[str, Tuple[int, ...]] = {"router": (E, width)}
+        if m["router"].get("bias", True):
+            out["router.b"] = (E,)
         parts = [(f"e{e}", m["expert"]["ff"]) for e in range(E)]
         if m.get("shared") is not None:
             parts.append(("shared", m["shared"]["ff"]))
@@ -72,7 +82,9 @@ class ExpertFF:
         return out
 
     def __call__(self, h: torch.Tensor) -> "ops.ExpertSum":
-        routing = ops.route_experts(h, self.w_router, self.b_router, self.top, self.experts)
+        routing = ops.route_experts(
+            h, self.w_router, self.b_router, self.top, self.experts, self.scale
+        )
         rows = ops.expert_rows(h, routing, self.experts, self.limit)
         shared = None
         if self.shared is not None:

@@ -3,11 +3,13 @@ several times in a row with the same weights.
 
 The residual stream is fp32; a sublayer's output stays pending, with its own
 norm where the design has one, and is added by the next norm's kernel
-(ops.add_layernorm, ops.add_tanh_norm). A loop pass starts by replacing the
+(ops.add_layernorm, ops.add_tanh_norm, ops.add_rms_norm). Where mixer and
+feed-forward are parallel, both of their outputs are pending together, and
+one kernel makes the two norms of the next layer. A loop pass starts by replacing the
 stream with W [stream; embedding output] (+ step[t]); each pass of a layer
 has its own cache view.
 
-Serves Lelisun and Filinex; another design built from these mixers and
+Serves Lelisun, Filinex and Mekevik; another design built from these mixers and
 feed-forwards needs only a configuration.
 """
 
@@ -61,7 +63,9 @@ class HybridModel:
         out = {"embed": (V, W), "head": (V, W)}
 
         def norm(name: str) -> None:
-            out[name] = out[name + ".b"] = (W,)
+            out[name] = (W,)
+            if config.norm != "rms":
+                out[name + ".b"] = (W,)
             if config.norm == "tanh":
                 out[name + ".alpha"] = ()
 
@@ -110,6 +114,8 @@ class HybridModel:
                 return t.fill_(2.0 if name.endswith((".f.b", ".a2.b")) else 0.0)
             if leaf == "dt_bias":
                 return t.fill_(-2.0)
+            if leaf in ("pb", "vmix"):
+                return t.fill_(-4.0 if leaf == "pb" else 0.5)
             if leaf == "w0":
                 return t.normal_(-1.5, 1.0, generator=gen)
             if ".mu." in name:
@@ -131,6 +137,8 @@ class HybridModel:
             return source(name).to(self.device).float().contiguous()
 
         def norm(name: str):
+            if c.norm == "rms":
+                return (vec(name),)
             parts = (vec(name), vec(name + ".b"))
             return parts + (float(source(name + ".alpha")),) if c.norm == "tanh" else parts
 
@@ -162,6 +170,10 @@ class HybridModel:
                 )
             self.layers.append(ent)
         self.final_norm = norm("final.norm")
+        if c.logit_scale != 1.0:  # the norm's last factors take it in
+            self.final_norm = tuple(t * c.logit_scale for t in self.final_norm[:2]) + (
+                self.final_norm[2:]
+            )
         self.head = mat("head")
 
     def _rope(self, base: float, dims: int) -> torch.Tensor:
@@ -173,17 +185,21 @@ class HybridModel:
         return self._ropes[key]
 
     # ---- forward ----
-    def _norm(self, x, delta, post, norm, vec=None, replace=False) -> torch.Tensor:
+    def _norm(self, x, pending, post, norm, vec=None, replace=False) -> torch.Tensor:
         """Add the pending sublayer output (through its own norm, ``post``)
         to the stream, or replace the stream by it; the normed rows."""
+        if self.config.norm == "rms":
+            return ops.add_rms_norm(x, pending, norm, self.config.norm_eps, self.dtype)[0]
+        delta = pending[0] if pending else None
         if self.config.norm == "tanh":
             return ops.add_tanh_norm(x, delta, post, norm, self.dtype, replace=replace)
         return ops.add_layernorm(
             x, delta, *norm, self.config.norm_eps, self.dtype, vec=vec, replace=replace
         )
 
-    def _cast(self, x, delta, post, out) -> None:
+    def _cast(self, x, pending, post, out) -> None:
         """The same addition; the stream itself goes to ``out``."""
+        delta = pending[0] if pending else None
         if self.config.norm == "tanh":
             ops.add_tanh_norm(x, delta, post, None, self.dtype, out=out)
         else:
@@ -204,26 +220,34 @@ class HybridModel:
             x = ops.embed_scaled(batch.token_ids, self.embed, c.embed_scale, x0)
         else:
             x = ops.embed_tanh_norm(batch.token_ids, self.embed, self.embed_norm, x0)
-        delta = post = None
+        pending, post = (), None
         for r, (i, t) in enumerate(c.runs()):
             layer = self.layers[i]
+            mixer, mlp = layer["mixer"], layer["mlp"]
+            if c.parallel_mlp and mlp is not None:
+                h, h2 = ops.add_rms_norm(
+                    x, pending, layer["norm1"] + layer["norm2"], c.norm_eps, self.dtype
+                )
+                pending = (mixer(h, batch, cache.runs[r], plan), mlp(h2))
+                continue
             if t is None:
-                h = self._norm(x, delta, post, layer["norm1"])
+                h = self._norm(x, pending, post, layer["norm1"])
             else:
-                self._cast(x, delta, post, both[:, :W])
+                self._cast(x, pending, post, both[:, :W])
                 h = self._norm(
-                    x, ops.linear_f32(both, self.loop_in), None, layer["norm1"],
+                    x, (ops.linear_f32(both, self.loop_in),), None, layer["norm1"],
                     vec=self.loop_step[t], replace=True,
                 )
-            delta, post = layer["mixer"](h, batch, cache.runs[r], plan), layer["norm1b"]
-            if layer["mlp"] is not None:
-                h = self._norm(x, delta, post, layer["norm2"])
-                delta, post = layer["mlp"](h), layer["norm2b"]
+            pending, post = (mixer(h, batch, cache.runs[r], plan),), layer["norm1b"]
+            if mlp is not None:
+                h = self._norm(x, pending, post, layer["norm2"])
+                pending, post = (mlp(h),), layer["norm2b"]
         if batch.logits_indices is not None:
-            x, delta = x[batch.logits_indices], delta[batch.logits_indices]
+            pick = batch.logits_indices
+            x, pending = x[pick], tuple(d[pick] for d in pending)
             if x.shape[0] == 0:
                 return torch.empty(0, c.vocab_size, dtype=torch.float32, device=self.device)
-        h = self._norm(x, delta, post, self.final_norm)
+        h = self._norm(x, pending, post, self.final_norm)
         logits = ops.linear_f32(h, self.head)
         if c.logit_softcap is not None:
             ops.soft_cap_(logits, c.logit_softcap)

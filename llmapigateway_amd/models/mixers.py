@@ -269,6 +269,65 @@ class GatedAttention:
         )
 
 
+class SigmoidAttention:
+    """Grouped-query attention over the last ``window`` tokens without
+    rotation or softmax: a key weighs sigmoid(score + a learned bias of its
+    distance and the head), and learned mixes of all heads' weights go to the
+    values. Queries and keys are normed over all heads at once; every output
+    value has a sigmoid gate. Layers with ``v_mix``, after the first of them,
+    blend their values with the first one's."""
+
+    plans = ("head_tiles",)  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.H, self.G, self.eps = m["heads"], m["kv_heads"], eps
+        self.scale, self.window, self.v_mix = float(m["scale"]), m["window"], m.get("v_mix")
+        w_in, self.cut = _stack([(n, get(n)) for n in ("q", "k", "v", "g")])
+        self.w = {"in": w_in, "o": get("o")}
+        self.q_norm, self.k_norm = vec("q.norm"), vec("k.norm")
+        self.talk = get("talk")
+        self.bias = ops.distance_bias(vec("rel"), vec("pb"), m["bias_max"], self.window)
+        self.blend = float(vec("vmix")) if self.v_mix else 0.0
+        add_decode_twins(self.w, ("in", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H, G = m["heads"], m["kv_heads"]
+        out: Dict[str, Tuple[int, ...]] = {
+            "q": (H * m["dim"], width), "k": (G * m["dim"], width),
+            "v": (G * m["vdim"], width), "q.norm": (H * m["dim"],),
+            "k.norm": (G * m["dim"],), "rel": (m["bias_rows"], H), "talk": (H, H), "pb": (H,),
+            "g": (H * m["vdim"], width), "o": (width, H * m["vdim"]),
+        }
+        if m.get("v_mix"):
+            out["vmix"] = ()
+        return out
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        return CacheSpec({"k": m["kv_heads"] * m["dim"], "v": m["kv_heads"] * m["vdim"]}, {})
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        q, k, v, g = (u[:, lo:hi] for lo, hi in self.cut.values())
+        first = None
+        if self.v_mix:
+            first = plan.carry.get("v_first")
+            if first is None:
+                plan.carry["v_first"] = v
+        q = ops.qkv_rows(
+            q, k, v, self.q_norm, self.k_norm, self.eps, self.blend, first, cache["k"],
+            cache["v"], batch.slot_mapping,
+        )
+        out = torch.empty(h.shape[0], w["o"].shape[1], dtype=h.dtype, device=h.device)
+        ops.sigmoid_attention(
+            out, q, cache["k"], cache["v"], self.H, self.G, self.scale, self.bias, self.talk,
+            self.window, g, batch.positions, batch.segs, plan,
+        )
+        return ops.linear(out, w["o"], w.get("o_swz"))
+
+
 class GatedLinearAttention:
     """Linear attention with a decay per key channel, sigmoid(z)^(1/tau) of a
     low-rank projection z, head-wise RMS norm and a silu gate."""
@@ -407,5 +466,5 @@ class WKV:
 
 MIXERS = {
     "latent_attention": LatentAttention, "mamba2": Mamba2, "mlstm": MLSTM,
-    "parallel": Parallel, "wkv": WKV,
+    "parallel": Parallel, "wkv": WKV, "sigmoid_attention": SigmoidAttention,
 }

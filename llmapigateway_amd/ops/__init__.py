@@ -550,12 +550,14 @@ from .experts import (  # noqa: E402
 from .hybrid import (  # noqa: E402
     add_cast,
     add_layernorm,
+    add_rms_norm,
     add_tanh_norm,
     build_pair_rope_cache,
     can_unfold,
     causal_conv,
     decay_logs,
     decayed_kv,
+    distance_bias,
     embed_scaled,
     embed_tanh_norm,
     fold_queries,
@@ -570,6 +572,8 @@ from .hybrid import (  # noqa: E402
     page_write,
     paged_attention,
     plan_segments,
+    qkv_rows,
+    sigmoid_attention,
     soft_cap_,
     ssd,
     token_shift,

@@ -19,7 +19,7 @@ hipError_t launch_paged_tiles(void*, int64_t, const void*, int64_t, const void*,
 hipError_t launch_decay_logs(float*, const void*, int64_t, const void*, const float*, int, float, int, int, int, int, int, hipStream_t);
 hipError_t launch_decay_scan(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*, const float*, float, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
 hipError_t launch_decay_chunked(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, float*, const float*, float, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, const int*, const int*, const int*, int, int, void*, hipStream_t);
-hipError_t launch_route_topk(int*, float*, const float*, const float*, int, int, int, hipStream_t);
+hipError_t launch_route_topk(int*, float*, const float*, const float*, float, int, int, int, hipStream_t);
 hipError_t launch_route_plan(int*, int*, int*, const int*, int, int, int, int, int, hipStream_t);
 hipError_t launch_expert_product(void*, int64_t, const void*, int64_t, const void*, const int*, const int*, int, int, int, float, int, int, int, int, int, int, hipStream_t);
 }
@@ -314,7 +314,7 @@ void soft_cap(Tensor x, double cap) {
 
 // z [T, E] logits -> ids, weights [T, top], and the rows' places by expert
 void route(Tensor ids, Tensor weights, Tensor slot, Tensor row_token, Tensor tile_info,
-           Tensor z, Tensor bias, int64_t tile_rows) {
+           Tensor z, OptTensor bias, double scale, int64_t tile_rows) {
     TORCH_CHECK(z.dim() == 2 && ids.dim() == 2);
     const int64_t T = z.size(0), E = z.size(1), top = ids.size(1), nt = (tile_info.numel() - 1) / 4;
     f32_ptr(z, T * E, "z");
@@ -327,16 +327,17 @@ void route(Tensor ids, Tensor weights, Tensor slot, Tensor row_token, Tensor til
     TORCH_CHECK(tile_rows > 0 && nt >= std::min(T * top, E + T * top / tile_rows),
                 "route: too few tiles");
     CHECK_HIP(launch_route_topk(ids.data_ptr<int>(), weights.data_ptr<float>(),
-                                z.data_ptr<float>(), f32_ptr(bias, E, "bias"), T, E, top,
-                                current_stream()));
+                                z.data_ptr<float>(),
+                                has(bias) ? f32_ptr(*bias, E, "bias") : nullptr, (float)scale, T,
+                                E, top, current_stream()));
     CHECK_HIP(launch_route_plan(slot.data_ptr<int>(), row_token.data_ptr<int>(),
                                 tile_info.data_ptr<int>(), ids.data_ptr<int>(), T * top, top,
                                 E, tile_rows, nt, current_stream()));
 }
 
-// out[r] = w[e] x[token(r)] through the clamped GLU (glu), or w[e] x[r]
+// out[r] = w[e] x[token(r)] through a GLU (glu 1: clamped, 2: silu), or w[e] x[r]
 void expert_product(Tensor out, Tensor x, Tensor w, Tensor row_token, Tensor tile_info,
-                    int64_t tile_rows, bool glu, double limit) {
+                    int64_t tile_rows, int64_t glu, double limit) {
     const bool f32 = is_f32(x, "x"), frag = w.dim() == 5;
     same_type(x, w, "w");
     same_type(x, out, "out");
@@ -345,6 +346,7 @@ void expert_product(Tensor out, Tensor x, Tensor w, Tensor row_token, Tensor til
     check_rows(out, R, N, "out");
     check_rows(x, x.size(0), K, "x");
     TORCH_CHECK(reinterpret_cast<uintptr_t>(tile_info.data_ptr()) % 16 == 0, "tile_info: unaligned");
+    TORCH_CHECK(glu >= 0 && glu <= 2);
     TORCH_CHECK(x.size(0) > 0 && (glu || x.size(0) == R) && w.is_contiguous());
     int64_t nfrags = 0, ksteps = 0;
     if (frag) {

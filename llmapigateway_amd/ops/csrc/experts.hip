@@ -5,6 +5,8 @@
 //
 //   act[r] = glu(W_gate[e] h[token(r)], W_up[e] h[token(r)]),  out[r] = W_down[e] act[r]
 //
+// with the clamped GLU (rows.h) or silu(gate) * up.
+//
 // A group fills whole tiles of tile_rows rows; row_token is -1 in the rest.
 // The weighted sum over a token's experts is part of the stream kernel.
 //
@@ -19,14 +21,14 @@
 #define MAX_EXPERTS 1024
 
 // ---------------------------------------------------------------------------
-// One wave a token: the top logits (ties: the lower index) and the softmax
-// over them.
+// One wave a token: the top logits (ties: the lower index) and scale times the
+// softmax over them.
 // ---------------------------------------------------------------------------
 template <int PER>  // logits a lane
 __launch_bounds__(256)
 __global__ void route_topk_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ z,
-    const float* __restrict__ bias, int T, int E, int top) {
+    const float* __restrict__ bias, float scale, int T, int E, int top) {
     const int lane = threadIdx.x & 63;
     const size_t t = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (t >= T) return;
@@ -34,7 +36,7 @@ __global__ void route_topk_kernel(
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
         const int e = i * 64 + lane;
-        v[i] = e < E ? z[t * E + e] + bias[e] : -INFINITY;
+        v[i] = e < E ? z[t * E + e] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
     }
     float mine = -INFINITY, first = 0.f;
     int my_id = 0;
@@ -70,7 +72,7 @@ __global__ void route_topk_kernel(
     const float sum = wave_reduce_sum(p);
     if (lane < top) {
         ids[t * top + lane] = my_id;
-        weights[t * top + lane] = p / sum;
+        weights[t * top + lane] = p / sum * scale;
     }
 }
 
@@ -126,8 +128,14 @@ struct ExpertArgs {
     int max_tiles;
     int64_t ldx, ld_out;
     int N, K;                // output width (GLU: of act), input width
+    int silu;                // the GLU: silu(gate) * up, or clamped at limit
     float limit;
 };
+
+template <typename T>
+__device__ __forceinline__ float expert_glu(float g, float u, const ExpertArgs& a) {
+    return a.silu ? silu_glu<T>(g, u) : clamped_glu<T>(g, u, a.limit);
+}
 
 // ---------------------------------------------------------------------------
 // Any size: tiles of 16 rows x 16 outputs, weights [E, N (GLU: 2N), K]
@@ -164,7 +172,7 @@ __global__ void expert_any_kernel(ExpertArgs a) {
         }
     }
     if (n0 + col < a.N) {
-        if (GLU) acc = clamped_glu<T>(acc, up, a.limit);
+        if (GLU) acc = expert_glu<T>(acc, up, a);
         stf((T*)a.out + (size_t)(tile * 16 + row) * a.ld_out + n0 + col, acc);
     }
 }
@@ -172,10 +180,10 @@ __global__ void expert_any_kernel(ExpertArgs a) {
 __device__ __forceinline__ void store4(bf16* p, const f32x4& v) {
     *reinterpret_cast<uint2*>(p) = make_uint2(cvt_pk_bf16(v[0], v[1]), cvt_pk_bf16(v[2], v[3]));
 }
-__device__ __forceinline__ f32x4 glu4(const f32x4& g, const f32x4& u, float limit) {
+__device__ __forceinline__ f32x4 glu4(const f32x4& g, const f32x4& u, const ExpertArgs& a) {
     f32x4 o;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) o[r] = clamped_glu<bf16>(g[r], u[r], limit);
+    for (int r = 0; r < 4; ++r) o[r] = expert_glu<bf16>(g[r], u[r], a);
     return o;
 }
 
@@ -239,7 +247,7 @@ __global__ void expert_stream_kernel(ExpertArgs a, int nfrags, int ksteps) {
             const int i = it >> 1, pair = it & 1;
             const int row = tile * 16 * MF + i * 16 + r16;
             const int n = (nf0 / 2 + pair) * 16 + g * 4;
-            const f32x4 v = glu4(sum(i * 4 + pair * 2), sum(i * 4 + pair * 2 + 1), a.limit);
+            const f32x4 v = glu4(sum(i * 4 + pair * 2), sum(i * 4 + pair * 2 + 1), a);
             if (n < a.N) store4((bf16*)a.out + (size_t)row * a.ld_out + n, v);
         }
     } else {
@@ -348,7 +356,7 @@ __global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int n = (f0 / 2 + j) * 16 + g * 4;
-                if (n < a.N) store4(o + n, glu4(acc[2 * j][i], acc[2 * j + 1][i], a.limit));
+                if (n < a.N) store4(o + n, glu4(acc[2 * j][i], acc[2 * j + 1][i], a));
             }
         } else {
 #pragma unroll
@@ -364,16 +372,17 @@ __global__ void expert_tile_kernel(ExpertArgs a, int nfrags, int ksteps, int ntn
 // launchers
 // ---------------------------------------------------------------------------
 extern "C" hipError_t launch_route_topk(
-    int* ids, float* weights, const float* z, const float* bias, int T, int E, int top,
-    hipStream_t stream) {
+    int* ids, float* weights, const float* z, const float* bias, float scale, int T, int E,
+    int top, hipStream_t stream) {
     if (T <= 0) return hipSuccess;
     if (E > MAX_EXPERTS || top > 64 || top > E || top < 1) return hipErrorInvalidValue;
     const int grid = ceil_div_i(T, 4);
-    if (E <= 64) route_topk_kernel<1><<<grid, 256, 0, stream>>>(ids, weights, z, bias, T, E, top);
-    else if (E <= 256) route_topk_kernel<4><<<grid, 256, 0, stream>>>(ids, weights, z, bias, T, E, top);
-    else {
-        route_topk_kernel<16><<<grid, 256, 0, stream>>>(ids, weights, z, bias, T, E, top);
-    }
+#define GO(PER) \
+    route_topk_kernel<PER><<<grid, 256, 0, stream>>>(ids, weights, z, bias, scale, T, E, top)
+    if (E <= 64) GO(1);
+    else if (E <= 256) GO(4);
+    else GO(16);
+#undef GO
     HIP_CHECK_LAST();
     return hipSuccess;
 }
@@ -389,13 +398,15 @@ extern "C" hipError_t launch_route_plan(
     return hipSuccess;
 }
 
-// frag: weights in fragments (bf16), else dense [E, N or 2N, K] and tiles of 16 rows
+// glu: 0 none, 1 clamped, 2 silu; frag: weights in fragments (bf16), else dense
+// [E, N or 2N, K] and tiles of 16 rows
 extern "C" hipError_t launch_expert_product(
     void* out, int64_t ld_out, const void* x, int64_t ldx, const void* w, const int* row_token,
     const int* tile_info, int N, int K, int glu, float limit, int frag, int nfrags,
     int ksteps, int tile_rows, int max_tiles, int f32, hipStream_t stream) {
     if (max_tiles <= 0) return hipSuccess;
-    const ExpertArgs a = {out, x, w, row_token, tile_info, max_tiles, ldx, ld_out, N, K, limit};
+    const ExpertArgs a = {out, x, w, row_token, tile_info, max_tiles, ldx, ld_out, N, K,
+                          glu == 2, limit};
     if (!frag) {
         if (tile_rows != 16) return hipErrorInvalidValue;
         const dim3 grid(max_tiles, ceil_div_i(N, 16));

@@ -79,6 +79,11 @@ __device__ __forceinline__ float clamped_glu(float g, float u, float limit) {
     return g * s * (u + 1.f);
 }
 
+template <typename T>
+__device__ __forceinline__ float silu_glu(float g, float u) {
+    return g * (sizeof(T) == 4 ? sigmoid_f(g) : 1.f / (1.f + __expf(-g))) * u;
+}
+
 // threads per row: enough for VEC elements each, whole waves, at most 512
 inline int row_threads(int width, int vec) {
     int t = (width + vec - 1) / vec;

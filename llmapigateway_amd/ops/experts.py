@@ -102,14 +102,17 @@ def _tile_rows(choices: int, w: ExpertWeights) -> int:
     return 16 if mean <= 10 else 32 if mean <= 20 else 64 if mean <= 48 else 256
 
 
-def route_experts(h, w_router, bias, top: int, experts: ExpertWeights) -> Routing:
-    """The ``top`` experts of every row by logits h w_router^T + bias (fp32),
-    weighted by the softmax over the chosen logits."""
+def route_experts(
+    h, w_router, bias, top: int, experts: ExpertWeights, scale: float = 1.0
+) -> Routing:
+    """The ``top`` experts of every row by logits h w_router^T (+ bias; fp32),
+    weighted by ``scale`` times the softmax over the chosen logits."""
     from .hybrid import linear_f32
 
     z = linear_f32(h, w_router)
     if not h.is_cuda:
-        ids, weights = ref.route_experts(z + bias, top)
+        ids, weights = ref.route_experts(z if bias is None else z + bias, top)
+        weights *= scale
         slot = torch.arange(ids.numel(), dtype=torch.int32).view(ids.shape)
         return Routing(slot, weights, ids.int())
     T, dev = h.shape[0], h.device
@@ -121,20 +124,25 @@ def route_experts(h, w_router, bias, top: int, experts: ExpertWeights) -> Routin
     tile_info, ids, slot, row_token = ints.split(sizes)
     ids, slot = ids.view(T, top), slot.view(T, top)
     weights = torch.empty(T, top, dtype=torch.float32, device=dev)
-    hybrid_native().route(ids, weights, slot, row_token, tile_info, z, bias, rows)
+    hybrid_native().route(ids, weights, slot, row_token, tile_info, z, bias, scale, rows)
     return Routing(slot, weights, ids, row_token, tile_info, rows)
 
 
-def expert_rows(h, routing: Routing, w: ExpertWeights, limit: float) -> torch.Tensor:
-    """The chosen experts' outputs, a row each at routing.slot."""
+def expert_rows(
+    h, routing: Routing, w: ExpertWeights, limit: Optional[float]
+) -> torch.Tensor:
+    """The chosen experts' outputs, a row each at routing.slot; ``limit``: of
+    the clamped GLU, None for silu(gate) * up."""
     if not h.is_cuda:
         return ref.expert_rows(h, routing.ids, w.gate_up, w.down, limit)
     R, ext = routing.row_token.numel(), hybrid_native()
     act = torch.empty(R, w.ff, dtype=h.dtype, device=h.device)
     out = torch.empty(R, w.width, dtype=h.dtype, device=h.device)
     where = (routing.row_token, routing.tile_info, routing.tile_rows)
-    ext.expert_product(act, h, w.gate_up, *where, True, float(limit))
-    ext.expert_product(out, act, w.down, *where, False, 0.0)
+    ext.expert_product(
+        act, h, w.gate_up, *where, 2 if limit is None else 1, float(limit or 0.0)
+    )
+    ext.expert_product(out, act, w.down, *where, 0, 0.0)
     return out
 
 

@@ -8,8 +8,8 @@ takes any split of a sequence into segments.
 
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Optional, Tuple
+from dataclasses import dataclass, field
+from typing import Dict, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
@@ -57,18 +57,22 @@ class Tiles:
 
 @dataclass
 class SegmentPlan:
-    """How a step's rows go through the kernels; made once per step."""
+    """How a step's rows go through the kernels; made once per step.
+    ``carry``: rows that one layer leaves for later layers of the step."""
 
     unfold: Optional[Unfold] = None
     chunks: Optional[Chunks] = None
     tiles: Optional[Tiles] = None
+    head_tiles: Optional[Tiles] = None
+    carry: Dict[str, torch.Tensor] = field(default_factory=dict)
 
 
 CHUNK = 64            # rows per chunk of the chunked recurrences
 CHUNK_MIN_ROWS = 32   # shorter segments run token by token
 UNFOLD_RATIO = 16     # query-key pairs per key from which unfolding pays
 TILE_MIN_ROWS = 16    # shorter segments attend row by row
-PLANS = ("unfold", "chunks", "tiles")
+HEAD_TILE = 16        # query rows per tile where a tile holds all heads
+PLANS = ("unfold", "chunks", "tiles", "head_tiles")
 
 
 def plan_segments(batch, dtype, parts_of=PLANS) -> SegmentPlan:
@@ -92,7 +96,13 @@ def plan_segments(batch, dtype, parts_of=PLANS) -> SegmentPlan:
     keys = int((pl + ps).sum())
     pairs = float((pl * (ps + pl / 2.0)).sum())
     unfold = "unfold" in parts_of and nseg_p > 0 and pairs >= UNFOLD_RATIO * keys
-    tiled = np.nonzero(lens >= TILE_MIN_ROWS)[0] if "tiles" in parts_of else []
+    tiled = np.nonzero(lens >= TILE_MIN_ROWS)[0]
+    kinds = {}  # name of the tiled form -> rows per tile
+    if len(tiled):
+        if "tiles" in parts_of:
+            kinds["tiles"] = 128 if int(lens[tiled].max()) > 64 else 64
+        if "head_tiles" in parts_of:
+            kinds["head_tiles"] = HEAD_TILE
     if unfold:
         put("cu_q", np.concatenate([[0], np.cumsum(pl)]))
         put("cu_k", np.concatenate([[0], np.cumsum(pl + ps)]))
@@ -102,15 +112,17 @@ def plan_segments(batch, dtype, parts_of=PLANS) -> SegmentPlan:
         order = np.argsort(-(ps[seg] + off), kind="stable")  # longest first
         put("tile_seg", seg[order])
         put("tile_off", off[order])
-    if len(tiled):
+    for name, rows_t in kinds.items():
         n = lens[tiled]
-        rows_t = 128 if int(n.max()) > 64 else 64
         seg = np.repeat(tiled, -(-n // rows_t))
         off = np.concatenate([np.arange(0, k, rows_t) for k in n])
-        order = np.argsort(-(starts[seg] + off), kind="stable")  # longest first
-        put("at_seg", seg[order])
-        put("at_off", off[order])
-        put("at_rest", np.nonzero(np.repeat(lens < TILE_MIN_ROWS, lens))[0])
+        if name == "tiles":
+            order = np.argsort(-(starts[seg] + off), kind="stable")  # longest first
+            seg, off = seg[order], off[order]
+        put(name + "_seg", seg)
+        put(name + "_off", off)
+    if kinds:
+        put("tile_rest", np.nonzero(np.repeat(lens < TILE_MIN_ROWS, lens))[0])
     long = np.nonzero(lens >= CHUNK_MIN_ROWS)[0] if "chunks" in parts_of else np.empty(0, int)
     nchunk = (lens[long] + CHUNK - 1) // CHUNK
     if len(long):
@@ -141,11 +153,11 @@ def plan_segments(batch, dtype, parts_of=PLANS) -> SegmentPlan:
             tile_seg=got["tile_seg"], tile_off=got["tile_off"],
             tile_rows=tile_rows,
         )
-    if len(tiled):
-        plan.tiles = Tiles(
-            tile_seg=got["at_seg"], tile_off=got["at_off"], tile_rows=rows_t,
-            rest=got["at_rest"] if got["at_rest"].numel() else None,
-        )
+    for name, rows_t in kinds.items():
+        setattr(plan, name, Tiles(
+            tile_seg=got[name + "_seg"], tile_off=got[name + "_off"], tile_rows=rows_t,
+            rest=got["tile_rest"] if got["tile_rest"].numel() else None,
+        ))
     if len(long):
         plan.chunks = Chunks(
             maps=tuple(got[k] for k in ("segs", "first", "chunk_seg", "chunk_off")),
@@ -182,6 +194,27 @@ def add_layernorm(x, delta, w, b, eps: float, dtype, vec=None, replace: bool = F
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
     hybrid_native().add_layernorm(out, x, delta, vec, w, b, float(eps), replace)
     return out
+
+
+def add_rms_norm(x, deltas: Sequence, weights: Sequence[torch.Tensor], eps: float, dtype):
+    """x (fp32 stream, in place) += every one of deltas: at most one tensor
+    and one ExpertSum, or two tensors; returns, for each of one or two norm
+    weights, RMS norm(x) * weight in ``dtype``."""
+    if not x.is_cuda:
+        return ref.add_rms_norm(x, deltas, weights, eps, dtype)
+    outs = tuple(torch.empty(x.shape, dtype=dtype, device=x.device) for _ in weights)
+    parts = [d for d in deltas if not isinstance(d, ExpertSum)]
+    sums = [d for d in deltas if isinstance(d, ExpertSum)]
+    assert len(outs) in (1, 2) and len(parts) <= 2 and len(sums) <= (1 if len(parts) < 2 else 0)
+    e = sums[0] if sums else None
+    if e is not None and e.shared is not None:
+        raise NotImplementedError("RMS norm after experts with a shared one")
+    hybrid_native().add_rms_norm(
+        outs[0], outs[1] if len(outs) > 1 else None, x, *(parts + [None, None])[:2],
+        *((e.rows, e.slot, e.weights) if e is not None else (None, None, None)),
+        weights[0], weights[1] if len(outs) > 1 else None, float(eps),
+    )
+    return outs
 
 
 def add_cast(x, delta, out) -> None:
@@ -442,6 +475,82 @@ def paged_attention(out, q, k_pages, v_pages, H: int, G: int, sink, scale: float
         if nsplit > 1:
             pa, pm = _folded_scratch(q.device, n * H * nsplit * vdim, n * H * nsplit * 2)
     ext.paged_rows(*head, segs.row_seg, segs.tables, rows, nsplit, pa, pm)
+
+
+# ------------------------------- sigmoid attention over pages, mixed heads
+def distance_bias(rel: torch.Tensor, pb: torch.Tensor, bias_max: float, window: int):
+    """fp32 [distances, heads padded to 16]: rel[bucket(n), h] + pb[h] for
+    distances n = 0, 1, ...; the last row also serves all larger ones. rel
+    [B, H] has a row per distance below B/2, then rows of logarithmically
+    growing width up to distance bias_max, beyond which all share the last."""
+    B, H = rel.shape
+    half = B // 2
+    last = min(int(np.ceil(bias_max)), window - 1)
+    n = np.arange(last + 1)
+    # (the nudge: where the logarithms' ratio is an integer, rounding must
+    # not take the floor below it)
+    log = np.log(np.maximum(n, half) / half) / np.log(bias_max / half) * (B - half) + 1e-9
+    row = np.where(n < half, n, np.minimum(B - 1, half + np.floor(log).astype(np.int64)))
+    out = torch.zeros(last + 1, -(-H // 16) * 16, dtype=torch.float32, device=rel.device)
+    out[:, :H] = rel.float()[torch.from_numpy(row).to(rel.device)] + pb.float()
+    return out
+
+
+def qkv_rows(q, k, v, q_norm, k_norm, eps: float, blend: float, v_first, k_pages, v_pages,
+             slot_mapping) -> torch.Tensor:
+    """RMS norm over a whole row of q (returned) and of k; keys and values,
+    blended to (1 - blend) v + blend v_first where v_first is given, go to
+    their cache slots. q, k, v, v_first may be strided."""
+    if not q.is_cuda:
+        return ref.qkv_rows(q, k, v, q_norm, k_norm, eps, blend, v_first, k_pages, v_pages,
+                            slot_mapping)
+    out = torch.empty(q.shape, dtype=q.dtype, device=q.device)
+    hybrid_native().qkv_rows(
+        out, q, k, v, q_norm, k_norm, float(eps), float(blend), v_first, k_pages, v_pages,
+        slot_mapping,
+    )
+    return out
+
+
+def sigmoid_attention(out, q, k_pages, v_pages, H: int, G: int, scale: float, bias, talk,
+                      window: int, gate, positions, segs, plan: SegmentPlan) -> None:
+    """Every row's attention to the last ``window`` rows of its sequence's
+    pages (its own token among them). Weights sigmoid(scale q.k +
+    bias[distance]) (bias: distance_bias) are not normalized; head h takes
+    sum_g talk[h, g] of all heads' weights to the values of its key head. out
+    [T, H*vdim] is multiplied by sigmoid(gate) element by element. q, gate
+    and out may be strided."""
+    if not q.is_cuda:
+        return ref.sigmoid_attention(
+            out, q, k_pages, v_pages, H, G, scale, bias, talk, window, gate, positions, segs
+        )
+    ext = hybrid_native()
+    page, dim, vdim = k_pages.shape[1], k_pages.shape[2] // G, v_pages.shape[2] // G
+    head = (out, q, k_pages, v_pages, H, G, float(scale), bias, talk, int(window), gate,
+            positions)
+    mfma = (
+        q.dtype == torch.bfloat16 and page >= 16 and page & (page - 1) == 0 and H <= 64
+        and dim % 8 == 0 and vdim % 8 == 0 and dim <= 256 and vdim <= 256
+    )
+    rows, n = None, q.shape[0]
+    per_wave = -(-H // 8)  # a tile's 8 waves share the heads, no wave has two key heads
+    if (
+        mfma and plan.head_tiles is not None and per_wave <= 4 and H // G % per_wave == 0
+        and dim <= 128 and vdim <= 128
+    ):
+        t = plan.head_tiles
+        ext.sigmoid_tiles(*head, segs.tables, segs.cu, t.tile_seg, t.tile_off)
+        if t.rest is None:
+            return
+        rows, n = t.rest, t.rest.numel()
+    nsplit, part = 0, None
+    if mfma:
+        # fill the chip: splits only from shapes, so captured graphs hold
+        most = -(-min(segs.tables.shape[1] * page, window + 31) // 128)
+        nsplit = max(1, min(-(-512 // n), 16, most))
+        if nsplit > 1:
+            part, _ = _folded_scratch(q.device, n * H * nsplit * vdim, 0)
+    ext.sigmoid_rows(*head, segs.row_seg, segs.tables, rows, nsplit, part)
 
 
 # -------------------------------------- recurrences with a decay per channel

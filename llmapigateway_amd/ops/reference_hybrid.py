@@ -228,6 +228,43 @@ def paged_attention(out, q, k_pages, v_pages, H, G, sink, scale, cap, gate, out_
         out[t] = (o * (torch.sigmoid(gate[t].float()) * out_scale)[:, None]).view(-1)
 
 
+# ------------------------------- sigmoid attention over pages, mixed heads
+def add_rms_norm(x, deltas, weights, eps, dtype):
+    for d in deltas:
+        x.add_(d.float())
+    unit = _rms(x, eps)
+    return tuple((unit * w).to(dtype) for w in weights)
+
+
+def qkv_rows(q, k, v, q_norm, k_norm, eps, blend, v_first, k_pages, v_pages, slot_mapping):
+    vf = v.float()
+    if v_first is not None:
+        vf = (1.0 - blend) * vf + blend * v_first.float()
+    page_write(
+        (_rms(k.float(), eps) * k_norm).to(k.dtype), vf.to(v.dtype), k_pages, v_pages,
+        slot_mapping,
+    )
+    return (_rms(q.float(), eps) * q_norm).to(q.dtype)
+
+
+def sigmoid_attention(out, q, k_pages, v_pages, H, G, scale, bias, talk, window, gate,
+                      positions, segs):
+    T, bs = q.shape[0], k_pages.shape[1]
+    dim, vdim = k_pages.shape[2] // G, v_pages.shape[2] // G
+    for t in range(T):
+        p = int(positions[t])
+        lo = max(0, p - window + 1)
+        keys = torch.arange(lo, p + 1)
+        slots = segs.tables[int(segs.row_seg[t])].long()[keys // bs] * bs + keys % bs
+        k = k_pages.view(-1, G, dim)[slots].float().repeat_interleave(H // G, 1)
+        v = v_pages.view(-1, G, vdim)[slots].float().repeat_interleave(H // G, 1)
+        s = torch.einsum("hd,nhd->hn", q[t].float().view(H, dim), k) * scale
+        s = s + bias[(p - keys).clamp(max=bias.shape[0] - 1), :H].t()
+        w = talk.float() @ torch.sigmoid(s)
+        o = torch.einsum("hn,nhd->hd", w, v)
+        out[t] = o.reshape(-1) * torch.sigmoid(gate[t].float())
+
+
 # ------------------------------------- recurrences with a decay per channel
 def decay_logs(a, w2, bias, kind, tau):
     a = torch.tanh(a.float()) if kind == "exp" else a.float()
@@ -293,13 +330,19 @@ def clamped_glu(x, limit):
 
 
 def expert_rows(h, ids, gate_up, down, limit):
-    """[T * top, width]: row t * top + j is expert ids[t, j] on row t."""
+    """[T * top, width]: row t * top + j is expert ids[t, j] on row t.
+    limit None: silu(gate) * up."""
     T, top = ids.shape
     out = torch.empty(T * top, down.shape[1], dtype=h.dtype)
     flat = ids.reshape(-1)
     for e in flat.unique().tolist():
         rows = torch.nonzero(flat == e).view(-1)
-        act = clamped_glu(F.linear(h[rows // top], gate_up[e]), limit)
+        both = F.linear(h[rows // top], gate_up[e])
+        if limit is None:
+            g, u = both.float().chunk(2, -1)
+            act = (F.silu(g) * u).to(both.dtype)
+        else:
+            act = clamped_glu(both, limit)
         out[rows] = F.linear(act, down[e])
     return out
 
