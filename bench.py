@@ -64,7 +64,7 @@ def parse_args():
         "width, feed-forward (of experts: what a token uses) and number of "
         "layer runs",
     )
-    p.add_argument("--family", default="lelisun", choices=["lelisun", "filinex"],
+    p.add_argument("--family", default="lelisun", choices=["lelisun", "filinex", "mekevik"],
                    help="--mode layers: whose presets")
     p.add_argument("--sizes", default="small,base",
                    help="--mode layers: <family>-<size> presets, or any hybrid model")
@@ -210,7 +210,7 @@ def run_layers(args) -> None:
     def llama_like(c):
         m = next(e.mlp for e in c.layers if e.mlp)
         ff = m["ff"] if m["kind"] == "dense" else (
-            m["router"]["top"] * m["expert"]["ff"] + m["shared"]["ff"])
+            m["router"]["top"] * m["expert"]["ff"] + m.get("shared", {}).get("ff", 0))
         heads = c.hidden_size // 128 or 1
         return ModelConfig(
             name=f"llama of {c.name}", hidden_size=c.hidden_size, intermediate_size=ff,

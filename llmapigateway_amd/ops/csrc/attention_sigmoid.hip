@@ -133,6 +133,10 @@ __device__ __forceinline__ bf16x8 masked(bool keep, const bf16x8& f) {
     return as_frag(v);
 }
 
+// columns past a row's end are read from its start: of keys they meet zeros of
+// the query, of values they make outputs that nobody stores
+__device__ __forceinline__ uint32_t col_of(int c, int width) { return c < width ? c : 0; }
+
 // ---------------------------------------------------------------------------
 // Rows: one workgroup per (row, split of the keys); its 4 waves take 32 keys
 // of all key heads in turn. A chain of products in which every result is the
@@ -143,40 +147,47 @@ __device__ __forceinline__ bf16x8 masked(bool keep, const bf16x8& f) {
 //     (4g + r of two fragments of 16) are the k order of the operand
 //   O^T [value, head] += V^T M^T, M^T zeroed like Q; key order as in
 //     attention_paged.hip
-// Keys go from global memory into the fragments, values through the wave's
-// LDS tile. The waves' shares meet in LDS; several splits leave partial sums
-// for sigmoid_combine_kernel.
+// Keys, then values of 32 tokens and one key head at a time come by transfers
+// through a ring of LDS buffers of the wave's own, RING - 1 ahead, 16-byte
+// chunks (of values: pairs of them) XOR-swizzled by row on the source address.
+// The waves' shares meet in LDS; several splits leave partial sums for
+// sigmoid_combine_kernel.
 // ---------------------------------------------------------------------------
 template <int NB, int NDQ, int NDV>  // blocks of 16 heads; dim/32, vdim/16
 __launch_bounds__(SA_THREADS)
 __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, float* part) {
-    constexpr int LDV = NDV * 16 + 8, TILE = 32 * LDV, NK = (NB + 1) / 2;
-    __shared__ __align__(16) bf16 v_lds[4][TILE];
+    static_assert(NDV == 2 * NDQ, "rows of keys and values have one length in LDS");
+    constexpr int LD = NDV * 16, CH = LD / 8, PER = 64 / CH;  // values, chunks; rows a transfer
+    constexpr int RING = NDQ > 4 ? 2 : 4, AHEAD = (RING - 1) * (32 / PER);
+    constexpr int NK = (NB + 1) / 2;
+    __shared__ __align__(16) bf16 ring[4][RING][32 * LD];
     const size_t t = a.rows ? a.rows[blockIdx.x] : blockIdx.x;
     const int split = blockIdx.y, per = a.H / a.G;
     const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int pos = (int)a.positions[t];
+    const int pos = __builtin_amdgcn_readfirstlane((int)a.positions[t]);
     const int first = max(0, pos - a.window + 1), base = first & ~31;
     const int span = (pos + 1 - base + nsplit * 128 - 1) / (nsplit * 128) * 128;
     const int key_lo = base + split * span, key_hi = min(pos + 1, key_lo + span);
     const int* bt = a.tables + (size_t)a.row_seg[t] * a.max_blocks;
-    const int mask = (1 << page_shift) - 1;
-    const float scale2 = a.scale * LOG2E;
+    const int mask = (1 << page_shift) - 1, last = pos;
+    const float scale2 = -a.scale * LOG2E;
+    // this wave's steps of 32 keys: k_first, k_first + 128, ...
+    const int k_first = key_lo + wave * 32;
+    const int steps = k_first < key_hi ? (key_hi - k_first + 127) / 128 : 0;
 
     int key_head[NB];  // of this lane's head in each block
     bf16x8 qf[NB][NDQ], tf[NB][NK];
+    f32x4 far[NB];     // biases beyond the table, of heads 16b + 4g + r
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
         const int h = b * 16 + r16;
         key_head[b] = h < a.H ? h / per : -1;
         const bf16* qr = (const bf16*)a.q + t * a.ldq + (size_t)min(h, a.H - 1) * a.dim;
 #pragma unroll
-        for (int c = 0; c < NDQ; ++c) {
-            uint4 x = {0, 0, 0, 0};
-            if (c * 32 + g * 8 < a.dim) x = *reinterpret_cast<const uint4*>(qr + c * 32 + g * 8);
-            qf[b][c] = as_frag(x);
-        }
+        for (int c = 0; c < NDQ; ++c)
+            qf[b][c] = masked(c * 32 + g * 8 < a.dim, *reinterpret_cast<const bf16x8*>(
+                                                          qr + col_of(c * 32 + g * 8, a.dim)));
 #pragma unroll
         for (int kb = 0; kb < NK; ++kb) {
             uint16_t x[8];
@@ -189,6 +200,8 @@ __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, f
             }
             tf[b][kb] = *reinterpret_cast<const bf16x8*>(x);
         }
+        far[b] = *reinterpret_cast<const f32x4*>(a.bias + (size_t)(a.nbias - 1) * a.Hp +
+                                                 min(b * 16, a.Hp - 16) + g * 4);
     }
     f32x4 acc[NB][NDV];
 #pragma unroll
@@ -196,56 +209,72 @@ __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, f
 #pragma unroll
         for (int j = 0; j < NDV; ++j) acc[b][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
 
-    // rows of 16 keys from k0 in the pages; past the end any row that is there
-    const int last = pos;
-    auto page_row = [&](int k0) {
-        return (size_t)bt[min(k0, last) >> page_shift] << page_shift;
+    // pages of 32 steps, two a step (past the end: of the last key)
+    int pages = 0;
+    auto load_pages = [&](int step) {
+        const int k = k_first + (step + (lane >> 1)) * 128 + (lane & 1) * 16;
+        pages = bt[min(k, last) >> page_shift];
     };
-    auto load_k = [&](size_t b0, size_t b1, int k0, int gk, uint4* kreg) {
+    // the next transfers: step, key head (G and up: values), ring buffer
+    int p_step = 0, p_head = 0, p_buf = 0;
+    auto issue = [&] {
+        if (p_step >= steps) return false;
+        if (p_head == 0 && (p_step & 31) == 0) load_pages(p_step);
+        const bool is_v = p_head >= a.G;
+        const int width = is_v ? a.vdim : a.dim, ld = a.G * width;
+        const bf16* src = is_v ? (const bf16*)a.v + (size_t)(p_head - a.G) * a.vdim
+                               : (const bf16*)a.k + (size_t)p_head * a.dim;
+        const int k0 = k_first + p_step * 128, at = (p_step & 31) * 2;
+        const bf16* b0 =
+            src + ((size_t)__builtin_amdgcn_readlane(pages, at) << page_shift) * ld;
+        const bf16* b1 =
+            src + ((size_t)__builtin_amdgcn_readlane(pages, at + 1) << page_shift) * ld;
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            const int key = min(k0 + u * 16 + r16, last);
-            const size_t row = (u && k0 + 16 <= last ? b1 : b0) + (key & mask);
-            const bf16* p = (const bf16*)a.k + (row * a.G + gk) * a.dim;
-#pragma unroll
-            for (int c = 0; c < NDQ; ++c) {
-                kreg[u * NDQ + c] = (uint4){0, 0, 0, 0};
-                if (c * 32 + g * 8 < a.dim)
-                    kreg[u * NDQ + c] = *reinterpret_cast<const uint4*>(p + c * 32 + g * 8);
-            }
-        }
-    };
-    auto load_v = [&](size_t b0, size_t b1, int k0, int gk, uint4* vreg) {
-#pragma unroll
-        for (int u = 0; u < NDV; ++u) {
-            const int e = lane + u * 64, o = e / (NDV * 2), d = e % (NDV * 2) * 8;
+        for (int u = 0; u < 32 / PER; ++u) {
+            const int o = u * PER + lane / CH, c = lane % CH;
+            const int col = (is_v ? c ^ ((o & (NDV - 1) & 7) << 1) : c ^ (o & (CH - 1))) * 8;
             const int key = min(k0 + o, last);
-            const size_t row = (key >= k0 + 16 ? b1 : b0) + (key & mask);
-            vreg[u] = (uint4){0, 0, 0, 0};
-            if (d < a.vdim)
-                vreg[u] = *reinterpret_cast<const uint4*>(
-                    (const bf16*)a.v + (row * a.G + gk) * a.vdim + d);
+            // (past the last key its own page: that of the first half, or both are one)
+            const bf16* page = u * PER >= 16 && k0 + 16 <= last ? b1 : b0;
+            dma16(page + (uint32_t)((key & mask) * ld + col_of(col, width)),
+                  ring[wave][p_buf] + u * 512);
         }
+        p_buf = (p_buf + 1) % RING;
+        if (++p_head == 2 * a.G) {
+            p_head = 0;
+            ++p_step;
+        }
+        return true;
     };
-    bf16* vt = v_lds[wave];
-    uint4 kreg[2 * NDQ], vreg[NDV];
-    int k0 = key_lo + wave * 32;
-    size_t b0 = 0, b1 = 0;
-    if (k0 < key_hi) {
-        b0 = page_row(k0);
-        b1 = page_row(k0 + 16);
-        load_k(b0, b1, k0, 0, kreg);
-    }
-    for (; k0 < key_hi; k0 += 128) {
+    int buf = 0;
+    // starts a transfer into the buffer that was read last; the next buffer to
+    // read, once its transfer has landed
+    auto next_buffer = [&] {
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        if (issue()) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(AHEAD) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        const bf16* p = ring[wave][buf];
+        buf = (buf + 1) % RING;
+        return p;
+    };
+#pragma unroll
+    for (int i = 0; i < RING - 1; ++i) issue();
+
+    for (int step = 0; step < steps; ++step) {
+        const int k0 = k_first + step * 128;
         f32x4 s[NB][2];
 #pragma unroll
         for (int b = 0; b < NB; ++b) s[b][0] = s[b][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
         for (int gk = 0; gk < a.G; ++gk) {
-            uint4 kf[2 * NDQ];
+            const bf16* kt = next_buffer();
+            bf16x8 kf[2][NDQ];
 #pragma unroll
-            for (int i = 0; i < 2 * NDQ; ++i) kf[i] = kreg[i];
-            if (gk + 1 < a.G) load_k(b0, b1, k0, gk + 1, kreg);
-            else load_v(b0, b1, k0, 0, vreg);
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int c = 0; c < NDQ; ++c)
+                    kf[u][c] = *reinterpret_cast<const bf16x8*>(
+                        kt + (u * 16 + r16) * LD +
+                        (((c * 4 + g) ^ ((u * 16 + r16) & (CH - 1))) << 3));
 #pragma unroll
             for (int b = 0; b < NB; ++b) {
                 if (gk * per >= b * 16 + 16 || (gk + 1) * per <= b * 16) continue;
@@ -254,83 +283,73 @@ __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, f
                 for (int c = 0; c < NDQ; ++c) {
                     const bf16x8 qm = masked(mine, qf[b][c]);
 #pragma unroll
-                    for (int u = 0; u < 2; ++u)
-                        s[b][u] = mfma16(qm, as_frag(kf[u * NDQ + c]), s[b][u]);
+                    for (int u = 0; u < 2; ++u) s[b][u] = mfma16(qm, kf[u][c], s[b][u]);
                 }
             }
         }
         // weights of heads 16b + 4g + r, keys k0 + 16u + r16; their mix
-        bf16x8 pf[NB];
-        {
-            f32x4 m[NB][2];
+        const bool near = pos - (k0 + 31) < a.nbias - 1;
+        f32x4 m[NB][2];
 #pragma unroll
-            for (int u = 0; u < 2; ++u) {
-                const int key = k0 + u * 16 + r16, dist = pos - key;
-                const bool seen = key >= first && key < key_hi;
-                const float* br = a.bias + (size_t)max(0, min(dist, a.nbias - 1)) * a.Hp + g * 4;
-                bf16x8 hi[NK], lo[NK];
+        for (int u = 0; u < 2; ++u) {
+            const int key = k0 + u * 16 + r16;
+            const bool seen = key >= first && key < key_hi;
+            f32x4 bias[NB];
 #pragma unroll
-                for (int kb = 0; kb < NK; ++kb) {
-                    float w[8];
+            for (int b = 0; b < NB; ++b) bias[b] = far[b];
+            if (near) {
+                const float* br = a.bias +
+                                  (size_t)max(0, min(pos - key, a.nbias - 1)) * a.Hp + g * 4;
 #pragma unroll
-                    for (int half = 0; half < 2; ++half) {
-                        const int b = kb * 2 + half;
-                        if (b < NB && b * 16 < a.Hp) {
-                            const float4 bb = *reinterpret_cast<const float4*>(br + b * 16);
-                            const float bv[4] = {bb.x, bb.y, bb.z, bb.w};
+                for (int b = 0; b < NB; ++b)
+                    bias[b] = *reinterpret_cast<const f32x4*>(br + min(b * 16, a.Hp - 16));
+            }
+            bf16x8 hi[NK], lo[NK];
 #pragma unroll
-                            for (int r = 0; r < 4; ++r)
-                                w[half * 4 + r] =
-                                    seen ? sigmoid_2(fmaf(s[b < NB ? b : 0][u][r], scale2,
-                                                          bv[r] * LOG2E))
-                                         : 0.f;
-                        } else {
+            for (int kb = 0; kb < NK; ++kb) {
+                float w[8];
 #pragma unroll
-                            for (int r = 0; r < 4; ++r) w[half * 4 + r] = 0.f;
-                        }
-                    }
-                    split_frag(w, hi[kb], lo[kb]);
+                for (int j = 0; j < 8; ++j) {
+                    const int b = kb * 2 + j / 4, r = j % 4;
+                    w[j] = b < NB && seen
+                               ? __builtin_amdgcn_rcpf(
+                                     1.f + __builtin_amdgcn_exp2f(
+                                               fmaf(s[b < NB ? b : 0][u][r], scale2,
+                                                    bias[b < NB ? b : 0][r] * -LOG2E)))
+                               : 0.f;
                 }
-#pragma unroll
-                for (int b = 0; b < NB; ++b) {
-                    m[b][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                    for (int kb = 0; kb < NK; ++kb) {
-                        m[b][u] = mfma16(hi[kb], tf[b][kb], m[b][u]);
-                        m[b][u] = mfma16(lo[kb], tf[b][kb], m[b][u]);
-                    }
-                }
+                split_frag(w, hi[kb], lo[kb]);
             }
 #pragma unroll
             for (int b = 0; b < NB; ++b) {
-                uint4 v;
-                v.x = cvt_pk_bf16(m[b][0][0], m[b][0][1]);
-                v.y = cvt_pk_bf16(m[b][0][2], m[b][0][3]);
-                v.z = cvt_pk_bf16(m[b][1][0], m[b][1][1]);
-                v.w = cvt_pk_bf16(m[b][1][2], m[b][1][3]);
-                pf[b] = as_frag(v);
-            }
-        }
-        const size_t c0 = b0, c1 = b1;  // this tile's pages
-        if (k0 + 128 < key_hi) {
-            b0 = page_row(k0 + 128);
-            b1 = page_row(k0 + 144);
-        }
-        const bf16* r0 = vt + (g * 4 + (r16 >> 2)) * LDV + (r16 & 3) * 4;
-        for (int gk = 0; gk < a.G; ++gk) {
+                m[b][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int u = 0; u < NDV; ++u) {
-                const int e = lane + u * 64;
-                *reinterpret_cast<uint4*>(vt + e / (NDV * 2) * LDV + e % (NDV * 2) * 8) = vreg[u];
+                for (int kb = 0; kb < NK; ++kb) {
+                    m[b][u] = mfma16(hi[kb], tf[b][kb], m[b][u]);
+                    m[b][u] = mfma16(lo[kb], tf[b][kb], m[b][u]);
+                }
             }
-            if (gk + 1 < a.G) load_v(c0, c1, k0, gk + 1, vreg);
-            else if (k0 + 128 < key_hi) load_k(b0, b1, k0 + 128, 0, kreg);
+        }
+        bf16x8 pf[NB];
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            uint4 v;
+            v.x = cvt_pk_bf16(m[b][0][0], m[b][0][1]);
+            v.y = cvt_pk_bf16(m[b][0][2], m[b][0][3]);
+            v.z = cvt_pk_bf16(m[b][1][0], m[b][1][1]);
+            v.w = cvt_pk_bf16(m[b][1][2], m[b][1][3]);
+            pf[b] = as_frag(v);
+        }
+        const int vr = g * 4 + (r16 >> 2), sw = vr & (NDV - 1) & 7;
+        for (int gk = 0; gk < a.G; ++gk) {
+            const bf16* r0 = next_buffer() + vr * LD + (r16 & 3) * 4;
             bf16x8 pm[NB];
 #pragma unroll
             for (int b = 0; b < NB; ++b) pm[b] = masked(key_head[b] == gk, pf[b]);
 #pragma unroll
             for (int j = 0; j < NDV; ++j) {
-                const bf16x8 vf = tr_pair(r0 + j * 16, r0 + 16 * LDV + j * 16);
+                const bf16* p = r0 + ((j ^ sw) << 4);
+                const bf16x8 vf = tr_pair(p, p + 16 * LD);
 #pragma unroll
                 for (int b = 0; b < NB; ++b) {
                     if (gk * per >= b * 16 + 16 || (gk + 1) * per <= b * 16) continue;
@@ -340,7 +359,7 @@ __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, f
         }
     }
     // the waves' shares, 16 heads at a time: [vdim][16 heads] in each wave's tile
-    float* sh = reinterpret_cast<float*>(vt);
+    float* sh = reinterpret_cast<float*>(ring[wave][0]);
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
         if (b > 0) __syncthreads();
@@ -354,7 +373,7 @@ __global__ void sigmoid_rows_kernel(SigmoidArgs a, int page_shift, int nsplit, f
             if (h >= a.H) break;
             float o = 0.f;
 #pragma unroll
-            for (int w = 0; w < 4; ++w) o += reinterpret_cast<const float*>(v_lds[w])[d * 16 + c];
+            for (int w = 0; w < 4; ++w) o += reinterpret_cast<const float*>(ring[w][0])[d * 16 + c];
             const int at = h * a.vdim + d;
             if (nsplit == 1)
                 stf((bf16*)a.out + t * a.ld_out + at,
@@ -392,9 +411,12 @@ __global__ void sigmoid_combine_kernel(SigmoidArgs a, int nsplit, const float* _
 //   mix: each wave two rows, M^T [key, head] = W^T talk^T; back to LDS in
 //     place of the weights, by row: [head][32 keys]
 //   O^T [value, row] += V^T M^T of the wave's heads
-// Keys go into the fragments, 32 ahead; values by transfers into the wave's
+// Keys go into the fragments, a step ahead; values by transfers into the wave's
 // own LDS tile, 32-byte pairs of chunks XOR-swizzled by row on the source
 // address. 16-byte chunks of weights are swizzled likewise.
+//
+// Queries and sums of 4 heads of 128 take 192 of a lane's 256 registers: the
+// steps are kept apart (sched_barrier) so that their temporaries are, too.
 // ---------------------------------------------------------------------------
 template <int HW, int NDQ, int NDV>
 __launch_bounds__(512)
@@ -403,8 +425,12 @@ __global__ void sigmoid_tiles_kernel(
     const int* __restrict__ tile_seg, const int* __restrict__ tile_off, int ntiles) {
     constexpr int LDW = 32 * 32 + 8;  // a row's weights
     constexpr int LDB = 36;           // biases of a distance
-    __shared__ __align__(16) bf16 w_lds[2][16][LDW], v_lds[8][32 * NDV * 16];
+    constexpr bool FULL = HW * (NDQ + NDV) > 36;
+    __shared__ __align__(16) bf16 w_lds[2][16][LDW], v_lds[8][32 * NDV * 16], t_lds[2][64 * 8];
     __shared__ __align__(16) float b_lds[47][LDB];
+    // the last fragments of some heads' queries, where registers do not hold all
+    constexpr int QL = FULL ? 2 : 0;
+    __shared__ __align__(16) bf16 q_lds[8][QL > 0 ? QL : 1][64 * 8];
     // each XCD (8, round robin) takes a contiguous part of the tiles, whose
     // windows overlap
     const int share = (ntiles + 7) / 8;
@@ -415,18 +441,36 @@ __global__ void sigmoid_tiles_kernel(
     const int pos0 = (int)a.positions[q0];  // of the tile's first row
     const int* bt = a.tables + (size_t)seg * a.max_blocks;
     const int mask = (1 << page_shift) - 1;
-    const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    int lane = tid & 63, r16 = lane & 15, g = lane >> 4;
+    // what addresses are made of, made anew in every step: kept from one step
+    // to the next they would fill the registers
+    auto fresh_lane = [&] {
+        lane = threadIdx.x & 63;
+        asm volatile("" : "+v"(lane));
+        r16 = lane & 15;
+        g = lane >> 4;
+    };
     const int h0 = wave * HW;
     const bool active = h0 < a.H;
     const int gk = active ? h0 / (a.H / a.G) : 0;
-    const float scale2 = a.scale * LOG2E;
+    const float scale2 = -a.scale * LOG2E;
     const bf16 *kp = (const bf16*)a.k + (size_t)gk * a.dim;
     const bf16 *vp = (const bf16*)a.v + (size_t)gk * a.vdim;
+    const int ldk = a.G * a.dim, ldv = a.G * a.vdim;
     const int key_end = pos0 + nq, key_lo = max(0, pos0 - a.window + 1) & ~31;
 
     for (int e = tid; e < 2 * 16 * LDW / 8; e += 512)  // heads that are not there: finite
         reinterpret_cast<uint4*>(w_lds)[e] = (uint4){0, 0, 0, 0};
+    if (wave < 2) {  // talk^T as fragments: column = head 16b + r16, k = head 8g + j
+        const int h = wave * 16 + r16;
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            reinterpret_cast<uint16_t*>(t_lds[wave])[lane * 8 + j] =
+                h < a.H && g * 8 + j < a.H
+                    ? reinterpret_cast<const uint16_t*>(a.talk)[(size_t)h * a.H + g * 8 + j]
+                    : 0;
+    }
     bf16x8 qf[HW][NDQ];
     if (active) {
 #pragma unroll
@@ -435,24 +479,13 @@ __global__ void sigmoid_tiles_kernel(
                              (size_t)(h0 + i) * a.dim;
 #pragma unroll
             for (int c = 0; c < NDQ; ++c) {
-                uint4 x = {0, 0, 0, 0};
-                if (c * 32 + g * 8 < a.dim)
-                    x = *reinterpret_cast<const uint4*>(qr + c * 32 + g * 8);
-                qf[i][c] = as_frag(x);
+                qf[i][c] =
+                    masked(c * 32 + g * 8 < a.dim, *reinterpret_cast<const bf16x8*>(
+                                                       qr + col_of(c * 32 + g * 8, a.dim)));
+                if (i < QL && c == NDQ - 1)
+                    *reinterpret_cast<bf16x8*>(q_lds[wave][i < QL ? i : 0] + lane * 8) = qf[i][c];
             }
         }
-    }
-    bf16x8 tf[2];  // talk^T: column = head 16b + r16, k = head 8g + j
-#pragma unroll
-    for (int b = 0; b < 2; ++b) {
-        const int h = b * 16 + r16;
-        uint16_t x[8];
-#pragma unroll
-        for (int j = 0; j < 8; ++j)
-            x[j] = h < a.H && g * 8 + j < a.H
-                       ? reinterpret_cast<const uint16_t*>(a.talk)[(size_t)h * a.H + g * 8 + j]
-                       : 0;
-        tf[b] = *reinterpret_cast<const bf16x8*>(x);
     }
     f32x4 acc[HW][NDV];
 #pragma unroll
@@ -460,23 +493,18 @@ __global__ void sigmoid_tiles_kernel(
 #pragma unroll
         for (int j = 0; j < NDV; ++j) acc[i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
 
-    auto page_row = [&](int k0) {
-        return (size_t)bt[min(k0, key_end - 1) >> page_shift] << page_shift;
+    // the page of 16 keys from k0 (past the end: of the last key)
+    auto page_of = [&](int k0) { return bt[min(k0, key_end - 1) >> page_shift]; };
+    auto row_of = [&](int page) {
+        return (size_t)__builtin_amdgcn_readfirstlane(page) << page_shift;
     };
-    uint4 kreg[2 * NDQ];
-    auto load_k = [&](int k0, size_t b0, size_t b1) {
+    auto load_k = [&](bf16x8* kreg, int k0, size_t page) {
+        const bf16* base = kp + page * ldk;
+        const uint32_t at = (uint32_t)((min(k0 + r16, key_end - 1) & mask) * ldk);
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            const int key = min(k0 + u * 16 + r16, key_end - 1);
-            const size_t row = (u && k0 + 16 < key_end ? b1 : b0) + (key & mask);
-            const bf16* p = kp + row * a.G * a.dim;
-#pragma unroll
-            for (int c = 0; c < NDQ; ++c) {
-                kreg[u * NDQ + c] = (uint4){0, 0, 0, 0};
-                if (c * 32 + g * 8 < a.dim)
-                    kreg[u * NDQ + c] = *reinterpret_cast<const uint4*>(p + c * 32 + g * 8);
-            }
-        }
+        for (int c = 0; c < NDQ; ++c)
+            kreg[c] =
+                *reinterpret_cast<const bf16x8*>(base + at + col_of(c * 32 + g * 8, a.dim));
     };
     bf16* vt = v_lds[wave];
     auto stage_v = [&](int k0, size_t b0, size_t b1) {
@@ -486,88 +514,128 @@ __global__ void sigmoid_tiles_kernel(
             const int o = u * PER + lane / (NDV * 2), c = lane % (NDV * 2);
             const int d = ((((c >> 1) ^ (o & (NDV - 1) & 7)) << 1) | (c & 1)) * 8;
             const int key = min(k0 + o, key_end - 1);
-            const size_t row = (key >= k0 + 16 ? b1 : b0) + (key & mask);
-            dma16(vp + row * a.G * a.vdim + (d < a.vdim ? d : 0), vt + u * 512);
+            const bf16* base = vp + (u * PER >= 16 && k0 + 16 < key_end ? b1 : b0) * ldv;
+            dma16(base + (uint32_t)((key & mask) * ldv + col_of(d, a.vdim)), vt + u * 512);
         }
     };
-    // biases of distances dmin .. dmin + 46
+    // -log2(e) times the biases of distances dmin .. dmin + 46
     auto fill_bias = [&](int dmin) {
         for (int e = tid; e < 47 * 32; e += 512) {
             const int x = e >> 5, h = e & 31;
             if (h < a.Hp)
                 b_lds[x][h] =
-                    a.bias[(size_t)max(0, min(dmin + x, a.nbias - 1)) * a.Hp + h] * LOG2E;
+                    a.bias[(size_t)max(0, min(dmin + x, a.nbias - 1)) * a.Hp + h] * -LOG2E;
         }
     };
-    size_t b0 = page_row(key_lo), b1 = page_row(key_lo + 16);
-    if (active) load_k(key_lo, b0, b1);
+    f32x4 s[2][HW];
+    auto scores = [&](const bf16x8* kreg, int u) {
+#pragma unroll
+        for (int i = 0; i < HW; ++i) {
+            s[u][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int c = 0; c < NDQ; ++c) {
+                const bool spilt = i < QL && c == NDQ - 1;
+                const bf16x8 x = spilt ? *reinterpret_cast<const bf16x8*>(
+                                             q_lds[wave][spilt ? i : 0] + lane * 8)
+                                       : qf[i][c];
+                s[u][i] = mfma16(x, kreg[c], s[u][i]);
+            }
+        }
+    };
+    // s to weights of rows 4g + r, key k0 + 16u + r16, in LDS
+    auto weights = [&](int k0, int u) {
+        const int o = u * 16 + r16;
+        const bool edge = k0 + u * 16 + 15 > pos0 || k0 + u * 16 < pos0 + 16 - a.window;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int row = g * 4 + r;
+            const float* bv = &b_lds[row + 31 - o][h0];
+            float w[4];
+#pragma unroll
+            for (int i = 0; i < HW; ++i)
+                w[i] = __builtin_amdgcn_rcpf(
+                    1.f + __builtin_amdgcn_exp2f(fmaf(s[u][i][r], scale2, bv[i])));
+            if (edge) {
+                const int dist = pos0 + row - (k0 + o);
+                const bool seen = dist >= 0 && dist < a.window;
+#pragma unroll
+                for (int i = 0; i < HW; ++i) w[i] = seen ? w[i] : 0.f;
+            }
+#pragma unroll
+            for (int i = HW; i < 4; ++i) w[i] = 0.f;
+            if (FULL) __builtin_amdgcn_sched_barrier(0);
+            const uint32_t p0 = cvt_pk_bf16(w[0], w[1]), p1 = cvt_pk_bf16(w[2], w[3]);
+            float f[4];
+            unpack2(p0, f[0], f[1]);
+            unpack2(p1, f[2], f[3]);
+            const uint32_t l0 = cvt_pk_bf16(w[0] - f[0], w[1] - f[1]);
+            const uint32_t l1 = cvt_pk_bf16(w[2] - f[2], w[3] - f[3]);
+            auto at = [&](int h) {
+                return o * 32 + (((h >> 3) ^ ((o >> 2) & 3)) << 3) + (h & 7);
+            };
+            if (HW == 4) {
+                *reinterpret_cast<uint2*>(&w_lds[0][row][at(h0)]) = make_uint2(p0, p1);
+                *reinterpret_cast<uint2*>(&w_lds[1][row][at(h0)]) = make_uint2(l0, l1);
+            } else if (HW == 2) {
+                *reinterpret_cast<uint32_t*>(&w_lds[0][row][at(h0)]) = p0;
+                *reinterpret_cast<uint32_t*>(&w_lds[1][row][at(h0)]) = l0;
+            } else {
+                const uint16_t hs[4] = {(uint16_t)p0, (uint16_t)(p0 >> 16), (uint16_t)p1, 0};
+                const uint16_t ls[4] = {(uint16_t)l0, (uint16_t)(l0 >> 16), (uint16_t)l1, 0};
+#pragma unroll
+                for (int i = 0; i < HW; ++i) {
+                    *reinterpret_cast<uint16_t*>(&w_lds[0][row][at(h0 + i)]) = hs[i];
+                    *reinterpret_cast<uint16_t*>(&w_lds[1][row][at(h0 + i)]) = ls[i];
+                }
+            }
+        }
+    };
+    bf16x8 k_lo[NDQ], k_hi[NDQ];
+    int n0, n1;
+    // keys of the step at k0, which lie in pages p0 and p1; pages of the next one
+    auto load_step = [&](int k0, size_t p0, size_t p1) {
+        n0 = page_of(k0 + 32);
+        n1 = page_of(k0 + 48);
+        load_k(k_lo, k0, p0);
+        load_k(k_hi, k0 + 16, k0 + 16 < key_end ? p1 : p0);
+    };
+    size_t b0 = row_of(page_of(key_lo)), b1 = row_of(page_of(key_lo + 16));
+    load_step(key_lo, b0, b1);
     fill_bias(pos0 - key_lo - 31);
     __syncthreads();
 
     for (int k0 = key_lo; k0 < key_end; k0 += 32) {
-        f32x4 s[HW][2];
-        if (active) {
+        // Transfers are waited for by count: what load_step loads must be in
+        // before they start (this uses it), the next step's comes after them.
 #pragma unroll
-            for (int u = 0; u < 2; ++u)
-#pragma unroll
-                for (int i = 0; i < HW; ++i) {
-                    s[i][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                    for (int c = 0; c < NDQ; ++c)
-                        s[i][u] = mfma16(qf[i][c], as_frag(kreg[u * NDQ + c]), s[i][u]);
-                }
-            __builtin_amdgcn_sched_barrier(0);  // the keys are in: transfers after them
-            stage_v(k0, b0, b1);
-        }
+        for (int c = 0; c < NDQ; ++c) asm volatile("" : "+v"(k_lo[c]), "+v"(k_hi[c]));
+        asm volatile("" : "+v"(n0), "+v"(n1));
+        const size_t next0 = row_of(n0), next1 = row_of(n1);
+        fresh_lane();
+        __builtin_amdgcn_sched_barrier(0);
+        if (active) stage_v(k0, b0, b1);
+        scores(k_lo, 0);
+        scores(k_hi, 1);
+        __builtin_amdgcn_sched_barrier(0);
+        b0 = next0;
+        b1 = next1;
+        if (!FULL) load_step(k0 + 32, b0, b1);
         lds_barrier();  // the last tile's mixed weights are read
         if (active) {
-#pragma unroll
-            for (int u = 0; u < 2; ++u) {
-                const int o = u * 16 + r16;
-#pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const int row = g * 4 + r, dist = pos0 + row - (k0 + o);
-                    const bool seen = dist >= 0 && dist < a.window;
-                    const float* bv = &b_lds[row + 31 - o][h0];
-                    float w[4];
-#pragma unroll
-                    for (int i = 0; i < HW; ++i)
-                        w[i] = seen ? sigmoid_2(fmaf(s[i][u][r], scale2, bv[i])) : 0.f;
-#pragma unroll
-                    for (int i = HW; i < 4; ++i) w[i] = 0.f;
-                    const uint32_t p0 = cvt_pk_bf16(w[0], w[1]), p1 = cvt_pk_bf16(w[2], w[3]);
-                    float f[4];
-                    unpack2(p0, f[0], f[1]);
-                    unpack2(p1, f[2], f[3]);
-                    const uint32_t l0 = cvt_pk_bf16(w[0] - f[0], w[1] - f[1]);
-                    const uint32_t l1 = cvt_pk_bf16(w[2] - f[2], w[3] - f[3]);
-                    auto at = [&](int h) {
-                        return o * 32 + (((h >> 3) ^ ((o >> 2) & 3)) << 3) + (h & 7);
-                    };
-                    if (HW == 4) {
-                        *reinterpret_cast<uint2*>(&w_lds[0][row][at(h0)]) = make_uint2(p0, p1);
-                        *reinterpret_cast<uint2*>(&w_lds[1][row][at(h0)]) = make_uint2(l0, l1);
-                    } else if (HW == 2) {
-                        *reinterpret_cast<uint32_t*>(&w_lds[0][row][at(h0)]) = p0;
-                        *reinterpret_cast<uint32_t*>(&w_lds[1][row][at(h0)]) = l0;
-                    } else {
-                        const uint16_t hs[4] = {(uint16_t)p0, (uint16_t)(p0 >> 16), (uint16_t)p1, 0};
-                        const uint16_t ls[4] = {(uint16_t)l0, (uint16_t)(l0 >> 16), (uint16_t)l1, 0};
-#pragma unroll
-                        for (int i = 0; i < HW; ++i) {
-                            *reinterpret_cast<uint16_t*>(&w_lds[0][row][at(h0 + i)]) = hs[i];
-                            *reinterpret_cast<uint16_t*>(&w_lds[1][row][at(h0 + i)]) = ls[i];
-                        }
-                    }
-                }
-            }
+            weights(k0, 0);
+            weights(k0, 1);
         }
+        __builtin_amdgcn_sched_barrier(0);
+        if (FULL) load_step(k0 + 32, b0, b1);
+        const bool more = k0 + 32 < key_end;
         lds_barrier();  // all weights are there
+        fresh_lane();
         // the next tile's biases, unless both are all beyond the table
         const int dmin = pos0 - k0 - 31;
-        if (k0 + 32 < key_end && dmin - 32 < a.nbias - 1) fill_bias(dmin - 32);
+        if (more && dmin - 32 < a.nbias - 1) fill_bias(dmin - 32);
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
+            if (FULL) __builtin_amdgcn_sched_barrier(0);
             const int row = wave * 2 + i;
             bf16 *hi = w_lds[0][row], *lo = w_lds[1][row];
             f32x4 m[2][2];
@@ -578,8 +646,9 @@ __global__ void sigmoid_tiles_kernel(
                 const bf16x8 wl = *reinterpret_cast<const bf16x8*>(lo + at);
 #pragma unroll
                 for (int b = 0; b < 2; ++b) {
-                    m[u][b] = mfma16(wh, tf[b], (f32x4){0.f, 0.f, 0.f, 0.f});
-                    m[u][b] = mfma16(wl, tf[b], m[u][b]);
+                    const bf16x8 tf = *reinterpret_cast<const bf16x8*>(t_lds[b] + lane * 8);
+                    m[u][b] = mfma16(wh, tf, (f32x4){0.f, 0.f, 0.f, 0.f});
+                    m[u][b] = mfma16(wl, tf, m[u][b]);
                 }
             }
             // keys 16u + 4g + r of head 16b + r16, at 8g + 4u + r
@@ -594,14 +663,11 @@ __global__ void sigmoid_tiles_kernel(
                                    cvt_pk_bf16(m[u][b][2], m[u][b][3]));
                 }
         }
-        const bool more = k0 + 32 < key_end;
-        if (more) {
-            b0 = page_row(k0 + 32);
-            b1 = page_row(k0 + 48);
-        }
-        dma_barrier();  // mixed weights and values are there
+        __builtin_amdgcn_sched_barrier(0);
+        // mixed weights and values are there; the 2 NDQ keys after them need not be
+        asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(2 * NDQ) : "memory");
         if (active) {
-            if (more) load_k(k0 + 32, b0, b1);
+            fresh_lane();
             bf16x8 pf[HW];
 #pragma unroll
             for (int i = 0; i < HW; ++i) {
@@ -613,6 +679,7 @@ __global__ void sigmoid_tiles_kernel(
             const bf16* r0 = vt + vr * NDV * 16 + (r16 & 3) * 4;
 #pragma unroll
             for (int j = 0; j < NDV; ++j) {
+                if (FULL && j % 2 == 0) __builtin_amdgcn_sched_barrier(0);
                 const bf16* p = r0 + ((j ^ sw) << 4);
                 const bf16x8 vf = tr_pair(p, p + 16 * NDV * 16);
 #pragma unroll
@@ -632,8 +699,8 @@ __global__ void sigmoid_tiles_kernel(
 #pragma unroll
         for (int j = 0; j < NDV; ++j) {
             const int d = j * 16 + g * 4;  // vdim is a multiple of 8
+            const uint2 zz = *reinterpret_cast<const uint2*>(z + col_of(d, a.vdim));
             if (d >= a.vdim) continue;
-            const uint2 zz = *reinterpret_cast<const uint2*>(z + d);
             float f[4];
             unpack2(zz.x, f[0], f[1]);
             unpack2(zz.y, f[2], f[3]);
@@ -657,9 +724,11 @@ static SigmoidArgs sigmoid_args(
                        dim, vdim};
 }
 
-// sizes of the MFMA forms; pages of a power of two, at least 16 tokens
+// sizes of the MFMA forms: up to 64 heads of 128, or 32 of 256; pages of a
+// power of two, at least 16 tokens
 static bool sigmoid_mfma_ok(const SigmoidArgs& a) {
-    return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.H <= 64 &&
+    const int most = a.H <= 32 ? 256 : 128;
+    return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= most && a.vdim <= most && a.H <= 64 &&
            a.Hp % 16 == 0 && a.Hp >= a.H && a.block_size >= 16 &&
            (a.block_size & (a.block_size - 1)) == 0;
 }
@@ -691,15 +760,15 @@ extern "C" hipError_t launch_sigmoid_rows(
     const dim3 grid(nrows, nsplit);
 #define GO(NB, A, B) \
     sigmoid_rows_kernel<NB, A, B><<<grid, SA_THREADS, 0, stream>>>(a, shift, nsplit, part)
-#define SIZES(NB)                                   \
-    {                                               \
-        if (dim <= 64 && vdim <= 64) GO(NB, 2, 4);  \
-        else if (dim <= 128 && vdim <= 128) GO(NB, 4, 8); \
-        else GO(NB, 8, 16);                         \
+#define SIZES(GO1, GO2, GO4)    \
+    {                           \
+        if (H <= 16) GO1;       \
+        else if (H <= 32) GO2;  \
+        else GO4;               \
     }
-    if (H <= 16) SIZES(1)
-    else if (H <= 32) SIZES(2)
-    else SIZES(4)
+    if (dim <= 64 && vdim <= 64) SIZES(GO(1, 2, 4), GO(2, 2, 4), GO(4, 2, 4))
+    else if (dim <= 128 && vdim <= 128) SIZES(GO(1, 4, 8), GO(2, 4, 8), GO(4, 4, 8))
+    else SIZES(GO(1, 8, 16), GO(2, 8, 16), return hipErrorInvalidValue)
 #undef SIZES
 #undef GO
     HIP_CHECK_LAST();

@@ -528,9 +528,10 @@ def sigmoid_attention(out, q, k_pages, v_pages, H: int, G: int, scale: float, bi
     page, dim, vdim = k_pages.shape[1], k_pages.shape[2] // G, v_pages.shape[2] // G
     head = (out, q, k_pages, v_pages, H, G, float(scale), bias, talk, int(window), gate,
             positions)
+    most = 256 if H <= 32 else 128
     mfma = (
         q.dtype == torch.bfloat16 and page >= 16 and page & (page - 1) == 0 and H <= 64
-        and dim % 8 == 0 and vdim % 8 == 0 and dim <= 256 and vdim <= 256
+        and dim % 8 == 0 and vdim % 8 == 0 and dim <= most and vdim <= most
     )
     rows, n = None, q.shape[0]
     per_wave = -(-H // 8)  # a tile's 8 waves share the heads, no wave has two key heads
@@ -547,7 +548,7 @@ def sigmoid_attention(out, q, k_pages, v_pages, H: int, G: int, scale: float, bi
     if mfma:
         # fill the chip: splits only from shapes, so captured graphs hold
         most = -(-min(segs.tables.shape[1] * page, window + 31) // 128)
-        nsplit = max(1, min(-(-512 // n), 16, most))
+        nsplit = max(1, min(-(-256 // n), 16, most))
         if nsplit > 1:
             part, _ = _folded_scratch(q.device, n * H * nsplit * vdim, 0)
     ext.sigmoid_rows(*head, segs.row_seg, segs.tables, rows, nsplit, part)
