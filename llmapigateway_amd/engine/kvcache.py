@@ -285,7 +285,8 @@ class PagedKVCache:
 class HybridCache:
     """Per layer run (a looped layer counts once per pass): ``runs[r]`` maps
     a name to pages ``[num_blocks, block_size, row]`` in the compute dtype,
-    or to state ``[num_slots, ...]``, fp32 where the recurrence lives."""
+    or to state ``[num_slots, ...]``, fp32 where the recurrence lives. A layer
+    that reads another layer's keys and values has that layer's view."""
 
     fp8 = False
 
@@ -307,7 +308,12 @@ class HybridCache:
         self.num_blocks = num_blocks
         self.num_slots = num_slots
         self.runs: List[dict] = []
-        for spec in _run_specs(config):
+        first = {}  # layer -> the first run of it
+        for r, ((i, _), spec) in enumerate(zip(config.runs(), _run_specs(config))):
+            first.setdefault(i, r)
+            if config.kv_source(i) != i:  # another layer's pages
+                self.runs.append(self.runs[first[config.kv_source(i)]])
+                continue
             views = {
                 name: torch.zeros(num_blocks, block_size, row, dtype=dtype, device=device)
                 for name, row in spec.pages.items()

@@ -71,8 +71,8 @@ class HybridConfig:
     [start, stop) run ``times`` times with the same weights, each pass with
     its own cache.
 
-    The field set is what the Lelisun, Filinex and Mekevik config.json files
-    give and what their designs fix; ``max_positions`` is the framework's own
+    The field set is what the Lelisun, Filinex, Mekevik and Duratar config.json
+    files give and what their designs fix; ``max_positions`` is the framework's own
     bound (nothing in the designs limits it) and ``weights_dir`` says where
     the checkpoint lies (None: random init)."""
 
@@ -85,6 +85,9 @@ class HybridConfig:
     parallel_mlp: bool = False    # mixer and feed-forward read the same stream
     post_norm: bool = False       # a norm on every sublayer's output, too
     embed_norm: bool = False
+    scalar_norms: bool = False    # the stream's norms have one number for all coordinates
+    streams: int = 0              # hyper-connected copies of the stream (0: one, plainly summed)
+    layer_scale: bool = False     # a learned factor per coordinate of every sublayer's output
     embed_scale: float = 1.0
     loop: Optional[Tuple[int, int, int]] = None  # (start, stop, times)
     loop_step: bool = True        # a learned vector per loop pass
@@ -104,11 +107,18 @@ class HybridConfig:
             raise ValueError("mixer and feed-forward in parallel: RMS norms only")
         if self.norm == "rms" and self.loop is not None:
             raise ValueError("loops: layer norms and dynamic tanh only")
-        if self.norm != "tanh" and (self.post_norm or self.embed_norm):
+        if self.norm != "tanh" and (self.post_norm or self.embed_norm and not self.streams):
             raise ValueError("norms of sublayer outputs and of the embedding: dynamic tanh only")
+        if self.streams and (self.norm != "rms" or self.parallel_mlp or not self.embed_norm):
+            raise ValueError("streams: RMS norms, one also on the embedding, sublayers in turn")
+        if not 0 <= self.streams <= 16:
+            raise ValueError(f"{self.streams} streams: 16 at most")
+        if not self.streams and (self.scalar_norms or self.layer_scale):
+            raise ValueError("scalar norms and layer scales: hyper-connected streams only")
         for i, layer in enumerate(self.layers):
             try:
                 self._check_layer(layer)
+                self._check_kv_source(i)
             except ValueError as e:
                 raise ValueError(f"layer {i}: {e}") from None
         shared = {
@@ -139,6 +149,21 @@ class HybridConfig:
                 raise ValueError(f"bias_max {m['bias_max']} for {m['bias_rows']} rows")
             if not m["window"] >= 1:
                 raise ValueError(f"a window of {m['window']}")
+        elif layer.type == "rotary_attention":
+            if m["heads"] % m["kv_heads"]:
+                raise ValueError("kv_heads does not divide the heads")
+            if m["rot"]["dims"] % 2 or not 0 <= m["rot"]["dims"] <= m["dim"]:
+                raise ValueError(f"rot.dims {m['rot']['dims']} of {m['dim']}")
+            if not m["window"] >= 1 or not m["keep_first"] >= 0:
+                raise ValueError(f"a window of {m['window']}, {m['keep_first']} kept")
+        elif layer.type == "lightning":
+            if len(m["decay"]) != m["heads"] or not all(0 <= d <= 1 for d in m["decay"]):
+                raise ValueError(f"decay: a number within 0..1 for each of {m['heads']} heads")
+        elif layer.type == "channel_delta":
+            if m["heads"] % m["kv_heads"]:
+                raise ValueError("kv_heads does not divide the heads")
+            if not m["conv"] >= 1:
+                raise ValueError(f"a convolution of {m['conv']} taps")
         elif layer.type not in ("mlstm", "wkv"):
             raise ValueError(f"unknown mixer '{layer.type}'")
         if layer.mlp is None:
@@ -147,8 +172,22 @@ class HybridConfig:
             r = layer.mlp["router"]
             if not 1 <= r["top"] <= r["experts"]:
                 raise ValueError(f"router: top {r['top']} of {r['experts']} experts")
-        elif layer.mlp["kind"] != "dense":
+        elif layer.mlp["kind"] not in ("dense", "xielu"):
             raise ValueError(f"unknown feed-forward '{layer.mlp['kind']}'")
+
+    def _check_kv_source(self, i: int) -> None:
+        m = self.layers[i].mixer
+        j = m.get("kv_from")
+        if j is None:
+            return
+        if self.loop is not None:
+            raise ValueError("kv_from inside or beside a loop")
+        source = self.layers[j] if 0 <= j < i else None
+        if source is None or source.type != self.layers[i].type or "kv_from" in source.mixer:
+            raise ValueError(f"kv_from {j}: not an earlier layer with keys of its own")
+        for key in ("kv_heads", "dim", "vdim", "rot"):
+            if source.mixer[key] != m[key]:
+                raise ValueError(f"kv_from {j}: its {key} differs")
 
     @staticmethod
     def _common(raw: Dict[str, Any], layers) -> Dict[str, Any]:
@@ -215,6 +254,36 @@ class HybridConfig:
             **cls._common(raw, layers),
         )
 
+    @classmethod
+    def from_duratar_json(cls, raw: Dict[str, Any], name: str, weights_dir: Optional[str] = None):
+        """Duratar's config.json. The ranks of the low-rank projections are
+        only in the checkpoint's shapes."""
+        from .weights import open_checkpoint
+
+        ckpt = open_checkpoint(weights_dir)
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            m, kind, mlp = dict(e["mixer"]), e["type"], e.get("mlp")
+            if kind == "attention":
+                kind, mask = "rotary_attention", m.pop("mask")
+                m.update(window=mask["size"], keep_first=mask["keep_first"])
+            elif kind == "channel_delta":
+                m["decay_rank"] = ckpt.shape(f"l{i}.mix.a1")[0]
+                m["gate_rank"] = ckpt.shape(f"l{i}.mix.g1")[0]
+            elif kind != "lightning":
+                raise ValueError(f"layer {i}: unknown mixer '{kind}'")
+            if mlp is not None and mlp["kind"] == "dense":
+                mlp = dict(mlp, kind="xielu")
+            layers.append(HybridLayer(type=kind, mixer=m, mlp=mlp))
+        return cls(
+            name=name, norm="rms", embed_norm=True, scalar_norms=True, streams=raw["streams"],
+            layer_scale=True, weights_dir=weights_dir, **cls._common(raw, layers),
+        )
+
+    def kv_source(self, i: int) -> int:
+        """The layer whose cached keys and values layer i reads."""
+        return self.layers[i].mixer.get("kv_from", i)
+
     def runs(self) -> List[Tuple[int, Optional[int]]]:
         """The layers in the order they run, as (layer index, t): t is the
         number of the loop pass that this layer begins, None elsewhere."""
@@ -229,7 +298,8 @@ class HybridConfig:
     @property
     def prefix_cacheable(self) -> bool:
         return all(
-            layer.type in ("latent_attention", "sigmoid_attention") for layer in self.layers
+            layer.type in ("latent_attention", "sigmoid_attention", "rotary_attention")
+            for layer in self.layers
         )
 
     def scaled_for_tp(self, tp: int) -> "HybridConfig":
@@ -241,6 +311,7 @@ ARCHITECTURES = {
     "Lelisun": HybridConfig.from_json,
     "Filinex": HybridConfig.from_filinex_json,
     "Mekevik": HybridConfig.from_mekevik_json,
+    "Duratar": HybridConfig.from_duratar_json,
 }
 
 
@@ -336,6 +407,43 @@ def _mekevik_preset(
             HybridLayer("sigmoid_attention", mixer, mlps[i % 2]) for i in range(layers)
         ),
         embed_scale=width ** 0.5, logit_scale=0.5, max_positions=max_positions,
+    )
+
+
+def _duratar_preset(
+    name: str, width: int, vocab: int, heads: int, kv_heads: int, dim: int, window: int,
+    keep_first: int, delta_heads: int, delta_kv_heads: int, delta_dim: int, delta_vdim: int,
+    rank: int, mem_heads: int, mem_dim: int, ff: int, streams: int, layers: int,
+    max_positions: int = 32768,
+) -> HybridConfig:
+    """A Duratar whose layers repeat delta, attention, lightning, delta; every
+    second attention reads the keys and values of the one before it."""
+    delta = dict(
+        heads=delta_heads, kv_heads=delta_kv_heads, dim=delta_dim, vdim=delta_vdim, conv=4,
+        decay_rank=rank, gate_rank=rank,
+    )
+    attn = dict(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=2 * dim, scale=dim ** -0.5, diff=0.5,
+        window=window, keep_first=keep_first,
+        rot=dict(base=500000.0, dims=dim // 2, scaling=dict(
+            factor=8.0, low=1.0, high=4.0, original=8192)),
+    )
+    mem = dict(
+        heads=mem_heads, dim=mem_dim, vdim=mem_dim,
+        decay=[1.0 - 2.0 ** (-3 - 6 * i / mem_heads) for i in range(mem_heads)],
+    )
+    kinds = ("channel_delta", "rotary_attention", "lightning", "channel_delta")
+    out = []
+    for i in range(layers):
+        kind = kinds[i % 4]
+        m = (delta, attn, mem, delta)[i % 4]
+        if kind == "rotary_attention" and i % 8 == 5:
+            m = dict(m, kv_from=i - 4)
+        out.append(HybridLayer(kind, m, dict(kind="xielu", ff=ff)))
+    return HybridConfig(
+        name=name, vocab_size=vocab, hidden_size=width, layers=tuple(out), norm_eps=1e-6,
+        norm="rms", embed_norm=True, scalar_norms=True, streams=streams, layer_scale=True,
+        max_positions=max_positions,
     )
 
 
@@ -469,6 +577,24 @@ MODEL_PRESETS = {
         "mekevik-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=128, vdim=128,
         window=1024, bias_rows=32, bias_max=128, ff=14336, experts=64, top=8, expert_ff=1792,
         layers=16,
+    ),
+    # hyper-connected streams over delta-rule, differential-attention and
+    # lightning layers
+    "tiny-duratar": _duratar_preset(
+        "tiny-duratar", width=96, vocab=320, heads=4, kv_heads=2, dim=16, window=24,
+        keep_first=3, delta_heads=4, delta_kv_heads=2, delta_dim=24, delta_vdim=40, rank=8,
+        mem_heads=3, mem_dim=16, ff=112, streams=3, layers=6, max_positions=1024,
+    ),
+    # layers as wide as llama-1b's and llama-3-8b's
+    "duratar-small": _duratar_preset(
+        "duratar-small", width=2048, vocab=128256, heads=16, kv_heads=4, dim=64, window=1024,
+        keep_first=16, delta_heads=16, delta_kv_heads=16, delta_dim=128, delta_vdim=128,
+        rank=128, mem_heads=16, mem_dim=128, ff=8192, streams=4, layers=12,
+    ),
+    "duratar-base": _duratar_preset(
+        "duratar-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=64, window=1024,
+        keep_first=16, delta_heads=32, delta_kv_heads=32, delta_dim=128, delta_vdim=128,
+        rank=128, mem_heads=32, mem_dim=128, ff=14336, streams=4, layers=16,
     ),
     # small-but-real shape for 1-GPU kernel shakedown
     "llama-1b": ModelConfig(

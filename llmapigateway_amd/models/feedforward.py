@@ -41,6 +41,26 @@ class DenseFF:
         )
 
 
+class XieluFF:
+    """W_down xielu(W_up h): xielu(z) = softplus(p) z^2 + z/2 for z > 0, and
+    (1/2 + softplus(q)) (e^z - 1 - z) + z/2 else; p and q are learned."""
+
+    def __init__(self, m: dict, get: Getter, vec: Getter):
+        self.w = {"up": get("up"), "down": get("down")}
+        p, q = torch.nn.functional.softplus(vec("act").double(), threshold=1e9).tolist()
+        self.pos, self.neg = p, 0.5 + q
+        add_decode_twins(self.w, ("up", "down"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        return {"up": (m["ff"], width), "down": (width, m["ff"]), "act": (2,)}
+
+    def __call__(self, h: torch.Tensor) -> torch.Tensor:
+        w = self.w
+        z = ops.linear(h, w["up"], w.get("up_swz"))
+        return ops.linear(ops.xielu_(z, self.pos, self.neg), w["down"], w.get("down_swz"))
+
+
 class ExpertFF:
     """Experts of which a router picks ``top`` per token, and optionally a
     shared one for every token. An expert is a DenseFF, with or without a
@@ -94,4 +114,4 @@ class ExpertFF:
         return ops.ExpertSum(rows, routing.slot, routing.weights, shared)
 
 
-FEEDFORWARDS = {"dense": DenseFF, "moe": ExpertFF}
+FEEDFORWARDS = {"dense": DenseFF, "xielu": XieluFF, "moe": ExpertFF}

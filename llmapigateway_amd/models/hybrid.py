@@ -7,10 +7,11 @@ norm where the design has one, and is added by the next norm's kernel
 feed-forward are parallel, both of their outputs are pending together, and
 one kernel makes the two norms of the next layer. A loop pass starts by replacing the
 stream with W [stream; embedding output] (+ step[t]); each pass of a layer
-has its own cache view.
+has its own cache view. Hyper-connected streams (models/streams.py) take the
+place of the one stream where a design has them.
 
-Serves Lelisun, Filinex and Mekevik; another design built from these mixers and
-feed-forwards needs only a configuration.
+Serves Lelisun, Filinex, Mekevik and Duratar; another design built from these
+mixers and feed-forwards needs only a configuration.
 """
 
 from __future__ import annotations
@@ -24,6 +25,7 @@ from .batch import ForwardBatch
 from .configs import HybridConfig
 from .feedforward import FEEDFORWARDS
 from .mixers import MIXERS
+from .streams import HyperStreams
 from .weights import open_checkpoint
 
 
@@ -63,7 +65,7 @@ class HybridModel:
         out = {"embed": (V, W), "head": (V, W)}
 
         def norm(name: str) -> None:
-            out[name] = (W,)
+            out[name] = () if config.scalar_norms else (W,)
             if config.norm != "rms":
                 out[name + ".b"] = (W,)
             if config.norm == "tanh":
@@ -86,6 +88,12 @@ class HybridModel:
                 norm(f"l{i}.norm{n}")
                 if config.post_norm:
                     norm(f"l{i}.norm{n}b")
+                if config.layer_scale:
+                    out[f"l{i}.ls{n}"] = (W,)
+                if config.streams:
+                    S = config.streams
+                    out.update({f"l{i}.hc{n}.in": (S,), f"l{i}.hc{n}.out": (S,),
+                                f"l{i}.hc{n}.mix": (S, S)})
         return out
 
     def _source(self, seed: int):
@@ -108,8 +116,15 @@ class HybridModel:
         def draw(name: str) -> torch.Tensor:
             shape, leaf = shapes[name], name.rsplit(".", 1)[-1]
             t = torch.empty(shape, dtype=torch.float32, device=device)
-            if leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b", "D", "alpha"):
+            if leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b", "D", "alpha", "ls1", "ls2"):
                 return t.fill_(1.0)
+            if ".hc" in name:
+                t.normal_(0.0, 0.1, generator=gen)
+                if leaf == "mix":
+                    return t.add_(torch.eye(len(t), device=device))
+                return t.add_(1.0 if leaf == "out" else 1.0 / len(t))
+            if leaf in ("lq1", "lk1", "lq2", "lk2"):
+                return t.normal_(0.0, 0.1, generator=gen)
             if leaf == "b" or leaf == "A_log":
                 return t.fill_(2.0 if name.endswith((".f.b", ".a2.b")) else 0.0)
             if leaf == "dt_bias":
@@ -138,7 +153,8 @@ class HybridModel:
 
         def norm(name: str):
             if c.norm == "rms":
-                return (vec(name),)
+                w = vec(name)
+                return (w.expand(c.hidden_size).contiguous() if c.scalar_norms else w,)
             parts = (vec(name), vec(name + ".b"))
             return parts + (float(source(name + ".alpha")),) if c.norm == "tanh" else parts
 
@@ -160,6 +176,7 @@ class HybridModel:
                     self._rope,
                 ),
                 "mlp": None,
+                "ls1": vec(p + "ls1") if c.layer_scale else None,
             }
             if layer.mlp is not None:
                 ent["norm2"] = norm(p + "norm2")
@@ -168,7 +185,14 @@ class HybridModel:
                     layer.mlp,
                     lambda n, p=p: mat(f"{p}mlp.{n}"), lambda n, p=p: vec(f"{p}mlp.{n}"),
                 )
+                ent["ls2"] = vec(p + "ls2") if c.layer_scale else None
             self.layers.append(ent)
+        self.streams = None
+        if c.streams:
+            self.streams = HyperStreams(c.streams, [
+                tuple(vec(f"l{i}.hc{n}.{leaf}") for leaf in ("in", "mix", "out"))
+                for i, layer in enumerate(c.layers) for n in ("1", "2")[: 1 + bool(layer.mlp)]
+            ], self.device)
         self.final_norm = norm("final.norm")
         if c.logit_scale != 1.0:  # the norm's last factors take it in
             self.final_norm = tuple(t * c.logit_scale for t in self.final_norm[:2]) + (
@@ -176,11 +200,11 @@ class HybridModel:
             )
         self.head = mat("head")
 
-    def _rope(self, base: float, dims: int) -> torch.Tensor:
-        key = (float(base), int(dims))
+    def _rope(self, base: float, dims: int, scaling: Optional[dict] = None) -> torch.Tensor:
+        key = (float(base), int(dims), tuple(sorted((scaling or {}).items())))
         if key not in self._ropes:
             self._ropes[key] = ops.build_pair_rope_cache(
-                self.max_positions, dims, base, device=self.device
+                self.max_positions, dims, base, device=self.device, scaling=scaling
             )
         return self._ropes[key]
 
@@ -212,6 +236,8 @@ class HybridModel:
         c, W = self.config, self.config.hidden_size
         plan = ops.plan_segments(batch, self.dtype, self.plans)
         T = batch.token_ids.shape[0]
+        if self.streams is not None:
+            return self._step_streams(batch, cache, plan)
         both = x0 = None
         if c.loop is not None:  # [stream; embedding output], the loop's input
             both = torch.empty(T, 2 * W, dtype=self.dtype, device=self.device)
@@ -247,7 +273,29 @@ class HybridModel:
             x, pending = x[pick], tuple(d[pick] for d in pending)
             if x.shape[0] == 0:
                 return torch.empty(0, c.vocab_size, dtype=torch.float32, device=self.device)
-        h = self._norm(x, pending, post, self.final_norm)
+        return self._logits(self._norm(x, pending, post, self.final_norm))
+
+    def _step_streams(self, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        """step() over hyper-connected streams."""
+        c, st = self.config, self.streams
+        x = ops.embed_rms_norm(batch.token_ids, self.embed, self.embed_norm[0], c.norm_eps)
+        x, pending, q = x.unsqueeze(1), [], 0  # [T, stored streams, W]
+        for r, (i, _) in enumerate(c.runs()):
+            layer = self.layers[i]
+            h, x, pending = st.read(q, x, pending, layer["norm1"][0], c.norm_eps, self.dtype)
+            y = layer["mixer"](h, batch, cache.runs[r], plan)
+            pending, q = pending + [(y, layer["ls1"])], q + 1
+            if layer["mlp"] is not None:
+                h, x, pending = st.read(q, x, pending, layer["norm2"][0], c.norm_eps, self.dtype)
+                pending, q = pending + [(layer["mlp"](h), layer["ls2"])], q + 1
+        if batch.logits_indices is not None and batch.logits_indices.shape[0] == 0:
+            return torch.empty(0, c.vocab_size, dtype=torch.float32, device=self.device)
+        return self._logits(st.read(
+            q, x, pending, self.final_norm[0], c.norm_eps, self.dtype, batch.logits_indices
+        )[0])
+
+    def _logits(self, h: torch.Tensor) -> torch.Tensor:
+        c = self.config
         logits = ops.linear_f32(h, self.head)
         if c.logit_softcap is not None:
             ops.soft_cap_(logits, c.logit_softcap)

@@ -464,7 +464,173 @@ class WKV:
         return ops.linear(out, w["o"], w.get("o_swz"))
 
 
+class RotaryAttention:
+    """Grouped-query softmax attention over the last ``window`` tokens and the
+    first ``keep_first`` ones; queries and keys are RMS-normed per head and
+    rotated in halves on their first ``rot.dims`` dimensions. With ``diff`` it
+    is differential: every head has two maps of queries and keys over the same
+    values, and gives unit_rms(map 1 - lambda map 2) (1 - diff). With
+    ``kv_from`` its keys and values are another layer's, out of that layer's
+    cache."""
+
+    plans = ("tiles",)  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.H, self.G, self.dim, self.eps = m["heads"], m["kv_heads"], m["dim"], eps
+        self.scale, self.window, self.keep = float(m["scale"]), m["window"], m["keep_first"]
+        self.own = m.get("kv_from") is None
+        w_in, self.cut = _stack([(n, get(n)) for n in ("qkv" if self.own else "q")])
+        self.w = {"in": w_in, "o": get("o")}
+        self.q_norm, self.k_norm = vec("q.norm"), vec("k.norm") if self.own else None
+        self.cos_sin = rope(m["rot"]["base"], m["rot"]["dims"], m["rot"].get("scaling"))
+        self.maps, self.lam, self.gain = 1, 0.0, 1.0
+        if m.get("diff") is not None:
+            l1, l2 = (float((vec("lq" + n).double() * vec("lk" + n).double()).sum().exp())
+                      for n in "12")
+            self.maps, self.lam = 2, l1 - l2 + m["diff"]
+            self.gain = 1.0 - m["diff"]
+        add_decode_twins(self.w, ("in", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        maps = 2 if m.get("diff") is not None else 1
+        H, G, dim = m["heads"], m["kv_heads"], m["dim"]
+        out: Dict[str, Tuple[int, ...]] = {
+            "q": (H * maps * dim, width), "q.norm": (dim,), "o": (width, H * m["vdim"]),
+        }
+        if m.get("kv_from") is None:
+            out.update({
+                "k": (G * maps * dim, width), "v": (G * m["vdim"], width), "k.norm": (dim,),
+            })
+        if maps == 2:
+            out.update({n: (dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
+        return out
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        if m.get("kv_from") is not None:
+            return CacheSpec({}, {})
+        maps, G = 2 if m.get("diff") is not None else 1, m["kv_heads"]
+        return CacheSpec({"k": G * maps * m["dim"], "v": G * m["vdim"]}, {})
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        p = {name: u[:, lo:hi] for name, (lo, hi) in self.cut.items()}
+        q = ops.rotary_rows(
+            p["q"], p.get("k"), p.get("v"), self.q_norm, self.k_norm, self.eps, self.cos_sin,
+            batch.positions, cache["k"], cache["v"], batch.slot_mapping,
+        )
+        out = torch.empty(h.shape[0], w["o"].shape[1], dtype=h.dtype, device=h.device)
+        ops.window_attention(
+            out, q, cache["k"], cache["v"], self.H, self.G, self.maps, self.scale, self.window,
+            self.keep, self.lam, self.gain, self.eps, batch.positions, batch.segs, plan,
+        )
+        return ops.linear(out, w["o"], w.get("o_swz"))
+
+
+class Lightning:
+    """Linear attention with a fixed decay per head on silu'd queries, keys
+    and values; one RMS norm over all heads' outputs and a sigmoid gate."""
+
+    plans = ("chunks",)  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.H, self.dk, self.dv, self.eps = m["heads"], m["dim"], m["vdim"], eps
+        w_in, self.cut = _stack([(n, get(n)) for n in "qkvg"])
+        self.w = {"in": w_in, "o": get("o")}
+        self.norm = vec("norm")
+        self.decay = torch.tensor(m["decay"], dtype=torch.float32, device=self.norm.device)
+        add_decode_twins(self.w, ("in", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        kk, vv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+        return {
+            "q": (kk, width), "k": (kk, width), "v": (vv, width), "g": (vv, width),
+            "o": (width, vv), "norm": (vv,),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        return CacheSpec({}, {"S": ((m["heads"], m["vdim"], m["dim"]), True)})
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w = self.w
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        q, k, v, g = (u[:, lo:hi] for lo, hi in self.cut.values())
+        y = ops.fixed_decay_kv(
+            q, k, v, self.decay, self.H, self.dk, self.dv, cache["S"], batch.positions,
+            batch.segs, plan,
+        )
+        y = ops.gated_norm(y, g, self.norm, 1, self.eps, gate_first=False)
+        return ops.linear(y, w["o"], w.get("o_swz"))
+
+
+class ChannelDelta:
+    """Gated delta rule with a decay per key channel: short convolutions on
+    queries, keys and values, unit queries and keys, decays and output gates
+    from low-rank projections, a head-wise RMS norm."""
+
+    plans = ("chunks",)  # what it uses of a step's plan
+
+    def __init__(self, m: dict, eps: float, get: Getter, vec: Getter, rope: Callable):
+        self.H, self.G, self.eps = m["heads"], m["kv_heads"], eps
+        self.dk, self.dv = m["dim"], m["vdim"]
+        w_in, self.cut = _stack([(n, get(n)) for n in ("q", "k", "v", "a1", "g1", "b")])
+        self.w = {"in": w_in, "g2": get("g2"), "o": get("o")}
+        # the convolutions of q, k and v are one over their stacked columns
+        taps = w_in.new_zeros(self.cut["v"][1], m["conv"], dtype=torch.float32)
+        for n in "qkv":
+            taps[self.cut[n][0] : self.cut[n][1]] = vec(n + ".conv")
+        self.conv_t = taps.t().contiguous()
+        self.conv_b = torch.zeros_like(self.conv_t[0])
+        self.a2, self.dt_bias = get("a2"), vec("dt_bias")
+        self.rate = vec("A_log").exp().repeat_interleave(self.dk)
+        self.norm = vec("norm").repeat(self.H)  # shared by the heads
+        add_decode_twins(self.w, ("in", "g2", "o"))
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
+        H, qk, vv = m["heads"], m["kv_heads"] * m["dim"], m["heads"] * m["vdim"]
+        ra, rg, taps = m["decay_rank"], m["gate_rank"], m["conv"]
+        return {
+            "q": (qk, width), "k": (qk, width), "v": (vv, width), "q.conv": (qk, taps),
+            "k.conv": (qk, taps), "v.conv": (vv, taps), "b": (H, width), "A_log": (H,),
+            "a1": (ra, width), "a2": (H * m["dim"], ra), "dt_bias": (H * m["dim"],),
+            "g1": (rg, width), "g2": (vv, rg), "norm": (m["vdim"],), "o": (width, vv),
+        }
+
+    @staticmethod
+    def cache_spec(m: dict, width: int) -> CacheSpec:
+        channels = 2 * _pad8(m["kv_heads"] * m["dim"]) + m["heads"] * m["vdim"]
+        return CacheSpec({}, {
+            "S": ((m["heads"], m["vdim"], m["dim"]), True),
+            "conv": ((m["conv"] - 1, channels), False),
+        })
+
+    def __call__(self, h: torch.Tensor, batch: ForwardBatch, cache, plan) -> torch.Tensor:
+        w, cut = self.w, self.cut
+        u = ops.linear(h, w["in"], w.get("in_swz"))
+        x = ops.causal_conv(
+            u[:, : cut["v"][1]], self.conv_t, self.conv_b, cache["conv"], batch.positions,
+            batch.segs, plan,
+        )
+        a, g1, b = (u[:, slice(*cut[n])] for n in ("a1", "g1", "b"))
+        logw = ops.decay_logs(a, self.a2, self.dt_bias, "softplus", rate=self.rate)
+        q, k, v = (x[:, slice(*cut[n])] for n in "qkv")
+        y = ops.delta_kv(
+            q, k, v, logw, b, self.H, self.G, self.dk, self.dv, cache["S"], batch.positions,
+            batch.segs, plan,
+        )
+        gate = ops.linear(g1, w["g2"], w.get("g2_swz"))
+        out = torch.empty_like(y)
+        ops.head_norm_gate(out, y, gate, self.norm, self.H, self.eps, act="sigmoid")
+        return ops.linear(out, w["o"], w.get("o_swz"))
+
+
 MIXERS = {
     "latent_attention": LatentAttention, "mamba2": Mamba2, "mlstm": MLSTM,
     "parallel": Parallel, "wkv": WKV, "sigmoid_attention": SigmoidAttention,
+    "rotary_attention": RotaryAttention, "lightning": Lightning, "channel_delta": ChannelDelta,
 }

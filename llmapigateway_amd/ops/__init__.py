@@ -557,9 +557,12 @@ from .hybrid import (  # noqa: E402
     causal_conv,
     decay_logs,
     decayed_kv,
+    delta_kv,
     distance_bias,
+    embed_rms_norm,
     embed_scaled,
     embed_tanh_norm,
+    fixed_decay_kv,
     fold_queries,
     gated_norm,
     head_linear,
@@ -568,15 +571,19 @@ from .hybrid import (  # noqa: E402
     latent_attention_unfolded,
     latent_rows,
     linear_f32,
+    mix_streams,
     mlstm,
     page_write,
     paged_attention,
     plan_segments,
     qkv_rows,
+    rotary_rows,
     sigmoid_attention,
     soft_cap_,
     ssd,
     token_shift,
+    window_attention,
+    xielu_,
 )
 
 __all__ = [

@@ -389,12 +389,12 @@ def gated_norm(y, gate, w, groups: int, eps: float, gate_first: bool):
     return out
 
 
-def head_norm_gate(out, y, gate, w, heads: int, eps: float) -> None:
-    """out = RMS norm of y per head, times w, times silu(gate); out and gate
-    may be strided."""
+def head_norm_gate(out, y, gate, w, heads: int, eps: float, act: str = "silu") -> None:
+    """out = RMS norm of y per head, times w, times silu(gate) (act "sigmoid":
+    sigmoid(gate)); out and gate may be strided."""
     if not y.is_cuda:
-        return ref.head_norm_gate(out, y, gate, w, heads, eps)
-    hybrid_native().head_norm_gate(out, y, gate, w, heads, float(eps))
+        return ref.head_norm_gate(out, y, gate, w, heads, eps, act)
+    hybrid_native().head_norm_gate(out, y, gate, w, heads, float(eps), act == "sigmoid")
 
 
 # ------------------------------------------------------------- dynamic tanh
@@ -555,14 +555,17 @@ def sigmoid_attention(out, q, k_pages, v_pages, H: int, G: int, scale: float, bi
 
 
 # -------------------------------------- recurrences with a decay per channel
-def decay_logs(a, w2, bias, kind: str, tau: float) -> torch.Tensor:
-    """fp32 log decays [T, N] from a [T, rank] (may be strided): "sigmoid":
-    log sigmoid(z) / tau with z = a w2^T + bias; "exp": -e^z with
-    z = tanh(a) w2^T + bias."""
+DECAY_KINDS = {"sigmoid": 0, "exp": 1, "softplus": 2}
+
+
+def decay_logs(a, w2, bias, kind: str, tau: float = 1.0, rate=None) -> torch.Tensor:
+    """fp32 log decays [T, N] from a [T, rank] (may be strided), with
+    z = a w2^T + bias: "sigmoid": log sigmoid(z) / tau; "softplus":
+    -rate * softplus(z), rate [N]; "exp": -e^z of z = tanh(a) w2^T + bias."""
     if not a.is_cuda:
-        return ref.decay_logs(a, w2, bias, kind, tau)
+        return ref.decay_logs(a, w2, bias, kind, tau, rate)
     out = torch.empty(a.shape[0], w2.shape[0], dtype=torch.float32, device=a.device)
-    hybrid_native().decay_logs(out, a, w2, bias, kind == "exp", float(tau))
+    hybrid_native().decay_logs(out, a, w2, bias, DECAY_KINDS[kind], float(tau), rate)
     return out
 
 
@@ -593,6 +596,147 @@ def decayed_kv(q, k, v, logw, u, qscale: float, H: int, dk: int, dv: int, S, pos
         ext.decay_chunked(*args, *ch.maps)
     else:
         ext.decay_scan(*args, None)
+    return y
+
+
+# --------------------------------------------------- hyper-connected streams
+def embed_rms_norm(tokens, embed, w, eps: float) -> torch.Tensor:
+    """fp32 RMS norm(embed[token]) * w."""
+    if not embed.is_cuda:
+        return ref.embed_rms_norm(tokens, embed, w, eps)
+    x = torch.empty(tokens.shape[0], embed.shape[1], dtype=torch.float32, device=embed.device)
+    hybrid_native().embed_rms_norm(x, tokens, embed, w, float(eps))
+    return x
+
+
+def mix_streams(x, pending, coef, rewrite: bool, w, eps: float, dtype):
+    """Linear combinations of the rows x[:, s] (fp32 [T, streams, W]) and of
+    the pending sublayer outputs, (y [T, W], scale [W] or None) each: coef
+    [streams + pending, columns]. Returns (streams, RMS norm of the last
+    column's * w in ``dtype``); the streams are the other columns with
+    ``rewrite`` (in x's memory where it fits), x as it is without."""
+    if not x.is_cuda:
+        return ref.mix_streams(x, pending, coef, rewrite, w, eps, dtype)
+    T, S, W = x.shape
+    out = x
+    if rewrite and coef.shape[1] - 1 != S:
+        out = torch.empty(T, coef.shape[1] - 1, W, dtype=torch.float32, device=x.device)
+    h = torch.empty(T, W, dtype=dtype, device=x.device)
+    ys, scales = [y for y, _ in pending], [s for _, s in pending]
+    hybrid_native().mix_streams(h, out if rewrite else None, x, ys, scales, coef, w, float(eps))
+    return out, h
+
+
+def xielu_(z: torch.Tensor, pos: float, neg: float) -> torch.Tensor:
+    """z = pos z^2 + z/2 where z > 0, neg (e^z - 1 - z) + z/2 else, in place."""
+    if not z.is_cuda:
+        return ref.xielu_(z, pos, neg)
+    hybrid_native().xielu(z, float(pos), float(neg))
+    return z
+
+
+# ------------------------ rotary attention in a window, differential or plain
+def rotary_rows(q, k, v, q_norm, k_norm, eps: float, cos_sin, positions, k_pages, v_pages,
+                slot_mapping) -> torch.Tensor:
+    """RMS norm of every dim = q_norm.numel() values of q (returned) and k,
+    then the rotation of the first cos_sin.shape[1] of them in halves; keys
+    and values go to their cache slots (k None: another layer wrote them).
+    q, k, v may be strided."""
+    if not q.is_cuda:
+        return ref.rotary_rows(q, k, v, q_norm, k_norm, eps, cos_sin, positions, k_pages,
+                               v_pages, slot_mapping)
+    out = torch.empty(q.shape, dtype=q.dtype, device=q.device)
+    hybrid_native().rotary_rows(
+        out, q, k, v, q_norm, k_norm, float(eps), cos_sin, positions,
+        *((k_pages, v_pages, slot_mapping) if k is not None else (None, None, None)),
+    )
+    return out
+
+
+def window_attention(out, q, k_pages, v_pages, H: int, G: int, maps: int, scale: float,
+                     window: int, keep_first: int, lam: float, gain: float, eps: float,
+                     positions, segs, plan: SegmentPlan) -> None:
+    """Softmax attention of every row to its sequence's pages: a row at
+    position p sees j <= p with p - j < window or j < keep_first. A head has
+    ``maps`` (1 or 2) queries, a key head as many keys, all over the same
+    values: with one, out is its output; with two, a1 and a2, it is the RMS
+    norm of a1 - lam a2 over the head, times gain. q and out [T, H*vdim] may
+    be strided."""
+    window, keep_first = min(int(window), 1 << 30), min(int(keep_first), 1 << 30)
+    if not q.is_cuda:
+        return ref.window_attention(
+            out, q, k_pages, v_pages, H, G, maps, scale, window, keep_first, lam, gain, eps,
+            positions, segs,
+        )
+    ext = hybrid_native()
+    page = k_pages.shape[1]
+    dim, vdim = k_pages.shape[2] // (G * maps), v_pages.shape[2] // G
+    head = (out, q, k_pages, v_pages, H, G, maps, float(scale), window, keep_first, float(lam),
+            float(gain), float(eps), positions)
+    mfma = (
+        q.dtype == torch.bfloat16 and page >= 16 and page & (page - 1) == 0
+        and dim % 8 == 0 and vdim % 8 == 0 and dim * maps <= 256 and vdim <= 256
+    )
+    rows, n = None, q.shape[0]
+    if mfma and plan.tiles is not None:
+        t = plan.tiles
+        ext.window_tiles(
+            *head, segs.tables, segs.cu, t.tile_seg, t.tile_off, t.tile_rows
+        )
+        if t.rest is None:
+            return
+        rows, n = t.rest, t.rest.numel()
+    nsplit, pa, pm = 0, None, None
+    if mfma:
+        # fill the chip: splits only from shapes, so captured graphs hold
+        groups = n * G * -(-(H // G) * maps // 16)
+        most = -(-min(segs.tables.shape[1] * page, window + keep_first + 62) // 128)
+        nsplit = max(1, min(-(-512 // groups), 16, most))
+        if nsplit > 1:
+            cols = n * H * maps * nsplit
+            pa, pm = _folded_scratch(q.device, cols * vdim, cols * 2)
+    ext.window_rows(*head, segs.row_seg, segs.tables, rows, nsplit, pa, pm)
+
+
+# -------------------------------------------------- fixed decays, the delta rule
+def fixed_decay_kv(q, k, v, decay, H: int, dk: int, dv: int, S, positions, segs,
+                   plan: SegmentPlan) -> torch.Tensor:
+    """S = decay[h] S + k v^T per head on silu(q), silu(k), silu(v), read out
+    by q after the update. q, k, v may be strided and are consumed; S [slots,
+    H, dv, dk]."""
+    if not q.is_cuda:
+        return ref.fixed_decay_kv(q, k, v, decay, H, dk, dv, S, positions, segs)
+    y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    ext, ch = hybrid_native(), plan.chunks
+    args = (y, q, k, v, decay, H, dk, dv, S, positions, segs.cu, segs.slots)
+    if ch is not None and dk % 8 == 0 and dv % 8 == 0:
+        if ch.short is not None:
+            ext.fixed_scan(*args, ch.short)
+        for x in (q, k, v):
+            ext.silu(x)
+        ext.fixed_chunked(*args, *ch.maps)
+    else:
+        ext.fixed_scan(*args, None)
+    return y
+
+
+def delta_kv(q, k, v, logw, b, H: int, G: int, dk: int, dv: int, S, positions, segs,
+             plan: SegmentPlan) -> torch.Tensor:
+    """Gated delta rule per head: S = diag(e^logw) S, u = sigmoid(b) (v - S^T
+    k), S += k u^T, o = S^T q, on q and k [T, G*dk] divided by their lengths
+    (q also by sqrt(dk)); G divides H. q, k, v, b may be strided; logw [T,
+    H*dk] fp32 is consumed; S [slots, H, dv, dk]."""
+    if not q.is_cuda:
+        return ref.delta_kv(q, k, v, logw, b, H, G, dk, dv, S, positions, segs)
+    y = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    ext, ch = hybrid_native(), plan.chunks
+    args = (y, q, k, v, logw, b, H, G, dk, dv, S, positions, segs.cu, segs.slots)
+    if ch is not None and dk % 8 == 0 and dv % 8 == 0 and dk <= 256:
+        if ch.short is not None:
+            ext.delta_scan(*args, ch.short)
+        ext.delta_chunked(*args, *ch.maps)
+    else:
+        ext.delta_scan(*args, None)
     return y
 
 

@@ -7,15 +7,30 @@ rows; attention gathers its keys from the pages.
 
 from __future__ import annotations
 
+import math
+
 import torch
 import torch.nn.functional as F
 
 
-def build_pair_rope_cache(max_positions, dims, base, device="cpu") -> torch.Tensor:
+def build_pair_rope_cache(
+    max_positions, dims, base, device="cpu", scaling=None
+) -> torch.Tensor:
     """[max_positions, dims] fp32: dims/2 cosines, then dims/2 sines, of
     position * base^(-2i/dims). Angles are taken in float64: at position
-    p a fp32 angle is off by up to p * 2^-24."""
+    p a fp32 angle is off by up to p * 2^-24.
+
+    scaling (factor, low, high, original): frequencies that turn less than
+    ``low`` times within ``original`` positions are divided by ``factor``,
+    those that turn more than ``high`` times stay, linear in between."""
     inv = base ** (-torch.arange(0, dims, 2, dtype=torch.float64, device=device) / dims)
+    if scaling is not None:
+        turns = scaling["original"] * inv / (2.0 * math.pi)
+        low, high = scaling["low"], scaling["high"]
+        keep = (turns > high).double()
+        if high > low:
+            keep = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+        inv = inv * (keep + (1.0 - keep) / scaling["factor"])
     ang = torch.outer(torch.arange(max_positions, dtype=torch.float64, device=device), inv)
     return torch.cat([ang.cos(), ang.sin()], -1).float().contiguous()
 
@@ -266,9 +281,11 @@ def sigmoid_attention(out, q, k_pages, v_pages, H, G, scale, bias, talk, window,
 
 
 # ------------------------------------- recurrences with a decay per channel
-def decay_logs(a, w2, bias, kind, tau):
+def decay_logs(a, w2, bias, kind, tau, rate):
     a = torch.tanh(a.float()) if kind == "exp" else a.float()
     z = a @ w2.float().t() + bias
+    if kind == "softplus":
+        return -rate * F.softplus(z, threshold=1e9)
     return -torch.exp(z) if kind == "exp" else F.logsigmoid(z) / tau
 
 
@@ -311,10 +328,107 @@ def decayed_kv(q, k, v, logw, u, qscale, H, dk, dv, S, positions, segs):
     return y.view(T, H * dv).to(q.dtype)
 
 
-def head_norm_gate(out, y, gate, w, heads, eps):
+def head_norm_gate(out, y, gate, w, heads, eps, act):
     T, W = y.shape
     yf = _rms(y.float().view(T, heads, W // heads), eps).view(T, W) * w
-    out.copy_(yf * F.silu(gate.float()))
+    g = gate.float()
+    out.copy_(yf * (F.silu(g) if act == "silu" else torch.sigmoid(g)))
+
+
+# ------------------------------------------------------ hyper-connected streams
+def embed_rms_norm(tokens, embed, w, eps):
+    return _rms(embed[tokens].float(), eps) * w
+
+
+def mix_streams(x, pending, coef, rewrite, w, eps, dtype):
+    rows = [x[:, s] for s in range(x.shape[1])]
+    rows += [y.float() if scale is None else y.float() * scale for y, scale in pending]
+    out = torch.einsum("rtw,rc->tcw", torch.stack(rows), coef)
+    h = (_rms(out[:, -1], eps) * w).to(dtype)
+    return (out[:, :-1].contiguous() if rewrite else x), h
+
+
+def xielu_(z, pos, neg):
+    f = z.float()
+    n = f.clamp(max=0)
+    return z.copy_(torch.where(f > 0, pos * f * f, neg * (torch.expm1(n) - n)) + 0.5 * f)
+
+
+# ------------------------- rotary attention in a window, differential or plain
+def rotate_halves(x, positions, cos_sin):
+    """x [T, heads, D] fp32: dimensions i and i + dims/2 of the first
+    dims = cos_sin's width are a pair."""
+    half = cos_sin.shape[1] // 2
+    cs = cos_sin[positions][:, None]
+    c, s = cs[..., :half], cs[..., half:]
+    u, v = x[..., :half], x[..., half : 2 * half]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half :]], -1)
+
+
+def rotary_rows(q, k, v, q_norm, k_norm, eps, cos_sin, positions, k_pages, v_pages,
+                slot_mapping):
+    T, dim = q.shape[0], q_norm.numel()
+
+    def rows(x, w):
+        x = _rms(x.float().reshape(T, -1, dim), eps) * w
+        return rotate_halves(x, positions, cos_sin).reshape(T, -1).to(q.dtype)
+
+    if k is not None:
+        page_write(rows(k, k_norm), v, k_pages, v_pages, slot_mapping)
+    return rows(q, q_norm)
+
+
+def window_attention(out, q, k_pages, v_pages, H, G, maps, scale, window, keep_first, lam, gain,
+                     eps, positions, segs):
+    T, bs, per = q.shape[0], k_pages.shape[1], H // G
+    dim, vdim = k_pages.shape[2] // (G * maps), v_pages.shape[2] // G
+    for t in range(T):
+        p = int(positions[t])
+        lo = max(0, p - window + 1)
+        keys = torch.cat([torch.arange(min(lo, keep_first)), torch.arange(lo, p + 1)])
+        slots = segs.tables[int(segs.row_seg[t])].long()[keys // bs] * bs + keys % bs
+        k = k_pages.view(-1, G, maps, dim)[slots].float().repeat_interleave(per, 1)
+        v = v_pages.view(-1, G, vdim)[slots].float().repeat_interleave(per, 1)
+        s = torch.einsum("hmd,nhmd->hmn", q[t].float().view(H, maps, dim), k) * scale
+        o = torch.einsum("hmn,nhd->hmd", torch.softmax(s, -1), v)
+        o = o[:, 0] if maps == 1 else _rms(o[:, 0] - lam * o[:, 1], eps) * gain
+        out[t] = o.reshape(-1)
+
+
+# ----------------------------------------------- fixed decays, the delta rule
+def fixed_decay_kv(q, k, v, decay, H, dk, dv, S, positions, segs):
+    w = decay.log().clamp(min=-80.0)[:, None].expand(H, dk).reshape(1, -1)
+    return decayed_kv(
+        F.silu(q.float()), F.silu(k.float()), F.silu(v.float()), w.expand(q.shape[0], -1), None,
+        1.0, H, dk, dv, S, positions, segs,
+    ).to(q.dtype)
+
+
+def delta_kv(q, k, v, logw, b, H, G, dk, dv, S, positions, segs):
+    T = q.shape[0]
+
+    def unit(x):
+        x = x.float().reshape(T, G, dk)
+        x = x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + 1e-6)
+        return x.repeat_interleave(H // G, 1)
+
+    qf, kf, vf = unit(q) * dk ** -0.5, unit(k), v.float().reshape(T, H, dv)
+    w, beta = torch.exp(logw).view(T, H, 1, dk), torch.sigmoid(b.float())
+    y = torch.zeros(T, H, dv)
+    cu = segs.cu.tolist()
+    for s, slot in enumerate(segs.slots.tolist()):
+        if slot < 0:
+            continue
+        st = S[slot].clone()  # [H, dv, dk]
+        if int(positions[cu[s]]) == 0:
+            st.zero_()
+        for t in range(cu[s], cu[s + 1]):
+            st = w[t] * st
+            new = beta[t][:, None] * (vf[t] - (st * kf[t][:, None, :]).sum(-1))
+            st = st + new[:, :, None] * kf[t][:, None, :]
+            y[t] = (st * qf[t][:, None, :]).sum(-1)
+        S[slot] = st
+    return y.view(T, H * dv).to(q.dtype)
 
 
 # ------------------------------------------------------------------- experts
