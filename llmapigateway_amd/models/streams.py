@@ -25,7 +25,7 @@ DEFER = 4  # pending outputs from which reading them again costs what a rewrite 
 
 
 class Read(NamedTuple):
-    """coef [stored + pending, columns] fp32: the last column is what the
+    """coef [stored + pending, columns] fp32: the first column is what the
     sublayer reads; with ``rewrite`` the others are the new streams."""
 
     coef: torch.Tensor
@@ -45,7 +45,7 @@ class HyperStreams:
             read = rows @ w_in[:, None]
             rewrite = len(pending) >= DEFER and mix is not None
             self.reads.append(Read(
-                (torch.cat([rows, read], 1) if rewrite else read).float().contiguous().to(device),
+                (torch.cat([read, rows], 1) if rewrite else read).float().contiguous().to(device),
                 rewrite,
             ))
             if mix is None:

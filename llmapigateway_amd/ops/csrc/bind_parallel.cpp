@@ -9,14 +9,14 @@ extern "C" {
 hipError_t launch_stream_tanh(void*, int64_t, float*, const void*, int, const void*, const void*, const int*, const float*, int, const float*, const float*, float, const float*, const float*, float, int, int, int, int, int, hipStream_t);
 hipError_t launch_embed_tanh(float*, void*, int64_t, const int64_t*, const void*, const float*, const float*, float, int, int, int, int, hipStream_t);
 hipError_t launch_token_shift(void*, const void*, const float*, int, void*, const int64_t*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
-hipError_t launch_head_norm(void*, int64_t, const void*, const void*, int64_t, const float*, float, int, int, int, int, hipStream_t);
+hipError_t launch_head_norm(void*, int64_t, const void*, const void*, int64_t, const float*, float, int, int, int, int, int, hipStream_t);
 hipError_t launch_gated_norm(void*, int64_t, const void*, const void*, int64_t, const float*, float, int, int, int, int, int, int, hipStream_t);
 hipError_t launch_page_write(void*, void*, const void*, int64_t, const void*, int64_t, const int64_t*, int, int, int, int, int, hipStream_t);
 hipError_t launch_clamped_glu(void*, const void*, float, int, int, int, int, hipStream_t);
 hipError_t launch_soft_cap(float*, float, size_t, hipStream_t);
 hipError_t launch_paged_rows(void*, int64_t, const void*, int64_t, const void*, const void*, const float*, const void*, int64_t, float, float, float, const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, int, int, float*, float*, int, hipStream_t);
 hipError_t launch_paged_tiles(void*, int64_t, const void*, int64_t, const void*, const void*, const float*, const void*, int64_t, float, float, float, const int64_t*, const int*, int, int, int, int, int, int, const int*, const int*, const int*, int, int, hipStream_t);
-hipError_t launch_decay_logs(float*, const void*, int64_t, const void*, const float*, int, float, int, int, int, int, int, hipStream_t);
+hipError_t launch_decay_logs(float*, const void*, int64_t, const void*, const float*, const float*, int, float, int, int, int, int, int, hipStream_t);
 hipError_t launch_decay_scan(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*, const float*, float, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, int, int, hipStream_t);
 hipError_t launch_decay_chunked(void*, const void*, int64_t, const void*, int64_t, const void*, int64_t, float*, const float*, float, int, int, int, int, float*, const int64_t*, const int*, const int*, const int*, const int*, const int*, const int*, int, int, void*, hipStream_t);
 hipError_t launch_route_topk(int*, float*, const float*, const float*, float, int, int, int, hipStream_t);
@@ -116,7 +116,8 @@ void token_shift(Tensor out, Tensor h, Tensor mu, Tensor prev, Tensor positions,
 }
 
 // out = rms(y) per head * w * silu(gate)
-void head_norm_gate(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t heads, double eps) {
+void head_norm_gate(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t heads, double eps,
+                    bool sigmoid) {
     const bool f32 = is_f32(y, "y");
     same_type(y, gate, "gate");
     same_type(y, out, "out");
@@ -128,12 +129,13 @@ void head_norm_gate(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t heads, 
     const bool v = vec8({&out, &y, &gate, &w}, {gs});
     if (v && gs <= 512)
         CHECK_HIP(launch_head_norm(out.data_ptr(), out.stride(0), y.data_ptr(), gate.data_ptr(),
-                                   gate.stride(0), f32_ptr(w, W, "w"), (float)eps, heads, gs, T,
-                                   f32, current_stream()));
+                                   gate.stride(0), f32_ptr(w, W, "w"), (float)eps, heads, gs,
+                                   sigmoid, T, f32, current_stream()));
     else
         CHECK_HIP(launch_gated_norm(out.data_ptr(), out.stride(0), y.data_ptr(),
                                     gate.data_ptr(), gate.stride(0), f32_ptr(w, W, "w"),
-                                    (float)eps, heads, gs, 2, T, f32, v, current_stream()));
+                                    (float)eps, heads, gs, sigmoid ? 0 : 2, T, f32, v,
+                                    current_stream()));
 }
 
 void page_write(Tensor k, Tensor v, Tensor k_pages, Tensor v_pages, Tensor slot_mapping) {
@@ -220,17 +222,22 @@ void paged_tiles(Tensor out, Tensor q, Tensor k, Tensor v, int64_t H, int64_t G,
         current_stream()));
 }
 
-void decay_logs(Tensor out, Tensor a, Tensor w2, Tensor bias, bool exp_form, double tau) {
+// kind 0: log sigmoid(z) / tau, 1: -e^z, 2: -rate softplus(z)
+void decay_logs(Tensor out, Tensor a, Tensor w2, Tensor bias, int64_t kind, double tau,
+                OptTensor rate) {
     const bool f32 = is_f32(a, "a");
     same_type(a, w2, "w2");
     TORCH_CHECK(w2.dim() == 2 && w2.is_contiguous() && tau > 0);
+    TORCH_CHECK(kind >= 0 && kind <= 2 && has(rate) == (kind == 2));
     const int64_t T = a.size(0), N = w2.size(0), R = w2.size(1);
     check_rows(a, T, R, "a");
     f32_ptr(out, T * N, "out");
     const bool v = vec8({&a, &w2}, {R}) && N % 4 == 0 &&
-                   reinterpret_cast<uintptr_t>(bias.data_ptr()) % 16 == 0;
+                   reinterpret_cast<uintptr_t>(bias.data_ptr()) % 16 == 0 &&
+                   (kind != 2 || reinterpret_cast<uintptr_t>(rate->data_ptr()) % 16 == 0);
     CHECK_HIP(launch_decay_logs(out.data_ptr<float>(), a.data_ptr(), a.stride(0),
-                                w2.data_ptr(), f32_ptr(bias, N, "bias"), exp_form,
+                                w2.data_ptr(), f32_ptr(bias, N, "bias"),
+                                kind == 2 ? f32_ptr(*rate, N, "rate") : nullptr, kind,
                                 (float)(1.0 / tau), T, N, R, f32, v, current_stream()));
 }
 
@@ -368,7 +375,7 @@ void bind_parallel(pybind11::module_& m) {
     m.def("stream_tanh", &stream_tanh, "stream add + dynamic tanh");
     m.def("embed_tanh", &embed_tanh, "embedding + dynamic tanh into the fp32 stream");
     m.def("token_shift", &token_shift, "mixes of every row with the previous one");
-    m.def("head_norm_gate", &head_norm_gate, "head-wise RMS norm with a silu gate");
+    m.def("head_norm_gate", &head_norm_gate, "head-wise RMS norm with a silu or sigmoid gate");
     m.def("page_write", &page_write, "keys and values into cache pages");
     m.def("paged_rows", &paged_rows, "attention over pages, row by row");
     m.def("paged_tiles", &paged_tiles, "attention over pages, tiles of prompt rows");

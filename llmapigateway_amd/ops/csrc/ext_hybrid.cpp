@@ -7,6 +7,7 @@
 
 void bind_parallel(pybind11::module_& m);  // bind_parallel.cpp
 void bind_sigmoid(pybind11::module_& m);   // bind_sigmoid.cpp
+void bind_streams(pybind11::module_& m);   // bind_streams.cpp
 
 extern "C" {
 hipError_t launch_embed_scaled(float*, void*, int64_t, const int64_t*, const void*, float, int, int, int, int, hipStream_t);
@@ -370,5 +371,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("gated_norm", &gated_norm, "group RMS norm with a gate");
     bind_parallel(m);
     bind_sigmoid(m);
+    bind_streams(m);
     bind_shared(m);
 }

@@ -69,3 +69,30 @@ __device__ __forceinline__ void split_bf16(float v, uint16_t& hi, uint16_t& lo) 
     hi = f2bfbits(v);
     lo = f2bfbits(v - bfbits2f(hi));
 }
+// fp32 values as the sum of two bf16 fragments
+__device__ __forceinline__ void split_frag(const float* f, bf16x8& hi, bf16x8& lo) {
+    uint4 h, l;
+    uint32_t* hp = reinterpret_cast<uint32_t*>(&h);
+    uint32_t* lp = reinterpret_cast<uint32_t*>(&l);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        hp[i] = cvt_pk_bf16(f[2 * i], f[2 * i + 1]);
+        float a, b;
+        unpack2(hp[i], a, b);
+        lp[i] = cvt_pk_bf16(f[2 * i] - a, f[2 * i + 1] - b);
+    }
+    hi = as_frag(h);
+    lo = as_frag(l);
+}
+__device__ __forceinline__ void unpack8(const uint4& v, float* f) {
+    unpack2(v.x, f[0], f[1]);
+    unpack2(v.y, f[2], f[3]);
+    unpack2(v.z, f[4], f[5]);
+    unpack2(v.w, f[6], f[7]);
+}
+__device__ __forceinline__ void load8f(const float* p, float* f) {
+    const float4 a = reinterpret_cast<const float4*>(p)[0];
+    const float4 b = reinterpret_cast<const float4*>(p)[1];
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+}

@@ -1,5 +1,6 @@
-// Gated linear recurrences for gfx950, token by token: Mamba-2 (SSD) and
-// mLSTM over the segments of a flat batch, state in fp32.
+// Linear recurrences for gfx950, token by token: Mamba-2 (SSD), mLSTM and
+// fixed decays (lightning attention) over the segments of a flat batch, state
+// in fp32.
 //
 // A state matrix is kept transposed, [value dim][key dim], key dim dense: 16
 // lanes share a value row and hold its key dims as float4s, so state traffic
@@ -13,12 +14,15 @@
 #define SCAN_ROWS 64  // value rows per workgroup
 
 // ---------------------------------------------------------------------------
-// MLSTM = false: S <- exp(-e^A dt) S + dt x B^T, y = S C + D x
-// MLSTM = true:  S, n with log gates i, f and running maximum m;
-//                y = S q / (max(|n.q|, e^-m) + 1e-6)
+// SCAN_SSD:   S <- exp(-e^A dt) S + dt x B^T, y = S C + D x
+// SCAN_MLSTM: S, n with log gates i, f and running maximum m;
+//             y = S q / (max(|n.q|, e^-m) + 1e-6)
+// SCAN_FIXED: S <- decay S + silu(v) silu(k)^T, y = S silu(q)
 // Every 64-row tile of S keeps its own copy of n and m (they are read by
 // every tile and written at the end).
 // ---------------------------------------------------------------------------
+enum { SCAN_SSD, SCAN_MLSTM, SCAN_FIXED };
+
 struct ScanArgs {
     void* y;              // [T, H*dv]
     const void* q;        // SSD: C        rows of stride ldq, head stride via group
@@ -27,7 +31,7 @@ struct ScanArgs {
     int64_t ldq, ldk, ldv;
     const float* gates;   // SSD: raw dt [T, H]; mLSTM: raw i | f [T, 2H]
     const float* bias;    // SSD: dt_bias [H]; mLSTM: [2H]
-    const float* A_log;   // SSD [H]
+    const float* A_log;   // SSD [H]; fixed: the decays
     const float* D;       // SSD [H]
     float cap, qscale;
     int H, per_group, dk, dv;
@@ -40,9 +44,12 @@ struct ScanArgs {
     const int* seg_list;  // nullable: the segments to run
 };
 
-template <typename T, int E4, bool MLSTM>
+__device__ __forceinline__ float scan_silu(float z) { return z / (1.f + expf(-z)); }
+
+template <typename T, int E4, int KIND>
 __launch_bounds__(256)
 __global__ void scan_kernel(ScanArgs a) {
+    constexpr bool MLSTM = KIND == SCAN_MLSTM;
     const int seg = a.seg_list ? a.seg_list[blockIdx.x] : blockIdx.x;
     const int h = blockIdx.y, tile = blockIdx.z, tiles = gridDim.z;
     const int slot = a.slots[seg];
@@ -94,7 +101,19 @@ __global__ void scan_kernel(ScanArgs a) {
         const T* vp = (const T*)a.v + (size_t)t * a.ldv + (size_t)h * dv;
 #pragma unroll
         for (int r = 0; r < 4; ++r) v[r] = row0 + r < dv ? ldf(vp + row0 + r) : 0.f;
-        if (MLSTM) {
+        if (KIND == SCAN_FIXED) {
+#pragma unroll
+            for (int e = 0; e < E4; ++e)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    k[e][j] = scan_silu(k[e][j]);
+                    q[e][j] = scan_silu(q[e][j]);
+                }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = scan_silu(v[r]);
+            keep = a.A_log[h];
+            add = 1.f;
+        } else if (MLSTM) {
             const float* g = a.gates + (size_t)t * 2 * H;
             const float i = soft_cap_f(g[h] + a.bias[h], a.cap);
             const float f = log_sigmoid_f(soft_cap_f(g[H + h] + a.bias[H + h], a.cap));
@@ -134,7 +153,7 @@ __global__ void scan_kernel(ScanArgs a) {
                 }
             o[r] = row16_sum(s);
         }
-        const float dh = MLSTM ? 0.f : a.D[h];
+        const float dh = KIND == SCAN_SSD ? a.D[h] : 0.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r)
             if (l16 == r && row0 + r < dv)
@@ -151,13 +170,13 @@ __global__ void scan_kernel(ScanArgs a) {
     }
 }
 
-template <typename T, bool MLSTM>
+template <typename T, int KIND>
 static hipError_t scan_go(const ScanArgs& a, int nseg, hipStream_t stream) {
     const dim3 grid(nseg, a.H, ceil_div_i(a.dv, SCAN_ROWS));
-    if (a.dk <= 64) scan_kernel<T, 1, MLSTM><<<grid, 256, 0, stream>>>(a);
-    else if (a.dk <= 128) scan_kernel<T, 2, MLSTM><<<grid, 256, 0, stream>>>(a);
-    else if (a.dk <= 256) scan_kernel<T, 4, MLSTM><<<grid, 256, 0, stream>>>(a);
-    else if (a.dk <= 512) scan_kernel<T, 8, MLSTM><<<grid, 256, 0, stream>>>(a);
+    if (a.dk <= 64) scan_kernel<T, 1, KIND><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 128) scan_kernel<T, 2, KIND><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 256) scan_kernel<T, 4, KIND><<<grid, 256, 0, stream>>>(a);
+    else if (a.dk <= 512) scan_kernel<T, 8, KIND><<<grid, 256, 0, stream>>>(a);
     else return hipErrorInvalidValue;
     HIP_CHECK_LAST();
     return hipSuccess;
@@ -179,7 +198,7 @@ extern "C" hipError_t launch_ssd_scan(
     a.gates = dt; a.bias = dt_bias; a.A_log = A_log; a.D = D;
     a.H = H; a.per_group = H / G; a.dk = N; a.dv = P;
     a.S = S; a.positions = positions; a.cu = cu; a.slots = slots; a.seg_list = seg_list;
-    return f32 ? scan_go<float, false>(a, nseg, stream) : scan_go<bf16, false>(a, nseg, stream);
+    return f32 ? scan_go<float, SCAN_SSD>(a, nseg, stream) : scan_go<bf16, SCAN_SSD>(a, nseg, stream);
 }
 
 extern "C" hipError_t launch_mlstm_scan(
@@ -194,5 +213,18 @@ extern "C" hipError_t launch_mlstm_scan(
     a.H = H; a.per_group = 1; a.dk = dk; a.dv = dv;
     a.S = S; a.n = n; a.m = m;
     a.positions = positions; a.cu = cu; a.slots = slots; a.seg_list = seg_list;
-    return f32 ? scan_go<float, true>(a, nseg, stream) : scan_go<bf16, true>(a, nseg, stream);
+    return f32 ? scan_go<float, SCAN_MLSTM>(a, nseg, stream) : scan_go<bf16, SCAN_MLSTM>(a, nseg, stream);
+}
+
+extern "C" hipError_t launch_fixed_scan(
+    void* y, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
+    int64_t ldv, const float* decay, int H, int dk, int dv, float* S,
+    const int64_t* positions, const int* cu, const int* slots, const int* seg_list, int nseg,
+    int f32, hipStream_t stream) {
+    if (nseg <= 0) return hipSuccess;
+    ScanArgs a = {};
+    a.y = y; a.q = q; a.k = k; a.v = v; a.ldq = ldq; a.ldk = ldk; a.ldv = ldv;
+    a.A_log = decay; a.H = H; a.per_group = 1; a.dk = dk; a.dv = dv; a.S = S;
+    a.positions = positions; a.cu = cu; a.slots = slots; a.seg_list = seg_list;
+    return f32 ? scan_go<float, SCAN_FIXED>(a, nseg, stream) : scan_go<bf16, SCAN_FIXED>(a, nseg, stream);
 }

@@ -1,6 +1,7 @@
-// Gated linear recurrences for gfx950 in chunks of 64 rows, on MFMA (bf16
-// data, fp32 state): the prompt form of recurrence.hip's scan. With the
-// chunk's inclusive sums F of the log decays,
+// Linear recurrences for gfx950 in chunks of 64 rows, on MFMA (bf16 data,
+// fp32 state): the prompt form of recurrence.hip's scan. Fixed decays are the
+// SSD form with dt = 1 and D = 0, on rows that silu has gone over already. With
+// the chunk's inclusive sums F of the log decays,
 //
 //   SSD:   P[t,s] = (q_t.k_s) e^(F_t-F_s) dt_s
 //          y_t    = sum_{s<=t} P[t,s] v_s + e^(F_t) S_in q_t + D v_t
@@ -57,7 +58,7 @@ __device__ __forceinline__ float wave_scan_max(float v, int lane) {
 }
 
 // a wave per (chunk, head), a lane per row
-template <bool MLSTM>
+template <bool MLSTM, bool FIXED = false>
 __global__ void chunk_gates_kernel(ChunkArgs a) {
     const int c = blockIdx.x, lane = threadIdx.x & 63;
     const int h = blockIdx.y * 4 + (threadIdx.x >> 6);
@@ -67,7 +68,11 @@ __global__ void chunk_gates_kernel(ChunkArgs a) {
     float decay = 0.f, in = 0.f;
     if (lane < n) {
         const size_t t = r0 + lane;
-        if (MLSTM) {
+        if (FIXED) {
+            // e^-80 is as good as 0, and sums of 64 of them keep their precision
+            decay = fmaxf(logf(a.A_log[h]), -80.f);
+            in = 1.f;
+        } else if (MLSTM) {
             const float* g = a.gates + t * 2 * H;
             in = soft_cap_f(g[h] + a.bias[h], a.cap);
             decay = log_sigmoid_f(soft_cap_f(g[H + h] + a.bias[H + h], a.cap));
@@ -405,7 +410,7 @@ __global__ void chunk_out_kernel(ChunkArgs a) {
             o[j] = mfma16(pl, vf, o[j]);
         }
     }
-    const float skip = MLSTM ? 0.f : a.D[h];
+    const float skip = MLSTM || a.D == nullptr ? 0.f : a.D[h];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int t = wave * 16 + g * 4 + r;
@@ -420,13 +425,13 @@ __global__ void chunk_out_kernel(ChunkArgs a) {
     }
 }
 
-template <bool MLSTM>
+template <bool MLSTM, bool FIXED = false>
 static hipError_t chunked_go(const ChunkArgs& a, int nsegs, int nchunks, hipStream_t stream) {
     if (nchunks <= 0) return hipSuccess;
     if (a.dk % 8 || a.dv % 8 || a.ldq % 8 || a.ldk % 8 || a.ldv % 8)
         return hipErrorInvalidValue;
     const int vt = ceil_div_i(a.dv, 64), kt = ceil_div_i(a.dk, 64);
-    chunk_gates_kernel<MLSTM><<<dim3(nchunks, ceil_div_i(a.H, 4)), 256, 0, stream>>>(a);
+    chunk_gates_kernel<MLSTM, FIXED><<<dim3(nchunks, ceil_div_i(a.H, 4)), 256, 0, stream>>>(a);
     HIP_CHECK_LAST();
     state_pass_kernel<MLSTM><<<dim3(nsegs, a.H, vt * kt), 256, 0, stream>>>(a);
     HIP_CHECK_LAST();
@@ -482,4 +487,23 @@ extern "C" hipError_t launch_mlstm_chunked(
     a.s_lo = a.s_hi + (size_t)nchunks * H * dv * dk;
     a.n_in = n_in; a.m_in = m_in;
     return chunked_go<true>(a, nsegs, nchunks, stream);
+}
+
+extern "C" hipError_t launch_fixed_chunked(
+    void* y, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
+    int64_t ldv, const float* decay, int T, int H, int dk, int dv, float* S,
+    const int64_t* positions, const int* cu, const int* slots, const int* segs,
+    const int* first, const int* chunk_seg, const int* chunk_off, int nsegs, int nchunks,
+    float* Fb, void* planes, hipStream_t stream) {
+    ChunkArgs a = {};
+    a.y = (bf16*)y; a.q = (const bf16*)q; a.k = (const bf16*)k; a.v = (const bf16*)v;
+    a.ldq = ldq; a.ldk = ldk; a.ldv = ldv;
+    a.A_log = decay;
+    a.T = T; a.H = H; a.per_group = 1; a.dk = dk; a.dv = dv; a.S = S;
+    a.positions = positions; a.cu = cu; a.slots = slots; a.segs = segs; a.first = first;
+    a.chunk_seg = chunk_seg; a.chunk_off = chunk_off;
+    a.F = Fb; a.b = Fb + (size_t)H * T;
+    a.s_hi = (uint16_t*)planes;
+    a.s_lo = a.s_hi + (size_t)nchunks * H * dv * dk;
+    return chunked_go<false, true>(a, nsegs, nchunks, stream);
 }

@@ -24,67 +24,45 @@
 #define CH 64  // rows per chunk
 #define LDT (CH + 8)
 
-// fp32 values as the sum of two bf16 fragments
-__device__ __forceinline__ void split_frag(const float* f, bf16x8& hi, bf16x8& lo) {
-    uint4 h, l;
-    uint32_t* hp = reinterpret_cast<uint32_t*>(&h);
-    uint32_t* lp = reinterpret_cast<uint32_t*>(&l);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        hp[i] = cvt_pk_bf16(f[2 * i], f[2 * i + 1]);
-        float a, b;
-        unpack2(hp[i], a, b);
-        lp[i] = cvt_pk_bf16(f[2 * i] - a, f[2 * i + 1] - b);
-    }
-    hi = as_frag(h);
-    lo = as_frag(l);
-}
-__device__ __forceinline__ void unpack8(const uint4& v, float* f) {
-    unpack2(v.x, f[0], f[1]);
-    unpack2(v.y, f[2], f[3]);
-    unpack2(v.z, f[4], f[5]);
-    unpack2(v.w, f[6], f[7]);
-}
-__device__ __forceinline__ void load8f(const float* p, float* f) {
-    const float4 a = reinterpret_cast<const float4*>(p)[0];
-    const float4 b = reinterpret_cast<const float4*>(p)[1];
-    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
-    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
-}
-
 // ---------------------------------------------------------------------------
 // log decays from z = act(a) W2^T + bias
-//   EXP:  act = tanh, log w = -e^z          (w = exp(-exp(z)))
-//   else: act = id,   log w = log sigmoid(z) / tau
+//   LOG_EXP:      act = tanh, log w = -e^z            (w = exp(-exp(z)))
+//   LOG_SIGMOID:  act = id,   log w = log sigmoid(z) * c,   c = 1 / tau
+//   LOG_SOFTPLUS: act = id,   log w = -softplus(z) * c,     c = rate[channel]
 // ---------------------------------------------------------------------------
-template <bool EXP>
-__device__ __forceinline__ float log_decay(float z, float inv_tau) {
+enum { LOG_SIGMOID, LOG_EXP, LOG_SOFTPLUS };
+
+template <int KIND>
+__device__ __forceinline__ float log_decay(float z, float c) {
     // e^-80 is as good as 0, and sums of 64 of them keep their precision
-    return fmaxf(EXP ? -expf(z) : log_sigmoid_f(z) * inv_tau, -80.f);
+    if (KIND == LOG_EXP) return fmaxf(-expf(z), -80.f);
+    return fmaxf(log_sigmoid_f(KIND == LOG_SOFTPLUS ? -z : z) * c, -80.f);
 }
 
 // the same for bf16 steps, whose z has bf16 rounding in it: hardware exponential
 // and logarithm, log(1 + x) by its series where x is small
-template <bool EXP>
-__device__ __forceinline__ float log_decay_fast(float z, float inv_tau) {
-    if (EXP) return fmaxf(-__expf(z), -80.f);
+template <int KIND>
+__device__ __forceinline__ float log_decay_fast(float z, float c) {
+    if (KIND == LOG_EXP) return fmaxf(-__expf(z), -80.f);
+    if (KIND == LOG_SOFTPLUS) z = -z;
     const float x = __expf(-fabsf(z));
     const float l = x < 0.02f ? x * (1.f + x * (-0.5f + x * (1.f / 3.f))) : __logf(1.f + x);
-    return fmaxf((fminf(z, 0.f) - l) * inv_tau, -80.f);
+    return fmaxf((fminf(z, 0.f) - l) * c, -80.f);
 }
 
 #define DL_ROWS 8
-template <typename T, bool EXP>
+template <typename T, int KIND>
 __launch_bounds__(256)
 __global__ void decay_logs_any_kernel(
     float* __restrict__ out, const T* __restrict__ a, int64_t lda, const T* __restrict__ w2,
-    const float* __restrict__ bias, float inv_tau, int rows, int N, int R) {
+    const float* __restrict__ bias, const float* __restrict__ rate, float inv_tau, int rows,
+    int N, int R) {
     extern __shared__ float act[];  // [DL_ROWS][R]
     const int t0 = blockIdx.x * DL_ROWS, n = blockIdx.y * 256 + threadIdx.x;
     for (int e = threadIdx.x; e < DL_ROWS * R; e += 256) {
         const int t = t0 + e / R;
         const float v = t < rows ? ldf(a + (size_t)t * lda + e % R) : 0.f;
-        act[e] = EXP ? tanhf(v) : v;
+        act[e] = KIND == LOG_EXP ? tanhf(v) : v;
     }
     __syncthreads();
     if (n >= N) return;
@@ -98,16 +76,19 @@ __global__ void decay_logs_any_kernel(
     }
 #pragma unroll
     for (int i = 0; i < DL_ROWS; ++i)
-        if (t0 + i < rows) out[(size_t)(t0 + i) * N + n] = log_decay<EXP>(z[i], inv_tau);
+        if (t0 + i < rows)
+            out[(size_t)(t0 + i) * N + n] =
+                log_decay<KIND>(z[i], KIND == LOG_SOFTPLUS ? rate[n] : inv_tau);
 }
 
 // MFMA form: a wave takes 16 rows x 64 channels; C fragments hold [channel][row]
-template <bool EXP>
+template <int KIND>
 __launch_bounds__(256)
 __global__ void decay_logs_mfma_kernel(
     float* __restrict__ out, const bf16* __restrict__ a, int64_t lda,
-    const bf16* __restrict__ w2, const float* __restrict__ bias, float inv_tau, int rows,
-    int N, int R) {
+    const bf16* __restrict__ w2, const float* __restrict__ bias,
+    const float* __restrict__ rate, float inv_tau, int rows, int N, int R) {
+    constexpr bool EXP = KIND == LOG_EXP;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, g = lane >> 4;
     const int t = (blockIdx.x * 4 + wave) * 16 + r16, n0 = blockIdx.y * 64;
     if ((blockIdx.x * 4 + wave) * 16 >= rows) return;
@@ -141,9 +122,11 @@ __global__ void decay_logs_mfma_kernel(
         const int n = n0 + j * 16 + g * 4;
         if (n >= N) continue;  // N is a multiple of 4
         const float4 b = *reinterpret_cast<const float4*>(bias + n);
+        float4 c = make_float4(inv_tau, inv_tau, inv_tau, inv_tau);
+        if (KIND == LOG_SOFTPLUS) c = *reinterpret_cast<const float4*>(rate + n);
         *reinterpret_cast<float4*>(out + (size_t)t * N + n) = make_float4(
-            log_decay_fast<EXP>(acc[j][0] + b.x, inv_tau), log_decay_fast<EXP>(acc[j][1] + b.y, inv_tau),
-            log_decay_fast<EXP>(acc[j][2] + b.z, inv_tau), log_decay_fast<EXP>(acc[j][3] + b.w, inv_tau));
+            log_decay_fast<KIND>(acc[j][0] + b.x, c.x), log_decay_fast<KIND>(acc[j][1] + b.y, c.y),
+            log_decay_fast<KIND>(acc[j][2] + b.z, c.z), log_decay_fast<KIND>(acc[j][3] + b.w, c.w));
     }
 }
 
@@ -611,34 +594,46 @@ __global__ void decay_out_kernel(DecayArgs a) {
 // ---------------------------------------------------------------------------
 // vec: bf16, R a multiple of 8, N of 4, rows aligned for 16-byte loads
 extern "C" hipError_t launch_decay_logs(
-    float* out, const void* a, int64_t lda, const void* w2, const float* bias, int exp_form,
-    float inv_tau, int rows, int N, int R, int f32, int vec, hipStream_t stream) {
+    float* out, const void* a, int64_t lda, const void* w2, const float* bias,
+    const float* rate, int kind, float inv_tau, int rows, int N, int R, int f32, int vec,
+    hipStream_t stream) {
     if (rows <= 0) return hipSuccess;
-    if (!f32 && vec) {
-        const dim3 grid(ceil_div_i(rows, 64), ceil_div_i(N, 64));
-        if (exp_form)
-            decay_logs_mfma_kernel<true><<<grid, 256, 0, stream>>>(
-                out, (const bf16*)a, lda, (const bf16*)w2, bias, inv_tau, rows, N, R);
-        else
-            decay_logs_mfma_kernel<false><<<grid, 256, 0, stream>>>(
-                out, (const bf16*)a, lda, (const bf16*)w2, bias, inv_tau, rows, N, R);
-        HIP_CHECK_LAST();
-        return hipSuccess;
-    }
-    const dim3 grid(ceil_div_i(rows, DL_ROWS), ceil_div_i(N, 256));
-    const size_t lds = (size_t)DL_ROWS * R * sizeof(float);
+    if (kind < LOG_SIGMOID || kind > LOG_SOFTPLUS || (kind == LOG_SOFTPLUS) != (rate != nullptr))
+        return hipErrorInvalidValue;
+    const bool mfma = !f32 && vec;
+    const dim3 grid = mfma ? dim3(ceil_div_i(rows, 64), ceil_div_i(N, 64))
+                           : dim3(ceil_div_i(rows, DL_ROWS), ceil_div_i(N, 256));
+    const size_t lds = mfma ? 0 : (size_t)DL_ROWS * R * sizeof(float);
     if (lds > 48 * 1024) return hipErrorInvalidValue;
-#define GO(T, E)                                                              \
-    decay_logs_any_kernel<T, E><<<grid, 256, lds, stream>>>(                  \
-        out, (const T*)a, lda, (const T*)w2, bias, inv_tau, rows, N, R)
-    if (f32) {
-        if (exp_form) GO(float, true);
-        else GO(float, false);
-    } else {
-        if (exp_form) GO(bf16, true);
-        else GO(bf16, false);
+#define GO(K)                                                                            \
+    {                                                                                    \
+        if (mfma)                                                                        \
+            decay_logs_mfma_kernel<K><<<grid, 256, 0, stream>>>(                         \
+                out, (const bf16*)a, lda, (const bf16*)w2, bias, rate, inv_tau, rows, N, R); \
+        else if (f32)                                                                    \
+            decay_logs_any_kernel<float, K><<<grid, 256, lds, stream>>>(                 \
+                out, (const float*)a, lda, (const float*)w2, bias, rate, inv_tau, rows, N, R); \
+        else                                                                             \
+            decay_logs_any_kernel<bf16, K><<<grid, 256, lds, stream>>>(                  \
+                out, (const bf16*)a, lda, (const bf16*)w2, bias, rate, inv_tau, rows, N, R); \
     }
+    if (kind == LOG_EXP) GO(LOG_EXP)
+    else if (kind == LOG_SOFTPLUS) GO(LOG_SOFTPLUS)
+    else GO(LOG_SIGMOID)
 #undef GO
+    HIP_CHECK_LAST();
+    return hipSuccess;
+}
+
+// F in place: the sums of logw [T, N] within every chunk of 64 rows
+extern "C" hipError_t launch_decay_sums(
+    float* logw, int N, const int* cu, const int* chunk_seg, const int* chunk_off, int nchunks,
+    hipStream_t stream) {
+    if (nchunks <= 0) return hipSuccess;
+    DecayArgs a = {};
+    a.logw = logw; a.H = 1; a.dk = N;
+    a.cu = cu; a.chunk_seg = chunk_seg; a.chunk_off = chunk_off;
+    decay_sums_kernel<<<dim3(nchunks, ceil_div_i(N, 256)), 256, 0, stream>>>(a);
     HIP_CHECK_LAST();
     return hipSuccess;
 }

@@ -13,6 +13,10 @@ __device__ __forceinline__ float tanh_of(float z) {
     return sizeof(T) == 4 ? tanhf(z) : tanh_fast(z);
 }
 template <typename T>
+__device__ __forceinline__ float sigmoid_of(float z) {
+    return sizeof(T) == 4 ? sigmoid_f(z) : 1.f / (1.f + __expf(-z));
+}
+template <typename T>
 __device__ __forceinline__ float silu_of(float z) {
     return sizeof(T) == 4 ? z * sigmoid_f(z) : z / (1.f + __expf(-z));
 }
@@ -162,10 +166,10 @@ __global__ void shift_state_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// out = rms(y) * w * silu(gate) per head of gs values: LG lanes a head, 8
-// values a lane, several heads a wave
+// out = rms(y) * w * silu(gate) (or sigmoid(gate)) per head of gs values: LG
+// lanes a head, 8 values a lane, several heads a wave
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, bool SIGMOID>
 __launch_bounds__(256)
 __global__ void head_norm_kernel(
     T* __restrict__ out, int64_t ld_out, const T* __restrict__ y, const T* __restrict__ gate,
@@ -188,7 +192,8 @@ __global__ void head_norm_kernel(
     load_vec<8>(gate + t * ld_gate + c, z);
     load_vec<8>(w + c, wv);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) f[j] *= inv * wv[j] * silu_of<T>(z[j]);
+    for (int j = 0; j < 8; ++j)
+        f[j] *= inv * wv[j] * (SIGMOID ? sigmoid_of<T>(z[j]) : silu_of<T>(z[j]));
     store_vec<8>(out + t * ld_out + c, f);
 }
 
@@ -307,7 +312,8 @@ extern "C" hipError_t launch_token_shift(
 // gs a multiple of 8, at most 512; everything aligned for 8-element accesses
 extern "C" hipError_t launch_head_norm(
     void* out, int64_t ld_out, const void* y, const void* gate, int64_t ld_gate,
-    const float* w, float eps, int groups, int gs, int rows, int f32, hipStream_t stream) {
+    const float* w, float eps, int groups, int gs, int sigmoid, int rows, int f32,
+    hipStream_t stream) {
     if (rows <= 0) return hipSuccess;
     if (gs % 8 || gs > 512) return hipErrorInvalidValue;
     int lg = 1;
@@ -316,7 +322,8 @@ extern "C" hipError_t launch_head_norm(
     const unsigned blocks = (unsigned)((total * lg + 255) / 256);
     return pick(f32, 1, [&](auto form) {
         FORM(form);
-        head_norm_kernel<T><<<blocks, 256, 0, stream>>>(
+        auto kernel = sigmoid ? head_norm_kernel<T, true> : head_norm_kernel<T, false>;
+        kernel<<<blocks, 256, 0, stream>>>(
             (T*)out, ld_out, (const T*)y, (const T*)gate, ld_gate, w, eps, groups, gs, lg, total);
     });
 }

@@ -612,7 +612,7 @@ def embed_rms_norm(tokens, embed, w, eps: float) -> torch.Tensor:
 def mix_streams(x, pending, coef, rewrite: bool, w, eps: float, dtype):
     """Linear combinations of the rows x[:, s] (fp32 [T, streams, W]) and of
     the pending sublayer outputs, (y [T, W], scale [W] or None) each: coef
-    [streams + pending, columns]. Returns (streams, RMS norm of the last
+    [streams + pending, columns]. Returns (streams, RMS norm of the first
     column's * w in ``dtype``); the streams are the other columns with
     ``rewrite`` (in x's memory where it fits), x as it is without."""
     if not x.is_cuda:

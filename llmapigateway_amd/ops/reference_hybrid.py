@@ -344,8 +344,8 @@ def mix_streams(x, pending, coef, rewrite, w, eps, dtype):
     rows = [x[:, s] for s in range(x.shape[1])]
     rows += [y.float() if scale is None else y.float() * scale for y, scale in pending]
     out = torch.einsum("rtw,rc->tcw", torch.stack(rows), coef)
-    h = (_rms(out[:, -1], eps) * w).to(dtype)
-    return (out[:, :-1].contiguous() if rewrite else x), h
+    h = (_rms(out[:, 0], eps) * w).to(dtype)
+    return (out[:, 1:].contiguous() if rewrite else x), h
 
 
 def xielu_(z, pos, neg):

@@ -24,7 +24,9 @@ SOURCES = {
     "_H": ["ext_hybrid.cpp", "hybrid_rows.hip", "head_linear.hip", "attention_latent.hip",
            "recurrence.hip", "recurrence_chunked.hip", "bind_parallel.cpp", "tanh_rows.hip",
            "attention_paged.hip", "recurrence_decay.hip", "experts.hip", "bind_sigmoid.cpp",
-           "rms_rows.hip", "attention_sigmoid.hip", "activation.hip", "gemm_skinny.hip"],
+           "rms_rows.hip", "attention_sigmoid.hip", "bind_streams.cpp", "stream_rows.hip",
+           "attention_window.hip", "recurrence_delta.hip", "activation.hip",
+           "gemm_skinny.hip"],
 }
 wanted = os.environ.get("LLMAPI_EXT", "_C,_H").split(",")
 
