@@ -64,7 +64,8 @@ def parse_args():
         "width, feed-forward (of experts: what a token uses) and number of "
         "layer runs",
     )
-    p.add_argument("--family", default="lelisun", choices=["lelisun", "filinex", "mekevik"],
+    p.add_argument("--family", default="lelisun",
+                   choices=["lelisun", "filinex", "mekevik", "duratar"],
                    help="--mode layers: whose presets")
     p.add_argument("--sizes", default="small,base",
                    help="--mode layers: <family>-<size> presets, or any hybrid model")
@@ -200,7 +201,7 @@ class StepDriver:
 def run_layers(args) -> None:
     """Prefill and decode tokens/s of a hybrid decoder at a few sizes, each
     beside the closest dense model at equal width: as many Llama layers as
-    the hybrid runs layers, a feed-forward as wide as what a token uses."""
+    the hybrid runs layers, a feed-forward of the weights that a token uses."""
     device = "cuda:0" if torch.cuda.is_available() else "cpu"
     context = args.decode_context
     batches = [int(b) for b in args.decode_batches.split(",") if b]
@@ -210,7 +211,8 @@ def run_layers(args) -> None:
     def llama_like(c):
         m = next(e.mlp for e in c.layers if e.mlp)
         ff = m["ff"] if m["kind"] == "dense" else (
-            m["router"]["top"] * m["expert"]["ff"] + m.get("shared", {}).get("ff", 0))
+            m["router"]["top"] * m["expert"]["ff"] + m.get("shared", {}).get("ff", 0)
+        ) if m["kind"] == "moe" else m["ff"] * 2 // 3  # two matrices against a GLU's three
         heads = c.hidden_size // 128 or 1
         return ModelConfig(
             name=f"llama of {c.name}", hidden_size=c.hidden_size, intermediate_size=ff,

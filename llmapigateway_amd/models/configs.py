@@ -583,18 +583,19 @@ MODEL_PRESETS = {
     "tiny-duratar": _duratar_preset(
         "tiny-duratar", width=96, vocab=320, heads=4, kv_heads=2, dim=16, window=24,
         keep_first=3, delta_heads=4, delta_kv_heads=2, delta_dim=24, delta_vdim=40, rank=8,
-        mem_heads=3, mem_dim=16, ff=112, streams=3, layers=6, max_positions=1024,
+        mem_heads=3, mem_dim=16, ff=96, streams=3, layers=6, max_positions=1024,
     ),
-    # layers as wide as llama-1b's and llama-3-8b's
+    # layers as wide as llama-1b's and llama-3-8b's, feed-forwards of as many
+    # weights (two matrices instead of three)
     "duratar-small": _duratar_preset(
         "duratar-small", width=2048, vocab=128256, heads=16, kv_heads=4, dim=64, window=1024,
         keep_first=16, delta_heads=16, delta_kv_heads=16, delta_dim=128, delta_vdim=128,
-        rank=128, mem_heads=16, mem_dim=128, ff=8192, streams=4, layers=12,
+        rank=128, mem_heads=16, mem_dim=128, ff=12288, streams=4, layers=12,
     ),
     "duratar-base": _duratar_preset(
         "duratar-base", width=4096, vocab=128256, heads=32, kv_heads=8, dim=64, window=1024,
         keep_first=16, delta_heads=32, delta_kv_heads=32, delta_dim=128, delta_vdim=128,
-        rank=128, mem_heads=32, mem_dim=128, ff=14336, streams=4, layers=16,
+        rank=128, mem_heads=32, mem_dim=128, ff=21504, streams=4, layers=16,
     ),
     # small-but-real shape for 1-GPU kernel shakedown
     "llama-1b": ModelConfig(

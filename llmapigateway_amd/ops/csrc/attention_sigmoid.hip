@@ -113,20 +113,6 @@ __device__ __forceinline__ float sigmoid_2(float s2) {
 }
 __device__ __forceinline__ float gate_2(float z) { return sigmoid_2(z * LOG2E); }
 
-// 8 fp32 as bf16 fragments of their leading and remaining halves
-__device__ __forceinline__ void split_frag(const float* f, bf16x8& hi, bf16x8& lo) {
-    uint4 h, l;
-    uint32_t *hp = &h.x, *lp = &l.x;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        float a, b;
-        hp[i] = cvt_pk_bf16(f[2 * i], f[2 * i + 1]);
-        unpack2(hp[i], a, b);
-        lp[i] = cvt_pk_bf16(f[2 * i] - a, f[2 * i + 1] - b);
-    }
-    hi = as_frag(h);
-    lo = as_frag(l);
-}
 __device__ __forceinline__ bf16x8 masked(bool keep, const bf16x8& f) {
     uint4 v = *reinterpret_cast<const uint4*>(&f);
     if (!keep) v = (uint4){0, 0, 0, 0};

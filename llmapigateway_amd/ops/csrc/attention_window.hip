@@ -452,10 +452,17 @@ __global__ void window_tiles_kernel(
     const int pos_last = ctx + min(nq, off + 16 * MR * NW) - 1;  // of the workgroup's rows
     const KeyTiles kt(ctx + off, pos_last, a.window, a.keep, 64);
     uint4 kreg[KV], vreg[VV];
+    int page[4];  // of the tile that is loaded next, per 16 keys: looked up a tile ahead
+    auto look_up = [&](int it) {
+        const int k0 = kt.key(min(it, kt.count - 1), 64);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) page[u] = bt[min(k0 + u * 16, pos_last) >> page_shift];
+    };
     auto load_tile = [&](int k0) {
-        auto row_of = [&](int key) {
-            key = min(key, pos_last);
-            return ((size_t)bt[key >> page_shift] << page_shift) + (key & mask);
+        auto row_of = [&](int o) {  // past the last key: any row
+            const int key = min(k0 + o, pos_last), u = (key - k0) >> 4;
+            const int p = u == 0 ? page[0] : u == 1 ? page[1] : u == 2 ? page[2] : page[3];
+            return ((size_t)p << page_shift) + (key & mask);
         };
 #pragma unroll
         for (int c = 0; c < KV; ++c) {
@@ -463,7 +470,7 @@ __global__ void window_tiles_kernel(
             kreg[c] = (uint4){0, 0, 0, 0};
             if (d < KD)
                 kreg[c] = *reinterpret_cast<const uint4*>(
-                    kp + row_of(k0 + e / (LQ / 8)) * a.G * KD + d);
+                    kp + row_of(e / (LQ / 8)) * a.G * KD + d);
         }
 #pragma unroll
         for (int c = 0; c < VV; ++c) {
@@ -471,11 +478,13 @@ __global__ void window_tiles_kernel(
             vreg[c] = (uint4){0, 0, 0, 0};
             if (d < a.vdim)
                 vreg[c] = *reinterpret_cast<const uint4*>(
-                    vp + row_of(k0 + e / (NDV * 2)) * a.G * a.vdim + d);
+                    vp + row_of(e / (NDV * 2)) * a.G * a.vdim + d);
         }
     };
     const int wp0 = ctx + wrow0, wp1 = wp0 + 16 * MR - 1;  // this wave's positions
+    look_up(0);
     load_tile(kt.key(0, 64));
+    look_up(1);
     for (int it = 0; it < kt.count; ++it) {
         const int k0 = kt.key(it, 64);
         __syncthreads();
@@ -490,7 +499,10 @@ __global__ void window_tiles_kernel(
             *reinterpret_cast<uint4*>(v_lds + e / (NDV * 2) * LDV + e % (NDV * 2) * 8) = vreg[c];
         }
         __syncthreads();
-        if (it + 1 < kt.count) load_tile(kt.key(it + 1, 64));
+        if (it + 1 < kt.count) {
+            load_tile(kt.key(it + 1, 64));
+            look_up(it + 2);
+        }
         // no row of this wave sees a key of the tile
         if (k0 > wp1 || (wp0 - (k0 + 63) >= a.window && k0 >= a.keep)) continue;
         const bool edge =  // some row does not see all keys
@@ -702,7 +714,6 @@ extern "C" hipError_t launch_window_tiles(
 #define GO(A, B, P)                                                                      \
     {                                                                                    \
         if (tile_rows == 64) GO3(A, B, 1, 4, P);                                         \
-        else if (B <= 8) GO3(A, B, (B <= 8 ? 2 : 1), (B <= 8 ? 4 : 8), P);               \
         else GO3(A, B, 1, 8, P);                                                         \
     }
     if (maps == 2) {

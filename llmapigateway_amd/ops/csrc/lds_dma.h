@@ -23,3 +23,12 @@ __device__ __forceinline__ void dma16(const bf16* src, const bf16* lds) {
     asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
                  ::"s"(at), "v"(src) : "memory", "m0");
 }
+// The same with everything but the lane's part uniform: 16 bytes a lane from
+// base + offset (bytes) to LDS byte address lds + 16*lane.
+__device__ __forceinline__ uint32_t lds_address(const void* p) {
+    return (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) char*)p;
+}
+__device__ __forceinline__ void dma16(const void* base, uint32_t offset, uint32_t lds) {
+    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2"
+                 ::"s"(lds), "v"(offset), "s"(base) : "memory", "m0");
+}

@@ -33,7 +33,7 @@
 #define CH 64  // rows per chunk
 #define LDT (CH + 8)
 #define STAGE 4096      // bf16 values of a transfer stage: 8 fragments
-#define RING 8          // stages in LDS
+#define RING 8          // stages in LDS, a power of two
 #define MAX_SPREAD 60.f
 
 struct DeltaArgs {
@@ -435,22 +435,26 @@ __global__ void delta_intra_kernel(DeltaArgs a) {
         f32x4 xt[2][4];
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
-            const int d = kk * 32 + u * 16 + r16;
+            const int d = kk * 32 + u * 16 + r16, dd = min(d, dk - 1);
             const bool in = d < dk;
-            const float Fl = in ? Fp[(size_t)(n - 1) * N + d] : 0.f;
+            const float Fl = Fp[(size_t)(n - 1) * N + dd];
             f32x4 R[4], K[4], x[4];
 #pragma unroll
             for (int i = 0; i < 4; ++i)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
+                    const int t = i * 16 + g * 4 + r, tt = min(t, n - 1);
+                    R[i][r] = Fp[(size_t)tt * N + dd];
+                    K[i][r] = ldf(kp + (size_t)tt * a.ldk + dd);
+                }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
                     const int t = i * 16 + g * 4 + r;
-                    R[i][r] = K[i][r] = 0.f;
-                    if (in && t < n) {
-                        const float k = ldf(kp + (size_t)t * a.ldk + d) * rk_lds[t];
-                        const float F = Fp[(size_t)t * N + d];
-                        R[i][r] = k * b_lds[t] * __expf(F);
-                        K[i][r] = k * __expf(Fl - F);
-                    }
+                    const float F = R[i][r], k = in && t < n ? K[i][r] * rk_lds[t] : 0.f;
+                    R[i][r] = k * b_lds[t] * __expf(F);
+                    K[i][r] = k * __expf(Fl - F);
                 }
 #pragma unroll
             for (int ks = 0; ks < 2; ++ks) {
@@ -472,15 +476,18 @@ __global__ void delta_intra_kernel(DeltaArgs a) {
     const int nvg = (dv + 31) / 32;
     float* u0 = a.u0 + ((size_t)c * H + h) * nvg * 2048;
     for (int vt = wave; vt < 2 * nvg; vt += 4) {
-        const int d = vt * 16 + r16;
+        const int d = vt * 16 + r16, dd = min(d, dv - 1);
         f32x4 R[4], x[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = i * 16 + g * 4 + r;
-                R[i][r] = d < dv && t < n ? ldf(vp + (size_t)t * a.ldv + d) * b_lds[t] : 0.f;
-            }
+            for (int r = 0; r < 4; ++r)
+                R[i][r] = ldf(vp + (size_t)min(i * 16 + g * 4 + r, n - 1) * a.ldv + dd);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)  // (rows past the last have a beta of 0)
+                R[i][r] = d < dv ? R[i][r] * b_lds[i * 16 + g * 4 + r] : 0.f;
         solve(R, x, nullptr);
 #pragma unroll
         for (int i = 0; i < 4; ++i)
@@ -499,6 +506,7 @@ template <int NC>
 __launch_bounds__(128)
 __global__ void delta_state_kernel(DeltaArgs a) {
     constexpr int NS = 3 * NC + 3;
+    static_assert((NS + RING - 1) / NS < 3, "chunks that stages are sent for");
     __shared__ __align__(16) bf16 ring[RING][STAGE];
     const int seg = a.segs[blockIdx.x], h = blockIdx.y, vg = blockIdx.z, nvg = gridDim.z;
     const int dk = a.dk, dv = a.dv, H = a.H;
@@ -516,82 +524,108 @@ __global__ void delta_state_kernel(DeltaArgs a) {
         S[j] = zero4();
         if (!fresh && v0 + r16 < dv && d < dk) S[j] = *reinterpret_cast<const f32x4*>(Sp + d);
     }
-    // the next stage to send for; past the last one, that one again
-    int to_chunk = c_lo, to_stage = 0, to_slot = 0;
-    auto send = [&]() {
-        const size_t ch = (size_t)to_chunk * H + h;
-        const bf16* src = to_stage == 0
-            ? reinterpret_cast<const bf16*>(a.u0 + (ch * nvg + vg) * 2048)
-            : a.frags + (ch * (3 * NC + 2) + to_stage - 1) * STAGE;
+    // Stages are numbered from the chunk that is being read; which one a
+    // position in the code sends for is known there. Past the segment's last
+    // chunk, that one again.
+    const bf16* fr[3];
+    const float* u0[3];
+    auto point = [&](int c) {
 #pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            const int at = wave * 2048 + u * 512;
-            dma16(src + at + lane * 8, &ring[to_slot][at]);
-        }
-        to_slot = to_slot + 1 == RING ? 0 : to_slot + 1;
-        if (to_stage + 1 < NS) {
-            ++to_stage;
-        } else if (to_chunk + 1 < c_hi) {
-            ++to_chunk;
-            to_stage = 0;
+        for (int i = 0; i < 3; ++i) {
+            const size_t ch = (size_t)min(c + i, c_hi - 1) * H + h;
+            fr[i] = a.frags + ch * (3 * NC + 2) * STAGE;
+            u0[i] = a.u0 + (ch * nvg + vg) * 2048;
         }
     };
-    int slot_in = 0;
-    // the next stage's data, here for both waves; the stage before has been read
-    auto next = [&]() -> const bf16* {
-        static_assert(4 * (RING - 2) == 24, "transfers that may be under way");
-        asm volatile("s_waitcnt vmcnt(24) lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        send();
-        const bf16* p = ring[slot_in];
-        slot_in = slot_in + 1 == RING ? 0 : slot_in + 1;
+    const uint32_t ring_at = lds_address(ring) + wave * 4096, lane_at = wave * 4096 + lane * 16;
+    uint32_t to_slot = 0, in_slot = 0;
+    auto send = [&](int stage) {
+        const int q = stage / NS, r = stage % NS;
+        const void* src = r == 0 ? (const void*)u0[q] : (const void*)(fr[q] + (r - 1) * STAGE);
+        const uint32_t to = ring_at + to_slot * (STAGE * 2);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) dma16(src, lane_at + u * 1024, to + u * 1024);
+        to_slot = (to_slot + 1) % RING;
+    };
+    // the data of stage j, here for both waves; the stage before it has been read
+    auto next = [&](int j) -> const bf16* {
+        // the transfers of later stages may be under way
+        asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(4 * (RING - 2)) : "memory");
+        send(j + RING - 1);
+        const bf16* p = ring[in_slot];
+        in_slot = (in_slot + 1) % RING;
         return p;
     };
-    auto frag = [&](const bf16* st, int i) {
-        return *reinterpret_cast<const bf16x8*>(st + i * 512 + lane * 8);
+    // a stage's fragments, read while the products of the stage before run
+    struct Stage {
+        bf16x8 f[8];
     };
-    for (int i = 0; i < RING - 1; ++i) send();
+    auto read = [&](Stage& x, const bf16* st, int first, int count) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            if (i < count)
+                x.f[i] = *reinterpret_cast<const bf16x8*>(st + (first + i) * 512 + lane * 8);
+    };
+    // c[i] += (hi + lo of x.f[2i], x.f[2i+1]) (bh + bl), or with the operands
+    // the other way round; the three products of a sum lie apart
+    auto products = [&](f32x4* c, const Stage& x, int n_c, bf16x8 bh, bf16x8 bl, bool left) {
+#pragma unroll
+        for (int p = 0; p < 3; ++p)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (i >= n_c) continue;
+                const bf16x8 m = x.f[2 * i + (p == 2)], b = p == 1 ? bl : bh;
+                c[i] = left ? mfma16(m, b, c[i]) : mfma16(b, m, c[i]);
+            }
+    };
+    point(c_lo);
+#pragma unroll
+    for (int i = 0; i < RING - 1; ++i) send(i);
+    Stage now, ahead;
+    read(ahead, next(0), wave * 4, 4);
     for (int c = c_lo; c < c_hi; ++c) {
         const int r0 = row_lo + (c - c_lo) * CH, n = min(CH, row_hi - r0);
-        f32x4 U[4], o[4];
-        const bf16* st = next();
+        point(c);
+        f32x4 U[4], o[4], keep[2 * NC];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            U[i] = *reinterpret_cast<const f32x4*>(
-                reinterpret_cast<const float*>(st) + wave * 1024 + i * 256 + lane * 4);
+            U[i] = *reinterpret_cast<const f32x4*>(&ahead.f[i]);
             o[i] = zero4();
         }
+        read(ahead, next(1), 0, 8);
         bf16x8 sh[NC], sl[NC];
 #pragma unroll
         for (int kk = 0; kk < NC; ++kk) split_pair(S[2 * kk], S[2 * kk + 1], sh[kk], sl[kk]);
 #pragma unroll
-        for (int kk = 0; kk < NC; ++kk) {
-            st = next();
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-                U[i] = mfma3(frag(st, i * 2), frag(st, i * 2 + 1), sh[kk], sl[kk], U[i]);
+        for (int kk = 0; kk < NC; ++kk) {  // W: [row][dv]
+            now = ahead;
+            read(ahead, next(2 + kk), 0, 8);
+            products(U, now, 4, sh[kk], sl[kk], true);
         }
 #pragma unroll
-        for (int kk = 0; kk < NC; ++kk) {  // [dv][row]
-            st = next();
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-                o[i] = mfma3(sh[kk], sl[kk], frag(st, i * 2), frag(st, i * 2 + 1), o[i]);
+        for (int kk = 0; kk < NC; ++kk) {  // Q: [dv][row]
+            now = ahead;
+            read(ahead, next(2 + NC + kk), 0, 8);
+            products(o, now, 4, sh[kk], sl[kk], false);
         }
         bf16x8 uh[2], ul[2];
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) split_pair(U[2 * ks], U[2 * ks + 1], uh[ks], ul[ks]);
-        st = next();
+        now = ahead;
+        {
+            const bf16* st = next(2 + 2 * NC);
+            read(ahead, st, 0, 4);
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-            o[i] = mfma3(uh[0], ul[0], frag(st, i * 2), frag(st, i * 2 + 1), o[i]);
-        st = next();
+            for (int j = 0; j < 2 * NC; ++j)
+                keep[j] = *reinterpret_cast<const f32x4*>(
+                    reinterpret_cast<const float*>(st + 2048) + j * 16 + g * 4);
+        }
+        products(o, now, 4, uh[0], ul[0], false);
+        now = ahead;
+        read(ahead, next(3 + 2 * NC), 0, 8);
+        products(o + 2, now, 2, uh[1], ul[1], false);
 #pragma unroll
-        for (int i = 2; i < 4; ++i)
-            o[i] = mfma3(uh[1], ul[1], frag(st, i * 2 - 4), frag(st, i * 2 - 3), o[i]);
-#pragma unroll
-        for (int j = 0; j < 2 * NC; ++j)
-            S[j] *= *reinterpret_cast<const f32x4*>(
-                reinterpret_cast<const float*>(st + 2048) + j * 16 + g * 4);
+        for (int j = 0; j < 2 * NC; ++j) S[j] *= keep[j];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int t = i * 16 + r16, d = v0 + g * 4;
@@ -601,13 +635,17 @@ __global__ void delta_state_kernel(DeltaArgs a) {
         }
 #pragma unroll
         for (int kk = 0; kk < NC; ++kk) {
-            st = next();
+            now = ahead;
+            if (kk + 1 < NC) read(ahead, next(4 + 2 * NC + kk), 0, 8);
+            else read(ahead, next(NS), wave * 4, 4);  // the next chunk's U0
 #pragma unroll
-            for (int u = 0; u < 2; ++u)
+            for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
-                for (int ks = 0; ks < 2; ++ks)
-                    S[2 * kk + u] = mfma3(frag(st, u * 4 + ks * 2), frag(st, u * 4 + ks * 2 + 1),
-                                          uh[ks], ul[ks], S[2 * kk + u]);
+                for (int p = 0; p < 3; ++p)
+#pragma unroll
+                    for (int u = 0; u < 2; ++u)
+                        S[2 * kk + u] = mfma16(now.f[u * 4 + ks * 2 + (p == 2)],
+                                               p == 1 ? ul[ks] : uh[ks], S[2 * kk + u]);
         }
     }
     dma_barrier();  // nothing is on its way to LDS when the workgroup ends
