@@ -25,16 +25,20 @@ __device__ __forceinline__ void load_dims(const T* p, int l16, int dk, float (*f
             f[e][j] = i < dk ? ldf(p + i) : 0.f;
         }
 }
-template <int E4>
+// STREAM: state that a step reads and writes once, past the caches
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float state4;
+template <int E4, bool STREAM = false>
 __device__ __forceinline__ void load_state(
     const float* p, int l16, int dk, bool vec, float (*f)[4]) {
 #pragma unroll
     for (int e = 0; e < E4; ++e) {
         const int i = 64 * e + 4 * l16;
         if (vec) {
-            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (i < dk) v = *reinterpret_cast<const float4*>(p + i);
-            f[e][0] = v.x; f[e][1] = v.y; f[e][2] = v.z; f[e][3] = v.w;
+            state4 v = {0.f, 0.f, 0.f, 0.f};
+            const state4* at = reinterpret_cast<const state4*>(p + i);
+            if (i < dk) v = STREAM ? __builtin_nontemporal_load(at) : *at;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) f[e][j] = v[j];
         } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j) f[e][j] = i + j < dk ? p[i + j] : 0.f;
@@ -48,9 +52,10 @@ __device__ __forceinline__ void store_state(
     for (int e = 0; e < E4; ++e) {
         const int i = 64 * e + 4 * l16;
         if (vec) {
-            if (i < dk)
-                *reinterpret_cast<float4*>(p + i) =
-                    make_float4(f[e][0], f[e][1], f[e][2], f[e][3]);
+            if (i < dk) {
+                const state4 v = {f[e][0], f[e][1], f[e][2], f[e][3]};
+                __builtin_nontemporal_store(v, reinterpret_cast<state4*>(p + i));
+            }
         } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j)

@@ -50,8 +50,8 @@ template <typename T, int E4, int KIND>
 __launch_bounds__(256)
 __global__ void scan_kernel(ScanArgs a) {
     constexpr bool MLSTM = KIND == SCAN_MLSTM;
-    const int seg = a.seg_list ? a.seg_list[blockIdx.x] : blockIdx.x;
-    const int h = blockIdx.y, tile = blockIdx.z, tiles = gridDim.z;
+    const int seg = a.seg_list ? a.seg_list[blockIdx.z] : blockIdx.z;
+    const int h = blockIdx.y, tile = blockIdx.x, tiles = gridDim.x;
     const int slot = a.slots[seg];
     const int r0 = a.cu[seg], r1 = a.cu[seg + 1];
     const int l16 = threadIdx.x & 15, grp = threadIdx.x >> 4;
@@ -75,7 +75,7 @@ __global__ void scan_kernel(ScanArgs a) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         if (!fresh && row0 + r < dv) {
-            load_state<E4>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
+            load_state<E4, true>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
         } else {
 #pragma unroll
             for (int e = 0; e < E4; ++e)
@@ -172,7 +172,7 @@ __global__ void scan_kernel(ScanArgs a) {
 
 template <typename T, int KIND>
 static hipError_t scan_go(const ScanArgs& a, int nseg, hipStream_t stream) {
-    const dim3 grid(nseg, a.H, ceil_div_i(a.dv, SCAN_ROWS));
+    const dim3 grid(ceil_div_i(a.dv, SCAN_ROWS), a.H, nseg);  // neighbours share a state
     if (a.dk <= 64) scan_kernel<T, 1, KIND><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 128) scan_kernel<T, 2, KIND><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 256) scan_kernel<T, 4, KIND><<<grid, 256, 0, stream>>>(a);

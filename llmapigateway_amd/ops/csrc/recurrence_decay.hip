@@ -90,8 +90,8 @@ __global__ void decay_logs_mfma_kernel(
     const float* __restrict__ rate, float inv_tau, int rows, int N, int R) {
     constexpr bool EXP = KIND == LOG_EXP;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, g = lane >> 4;
-    const int t = (blockIdx.x * 4 + wave) * 16 + r16, n0 = blockIdx.y * 64;
-    if ((blockIdx.x * 4 + wave) * 16 >= rows) return;
+    const int t = (blockIdx.y * 4 + wave) * 16 + r16, n0 = blockIdx.x * 64;
+    if ((blockIdx.y * 4 + wave) * 16 >= rows) return;
     f32x4 acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -155,11 +155,11 @@ struct DecayArgs {
 template <typename T, int E4, bool WKV>
 __launch_bounds__(256)
 __global__ void decay_scan_kernel(DecayArgs a) {
-    const int seg = a.seg_list ? a.seg_list[blockIdx.x] : blockIdx.x;
+    const int seg = a.seg_list ? a.seg_list[blockIdx.z] : blockIdx.z;
     const int h = blockIdx.y, slot = a.slots[seg];
     const int r0 = a.cu[seg], r1 = a.cu[seg + 1];
     const int l16 = threadIdx.x & 15, grp = threadIdx.x >> 4;
-    const int row0 = blockIdx.z * 64 + grp * 4;
+    const int row0 = blockIdx.x * 64 + grp * 4;
     const int dk = a.dk, dv = a.dv, H = a.H;
     T* y = (T*)a.y + (size_t)h * dv;
     if (slot < 0) {  // padding row
@@ -173,7 +173,7 @@ __global__ void decay_scan_kernel(DecayArgs a) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         if (!fresh && row0 + r < dv) {
-            load_state<E4>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
+            load_state<E4, true>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
         } else {
 #pragma unroll
             for (int e = 0; e < E4; ++e)
@@ -601,7 +601,7 @@ extern "C" hipError_t launch_decay_logs(
     if (kind < LOG_SIGMOID || kind > LOG_SOFTPLUS || (kind == LOG_SOFTPLUS) != (rate != nullptr))
         return hipErrorInvalidValue;
     const bool mfma = !f32 && vec;
-    const dim3 grid = mfma ? dim3(ceil_div_i(rows, 64), ceil_div_i(N, 64))
+    const dim3 grid = mfma ? dim3(ceil_div_i(N, 64), ceil_div_i(rows, 64))
                            : dim3(ceil_div_i(rows, DL_ROWS), ceil_div_i(N, 256));
     const size_t lds = mfma ? 0 : (size_t)DL_ROWS * R * sizeof(float);
     if (lds > 48 * 1024) return hipErrorInvalidValue;
@@ -640,7 +640,7 @@ extern "C" hipError_t launch_decay_sums(
 
 template <typename T, bool WKV>
 static hipError_t decay_scan_go(const DecayArgs& a, int nseg, hipStream_t stream) {
-    const dim3 grid(nseg, a.H, ceil_div_i(a.dv, 64));
+    const dim3 grid(ceil_div_i(a.dv, 64), a.H, nseg);  // neighbours share a state
     if (a.dk <= 64) decay_scan_kernel<T, 1, WKV><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 128) decay_scan_kernel<T, 2, WKV><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 256) decay_scan_kernel<T, 4, WKV><<<grid, 256, 0, stream>>>(a);

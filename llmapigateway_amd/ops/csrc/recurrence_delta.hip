@@ -61,11 +61,11 @@ struct DeltaArgs {
 template <typename T, int E4>
 __launch_bounds__(256)
 __global__ void delta_scan_kernel(DeltaArgs a) {
-    const int seg = a.seg_list ? a.seg_list[blockIdx.x] : blockIdx.x;
+    const int seg = a.seg_list ? a.seg_list[blockIdx.z] : blockIdx.z;
     const int h = blockIdx.y, hk = h / a.per, slot = a.slots[seg];
     const int r0 = a.cu[seg], r1 = a.cu[seg + 1];
     const int l16 = threadIdx.x & 15, grp = threadIdx.x >> 4;
-    const int row0 = blockIdx.z * 64 + grp * 4;
+    const int row0 = blockIdx.x * 64 + grp * 4;
     const int dk = a.dk, dv = a.dv, H = a.H;
     T* y = (T*)a.y + (size_t)h * dv;
     if (slot < 0) {  // padding row
@@ -79,7 +79,7 @@ __global__ void delta_scan_kernel(DeltaArgs a) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         if (!fresh && row0 + r < dv) {
-            load_state<E4>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
+            load_state<E4, true>(Sp + (size_t)(row0 + r) * dk, l16, dk, vec, S[r]);
         } else {
 #pragma unroll
             for (int e = 0; e < E4; ++e)
@@ -661,7 +661,7 @@ __global__ void delta_state_kernel(DeltaArgs a) {
 // ---------------------------------------------------------------------------
 template <typename T>
 static hipError_t delta_scan_go(const DeltaArgs& a, int nseg, hipStream_t stream) {
-    const dim3 grid(nseg, a.H, ceil_div_i(a.dv, 64));
+    const dim3 grid(ceil_div_i(a.dv, 64), a.H, nseg);  // neighbours share a state
     if (a.dk <= 64) delta_scan_kernel<T, 1><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 128) delta_scan_kernel<T, 2><<<grid, 256, 0, stream>>>(a);
     else if (a.dk <= 256) delta_scan_kernel<T, 4><<<grid, 256, 0, stream>>>(a);

@@ -57,7 +57,8 @@ def test_wave_mode():
     assert d["config"]["mode"] == "closed-loop-waves"
 
 
-@pytest.mark.parametrize("family,runs", [("lelisun", 6), ("filinex", 3), ("mekevik", 3)])
+@pytest.mark.parametrize("family,runs", [("lelisun", 6), ("filinex", 3), ("mekevik", 3),
+                                          ("duratar", 6)])
 def test_layers_mode(family, runs):
     d = run_bench(["--mode", "layers", "--family", family, "--sizes", f"tiny-{family}",
                    "--prefill-shapes", "2x16", "--decode-batches", "2", "--decode-context", "16"])
