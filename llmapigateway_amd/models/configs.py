@@ -266,7 +266,7 @@ class HybridConfig:
             m, kind, mlp = dict(e["mixer"]), e["type"], e.get("mlp")
             if kind == "attention":
                 kind, mask = "rotary_attention", m.pop("mask")
-                m.update(window=mask["size"], keep_first=mask["keep_first"])
+                m.update(window=mask["size"], keep_first=mask.get("keep_first", 0))
             elif kind == "channel_delta":
                 m["decay_rank"] = ckpt.shape(f"l{i}.mix.a1")[0]
                 m["gate_rank"] = ckpt.shape(f"l{i}.mix.g1")[0]
