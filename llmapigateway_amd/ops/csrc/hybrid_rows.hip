@@ -361,33 +361,50 @@ __global__ void conv_state_kernel(
     }
 }
 
-// one row per segment: convolve and shift in one launch
-template <typename T, int VEC>
+// one row per segment: convolve and shift in one launch. TAPS 0: any number;
+// otherwise all of a channel's inputs are loaded before the first is stored
+template <typename T, int VEC, int TAPS>
 __global__ void conv_step_kernel(
     T* __restrict__ y, const T* __restrict__ x, int64_t ldx, const float* __restrict__ w_t,
     const float* __restrict__ b, T* __restrict__ state,
-    const int64_t* __restrict__ positions, const int* __restrict__ slots, int C, int taps) {
+    const int64_t* __restrict__ positions, const int* __restrict__ slots, int C, int any_taps) {
     const size_t t = blockIdx.x;
     const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
     if (c >= C) return;
-    const int slot = slots[t];
-    const bool fresh = positions[t] == 0;
-    float acc[VEC], f[VEC], wv[VEC];
+    const int slot = slots[t], taps = TAPS ? TAPS : any_taps;
+    const bool empty = slot < 0 || positions[t] == 0;
+    float acc[VEC];
     load_vec<VEC>(b + c, acc);
     T* st = state + (size_t)(slot < 0 ? 0 : slot) * (taps - 1) * C + c;
-    for (int k = 0; k < taps; ++k) {
+    auto load = [&](int k, float* f) {
         if (k == taps - 1) {
             load_vec<VEC>(x + t * ldx + c, f);
-        } else if (slot < 0 || fresh) {
+        } else if (empty) {
 #pragma unroll
             for (int j = 0; j < VEC; ++j) f[j] = 0.f;
         } else {
             load_vec<VEC>(st + (size_t)k * C, f);
         }
+    };
+    auto take = [&](int k, const float* f) {
+        float wv[VEC];
         load_vec<VEC>(w_t + (size_t)k * C + c, wv);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * f[j];
         if (k > 0 && slot >= 0) store_vec<VEC>(st + (size_t)(k - 1) * C, f);
+    };
+    if (TAPS) {
+        float f[TAPS ? TAPS : 1][VEC];
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) load(k, f[k]);
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) take(k, f[k]);
+    } else {
+        for (int k = 0; k < taps; ++k) {
+            float f[VEC];
+            load(k, f);
+            take(k, f);
+        }
     }
 #pragma unroll
     for (int j = 0; j < VEC; ++j) acc[j] *= sigmoid_f(acc[j]);
@@ -484,7 +501,8 @@ extern "C" hipError_t launch_causal_conv(
     if (rows == nseg)
         return pick(f32, vec8, [&](auto form) {
             FORM(form);
-            conv_step_kernel<T, V><<<dim3(rows, cb), th, 0, stream>>>(
+            auto kernel = taps == 4 ? conv_step_kernel<T, V, 4> : conv_step_kernel<T, V, 0>;
+            kernel<<<dim3(rows, cb), th, 0, stream>>>(
                 (T*)y, (const T*)x, ldx, w_t, b, (T*)state, positions, slots, C, taps);
         });
     return pick(f32, vec8, [&](auto form) {

@@ -95,25 +95,37 @@ __global__ void decay_logs_mfma_kernel(
     f32x4 acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    for (int r0 = 0; r0 < R; r0 += 32) {
-        const int r = r0 + g * 8;
-        float f[8];
-        bf16x8 hi, lo;
-        uint4 x = {0, 0, 0, 0};
-        if (r < R && t < rows) x = *reinterpret_cast<const uint4*>(a + (size_t)t * lda + r);
-        unpack8(x, f);
-        if (EXP) {
+    // 128 of the rank at a time, all loads ahead of the products; past an end
+    // any row, or rank 0 against zeros
+    const bf16* ar = a + (size_t)min(t, rows - 1) * lda;
+    const bf16* wr[4];
 #pragma unroll
-            for (int i = 0; i < 8; ++i) f[i] = tanh_fast(f[i]);
+    for (int j = 0; j < 4; ++j) wr[j] = w2 + (size_t)min(n0 + j * 16 + r16, N - 1) * R;
+    for (int r0 = 0; r0 < R; r0 += 128) {
+        uint4 x[4], w[4][4];
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            const int r = r0 + s * 32 + g * 8, rr = r < R ? r : 0;
+            x[s] = *reinterpret_cast<const uint4*>(ar + rr);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) w[s][j] = *reinterpret_cast<const uint4*>(wr[j] + rr);
+            if (r >= R) x[s] = (uint4){0, 0, 0, 0};
         }
-        split_frag(f, hi, lo);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            uint4 w = {0, 0, 0, 0};
-            const int n = n0 + j * 16 + r16;
-            if (r < R && n < N) w = *reinterpret_cast<const uint4*>(w2 + (size_t)n * R + r);
-            acc[j] = mfma16(as_frag(w), hi, acc[j]);
-            if (EXP) acc[j] = mfma16(as_frag(w), lo, acc[j]);
+        for (int s = 0; s < 4; ++s) {
+            float f[8];
+            bf16x8 hi, lo;
+            unpack8(x[s], f);
+            if (EXP) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) f[i] = tanh_fast(f[i]);
+            }
+            split_frag(f, hi, lo);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                acc[j] = mfma16(as_frag(w[s][j]), hi, acc[j]);
+                if (EXP) acc[j] = mfma16(as_frag(w[s][j]), lo, acc[j]);
+            }
         }
     }
     if (t >= rows) return;

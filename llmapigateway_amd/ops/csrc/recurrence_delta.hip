@@ -246,54 +246,72 @@ __global__ void delta_intra_kernel(DeltaArgs a) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) P[j] = A[j] = zero4();
     if (b0 < n) {
+        bf16x8 qh[NC], ql[NC], kh[NC], kl[NC];
+        float R[NC][8];
+        uint32_t far = 0;  // slices of the key dims whose own block does not factor
+#pragma unroll
         for (int cc = 0; cc < NC; ++cc) {
-            const int d = cc * 32 + g * 8;
-            const bool in = d < dk;
-            const int dd = in ? d : 0;
-            uint4 qraw = *reinterpret_cast<const uint4*>(qp + (size_t)t_own * a.ldq + dd);
-            uint4 kraw = *reinterpret_cast<const uint4*>(kp + (size_t)t_own * a.ldk + dd);
-            if (!in) qraw = kraw = (uint4){0, 0, 0, 0};
-            float E[8], R[8], f[8], spread = 0.f;
+            const int d = cc * 32 + g * 8, dd = d < dk ? d : 0;
+            uint4 q = *reinterpret_cast<const uint4*>(qp + (size_t)t_own * a.ldq + dd);
+            uint4 k = *reinterpret_cast<const uint4*>(kp + (size_t)t_own * a.ldk + dd);
+            if (d >= dk) q = k = (uint4){0, 0, 0, 0};
+            float E[8], f[8], spread = 0.f;
             load8f(Fp + (size_t)t_own * N + dd, E);
             if (b0 > 0) {
-                load8f(Fp + (size_t)(b0 - 1) * N + dd, R);
+                load8f(Fp + (size_t)(b0 - 1) * N + dd, R[cc]);
             } else {
 #pragma unroll
-                for (int i = 0; i < 8; ++i) R[i] = 0.f;
+                for (int i = 0; i < 8; ++i) R[cc][i] = 0.f;
             }
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
-                spread = fmaxf(spread, R[i] - E[i]);
-                E[i] = __expf(E[i] - R[i]);
+                spread = fmaxf(spread, R[cc][i] - E[i]);
+                E[i] = __expf(E[i] - R[cc][i]);
             }
-            const bool factors = !__any(spread > MAX_SPREAD);
-            bf16x8 qh, ql, kh, kl;
-            unpack8(qraw, f);
+            if (__any(spread > MAX_SPREAD)) far |= 1u << cc;
+            unpack8(q, f);
 #pragma unroll
             for (int i = 0; i < 8; ++i) f[i] *= E[i];
-            split_frag(f, qh, ql);
-            unpack8(kraw, f);
+            split_frag(f, qh[cc], ql[cc]);
+            unpack8(k, f);
 #pragma unroll
             for (int i = 0; i < 8; ++i) f[i] *= E[i];
-            split_frag(f, kh, kl);
+            split_frag(f, kh[cc], kl[cc]);
+        }
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                if (j > wave || (j == wave && !factors)) continue;
-                const int s = min(j * 16 + r16, n - 1);
-                float Fs[8], k[8];
+        for (int j = 0; j < 4; ++j) {
+            if (j > wave) continue;
+            const int s = min(j * 16 + r16, n - 1);
+            uint4 k[NC];
+            float Fs[NC][8];
+#pragma unroll
+            for (int cc = 0; cc < NC; ++cc) {
+                const int d = cc * 32 + g * 8, dd = d < dk ? d : 0;
+                k[cc] = *reinterpret_cast<const uint4*>(kp + (size_t)s * a.ldk + dd);
+                load8f(Fp + (size_t)s * N + dd, Fs[cc]);
+            }
+#pragma unroll
+            for (int cc = 0; cc < NC; ++cc) {
+                float f[8];
                 bf16x8 sh, sl;
-                unpack8(*reinterpret_cast<const uint4*>(kp + (size_t)s * a.ldk + dd), k);
-                load8f(Fp + (size_t)s * N + dd, Fs);
+                unpack8(k[cc], f);
 #pragma unroll
-                for (int i = 0; i < 8; ++i) k[i] *= __expf(R[i] - Fs[i]);
-                split_frag(k, sh, sl);
-                P[j] = mfma3(qh, ql, sh, sl, P[j]);
-                A[j] = mfma3(kh, kl, sh, sl, A[j]);
+                for (int i = 0; i < 8; ++i) f[i] *= __expf(R[cc][i] - Fs[cc][i]);
+                split_frag(f, sh, sl);
+                if (j == wave && (far >> cc & 1)) continue;
+                P[j] = mfma3(qh[cc], ql[cc], sh, sl, P[j]);
+                A[j] = mfma3(kh[cc], kl[cc], sh, sl, A[j]);
             }
-            if (factors) continue;
-            // this block, row by row: row tt against k_s g_(s+1) .. g_tt, the
-            // decayed keys carried from row to row; lane r16 holds key r16 (0
-            // before its row is there)
+        }
+        // the other slices of the own block, row by row: row tt against k_s
+        // g_(s+1) .. g_tt, the decayed keys carried from row to row; lane r16
+        // holds key r16 (0 before its row is there)
+        for (int cc = 0; cc < NC; ++cc) {
+            if (!(far >> cc & 1)) continue;
+            const int d = cc * 32 + g * 8, dd = d < dk ? d : 0;
+            uint4 qraw = *reinterpret_cast<const uint4*>(qp + (size_t)t_own * a.ldq + dd);
+            uint4 kraw = *reinterpret_cast<const uint4*>(kp + (size_t)t_own * a.ldk + dd);
+            if (d >= dk) qraw = kraw = (uint4){0, 0, 0, 0};
             float k[8], kt[8];
             unpack8(kraw, k);
             {
