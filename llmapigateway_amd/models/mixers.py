@@ -588,7 +588,7 @@ class ChannelDelta:
         self.a2, self.dt_bias = get("a2"), vec("dt_bias")
         self.rate = vec("A_log").exp().repeat_interleave(self.dk)
         self.norm = vec("norm").repeat(self.H)  # shared by the heads
-        add_decode_twins(self.w, ("in", "g2", "o"))
+        add_decode_twins(self.w, ("in", "o"))
 
     @staticmethod
     def shapes(m: dict, width: int) -> Dict[str, Tuple[int, ...]]:
@@ -623,7 +623,7 @@ class ChannelDelta:
             q, k, v, logw, b, self.H, self.G, self.dk, self.dv, cache["S"], batch.positions,
             batch.segs, plan,
         )
-        gate = ops.linear(g1, w["g2"], w.get("g2_swz"))
+        gate = ops.linear(g1, w["g2"])
         out = torch.empty_like(y)
         ops.head_norm_gate(out, y, gate, self.norm, self.H, self.eps, act="sigmoid")
         return ops.linear(out, w["o"], w.get("o_swz"))
